@@ -138,7 +138,10 @@ def _prefill_attention_gpu(q, k, v, scale, causal_offset, softcap, sliding_windo
     Hkv, S = k.shape[1], k.shape[2]
     G = Hq // Hkv
     qg = q.view(B, Hkv, G, Tq, Dk)
-    scores = torch.matmul(qg, k.unsqueeze(2).transpose(-1, -2)).float() * scale
+    # contiguous K^T: a batched bf16 product with a transposed-view operand
+    # is not safe in this torch/hipBLASLt build
+    kt = k.unsqueeze(2).transpose(-1, -2).contiguous()
+    scores = torch.matmul(qg, kt).float() * scale
     if softcap and softcap > 0:
         scores = torch.tanh(scores / softcap) * softcap
     qpos = torch.arange(Tq, device=q.device)[:, None] + causal_offset

@@ -5,6 +5,24 @@
 #include "hip_common.h"
 
 // ---------------------------------------------------------------------------
+// Fill with zero (fp32), grid-stride.
+// ---------------------------------------------------------------------------
+
+__global__ void zero_f32_kernel(float* __restrict__ p, long n) {
+  const long stride = (long)gridDim.x * blockDim.x;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
+       i += stride)
+    p[i] = 0.0f;
+}
+
+extern "C" void launch_zero_f32(float* p, long n, hipStream_t stream) {
+  if (n <= 0) return;
+  const long want = (n + 255) / 256;
+  const unsigned grid = (unsigned)min(want, (long)4096);
+  zero_f32_kernel<<<dim3(grid), dim3(256), 0, stream>>>(p, n);
+}
+
+// ---------------------------------------------------------------------------
 // RMSNorm: y = x / rms(x) * (w + w_off).  One block per row.
 // Optional fused residual: h = x + r; y = norm(h); h written back.
 // ---------------------------------------------------------------------------

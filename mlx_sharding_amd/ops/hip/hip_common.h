@@ -1,6 +1,5 @@
 // Common helpers for the gfx950 (CDNA4) kernels.
-// Wave size is 64 on CDNA — every reduction below is wave64-shaped
-// (see /opt/skills/guides/cdna_hip_programming.md §1).
+// Wave size is 64 on CDNA — every reduction below is wave64-shaped.
 #pragma once
 
 #include <hip/hip_runtime.h>
@@ -76,6 +75,10 @@ __device__ __forceinline__ float block_max(float v, float* scratch) {
   __syncthreads();
   return r;
 }
+
+// Clears a float buffer with a kernel (elementwise.hip): a memset node inside
+// a captured hipGraph is not reliable on replay, a kernel node is.
+extern "C" void launch_zero_f32(float* p, long n, hipStream_t stream);
 
 #define HIP_CHECK_LAST()                                                     \
   do {                                                                       \

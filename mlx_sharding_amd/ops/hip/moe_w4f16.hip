@@ -537,7 +537,7 @@ extern "C" void launch_w4f16_gemv(const void* x, const void* wq,
                                   float* yf, int nk, int M, int O, int H,
                                   int gs, int bits, hipStream_t stream) {
   if (nk > 1)
-    (void)hipMemsetAsync(yf, 0, (size_t)M * O * sizeof(float), stream);
+    launch_zero_f32(yf, (long)M * O, stream);
 #define GV_GS(BB)                                                           \
   do {                                                                      \
     if (gs == 32)                                                           \

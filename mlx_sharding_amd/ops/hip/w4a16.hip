@@ -489,7 +489,7 @@ extern "C" void launch_bf16_gemv_mfma(const void* x, const void* w, void* y,
   const int mz = (M + 15) / 16;
   dim3 grid((unsigned)gx, (unsigned)nk);
   if (nk > 1) {
-    (void)hipMemsetAsync(yf, 0, (size_t)M * O * sizeof(float), stream);
+    launch_zero_f32(yf, (long)M * O, stream);
   }
   float* yfp = nk > 1 ? yf : nullptr;
 #define DG_CASE(Z)                                                           \
@@ -649,7 +649,7 @@ extern "C" void launch_bf16_gemm_m64(const void* x, const void* w, void* y,
   const int gx = (O + DM_WAVES * 16 * DM_R - 1) / (DM_WAVES * 16 * DM_R);
   const size_t smem = (size_t)64 * DM_LDS * sizeof(short);
   if (nk > 1)
-    (void)hipMemsetAsync(yf, 0, (size_t)M * O * sizeof(float), stream);
+    launch_zero_f32(yf, (long)M * O, stream);
   float* yfp = nk > 1 ? yf : nullptr;
   bf16_gemm_m64_kernel<DM_R><<<dim3((unsigned)gx, (unsigned)nk),
                                dim3(DM_BLOCK), smem, stream>>>(
@@ -698,7 +698,7 @@ extern "C" void launch_w4a16_mfma(const void* x, const void* wq,
   const size_t smem = QM_MTOK * QM_LDS * sizeof(short);
   dim3 grid((unsigned)gx, (unsigned)nk, (unsigned)mz);
   if (nk > 1)
-    (void)hipMemsetAsync(yf, 0, (size_t)M * O * sizeof(float), stream);
+    launch_zero_f32(yf, (long)M * O, stream);
   float* yfp = nk > 1 ? yf : nullptr;
   if (bits == 4)
     w4a16_mfma_kernel<4><<<grid, dim3(QM_BLOCK), smem, stream>>>(

@@ -17,6 +17,10 @@ from setuptools import find_packages, setup
 ROOT = Path(__file__).parent
 HIP_DIR = ROOT / "mlx_sharding_amd" / "ops" / "hip"
 
+# scalar fp32 math only: the packed v_pk_*_f32 forms the optimizer makes out
+# of ordinary float code are kept out of every kernel
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
 ext_modules = []
 cmdclass = {}
 hip_sources = sorted(str(p) for p in HIP_DIR.glob("*.hip") if not p.name.endswith("_hip.hip")) + \
@@ -32,7 +36,8 @@ if hip_sources and os.environ.get("MLXS_AMD_SKIP_EXT", "0") != "1":
                 sources=hip_sources,
                 extra_compile_args={
                     "cxx": ["-O3", "-std=c++17"],
-                    "nvcc": ["-O3", "-std=c++17", "--offload-arch=gfx950"],
+                    "nvcc": ["-O3", "-std=c++17", "--offload-arch=gfx950",
+                             *NO_PACKED_FP32],
                 },
             )
         ]
