@@ -1,0 +1,681 @@
+// Gated delta rule over a ragged batch, state in slots.
+//
+//   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//
+// with q, k, v behind a short causal convolution and silu, q and k unit
+// vectors, one decay g per head.  The state [D, V] and everything that enters
+// the recurrence are fp32 in either element type.
+//
+//  * short portions (decoding): one kernel does convolution, norms, gates,
+//    recurrence, output norm and gate; the state lives in registers.
+//  * long portions: chunks of 64 tokens.  With G the running log decay of the
+//    chunk, S0 the state before it, and
+//        L[i,j] = beta_i exp(G_i - G_j) k_i.k_j   (j < i)
+//        A[i,j] =        exp(G_i - G_j) q_i.k_j   (j <= i)
+//    the writes are U = (I + L)^-1 diag(beta) (V - diag(exp G) K S0), the
+//    outputs O = diag(exp G) Q S0 + A U, and the next state
+//    exp(G_last) S0 + K^T diag(exp(G_last - G)) U.  One kernel makes
+//    (I + L)^-1 diag(beta) and A of all chunks at once, a second walks the
+//    chunks of a (request, head, 16 value columns).  All products run on the
+//    fp32 matrix cores.
+//
+// A request at position 0 starts from a zero state whatever its slot holds.
+#include "ragged_common.h"
+
+#define DR_CHUNK 64
+#define DR_MAXTAPS 8
+#define DR_SHORT 16  // most tokens of a short portion
+
+struct DeltaDims {
+  int KH, H, D, V, taps;
+  int qc, kc, vc, gc, ac, bc;  // column offsets in a projection row
+  long ystride;
+};
+
+__device__ __forceinline__ float log_decay(float a, float A_log, float dt) {
+  return -expf(A_log) * softplus_f(a + dt);
+}
+
+// ---------------------------------------------------------------------------
+// Short portions.  Block = (request, q/k head); its r = H / KH value heads
+// follow one another.  Threads: VT along V (power of two), DG groups along D,
+// RPT state rows per thread.
+// ---------------------------------------------------------------------------
+
+template <typename T, int RPT, int NT>
+__global__ __launch_bounds__(NT) void delta_short_kernel(
+    const T* __restrict__ y, const T* __restrict__ conv_w,
+    const T* __restrict__ A_log, const T* __restrict__ dt_bias,
+    const T* __restrict__ norm_w, float* __restrict__ state,
+    T* __restrict__ conv_state, T* __restrict__ out,
+    const int* __restrict__ cu, const int* __restrict__ pos0,
+    const int* __restrict__ slots, DeltaDims dm, int VT, float q_scale,
+    float eps) {
+  const int e = blockIdx.x;
+  const int kh = blockIdx.y;
+  const int t0 = cu[e];
+  const int n = min(cu[e + 1] - t0, DR_SHORT);
+  const bool fresh = pos0[e] == 0;
+  const long slot = slots[e];
+  const int D = dm.D, V = dm.V;
+  const int DG = NT / VT;
+  const int tid = threadIdx.x;
+  const int lane = tid & (WAVE - 1);
+  const int wid = tid / WAVE;
+  const int C = 2 * dm.KH * D + dm.H * V;
+  const int hist = dm.taps - 1;
+
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  float* qk = reinterpret_cast<float*>(smem);  // [n][2][D]
+  float* kq = qk + (long)n * 2 * D;            // [n]
+  float* vb = kq + DR_SHORT;                   // [n][V]
+  float* red = vb + (long)n * V;               // [2][DG][VT]
+  float* scratch = red + 2 * NT;               // [NT / WAVE]
+
+  // convolution + silu of channel c (column col of y) for all n tokens
+  auto convolve = [&](int c, int col, float* dst, int dstep) {
+    float w[DR_MAXTAPS], x[DR_MAXTAPS];
+    T* cs = conv_state + (slot * C + c) * hist;
+    // taps sit at the end of w/x, so the index of the newest is fixed
+    const int pad = DR_MAXTAPS - dm.taps;
+#pragma unroll
+    for (int j = 0; j < DR_MAXTAPS; ++j) {
+      w[j] = j >= pad ? (float)conv_w[(long)c * dm.taps + j - pad] : 0.0f;
+      x[j] = (j >= pad && j < DR_MAXTAPS - 1 && !fresh) ? (float)cs[j - pad]
+                                                        : 0.0f;
+    }
+    for (int t = 0; t < n; ++t) {
+      x[DR_MAXTAPS - 1] = (float)y[(long)(t0 + t) * dm.ystride + col];
+      float a = 0.0f;
+#pragma unroll
+      for (int j = 0; j < DR_MAXTAPS; ++j) a += w[j] * x[j];
+      dst[(long)t * dstep] = silu_f(a);
+#pragma unroll
+      for (int j = 0; j < DR_MAXTAPS - 1; ++j) x[j] = x[j + 1];
+    }
+    // x[j] now holds the input one step older than slot j + 1: the last
+    // taps - 1 inputs are x[pad .. MAXTAPS - 2]
+#pragma unroll
+    for (int j = 0; j < DR_MAXTAPS - 1; ++j)
+      if (j >= pad) cs[j - pad] = (T)x[j];
+  };
+
+  for (int i = tid; i < 2 * D; i += NT) {
+    const int which = i / D, d = i - which * D;
+    const int c = which * dm.KH * D + kh * D + d;
+    convolve(c, (which ? dm.kc : dm.qc) + kh * D + d, qk + i, 2 * D);
+  }
+  __syncthreads();
+  for (int r = wid; r < 2 * n; r += NT / WAVE) {
+    float* row = qk + (long)r * D;
+    float ss = 0.0f;
+    for (int d = lane; d < D; d += WAVE) ss += row[d] * row[d];
+    ss = wave_sum(ss);
+    const float s = (r & 1 ? 1.0f : q_scale) / sqrtf(ss + 1e-6f);
+    for (int d = lane; d < D; d += WAVE) row[d] *= s;
+  }
+  __syncthreads();
+  for (int t = wid; t < n; t += NT / WAVE) {
+    float a = 0.0f;
+    for (int d = lane; d < D; d += WAVE)
+      a += qk[(long)t * 2 * D + d] * qk[(long)t * 2 * D + D + d];
+    a = wave_sum(a);
+    if (lane == 0) kq[t] = a;
+  }
+
+  const int v = tid & (VT - 1);
+  const int dg = tid / VT;
+  const int d0 = dg * RPT;
+  const int rep = dm.H / dm.KH;
+  for (int hh = 0; hh < rep; ++hh) {
+    const int h = kh * rep + hh;
+    __syncthreads();
+    for (int i = tid; i < V; i += NT)
+      convolve(2 * dm.KH * D + h * V + i, dm.vc + h * V + i, vb + i, V);
+    float S[RPT];
+    float* sp = state + ((slot * dm.H + h) * (long)D + d0) * V + v;
+#pragma unroll
+    for (int i = 0; i < RPT; ++i)
+      S[i] = (!fresh && v < V && d0 + i < D) ? sp[(long)i * V] : 0.0f;
+    __syncthreads();
+    const float Al = (float)A_log[h], dt = (float)dt_bias[h];
+    for (int t = 0; t < n; ++t) {
+      const T* yt = y + (long)(t0 + t) * dm.ystride;
+      const float g = expf(log_decay((float)yt[dm.ac + h], Al, dt));
+      const float beta = sigmoid_f((float)yt[dm.bc + h]);
+      const float* qr = qk + (long)t * 2 * D;
+      const float* kr = qr + D;
+      float sk = 0.0f, sq = 0.0f;
+#pragma unroll
+      for (int i = 0; i < RPT; ++i)
+        if (d0 + i < D) {
+          sk += S[i] * kr[d0 + i];
+          sq += S[i] * qr[d0 + i];
+        }
+      red[dg * VT + v] = sk;
+      red[NT + dg * VT + v] = sq;
+      __syncthreads();
+      sk = 0.0f;
+      sq = 0.0f;
+      for (int i = 0; i < DG; ++i) {
+        sk += red[i * VT + v];
+        sq += red[NT + i * VT + v];
+      }
+      const float vv = v < V ? vb[(long)t * V + v] : 0.0f;
+      const float u = beta * (vv - g * sk);
+      const float o = g * sq + kq[t] * u;
+#pragma unroll
+      for (int i = 0; i < RPT; ++i)
+        if (d0 + i < D) S[i] = g * S[i] + kr[d0 + i] * u;
+      const bool mine = dg == 0 && v < V;
+      const float ss = block_sum<NT>(mine ? o * o : 0.0f, scratch);
+      if (mine) {
+        const float gate = silu_f((float)yt[dm.gc + h * V + v]);
+        out[(long)(t0 + t) * ((long)dm.H * V) + h * V + v] =
+            (T)(o / sqrtf(ss / (float)V + eps) * (float)norm_w[v] * gate);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < RPT; ++i)
+      if (v < V && d0 + i < D) sp[(long)i * V] = S[i];
+  }
+}
+
+static int pow2_at_least(int v) {
+  int p = 16;
+  while (p < v) p *= 2;
+  return p;
+}
+
+// state rows per thread, or 0 if the head is too large for the kernel
+extern "C" int delta_short_rows(int D, int V, int nt) {
+  const int vt = pow2_at_least(V);
+  if (vt > nt) return 0;
+  const int need = (D + nt / vt - 1) / (nt / vt);
+  for (int r : {4, 16, 32, 64, 128})
+    if (need <= r) return r;
+  return 0;
+}
+
+#define DR_NT 512
+
+template <typename T>
+static void delta_short_t(const void* y, const void* conv_w, const void* A_log,
+                          const void* dt_bias, const void* norm_w,
+                          float* state, void* conv_state, void* out,
+                          const int* cu, const int* pos0, const int* slots,
+                          const DeltaDims& dm, int n_req, int max_len,
+                          float eps, hipStream_t stream) {
+  const int vt = pow2_at_least(dm.V);
+  const int rpt = delta_short_rows(dm.D, dm.V, DR_NT);
+  const size_t smem = ((size_t)max_len * (2 * dm.D + dm.V) + DR_SHORT +
+                       2 * DR_NT + DR_NT / WAVE) * sizeof(float);
+  const float q_scale = 1.0f / sqrtf((float)dm.D);
+  dim3 grid((unsigned)n_req, (unsigned)dm.KH), block(DR_NT);
+#define DS_GO(R)                                                             \
+  do {                                                                       \
+    if (smem > 65536)                                                        \
+      (void)hipFuncSetAttribute(                                             \
+          reinterpret_cast<const void*>(&delta_short_kernel<T, R, DR_NT>),   \
+          hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);            \
+    delta_short_kernel<T, R, DR_NT><<<grid, block, smem, stream>>>(          \
+        (const T*)y, (const T*)conv_w, (const T*)A_log, (const T*)dt_bias,   \
+        (const T*)norm_w, state, (T*)conv_state, (T*)out, cu, pos0, slots,   \
+        dm, vt, q_scale, eps);                                               \
+  } while (0)
+  switch (rpt) {
+    case 4: DS_GO(4); break;
+    case 16: DS_GO(16); break;
+    case 32: DS_GO(32); break;
+    case 64: DS_GO(64); break;
+    case 128: DS_GO(128); break;
+    default: break;
+  }
+#undef DS_GO
+}
+
+extern "C" void launch_delta_short(const void* y, const void* conv_w,
+                                   const void* A_log, const void* dt_bias,
+                                   const void* norm_w, float* state,
+                                   void* conv_state, void* out, const int* cu,
+                                   const int* pos0, const int* slots,
+                                   const DeltaDims* dm, int n_req, int max_len,
+                                   float eps, bool f32, hipStream_t stream) {
+  if (f32)
+    delta_short_t<float>(y, conv_w, A_log, dt_bias, norm_w, state, conv_state,
+                         out, cu, pos0, slots, *dm, n_req, max_len, eps,
+                         stream);
+  else
+    delta_short_t<__bf16>(y, conv_w, A_log, dt_bias, norm_w, state, conv_state,
+                          out, cu, pos0, slots, *dm, n_req, max_len, eps,
+                          stream);
+}
+
+// ---------------------------------------------------------------------------
+// Long portions, step 1: convolution, silu, unit norms, gates.
+// Block per token.  q, k -> fp32 [n, KH, Dp] (zero padded), v -> T [n, H, Vp],
+// log decay and beta -> fp32 [n, H].
+// ---------------------------------------------------------------------------
+
+#define DC_BLOCK 256
+#define DC_MAXD 8  // D <= 64 * DC_MAXD
+
+template <typename T>
+__global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
+    const T* __restrict__ y, const T* __restrict__ conv_w,
+    const T* __restrict__ A_log, const T* __restrict__ dt_bias,
+    const T* __restrict__ conv_state, float* __restrict__ qo,
+    float* __restrict__ ko, T* __restrict__ vo, float* __restrict__ lg,
+    float* __restrict__ bt, const int* __restrict__ cu,
+    const int* __restrict__ pos0, const int* __restrict__ slots,
+    const int* __restrict__ tok_entry, int tok_base, DeltaDims dm, int Dp,
+    int Vp, float q_scale) {
+  const long i = blockIdx.x;              // row among the long tokens
+  const long t = tok_base + i;
+  const int e = tok_entry[t];
+  const int rel = (int)(t - cu[e]);       // place within the portion
+  const bool fresh = pos0[e] == 0;
+  const int hist = dm.taps - 1;
+  const int D = dm.D, V = dm.V;
+  const int C = 2 * dm.KH * D + dm.H * V;
+  const T* cs = conv_state + (long)slots[e] * C * hist;
+  const T* yt = y + t * dm.ystride;
+
+  auto conv = [&](int c, int col) {
+    float a = 0.0f;
+    for (int j = 0; j < dm.taps; ++j) {
+      const int s = rel - hist + j;
+      float x;
+      if (s >= 0)
+        x = (float)yt[col + (long)(j - hist) * dm.ystride];
+      else
+        x = fresh ? 0.0f : (float)cs[(long)c * hist + hist + s];
+      a += (float)conv_w[(long)c * dm.taps + j] * x;
+    }
+    return silu_f(a);
+  };
+
+  const int lane = threadIdx.x & (WAVE - 1);
+  const int wid = threadIdx.x / WAVE;
+  for (int hq = wid; hq < 2 * dm.KH; hq += DC_BLOCK / WAVE) {
+    const int which = hq / dm.KH, kh = hq - which * dm.KH;
+    float x[DC_MAXD];
+    float ss = 0.0f;
+#pragma unroll
+    for (int u = 0; u < DC_MAXD; ++u) {
+      const int d = lane + u * WAVE;
+      x[u] = 0.0f;
+      if (d < D) {
+        x[u] = conv(which * dm.KH * D + kh * D + d,
+                    (which ? dm.kc : dm.qc) + kh * D + d);
+        ss += x[u] * x[u];
+      }
+    }
+    ss = wave_sum(ss);
+    const float s = (which ? 1.0f : q_scale) / sqrtf(ss + 1e-6f);
+    float* dst = (which ? ko : qo) + (i * dm.KH + kh) * Dp;
+#pragma unroll
+    for (int u = 0; u < DC_MAXD; ++u) {
+      const int d = lane + u * WAVE;
+      if (d < Dp) dst[d] = x[u] * s;
+    }
+  }
+  for (int j = threadIdx.x; j < dm.H * Vp; j += DC_BLOCK) {
+    const int h = j / Vp, v = j - h * Vp;
+    vo[i * ((long)dm.H * Vp) + j] =
+        v < V ? (T)conv(2 * dm.KH * D + h * V + v, dm.vc + h * V + v) : (T)0.0f;
+  }
+  for (int h = threadIdx.x; h < dm.H; h += DC_BLOCK) {
+    lg[i * dm.H + h] =
+        log_decay((float)yt[dm.ac + h], (float)A_log[h], (float)dt_bias[h]);
+    bt[i * dm.H + h] = sigmoid_f((float)yt[dm.bc + h]);
+  }
+}
+
+// The last taps - 1 inputs of every channel; runs after the convolution.
+template <typename T>
+__global__ __launch_bounds__(DC_BLOCK) void delta_conv_state_kernel(
+    const T* __restrict__ y, T* __restrict__ conv_state,
+    const int* __restrict__ cu, const int* __restrict__ pos0,
+    const int* __restrict__ slots, int n_short, DeltaDims dm) {
+  const int e = n_short + blockIdx.x;
+  const int c = blockIdx.y * DC_BLOCK + threadIdx.x;
+  const int D = dm.D, V = dm.V;
+  const int nq = dm.KH * D;
+  const int C = 2 * nq + dm.H * V;
+  if (c >= C) return;
+  const int col = c < nq ? dm.qc + c
+                         : (c < 2 * nq ? dm.kc + c - nq : dm.vc + c - 2 * nq);
+  const int hist = dm.taps - 1;
+  const int t0 = cu[e], n = cu[e + 1] - t0;
+  const bool fresh = pos0[e] == 0;
+  T* cs = conv_state + ((long)slots[e] * C + c) * hist;
+  for (int j = 0; j < hist; ++j) {  // ascending: reads stay ahead of writes
+    const int s = n - hist + j;
+    if (s >= 0)
+      cs[j] = y[(long)(t0 + s) * dm.ystride + col];
+    else
+      cs[j] = fresh ? (T)0.0f : cs[hist + s];
+  }
+}
+
+// ---------------------------------------------------------------------------
+// Step 2, all chunks at once.  Block = (chunk, head), 4 waves; wave w makes
+// rows 16w..16w+15 of the two Gram matrices, wave 0 then inverts I + L, one
+// column per lane.
+//   tm [chunks, H, 64, 64]  (I + L)^-1 diag(beta)
+//   am [chunks, H, 64, 64]  A (lower tiles only)
+//   ge [chunks, H, 2, 64]   exp(G), exp(G_last - G)
+// ---------------------------------------------------------------------------
+
+#define DR_LS 68
+
+__global__ __launch_bounds__(256) void delta_chunk_kernel(
+    const float* __restrict__ qn, const float* __restrict__ kn,
+    const float* __restrict__ lg, const float* __restrict__ bt,
+    float* __restrict__ tm, float* __restrict__ am, float* __restrict__ ge,
+    const int* __restrict__ chunks, int tok_base, int KH, int H, int Dp) {
+  const int c = blockIdx.x, h = blockIdx.y;
+  const int kh = h / (H / KH);
+  const int i0 = chunks[2 * c] - tok_base;
+  const int len = chunks[2 * c + 1];
+  const int tid = threadIdx.x;
+  const int lane = tid & (WAVE - 1);
+  const int wid = tid / WAVE;
+  const int lr = lane & 15, g4 = lane >> 4;
+
+  __shared__ double gs[DR_CHUNK];
+  __shared__ float bs[DR_CHUNK];
+  __shared__ __attribute__((aligned(16))) float ls[DR_CHUNK * DR_LS];
+
+  const long ch = (long)c * H + h;
+  if (wid == 0) {
+    // running sum of log decays; differences of it must stay exact to fp32,
+    // also behind strong decays, hence double
+    const bool in = lane < len;
+    double g = in ? (double)lg[(long)(i0 + lane) * H + h] : 0.0;
+#pragma unroll
+    for (int off = 1; off < WAVE; off <<= 1) {
+      const double o = __shfl_up(g, off, WAVE);
+      if (lane >= off) g += o;
+    }
+    const double last = __shfl(g, WAVE - 1, WAVE);
+    gs[lane] = g;
+    bs[lane] = in ? bt[(long)(i0 + lane) * H + h] : 0.0f;
+    ge[ch * 128 + lane] = expf((float)g);
+    ge[ch * 128 + 64 + lane] = expf((float)(last - g));
+  }
+
+  f32x4 kk[4], qk[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    kk[j] = f32x4{0, 0, 0, 0};
+    qk[j] = f32x4{0, 0, 0, 0};
+  }
+  const int ra = wid * 16 + lr;
+  const f32x4 zero = {0, 0, 0, 0};
+  const float* kbase = kn + ((long)i0 * KH + kh) * Dp + g4 * 4;
+  const float* qbase = qn + ((long)i0 * KH + kh) * Dp + g4 * 4;
+  const long rstride = (long)KH * Dp;
+  for (int d = 0; d < Dp; d += 16) {
+    const f32x4 ka = ra < len ? load4(kbase + ra * rstride + d) : zero;
+    const f32x4 qa = ra < len ? load4(qbase + ra * rstride + d) : zero;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j > wid) continue;
+      const int rb = j * 16 + lr;
+      const f32x4 kb = rb < len ? load4(kbase + rb * rstride + d) : zero;
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        kk[j] = mma4(ka[s], kb[s], kk[j]);
+        qk[j] = mma4(qa[s], kb[s], qk[j]);
+      }
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    if (j > wid) continue;
+    const int col = j * 16 + lr;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = wid * 16 + g4 * 4 + r;
+      const float dec = col <= row ? expf((float)(gs[row] - gs[col])) : 0.0f;
+      ls[row * DR_LS + col] = col < row ? bs[row] * dec * kk[j][r] : 0.0f;
+      am[ch * 4096 + row * 64 + col] = dec * qk[j][r];
+    }
+  }
+  __syncthreads();
+  if (wid != 0) return;
+  float x[DR_CHUNK];
+  const float bc = bs[lane];
+#pragma unroll
+  for (int i = 0; i < DR_CHUNK; ++i) {
+    float a0 = i == lane ? 1.0f : 0.0f, a1 = 0.0f, a2 = 0.0f, a3 = 0.0f;
+    const float* row = ls + i * DR_LS;
+#pragma unroll
+    for (int j = 0; j + 4 <= i; j += 4) {
+      const f32x4 l4 = load4(row + j);
+      a0 -= l4[0] * x[j];
+      a1 -= l4[1] * x[j + 1];
+      a2 -= l4[2] * x[j + 2];
+      a3 -= l4[3] * x[j + 3];
+    }
+#pragma unroll
+    for (int j = i & ~3; j < i; ++j) a0 -= row[j] * x[j];
+    x[i] = (a0 + a1) + (a2 + a3);
+    tm[ch * 4096 + i * 64 + lane] = x[i] * bc;
+  }
+}
+
+// ---------------------------------------------------------------------------
+// Step 3: the walk.  Block = (value column tile, head, request), 4 waves;
+// wave w owns token rows 16w..16w+15 of a chunk and state row tiles w, w+4,...
+// A operands come straight from global memory as vectors (the contraction
+// order inside 16 is permuted the same way on both sides).
+// ---------------------------------------------------------------------------
+
+template <typename T>
+__global__ __launch_bounds__(256) void delta_walk_kernel(
+    const float* __restrict__ qn, const float* __restrict__ kn,
+    const T* __restrict__ vn, const float* __restrict__ tm,
+    const float* __restrict__ am, const float* __restrict__ ge,
+    float* __restrict__ state, float* __restrict__ o,
+    const int* __restrict__ chunks, const int* __restrict__ chunk_cu,
+    const int* __restrict__ pos0, const int* __restrict__ slots, int n_short,
+    int tok_base, int KH, int H, int D, int Dp, int V, int Vp) {
+  const int v0 = blockIdx.x * 16;
+  const int h = blockIdx.y;
+  const int e = blockIdx.z;
+  const int kh = h / (H / KH);
+  const int tid = threadIdx.x;
+  const int lane = tid & (WAVE - 1);
+  const int wid = tid / WAVE;
+  const int lr = lane & 15, g4 = lane >> 4;
+
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  float* ss = reinterpret_cast<float*>(smem);  // [Dp][17] state columns
+  float* xs = ss + Dp * 17;                    // [64][17] V - exp(G) K S
+  float* us = xs + 64 * 17;                    // [64][17] U
+  float* uw = us + 64 * 17;                    // [64][17] exp(G_last - G) U
+
+  const bool fresh = pos0[n_short + e] == 0;
+  float* sg = state + ((long)slots[n_short + e] * H + h) * (long)D * V;
+  for (int i = tid; i < Dp * 16; i += 256) {
+    const int d = i >> 4, v = v0 + (i & 15);
+    ss[d * 17 + (i & 15)] =
+        (!fresh && d < D && v < V) ? sg[(long)d * V + v] : 0.0f;
+  }
+  __syncthreads();
+
+  const long rstride = (long)KH * Dp;
+  const f32x4 zero = {0, 0, 0, 0};
+  const int row = wid * 16 + lr;            // A-operand row
+  for (int c = chunk_cu[e]; c < chunk_cu[e + 1]; ++c) {
+    const int i0 = chunks[2 * c] - tok_base;
+    const int len = chunks[2 * c + 1];
+    const long ch = (long)c * H + h;
+    const float* kp = kn + ((long)i0 * KH + kh) * Dp;
+    const float* qp = qn + ((long)i0 * KH + kh) * Dp;
+    const float* gc = ge + ch * 128;
+
+    f32x4 ks = zero, qs = zero;
+    {
+      const float* ka = kp + row * rstride + g4 * 4;
+      const float* qa = qp + row * rstride + g4 * 4;
+      const bool in = row < len;
+#pragma unroll 4
+      for (int d = 0; d < Dp; d += 16) {
+        const f32x4 a = in ? load4(ka + d) : zero;
+        const f32x4 b = in ? load4(qa + d) : zero;
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          const float sv = ss[(d + g4 * 4 + s) * 17 + lr];
+          ks = mma4(a[s], sv, ks);
+          qs = mma4(b[s], sv, qs);
+        }
+      }
+    }
+    float gr[4], gl[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = wid * 16 + g4 * 4 + r;
+      gr[r] = gc[i];
+      gl[r] = gc[64 + i];
+      const float v =
+          i < len ? (float)vn[((long)(i0 + i) * H + h) * Vp + v0 + lr] : 0.0f;
+      xs[i * 17 + lr] = v - gr[r] * ks[r];
+    }
+    __syncthreads();
+    f32x4 u = zero;
+    const float* ta = tm + ch * 4096 + row * 64 + g4 * 4;
+    for (int j = 0; j <= wid; ++j) {
+      const f32x4 a = load4(ta + j * 16);
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+        u = mma4(a[s], xs[(j * 16 + g4 * 4 + s) * 17 + lr], u);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = wid * 16 + g4 * 4 + r;
+      us[i * 17 + lr] = u[r];
+      uw[i * 17 + lr] = u[r] * gl[r];
+    }
+    __syncthreads();
+    f32x4 oc;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) oc[r] = gr[r] * qs[r];
+    const float* aa = am + ch * 4096 + row * 64 + g4 * 4;
+    for (int j = 0; j <= wid; ++j) {
+      const f32x4 a = load4(aa + j * 16);
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+        oc = mma4(a[s], us[(j * 16 + g4 * 4 + s) * 17 + lr], oc);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = wid * 16 + g4 * 4 + r;
+      if (i < len) o[((long)(i0 + i) * H + h) * Vp + v0 + lr] = oc[r];
+    }
+    const float g_all = gc[63];
+    for (int d0 = wid * 16; d0 < Dp; d0 += 64) {
+      f32x4 sn;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        sn[r] = g_all * ss[(d0 + g4 * 4 + r) * 17 + lr];
+      const float* ka = kp + d0 + lr;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          const int i = j * 16 + g4 * 4 + s;
+          const float a = i < len ? ka[i * rstride] : 0.0f;
+          sn = mma4(a, uw[i * 17 + lr], sn);
+        }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ss[(d0 + g4 * 4 + r) * 17 + lr] = sn[r];
+    }
+    __syncthreads();
+  }
+  for (int i = tid; i < Dp * 16; i += 256) {
+    const int d = i >> 4, v = v0 + (i & 15);
+    if (d < D && v < V) sg[(long)d * V + v] = ss[d * 17 + (i & 15)];
+  }
+}
+
+// ---------------------------------------------------------------------------
+// Step 4: output norm over V, weight, silu gate.  One wave per (token, head).
+// ---------------------------------------------------------------------------
+
+template <typename T>
+__global__ __launch_bounds__(256) void delta_gate_kernel(
+    const float* __restrict__ o, const T* __restrict__ y,
+    const T* __restrict__ norm_w, T* __restrict__ out, long n, int tok_base,
+    DeltaDims dm, int Vp, float eps) {
+  const long wi = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
+  if (wi >= n * dm.H) return;
+  const int lane = threadIdx.x & (WAVE - 1);
+  const long i = wi / dm.H;
+  const int h = (int)(wi - i * dm.H);
+  const float* orow = o + wi * Vp;
+  float ss = 0.0f;
+  for (int v = lane; v < dm.V; v += WAVE) ss += orow[v] * orow[v];
+  ss = wave_sum(ss);
+  const float inv = 1.0f / sqrtf(ss / (float)dm.V + eps);
+  const T* gr = y + (tok_base + i) * dm.ystride + dm.gc + (long)h * dm.V;
+  T* dst = out + (tok_base + i) * ((long)dm.H * dm.V) + (long)h * dm.V;
+  for (int v = lane; v < dm.V; v += WAVE)
+    dst[v] = (T)(orow[v] * inv * (float)norm_w[v] * silu_f((float)gr[v]));
+}
+
+struct DeltaLongArgs {
+  const void *y, *conv_w, *A_log, *dt_bias, *norm_w;
+  float* state;
+  void *conv_state, *out;
+  float *qn, *kn, *lg, *bt, *tm, *am, *ge, *o;
+  void* vn;
+  const int *cu, *pos0, *slots, *tok_entry, *chunks, *chunk_cu;
+  int n_short, n_long, tok_base, n_chunks, Dp, Vp;
+  long n_tok;
+  float eps;
+};
+
+template <typename T>
+static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
+                         hipStream_t stream) {
+  const int C = 2 * dm.KH * dm.D + dm.H * dm.V;
+  const float q_scale = 1.0f / sqrtf((float)dm.D);
+  dim3 block(DC_BLOCK);
+  dim3 g1((unsigned)a.n_tok);
+  delta_conv_kernel<T><<<g1, block, 0, stream>>>(
+      (const T*)a.y, (const T*)a.conv_w, (const T*)a.A_log,
+      (const T*)a.dt_bias, (const T*)a.conv_state, a.qn, a.kn, (T*)a.vn, a.lg,
+      a.bt, a.cu, a.pos0, a.slots, a.tok_entry, a.tok_base, dm, a.Dp, a.Vp,
+      q_scale);
+  dim3 g2((unsigned)a.n_long, (unsigned)((C + DC_BLOCK - 1) / DC_BLOCK));
+  if (dm.taps > 1)
+    delta_conv_state_kernel<T><<<g2, block, 0, stream>>>(
+        (const T*)a.y, (T*)a.conv_state, a.cu, a.pos0, a.slots, a.n_short, dm);
+  dim3 g3((unsigned)a.n_chunks, (unsigned)dm.H);
+  delta_chunk_kernel<<<g3, block, 0, stream>>>(
+      a.qn, a.kn, a.lg, a.bt, a.tm, a.am, a.ge, a.chunks, a.tok_base, dm.KH,
+      dm.H, a.Dp);
+  const size_t smem = ((size_t)a.Dp + 3 * 64) * 17 * sizeof(float);
+  dim3 g4((unsigned)(a.Vp / 16), (unsigned)dm.H, (unsigned)a.n_long);
+  delta_walk_kernel<T><<<g4, block, smem, stream>>>(
+      a.qn, a.kn, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,
+      a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, dm.KH, dm.H, dm.D,
+      a.Dp, dm.V, a.Vp);
+  dim3 g5((unsigned)((a.n_tok * dm.H + 3) / 4));
+  delta_gate_kernel<T><<<g5, block, 0, stream>>>(
+      a.o, (const T*)a.y, (const T*)a.norm_w, (T*)a.out, a.n_tok, a.tok_base,
+      dm, a.Vp, a.eps);
+}
+
+extern "C" void launch_delta_long(const DeltaLongArgs* a, const DeltaDims* dm,
+                                  bool f32, hipStream_t stream) {
+  if (f32)
+    delta_long_t<float>(*a, *dm, stream);
+  else
+    delta_long_t<__bf16>(*a, *dm, stream);
+}

@@ -1,0 +1,267 @@
+// Norms around a 32-bit residual stream, and the short-row work of paged
+// latent attention (latent norm, rotation, append, gather).
+#include "ragged_common.h"
+
+#define RN_BLOCK 256
+
+// ---------------------------------------------------------------------------
+// One sublayer boundary in one kernel, one block per row:
+//   x += rms(y) * (w_post + off)      (y == null: x unchanged)
+//   h  = rms(x) * (w_next + off)      (w_next == null: no h)
+// x is the fp32 residual; y and h are T.  NR > 0 keeps the row in registers
+// (NR groups of VEC elements per thread); NR == 0 re-reads it.
+// ---------------------------------------------------------------------------
+
+template <typename T, int VEC>
+__device__ __forceinline__ void rn_load(const T* p, float (&o)[VEC]) {
+  if constexpr (VEC == 4) {
+    f32x4 v = load4(p);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = v[j];
+  } else {
+    o[0] = (float)p[0];
+  }
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void rn_store(T* p, const float (&o)[VEC]) {
+  if constexpr (VEC == 4) {
+    store4(p, f32x4{o[0], o[1], o[2], o[3]});
+  } else {
+    p[0] = (T)o[0];
+  }
+}
+
+template <typename T, int VEC, int NR>
+__global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
+    float* __restrict__ x, const T* __restrict__ y, long ystride,
+    const T* __restrict__ w_post, const T* __restrict__ w_next,
+    T* __restrict__ h, int W, float eps, float off) {
+  __shared__ float scratch[RN_BLOCK / WAVE];
+  const long row = blockIdx.x;
+  float* xr = x + row * W;
+  const T* yr = y ? y + row * ystride : nullptr;
+  T* hr = h ? h + row * W : nullptr;
+  const int step = RN_BLOCK * VEC;
+  constexpr int NA = NR > 0 ? NR : 1;
+  float xv[NA][VEC];
+
+  float inv_y = 0.0f;
+  float yv[NA][VEC];
+  if (yr) {
+    float ss = 0.0f;
+    if constexpr (NR > 0) {
+#pragma unroll
+      for (int i = 0; i < NR; ++i) {
+        const int c = i * step + threadIdx.x * VEC;
+        if (c < W) {
+          rn_load<T, VEC>(yr + c, yv[i]);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) ss += yv[i][j] * yv[i][j];
+        }
+      }
+    } else {
+      for (int c = threadIdx.x * VEC; c < W; c += step) {
+        rn_load<T, VEC>(yr + c, yv[0]);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss += yv[0][j] * yv[0][j];
+      }
+    }
+    ss = block_sum<RN_BLOCK>(ss, scratch);
+    inv_y = 1.0f / sqrtf(ss / (float)W + eps);
+  }
+
+  float ss = 0.0f;
+  auto update = [&](int c, float (&xa)[VEC], float (&ya)[VEC]) {
+    rn_load<float, VEC>(xr + c, xa);
+    if (yr) {
+      float wv[VEC];
+      rn_load<T, VEC>(w_post + c, wv);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) xa[j] += ya[j] * inv_y * (wv[j] + off);
+      rn_store<float, VEC>(xr + c, xa);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss += xa[j] * xa[j];
+  };
+  if constexpr (NR > 0) {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      const int c = i * step + threadIdx.x * VEC;
+      if (c < W) update(c, xv[i], yv[i]);
+    }
+  } else {
+    for (int c = threadIdx.x * VEC; c < W; c += step) {
+      if (yr) rn_load<T, VEC>(yr + c, yv[0]);
+      update(c, xv[0], yv[0]);
+    }
+  }
+  if (!hr) return;
+  ss = block_sum<RN_BLOCK>(ss, scratch);
+  const float inv = 1.0f / sqrtf(ss / (float)W + eps);
+  auto emit = [&](int c, float (&xa)[VEC]) {
+    float wv[VEC], o[VEC];
+    rn_load<T, VEC>(w_next + c, wv);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) o[j] = xa[j] * inv * (wv[j] + off);
+    rn_store<T, VEC>(hr + c, o);
+  };
+  if constexpr (NR > 0) {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      const int c = i * step + threadIdx.x * VEC;
+      if (c < W) emit(c, xv[i]);
+    }
+  } else {
+    for (int c = threadIdx.x * VEC; c < W; c += step) {
+      rn_load<float, VEC>(xr + c, xv[0]);
+      emit(c, xv[0]);
+    }
+  }
+}
+
+template <typename T>
+static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
+                       const void* wn, void* h, long rows, int W, float eps,
+                       float off, hipStream_t stream) {
+  const bool vec = W % 4 == 0 && ystride % 4 == 0 &&
+                   ((uintptr_t)y) % 16 == 0;
+  const int nr = (W + RN_BLOCK * 4 - 1) / (RN_BLOCK * 4);
+  dim3 grid((unsigned)rows), block(RN_BLOCK);
+#define RN_GO(V, N)                                                        \
+  add_norm_kernel<T, V, N><<<grid, block, 0, stream>>>(                    \
+      (float*)x, (const T*)y, ystride, (const T*)wp, (const T*)wn, (T*)h, W, \
+      eps, off)
+  if (!vec)
+    RN_GO(1, 0);
+  else if (nr <= 1)
+    RN_GO(4, 1);
+  else if (nr <= 2)
+    RN_GO(4, 2);
+  else if (nr <= 4)
+    RN_GO(4, 4);
+  else if (nr <= 8)
+    RN_GO(4, 8);
+  else
+    RN_GO(4, 0);
+#undef RN_GO
+}
+
+extern "C" void launch_add_norm(void* x, const void* y, long ystride,
+                                const void* wp, const void* wn, void* h,
+                                long rows, int W, float eps, float off,
+                                bool f32, hipStream_t stream) {
+  if (f32)
+    add_norm_t<float>(x, y, ystride, wp, wn, h, rows, W, eps, off, stream);
+  else
+    add_norm_t<__bf16>(x, y, ystride, wp, wn, h, rows, W, eps, off, stream);
+}
+
+// ---------------------------------------------------------------------------
+// Latent row work, one block per token:
+//   pool[row(token)] = [ rms(d[:rank]) * w | 0 | rotate(d[rank:]) | 0 ]
+//   q[token, h, qoff : qoff + rot] rotated in place for every head
+// Rows are rankp + rotp wide; rotation pairs neighbours; cos/sin [*, rot/2].
+// dkv == null (the layer reads another layer's rows): only q is rotated.
+// ---------------------------------------------------------------------------
+
+template <typename T>
+__global__ __launch_bounds__(RN_BLOCK) void latent_append_kernel(
+    const T* __restrict__ dkv, long dstride, const T* __restrict__ norm_w,
+    float eps, T* __restrict__ pool, T* __restrict__ q, long qstride, int H,
+    int dq, int qoff, int rank, int rankp, int rot, int rotp,
+    const float* __restrict__ cost, const float* __restrict__ sint,
+    const int* __restrict__ tok_pos, const int* __restrict__ tok_entry,
+    const int* __restrict__ pages, int P) {
+  __shared__ float scratch[RN_BLOCK / WAVE];
+  const long t = blockIdx.x;
+  const int pos = tok_pos[t];
+  const int half = rot / 2;
+  const float* c = cost + (long)pos * half;
+  const float* s = sint + (long)pos * half;
+
+  T* qt = q + t * qstride + qoff;
+  for (int i = threadIdx.x; i < H * half; i += RN_BLOCK) {
+    const int h = i / half, p = i - h * half;
+    T* a = qt + (long)h * dq + 2 * p;
+    const float u = (float)a[0], v = (float)a[1];
+    a[0] = (T)(u * c[p] - v * s[p]);
+    a[1] = (T)(v * c[p] + u * s[p]);
+  }
+  if (!dkv) return;
+
+  const T* d = dkv + t * dstride;
+  const long page = pages[(long)tok_entry[t] * P + pos / RG_PAGE];
+  T* row = pool + (page * RG_PAGE + pos % RG_PAGE) * (long)(rankp + rotp);
+  float ss = 0.0f;
+  for (int i = threadIdx.x; i < rank; i += RN_BLOCK) {
+    const float v = (float)d[i];
+    ss += v * v;
+  }
+  ss = block_sum<RN_BLOCK>(ss, scratch);
+  const float inv = 1.0f / sqrtf(ss / (float)rank + eps);
+  for (int i = threadIdx.x; i < rankp; i += RN_BLOCK)
+    row[i] = i < rank ? (T)((float)d[i] * inv * (float)norm_w[i]) : (T)0.0f;
+  for (int p = threadIdx.x; p < rotp / 2; p += RN_BLOCK) {
+    float o0 = 0.0f, o1 = 0.0f;
+    if (p < half) {
+      const float u = (float)d[rank + 2 * p], v = (float)d[rank + 2 * p + 1];
+      o0 = u * c[p] - v * s[p];
+      o1 = v * c[p] + u * s[p];
+    }
+    row[rankp + 2 * p] = (T)o0;
+    row[rankp + 2 * p + 1] = (T)o1;
+  }
+}
+
+extern "C" void launch_latent_append(
+    const void* dkv, long dstride, const void* norm_w, float eps, void* pool,
+    void* q, long qstride, int H, int dq, int qoff, int rank, int rankp,
+    int rot, int rotp, const float* cost, const float* sint,
+    const int* tok_pos, const int* tok_entry, const int* pages, int P,
+    long n_tok, bool f32, hipStream_t stream) {
+  dim3 grid((unsigned)n_tok), block(RN_BLOCK);
+#define LA_GO(T)                                                            \
+  latent_append_kernel<T><<<grid, block, 0, stream>>>(                      \
+      (const T*)dkv, dstride, (const T*)norm_w, eps, (T*)pool, (T*)q,       \
+      qstride, H, dq, qoff, rank, rankp, rot, rotp, cost, sint, tok_pos,    \
+      tok_entry, pages, P)
+  if (f32)
+    LA_GO(float);
+  else
+    LA_GO(__bf16);
+#undef LA_GO
+}
+
+// ---------------------------------------------------------------------------
+// Pages -> contiguous rows.  One block per page: blocks[i] = (page, first
+// destination row, valid rows); rows past the valid ones become zero.
+// ---------------------------------------------------------------------------
+
+template <typename T>
+__global__ __launch_bounds__(RN_BLOCK) void latent_gather_kernel(
+    const T* __restrict__ pool, T* __restrict__ dst,
+    const int* __restrict__ blocks, int W) {
+  const int* b = blocks + (long)blockIdx.x * 3;
+  const T* src = pool + (long)b[0] * RG_PAGE * W;
+  T* out = dst + (long)b[1] * W;
+  const int nvec = W / 8;
+  const int valid = b[2] * nvec;
+  for (int i = threadIdx.x; i < RG_PAGE * nvec; i += RN_BLOCK) {
+    if (i < valid)
+      copy8(out + (long)i * 8, src + (long)i * 8);
+    else
+      zero8(out + (long)i * 8);
+  }
+}
+
+extern "C" void launch_latent_gather(const void* pool, void* dst,
+                                     const int* blocks, int n_blocks, int W,
+                                     bool f32, hipStream_t stream) {
+  dim3 grid((unsigned)n_blocks), block(RN_BLOCK);
+  if (f32)
+    latent_gather_kernel<float><<<grid, block, 0, stream>>>(
+        (const float*)pool, (float*)dst, blocks, W);
+  else
+    latent_gather_kernel<__bf16><<<grid, block, 0, stream>>>(
+        (const __bf16*)pool, (__bf16*)dst, blocks, W);
+}
