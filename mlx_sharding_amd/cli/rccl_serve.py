@@ -25,6 +25,7 @@ def main(argv=None):
     from transformers import AutoTokenizer
 
     from ..config import ModelConfig
+    from ..models import get_model_class
     from ..parallel.rccl import PipelineWorker, init_distributed, split_layers
     from ..parallel.rccl_serve import (RcclModelProvider, RcclPipeline)
     from ..server.openai_api import run
@@ -32,7 +33,8 @@ def main(argv=None):
 
     rank, world, device = init_distributed()
     cfg = ModelConfig.load(args.model)
-    s, e = split_layers(cfg.num_hidden_layers, world)[rank]
+    cuts = get_model_class(cfg.model_type).allowed_cuts(cfg)
+    s, e = split_layers(cfg.num_hidden_layers, world, cuts)[rank]
     q = (args.quantize, args.quantize_group_size) if args.quantize else None
     model, _ = load_model(args.model, s, e, device=str(device), quantize=q)
     worker = PipelineWorker(model, rank, world, device)

@@ -71,15 +71,19 @@ class ModelConfig:
 
     @property
     def num_hidden_layers(self) -> int:
-        return int(self.raw["num_hidden_layers"])
+        if "num_hidden_layers" in self.raw:
+            return int(self.raw["num_hidden_layers"])
+        return len(self.raw["layers"])  # configs that list their layers
 
     @property
     def hidden_size(self) -> int:
-        return int(self.raw["hidden_size"])
+        return int(self.raw["hidden_size"] if "hidden_size" in self.raw
+                   else self.raw["width"])
 
     @property
     def vocab_size(self) -> int:
-        return int(self.raw["vocab_size"])
+        return int(self.raw["vocab_size"] if "vocab_size" in self.raw
+                   else self.raw["vocab"])
 
     @property
     def quantization(self) -> Optional[QuantConfig]:
@@ -107,7 +111,9 @@ class ModelConfig:
 
     @classmethod
     def from_dict(cls, d: dict) -> "ModelConfig":
-        return cls(model_type=d["model_type"], raw=dict(d))
+        # configs without a model_type name their design in "architecture"
+        kind = d["model_type"] if "model_type" in d else d["architecture"].lower()
+        return cls(model_type=kind, raw=dict(d))
 
     @classmethod
     def load(cls, model_path: str | Path) -> "ModelConfig":

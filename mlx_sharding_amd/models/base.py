@@ -95,6 +95,9 @@ class StageModel(nn.Module):
     """
 
     rope_attn_scale: float = 1.0
+    # runs ragged batches over a PagedState (``run``, ``make_state``)
+    supports_ragged: bool = False
+    supports_quantization: bool = True
 
     def __init__(self, config: ModelConfig, shard: ShardSpec):
         super().__init__()
@@ -137,6 +140,16 @@ class StageModel(nn.Module):
         — casting activations to THAT truncates them to garbage)."""
         return next((q.dtype for q in self.parameters()
                      if q.is_floating_point()), torch.bfloat16)
+
+    @property
+    def hop_dtype(self) -> torch.dtype:
+        """Type of the hidden states handed from stage to stage."""
+        return self.fp_dtype
+
+    @classmethod
+    def allowed_cuts(cls, config: ModelConfig) -> Optional[List[int]]:
+        """Layer indices a stage may begin at; None: any."""
+        return None
 
     # -- cache ------------------------------------------------------------
     def cache_specs(self) -> List[Tuple[int, int, int]]:

@@ -75,6 +75,7 @@ def fuse_model(model) -> int:
     from .llama import LlamaAttention, LlamaMLP
     from .gemma2 import Gemma2Attention, Gemma2MLP
     from .deepseek_v2 import MLAAttention
+    from .mixers import GatedDelta, GatedMLP, LatentAttention
 
     n = 0
     for mod in model.modules():
@@ -87,6 +88,9 @@ def fuse_model(model) -> int:
                 n += 1
             elif isinstance(mod, MLAAttention) and not mod.q_lora_rank:
                 mod._fused_qkv = FusedColumns([mod.q_proj, mod.kv_a_proj_with_mqa])
+                n += 1
+            elif isinstance(mod, (GatedDelta, GatedMLP, LatentAttention)):
+                mod.prepare()
                 n += 1
         except AssertionError:
             continue  # mixed quant/bias group — leave unfused

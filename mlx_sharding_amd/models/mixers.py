@@ -1,0 +1,224 @@
+"""Token mixers and layer pieces for ragged batches.
+
+A mixer works on rows [tokens, width] of a ragged batch (ops.paged) and keeps
+what it needs between steps in its layer's store.  Every constant is a
+parameter, so designs combine them freely.  Parameters keep the checkpoint's
+shapes; ``prepare`` lays them out for the kernels (sibling projections in one
+GEMM, head sizes padded to the kernels' tiles) once they are on their device.
+"""
+
+from __future__ import annotations
+
+from typing import Optional
+
+import torch
+import torch.nn as nn
+import torch.nn.functional as F
+
+from .. import ops
+from ..ops import ragged
+from ..ops.paged import LayerStore, RaggedBatch, RowSpec, StateSpec
+from ..ops.ragged import DeltaShape, LatentShape, Rotary
+from .base import Linear, RMSNorm
+
+
+def _param(*shape, dtype) -> nn.Parameter:
+    return nn.Parameter(torch.empty(*shape, dtype=dtype), requires_grad=False)
+
+
+def _share(weight: torch.Tensor, *linears: Linear):
+    """Make the linears' weights views of the stacked one."""
+    off = 0
+    for lin in linears:
+        lin.weight.data = weight[off: off + lin.out_features]
+        off += lin.out_features
+
+
+class _Weight(nn.Module):
+    def __init__(self, *shape, dtype):
+        super().__init__()
+        self.weight = _param(*shape, dtype=dtype)
+
+
+class ConvLinear(Linear):
+    """A projection followed by a causal convolution over time per channel,
+    ``conv.weight`` [channels, taps], the last tap on the current token."""
+
+    def __init__(self, in_features: int, out_features: int, taps: int,
+                 dtype: torch.dtype):
+        super().__init__(in_features, out_features, dtype=dtype)
+        self.conv = _Weight(out_features, taps, dtype=dtype)
+
+
+class NormedLinear(Linear):
+    """A projection whose leading outputs are RMS-normed (``norm.weight``)."""
+
+    def __init__(self, in_features: int, out_features: int, normed: int,
+                 eps: float, dtype: torch.dtype):
+        super().__init__(in_features, out_features, dtype=dtype)
+        self.norm = RMSNorm(normed, eps, dtype=dtype)
+
+
+class LatentAttention(nn.Module):
+    """Causal softmax attention over a cached low-rank latent.
+
+    Cached per token: the normed latent (``rank``) and one rotated key part
+    shared by all heads (``rotary.dims``).  Keys are [W_uk c | rotated part],
+    values W_uv c.  Without ``own_rows`` the layer has no latent projection and
+    attends to the rows of another layer's store.
+    """
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, rank: int,
+                 rotary: Rotary, scale: float, eps: float,
+                 own_rows: bool = True, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.rotary, self.scale, self.eps = rotary, float(scale), eps
+        self.sizes = dict(heads=heads, dim=dim, rot=rotary.dims, vdim=vdim,
+                          rank=rank)
+        if rank > 1024:
+            raise ValueError(f"latent size {rank} is above 1024")
+        rot = rotary.dims
+        self.q = Linear(width, heads * (dim + rot), dtype=dtype)
+        self.dkv = NormedLinear(width, rank + rot, rank, eps, dtype) \
+            if own_rows else None
+        self.uk = Linear(rank, heads * dim, dtype=dtype)
+        self.uv = Linear(rank, heads * vdim, dtype=dtype)
+        self.o = Linear(heads * vdim, width, dtype=dtype)
+        self.ready = False
+
+    def store_spec(self) -> Optional[RowSpec]:
+        if self.dkv is None:
+            return None
+        return RowSpec(LatentShape(**self.sizes).width)
+
+    @torch.no_grad()
+    def prepare(self):
+        wq, wuk, wuv, wo = (m.weight.data for m in (self.q, self.uk, self.uv, self.o))
+        self.shape = sh = LatentShape(**self.sizes, f32=wq.dtype == torch.float32)
+        H, width = sh.heads, wq.shape[1]
+
+        w = wq.view(H, sh.dim + sh.rot, width)
+        w = torch.cat([F.pad(w[:, : sh.dim], (0, 0, 0, sh.dimp - sh.dim)),
+                       F.pad(w[:, sh.dim:], (0, 0, 0, sh.rotp - sh.rot))], 1)
+        w = w.reshape(H * sh.dq, width)
+        if self.dkv is not None:
+            w = torch.cat([w, self.dkv.weight.data])
+        w = F.pad(w, (0, 0, 0, -w.shape[0] % 8)).contiguous()
+        self.w_in = w
+        if sh.dq == sh.dim + sh.rot:
+            _share(w, self.q, *([self.dkv] if self.dkv is not None else []))
+
+        rpad = (0, sh.rankp - sh.rank)
+        uk = F.pad(wuk.view(H, sh.dim, sh.rank), (*rpad, 0, sh.dimp - sh.dim))
+        uv = F.pad(wuv.view(H, sh.vdim, sh.rank), (*rpad, 0, sh.vdp - sh.vdim))
+        self.w_uk = uk.reshape(H * sh.dimp, sh.rankp).contiguous()
+        self.w_uv = uv.reshape(H * sh.vdp, sh.rankp).contiguous()
+        # absorbed form: [H, dimp, rankp] into the query, [H, rankp, vdp] out
+        self.w_absorb = self.w_uk.view(H, sh.dimp, sh.rankp)
+        self.w_emit = self.w_uv.view(H, sh.vdp, sh.rankp).transpose(1, 2).contiguous()
+        wo = F.pad(wo.view(width, H, sh.vdim), (0, sh.vdp - sh.vdim))
+        self.w_o = wo.reshape(width, H * sh.vdp).contiguous()
+        self.ready = True
+
+    def forward(self, h: torch.Tensor, batch: RaggedBatch, store: LayerStore,
+                tables) -> torch.Tensor:
+        """store: the layer's own, or that of the layer it reads."""
+        if not self.ready:
+            self.prepare()
+        sh = self.shape
+        H, nq = sh.heads, sh.heads * sh.dq
+        y = ops.linear(h, self.w_in)
+        q = y[:, :nq]
+        dkv = norm_w = None
+        if self.dkv is not None:
+            dkv = y[:, nq: nq + sh.rank + sh.rot]
+            norm_w = self.dkv.norm.weight
+        ragged.latent_append(dkv, norm_w, self.eps, store, q, sh, *tables,
+                             batch)
+        n, n_req, max_len = batch.short_tokens, batch.n_short, batch.max_short
+        if not sh.expandable:
+            n, n_req, max_len = batch.n_tokens, batch.n_requests, batch.max_len
+        parts = []
+        if n:
+            qn = q[:n].unflatten(1, (H, sh.dq))[..., : sh.dimp]
+            q_abs = torch.bmm(qn.transpose(0, 1).contiguous(), self.w_absorb)
+            o = ragged.latent_attention_absorbed(q, q_abs, store, sh,
+                                                 self.scale, batch, n_req,
+                                                 max_len)
+            o = torch.bmm(o, self.w_emit)               # [H, n, vdp]
+            parts.append(o.transpose(0, 1).reshape(n, H * sh.vdp))
+        if n < batch.n_tokens:
+            parts.append(ragged.latent_attention_expanded(
+                q, store, self.w_uk, self.w_uv, sh, self.scale, batch))
+        out = parts[0] if len(parts) == 1 else torch.cat(parts)
+        return ops.linear(out, self.w_o)
+
+
+class GatedDelta(nn.Module):
+    """Gated delta rule: a linear recurrence with a fp32 matrix state per head
+    that forgets (one decay per head) and corrects (delta write), behind short
+    convolutions, with a normed and gated output."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, taps: int, eps: float,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.shape = DeltaShape(heads, kv_heads, dim, vdim, taps)
+        self.eps = eps
+        self.q = ConvLinear(width, kv_heads * dim, taps, dtype)
+        self.k = ConvLinear(width, kv_heads * dim, taps, dtype)
+        self.v = ConvLinear(width, heads * vdim, taps, dtype)
+        self.g = Linear(width, heads * vdim, dtype=dtype)
+        self.a = Linear(width, heads, dtype=dtype)
+        self.b = Linear(width, heads, dtype=dtype)
+        self.A_log = _param(heads, dtype=dtype)
+        self.dt_bias = _param(heads, dtype=dtype)
+        self.norm = RMSNorm(vdim, eps, dtype=dtype)
+        self.o = Linear(heads * vdim, width, dtype=dtype)
+        self.ready = False
+
+    def store_spec(self) -> StateSpec:
+        sh = self.shape
+        return StateSpec(sh.heads, sh.dim, sh.vdim, sh.channels, sh.taps - 1)
+
+    @torch.no_grad()
+    def prepare(self):
+        rows = (self.q, self.k, self.v, self.g, self.a, self.b)
+        self.w_in = torch.cat([m.weight.data for m in rows]).contiguous()
+        _share(self.w_in, *rows)
+        convs = (self.q, self.k, self.v)
+        self.w_conv = torch.cat([m.conv.weight.data for m in convs]).contiguous()
+        self.ready = True
+
+    def forward(self, h: torch.Tensor, batch: RaggedBatch,
+                store: LayerStore) -> torch.Tensor:
+        if not self.ready:
+            self.prepare()
+        y = ops.linear(h, self.w_in)
+        o = ragged.gated_delta(y, self.w_conv, self.A_log, self.dt_bias,
+                               self.norm.weight, store, self.shape, self.eps,
+                               batch)
+        return self.o(o)
+
+
+class GatedMLP(nn.Module):
+    """W_down (act(W_gate h) * W_up h)."""
+
+    ACTS = {"gelu_tanh": ops.geglu, "silu": ops.swiglu}
+
+    def __init__(self, width: int, ff: int, act: str,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.act = self.ACTS[act]
+        self.gate = Linear(width, ff, dtype=dtype)
+        self.up = Linear(width, ff, dtype=dtype)
+        self.down = Linear(ff, width, dtype=dtype)
+        self.fused = None
+
+    def prepare(self):
+        from .fuse import FusedColumns
+        self.fused = FusedColumns([self.gate, self.up])
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        g, u = self.fused(h) if self.fused is not None else (self.gate(h), self.up(h))
+        return self.down(self.act(g, u))

@@ -1,0 +1,224 @@
+"""Tuvutar stage model: gated-delta and latent-attention layers in any order.
+
+config.json: ``width``, ``vocab``, ``norm.eps`` and ``layers``, a list of
+{"type", "mixer", "mlp"}.  A layer is normed on both sides of each sublayer
+(norm weights stored around zero) on a 32-bit residual stream; ``mlp`` may be
+null.  A latent-attention layer with ``kv_from`` reads the rows that layer
+cached, so both live on the same pipeline stage.
+
+Tensors: ``embed``, ``l<i>.norm1`` / ``norm1b`` / ``norm2`` / ``norm2b``,
+``l<i>.mix.*``, ``l<i>.mlp.*``, ``final.norm``, ``head``.
+"""
+
+from __future__ import annotations
+
+from typing import Dict, List, Optional
+
+import torch
+import torch.nn as nn
+import torch.nn.functional as F
+
+from .. import ops
+from ..config import ModelConfig, ShardSpec
+from ..ops import ragged
+from ..ops.paged import PagedState, RaggedBatch, RaggedCache, RaggedLayerCache
+from ..ops.ragged import Rotary
+from .base import Linear, RMSNorm, StageModel, owned_layer_indices
+from .mixers import GatedDelta, GatedMLP, LatentAttention
+
+NORM_OFFSET = 1.0  # norm weights are stored around zero
+
+# parameters that are not the ``weight`` of a module
+_BARE = ("A_log", "dt_bias")
+
+
+def _rotary(rot: dict) -> Rotary:
+    sc = rot.get("scaling")
+    if not sc:
+        return Rotary(int(rot["dims"]), float(rot["base"]))
+    return Rotary(int(rot["dims"]), float(rot["base"]), float(sc["factor"]),
+                  float(sc["original"]), float(sc["fast"]), float(sc["slow"]))
+
+
+def _mixer(kind: str, mx: dict, width: int, eps: float, dtype: torch.dtype):
+    if kind == "latent_attention":
+        rotary = _rotary(mx["rot"])
+        if rotary.dims != int(mx["rot_dim"]):
+            raise ValueError("the rotated part has rot_dim = rot.dims dimensions")
+        return LatentAttention(
+            width, int(mx["heads"]), int(mx["dim"]), int(mx["vdim"]),
+            int(mx["kv_rank"]), rotary, float(mx["scale"]), eps,
+            own_rows=mx.get("kv_from") is None, dtype=dtype)
+    if kind == "delta":
+        return GatedDelta(width, int(mx["heads"]), int(mx["kv_heads"]),
+                          int(mx["dim"]), int(mx["vdim"]), int(mx["conv"]),
+                          eps, dtype=dtype)
+    raise ValueError(f"unknown mixer type {kind!r}")
+
+
+class TuvutarLayer(nn.Module):
+    def __init__(self, spec: dict, width: int, eps: float, dtype: torch.dtype):
+        super().__init__()
+        mx = spec["mixer"]
+        self.norm1 = RMSNorm(width, eps, NORM_OFFSET, dtype)
+        self.norm1b = RMSNorm(width, eps, NORM_OFFSET, dtype)
+        self.mix = _mixer(spec["type"], mx, width, eps, dtype)
+        src = mx.get("kv_from")
+        self.source: Optional[int] = None if src is None else int(src)
+        mlp = spec.get("mlp")
+        self.mlp = None
+        if mlp is not None:
+            if mlp["kind"] != "dense":
+                raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+            self.norm2 = RMSNorm(width, eps, NORM_OFFSET, dtype)
+            self.norm2b = RMSNorm(width, eps, NORM_OFFSET, dtype)
+            self.mlp = GatedMLP(width, int(mlp["ff"]), "gelu_tanh", dtype)
+
+
+class TuvutarStageModel(StageModel):
+    model_type = "tuvutar"
+    supports_ragged = True
+    supports_quantization = False
+
+    def __init__(self, config: ModelConfig, shard: ShardSpec, quant_for=None,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__(config, shard)
+        W, self.eps = config.hidden_size, float(config["norm"]["eps"])
+        specs = config["layers"]
+        if shard.is_first:
+            self.embed = nn.Embedding(config.vocab_size, W, dtype=dtype)
+        for i in owned_layer_indices(shard):
+            layer = TuvutarLayer(specs[i], W, self.eps, dtype)
+            self.add_module(f"l{i}", layer)
+            j = layer.source
+            if j is not None and not (shard.owns(j) and j < i):
+                raise ValueError(
+                    f"layer {i} reads the rows of layer {j}, which stage "
+                    f"[{shard.start_layer}, {shard.end_layer}) does not run "
+                    f"before it")
+        if shard.is_last:
+            self.final = nn.Module()
+            self.final.norm = RMSNorm(W, self.eps, NORM_OFFSET, dtype)
+            self.head = Linear(W, config.vocab_size, dtype=dtype)
+        self._tables: Dict = {}
+
+    # -- layers ------------------------------------------------------------
+    def layer(self, i: int) -> TuvutarLayer:
+        return getattr(self, f"l{i}")
+
+    def layer_items(self):
+        return [(i, self.layer(i)) for i in owned_layer_indices(self.shard)]
+
+    @classmethod
+    def allowed_cuts(cls, config: ModelConfig) -> List[int]:
+        """Layer indices a pipeline stage may begin at: not between a layer
+        and one that reads its rows."""
+        n = config.num_hidden_layers
+        bad = set()
+        for i, spec in enumerate(config["layers"]):
+            j = spec["mixer"].get("kv_from")
+            if j is not None:
+                bad.update(range(int(j) + 1, i + 1))
+        return [c for c in range(1, n) if c not in bad]
+
+    @property
+    def hop_dtype(self) -> torch.dtype:
+        return torch.float32  # stages hand on the residual stream
+
+    # -- weights -----------------------------------------------------------
+    @classmethod
+    def owns_key(cls, key: str, shard: ShardSpec) -> bool:
+        top = key.split(".")[0]
+        if top == "embed":
+            return shard.is_first
+        if top in ("final", "head"):
+            return shard.is_last
+        return top[:1] == "l" and top[1:].isdigit() and shard.owns(int(top[1:]))
+
+    @classmethod
+    def sanitize(cls, weights, shard: ShardSpec):
+        out = {}
+        for k, v in weights.items():
+            if cls.owns_key(k, shard):
+                if k.rsplit(".", 1)[-1] not in (*_BARE, "weight"):
+                    k = f"{k}.weight"
+                out[k] = v
+        return out
+
+    # -- cache -------------------------------------------------------------
+    def store_specs(self) -> List:
+        return [layer.mix.store_spec() for _, layer in self.layer_items()]
+
+    def make_state(self, max_tokens: int, max_requests: int) -> PagedState:
+        p = next(self.parameters())
+        return PagedState(self.store_specs(), max_tokens, max_requests,
+                          p.dtype, p.device)
+
+    def make_cache(self, dtype: Optional[torch.dtype] = None,
+                   batch_size: int = 1, device=None) -> List[RaggedLayerCache]:
+        p = next(self.parameters())
+        shared = RaggedCache(self.store_specs(), batch_size, dtype or p.dtype,
+                             device if device is not None else p.device)
+        return [RaggedLayerCache(shared, i) for i in range(self.shard.n_layers)]
+
+    # -- forward -----------------------------------------------------------
+    def _rotation(self, rotary: Rotary, n: int, device):
+        got = self._tables.get(rotary)
+        if got is None or got[0].shape[0] < n or got[0].device != device:
+            rows = max(1024, 1 << max(n - 1, 1).bit_length())
+            got = self._tables[rotary] = rotary.tables(rows, device)
+        return got
+
+    @torch.no_grad()
+    def run(self, x: torch.Tensor, batch: RaggedBatch, state: PagedState,
+            rows: Optional[torch.Tensor] = None,
+            layer_outputs: Optional[list] = None) -> torch.Tensor:
+        """One ragged forward.  x: token ids [N] on the first stage, else the
+        residual [N, width]; rows select the tokens that go through the head.
+        Returns the residual, or fp32 logits on the last stage."""
+        if self.shard.is_first:
+            x = F.embedding(x, self.embed.weight).float()
+        else:
+            x = x.float().contiguous().clone()
+        dtype = next(self.parameters()).dtype
+        norm = lambda y, post, nxt: ragged.add_norm(  # noqa: E731
+            x, y, None if post is None else post.weight,
+            None if nxt is None else nxt.weight, self.eps, NORM_OFFSET, dtype)
+        items = self.layer_items()
+        first = self.shard.start_layer
+        h = norm(None, None, items[0][1].norm1)
+        for k, (i, layer) in enumerate(items):
+            if k + 1 < len(items):
+                after = items[k + 1][1].norm1
+            else:
+                after = self.final.norm if self.shard.is_last else None
+            if isinstance(layer.mix, LatentAttention):
+                src = i if layer.source is None else layer.source
+                y = layer.mix(h, batch, state.layers[src - first],
+                              self._rotation(layer.mix.rotary, batch.max_pos,
+                                             x.device))
+            else:
+                y = layer.mix(h, batch, state.layers[k])
+            if layer.mlp is None:
+                h = norm(y, layer.norm1b, after)
+            else:
+                h = norm(y, layer.norm1b, layer.norm2)
+                h = norm(layer.mlp(h), layer.norm2b, after)
+            if layer_outputs is not None:
+                layer_outputs.append(x.clone())
+        if not self.shard.is_last:
+            return x
+        if rows is not None:
+            h = h.index_select(0, rows)
+        return self.head(h).float()
+
+    def forward(self, x: torch.Tensor, cache: Optional[List] = None) -> torch.Tensor:
+        B, T = x.shape[:2]
+        if cache is None:
+            cache = self.make_cache(batch_size=B, device=x.device)
+        shared = cache[0].shared
+        if B != shared.batch_size:
+            raise ValueError(f"cache batch mismatch: {shared.batch_size} vs {B}")
+        y = self.run(x.reshape(B * T, *x.shape[2:]), shared.next_batch(T),
+                     shared.state)
+        return y.view(B, T, -1)

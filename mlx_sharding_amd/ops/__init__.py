@@ -155,15 +155,27 @@ def _prefill_attention_gpu(q, k, v, scale, causal_offset, softcap, sliding_windo
     return out.reshape(B, Hq, Tq, v.shape[3])
 
 
+def _glu(gate, up, gelu: bool):
+    # both extensions carry the bf16 kernel; 32-bit activations and odd
+    # widths are the ragged one's
+    ext = _load_ext()
+    if ext is None or gate.dtype != torch.bfloat16 or gate.shape[-1] % 4:
+        from .ragged import hip_ragged
+        ragged = hip_ragged()
+        if ragged is not None:
+            return ragged.glu(gate, up, gelu)
+    return _require_ext("glu").glu(gate, up, gelu)
+
+
 def swiglu(gate, up):
     if _use_hip(gate):
-        return _require_ext("swiglu").glu(gate, up, False)
+        return _glu(gate, up, False)
     return ref.swiglu(gate, up)
 
 
 def geglu(gate, up):
     if _use_hip(gate):
-        return _require_ext("geglu").glu(gate, up, True)
+        return _glu(gate, up, True)
     return ref.geglu(gate, up)
 
 

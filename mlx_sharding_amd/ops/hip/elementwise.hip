@@ -167,6 +167,46 @@ __global__ void glu_strided_kernel(const short* __restrict__ gate,
   }
 }
 
+// Any element type, width and alignment (one element per step).
+template <typename T, bool GELU>
+__global__ void glu_any_kernel(const T* __restrict__ gate,
+                               const T* __restrict__ up, T* __restrict__ y,
+                               long rows, int I, long gstride, long ustride) {
+  const long total = rows * I;
+  const long stride = (long)gridDim.x * blockDim.x;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+       i += stride) {
+    const long r = i / I;
+    const int c = (int)(i - r * I);
+    const float x = (float)gate[r * gstride + c];
+    const float u = (float)up[r * ustride + c];
+    float a;
+    if (GELU) {
+      a = 0.5f * x *
+          (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+    } else {
+      a = x / (1.0f + expf(-x));
+    }
+    y[i] = (T)(a * u);
+  }
+}
+
+extern "C" void launch_glu_any(const void* gate, const void* up, void* y,
+                               long rows, int I, long gstride, long ustride,
+                               bool gelu, bool f32, hipStream_t stream) {
+  const long want = (rows * I + 255) / 256;
+  const unsigned grid = (unsigned)max(1L, min(want, 2048L));
+#define GA_GO(T, G)                                                          \
+  glu_any_kernel<T, G><<<dim3(grid), dim3(256), 0, stream>>>(                \
+      (const T*)gate, (const T*)up, (T*)y, rows, I, gstride, ustride)
+  if (f32) {
+    if (gelu) GA_GO(float, true); else GA_GO(float, false);
+  } else {
+    if (gelu) GA_GO(__bf16, true); else GA_GO(__bf16, false);
+  }
+#undef GA_GO
+}
+
 extern "C" void launch_glu_strided(const void* gate, const void* up, void* y,
                                    long rows, int I, long gstride,
                                    long ustride, bool gelu,

@@ -1,0 +1,456 @@
+// Python bindings of the ragged-batch kernels (extension _hip_ragged).
+// Every operand's device, type, shape and alignment is checked here, before
+// anything is launched.
+
+#include <torch/extension.h>
+#include <c10/hip/HIPStream.h>
+
+#include "ragged_prefill.h"
+
+extern "C" {
+void launch_glu_strided(const void*, const void*, void*, long, int, long, long,
+                        bool, hipStream_t);
+void launch_glu_any(const void*, const void*, void*, long, int, long, long,
+                    bool, bool, hipStream_t);
+void launch_add_norm(void*, const void*, long, const void*, const void*, void*,
+                     long, int, float, float, bool, hipStream_t);
+void launch_latent_append(const void*, long, const void*, float, void*, void*,
+                          long, int, int, int, int, int, int, int,
+                          const float*, const float*, const int*, const int*,
+                          const int*, int, long, bool, hipStream_t);
+void launch_latent_gather(const void*, void*, const int*, int, int, bool,
+                          hipStream_t);
+void launch_latent_attn_short(const void*, const void*, const void*, void*,
+                              float*, float*, const int*, const int*,
+                              const int*, int, int, int, long, int, int, int,
+                              int, float, int, int, int, bool, hipStream_t);
+void launch_latent_attn_long_bf16(const LatentLongArgs*, int, int,
+                                  hipStream_t);
+void launch_latent_attn_long_f32(const LatentLongArgs*, int, int, hipStream_t);
+int delta_short_rows(int, int, int);
+}
+
+struct DeltaDims {
+  int KH, H, D, V, taps;
+  int qc, kc, vc, gc, ac, bc;
+  long ystride;
+};
+
+struct DeltaLongArgs {
+  const void *y, *conv_w, *A_log, *dt_bias, *norm_w;
+  float* state;
+  void *conv_state, *out;
+  float *qn, *kn, *lg, *bt, *tm, *am, *ge, *o;
+  void* vn;
+  const int *cu, *pos0, *slots, *tok_entry, *chunks, *chunk_cu;
+  int n_short, n_long, tok_base, n_chunks, Dp, Vp;
+  long n_tok;
+  float eps;
+};
+
+extern "C" {
+void launch_delta_short(const void*, const void*, const void*, const void*,
+                        const void*, float*, void*, void*, const int*,
+                        const int*, const int*, const DeltaDims*, int, int,
+                        float, bool, hipStream_t);
+void launch_delta_long(const DeltaLongArgs*, const DeltaDims*, bool,
+                       hipStream_t);
+}
+
+namespace {
+
+using torch::Tensor;
+
+hipStream_t stream() { return c10::hip::getCurrentHIPStream().stream(); }
+
+bool is_f32(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda(), name, " must be on the GPU");
+  TORCH_CHECK(t.scalar_type() == torch::kFloat32 ||
+                  t.scalar_type() == torch::kBFloat16,
+              name, " must be float32 or bfloat16");
+  return t.scalar_type() == torch::kFloat32;
+}
+
+void check_like(const Tensor& t, const Tensor& as, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == as.scalar_type(), name,
+              " must be on the GPU with the activations' type");
+}
+
+void check_f32(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 &&
+                  t.is_contiguous(),
+              name, " must be contiguous float32 on the GPU");
+}
+
+const int* ints(const Tensor& t, int64_t at_least, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt32 &&
+                  t.is_contiguous() && t.numel() >= at_least,
+              name, " must be contiguous int32 on the GPU with at least ",
+              at_least, " elements");
+  return t.data_ptr<int>();
+}
+
+// [N, C] with unit column stride; returns the row stride
+long rows2(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.dim() == 2 && (t.stride(1) == 1 || t.size(1) == 1), name,
+              " must be [rows, columns] with unit column stride");
+  return t.size(0) > 1 ? t.stride(0) : std::max<long>(t.stride(0), t.size(1));
+}
+
+void aligned16(const Tensor& t, const char* name) {
+  TORCH_CHECK(((uintptr_t)t.data_ptr()) % 16 == 0, name,
+              " must be 16-byte aligned");
+}
+
+Tensor glu(Tensor gate, Tensor up, bool gelu) {
+  const bool f32 = is_f32(gate, "gate");
+  check_like(up, gate, "up");
+  TORCH_CHECK(gate.sizes() == up.sizes() && gate.dim() >= 1);
+  const long I = gate.size(-1);
+  auto g = gate.reshape({-1, I}), u = up.reshape({-1, I});
+  if (g.stride(1) != 1) g = g.contiguous();
+  if (u.stride(1) != 1) u = u.contiguous();
+  auto y = torch::empty(gate.sizes(), gate.options());
+  const long rows = g.size(0);
+  if (rows == 0) return y;
+  const long gs = rows2(g, "gate"), us = rows2(u, "up");
+  const bool vec = !f32 && I % 4 == 0 && gs % 4 == 0 && us % 4 == 0 &&
+                   ((uintptr_t)g.data_ptr()) % 8 == 0 &&
+                   ((uintptr_t)u.data_ptr()) % 8 == 0;
+  if (vec)
+    launch_glu_strided(g.data_ptr(), u.data_ptr(), y.data_ptr(), rows, (int)I,
+                       gs, us, gelu, stream());
+  else
+    launch_glu_any(g.data_ptr(), u.data_ptr(), y.data_ptr(), rows, (int)I, gs,
+                   us, gelu, f32, stream());
+  return y;
+}
+
+// x [N, W] fp32 (updated in place when y is given); returns h or an empty
+// tensor when there is no following norm.
+Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
+                c10::optional<Tensor> w_next, Tensor like, double eps,
+                double off) {
+  check_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2, "x must be [rows, width]");
+  const bool f32 = is_f32(like, "like");
+  const long N = x.size(0), W = x.size(1);
+  long ys = W;
+  if (y) {
+    check_like(*y, like, "y");
+    TORCH_CHECK(y->sizes() == x.sizes() && w_post, "y must match x");
+    ys = rows2(*y, "y");
+    check_like(*w_post, like, "w_post");
+    TORCH_CHECK(w_post->numel() == W && w_post->is_contiguous());
+  }
+  Tensor h;
+  if (w_next) {
+    check_like(*w_next, like, "w_next");
+    TORCH_CHECK(w_next->numel() == W && w_next->is_contiguous());
+    h = torch::empty({N, W}, like.options());
+  } else {
+    h = torch::empty({0}, like.options());
+  }
+  if (N == 0) return h;
+  launch_add_norm(x.data_ptr(), y ? y->data_ptr() : nullptr, ys,
+                  y ? w_post->data_ptr() : nullptr,
+                  w_next ? w_next->data_ptr() : nullptr,
+                  w_next ? h.data_ptr() : nullptr, N, (int)W, (float)eps,
+                  (float)off, f32, stream());
+  return h;
+}
+
+// q [N, >= H * dq], rotated in place at qoff of every head; dkv [N, rank+rot]
+// (optional) normed, rotated and written to its page rows.
+void latent_append(c10::optional<Tensor> dkv, c10::optional<Tensor> norm_w,
+                   double eps, Tensor pool, Tensor q, int64_t H, int64_t dq,
+                   int64_t qoff, int64_t rank, int64_t rankp, int64_t rot,
+                   int64_t rotp, Tensor cos, Tensor sin, Tensor tok_pos,
+                   Tensor tok_entry, Tensor pages) {
+  const bool f32 = is_f32(q, "q");
+  const long N = q.size(0);
+  const long qs = rows2(q, "q");
+  TORCH_CHECK(q.size(1) >= H * dq && qoff >= 0 && qoff + rot <= dq);
+  check_like(pool, q, "pool");
+  TORCH_CHECK(pool.is_contiguous() && pool.dim() == 2 &&
+              pool.size(1) == rankp + rotp);
+  check_f32(cos, "cos");
+  check_f32(sin, "sin");
+  TORCH_CHECK(rot % 2 == 0 && cos.size(1) == rot / 2 &&
+              sin.sizes() == cos.sizes());
+  TORCH_CHECK(rank <= rankp && rot <= rotp && rotp % 2 == 0);
+  TORCH_CHECK(pages.dim() == 2);
+  long ds = 0;
+  if (dkv) {
+    check_like(*dkv, q, "dkv");
+    ds = rows2(*dkv, "dkv");
+    TORCH_CHECK(dkv->size(0) == N && dkv->size(1) >= rank + rot && norm_w);
+    check_like(*norm_w, q, "norm_w");
+    TORCH_CHECK(norm_w->numel() == rank && norm_w->is_contiguous());
+  }
+  if (N == 0) return;
+  launch_latent_append(
+      dkv ? dkv->data_ptr() : nullptr, ds, dkv ? norm_w->data_ptr() : nullptr,
+      (float)eps, pool.data_ptr(), q.data_ptr(), qs, (int)H, (int)dq,
+      (int)qoff, (int)rank, (int)rankp, (int)rot, (int)rotp,
+      cos.data_ptr<float>(), sin.data_ptr<float>(), ints(tok_pos, N, "tok_pos"),
+      ints(tok_entry, N, "tok_entry"), ints(pages, 0, "pages"),
+      (int)pages.size(1), N, f32, stream());
+}
+
+Tensor latent_gather(Tensor pool, Tensor blocks, int64_t rows) {
+  const bool f32 = is_f32(pool, "pool");
+  TORCH_CHECK(pool.is_contiguous() && pool.dim() == 2 &&
+              pool.size(1) % 8 == 0 && pool.size(0) % RG_PAGE == 0);
+  TORCH_CHECK(blocks.dim() == 2 && blocks.size(1) == 3 &&
+              rows == blocks.size(0) * RG_PAGE);
+  auto out = torch::empty({rows, pool.size(1)}, pool.options());
+  if (rows)
+    launch_latent_gather(pool.data_ptr(), out.data_ptr(),
+                         ints(blocks, 0, "blocks"), (int)blocks.size(0),
+                         (int)pool.size(1), f32, stream());
+  return out;
+}
+
+// q_abs [H, Nt, rankp], q [N, >= H*dq] (rotated) -> [H, Nt, rankp]
+Tensor latent_attn_short(Tensor q_abs, Tensor q, Tensor pool, Tensor cu,
+                         Tensor pos0, Tensor pages, int64_t n_req,
+                         int64_t max_len, int64_t max_keys, int64_t dq,
+                         int64_t qoff, int64_t rotp, double scale) {
+  const bool f32 = is_f32(q_abs, "q_abs");
+  check_like(q, q_abs, "q");
+  check_like(pool, q_abs, "pool");
+  TORCH_CHECK(q_abs.dim() == 3 && q_abs.is_contiguous());
+  const long H = q_abs.size(0), Nt = q_abs.size(1), rankp = q_abs.size(2);
+  TORCH_CHECK(rankp % 64 == 0 && rankp <= 1024 && rotp % 32 == 0);
+  const long nd = rankp / 64;
+  TORCH_CHECK(nd == 1 || nd == 2 || nd == 4 || nd == 8 || nd == 16,
+              "latent width must be padded to 64 * 2^k");
+  TORCH_CHECK(pool.is_contiguous() && pool.size(1) == rankp + rotp);
+  const long qs = rows2(q, "q");
+  TORCH_CHECK(q.size(0) >= Nt && q.size(1) >= H * dq && qoff + rotp <= dq &&
+              qs % 8 == 0 && dq % 8 == 0 && qoff % 8 == 0);
+  aligned16(q, "q");
+  aligned16(q_abs, "q_abs");
+  TORCH_CHECK(pages.dim() == 2 && pages.size(0) >= n_req);
+  auto out = torch::empty_like(q_abs);
+  if (Nt == 0 || n_req == 0) return out;
+  const long tiles = (max_len * H + 15) / 16;
+  // enough blocks for the chip, at least two key tiles per slice
+  long nsplit = std::max<long>(1, 1024 / std::max<long>(1, n_req * tiles));
+  nsplit = std::min<long>(nsplit, std::max<long>(1, max_keys / 64));
+  nsplit = std::min<long>(nsplit, 64);
+  Tensor po, ml;
+  if (nsplit > 1) {
+    auto o = q_abs.options().dtype(torch::kFloat32);
+    po = torch::empty({H, Nt, nsplit, rankp}, o);
+    ml = torch::empty({H, Nt, nsplit, 2}, o);
+  }
+  launch_latent_attn_short(
+      q_abs.data_ptr(), q.data_ptr(), pool.data_ptr(), out.data_ptr(),
+      nsplit > 1 ? po.data_ptr<float>() : nullptr,
+      nsplit > 1 ? ml.data_ptr<float>() : nullptr, ints(cu, n_req + 1, "cu"),
+      ints(pos0, n_req, "pos0"), ints(pages, 0, "pages"), (int)pages.size(1),
+      (int)H, (int)Nt, qs, (int)dq, (int)qoff, (int)rankp, (int)rotp,
+      (float)scale, (int)n_req, (int)nsplit, (int)tiles, f32, stream());
+  return out;
+}
+
+// q [N, >= H*dq] (rotated), kx [St, H*dimp], lat [St, rankp+rotp],
+// vt [H*vdp, St] -> [N - tok_base, H*vdp]
+Tensor latent_attn_long(Tensor q, Tensor kx, Tensor lat, Tensor vt,
+                        Tensor tiles, Tensor cu, Tensor pos0, Tensor cuk,
+                        int64_t n_short, int64_t tok_base, int64_t H,
+                        int64_t dimp, int64_t rotp, double scale) {
+  const bool f32 = is_f32(q, "q");
+  check_like(kx, q, "kx");
+  check_like(lat, q, "lat");
+  check_like(vt, q, "vt");
+  const long dq = dimp + rotp;
+  const long St = lat.size(0);
+  const long vdp = vt.size(0) / H;
+  TORCH_CHECK(kx.is_contiguous() && kx.size(0) == St && kx.size(1) == H * dimp);
+  TORCH_CHECK(lat.is_contiguous() && lat.dim() == 2 && lat.size(1) > rotp);
+  TORCH_CHECK(vt.is_contiguous() && vt.size(1) == St && vt.size(0) == H * vdp);
+  TORCH_CHECK(St % LP_KT == 0 && dimp % 32 == 0 && rotp % 32 == 0);
+  const long qs = rows2(q, "q");
+  TORCH_CHECK(q.size(1) >= H * dq && qs % 8 == 0);
+  aligned16(q, "q");
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2);
+  const int step = f32 ? 4 : 2;
+  const int nks = (int)((dq / 32 + step - 1) / step) * step;
+  const int ndh = (int)(vdp / 16);
+  const bool ok_k = nks <= 8;
+  const bool ok_v = f32 ? (ndh == 4 || ndh == 16)
+                        : (ndh == 2 || ndh == 4 || ndh == 8 || ndh == 16);
+  TORCH_CHECK(ok_k && ok_v && vdp % 16 == 0, "unsupported head shape ", dq,
+              "/", vdp);
+  auto out = torch::empty({q.size(0) - tok_base, H * vdp}, q.options());
+  LatentLongArgs a;
+  a.q = q.data_ptr();
+  a.kx = kx.data_ptr();
+  a.lat = lat.data_ptr();
+  a.vt = vt.data_ptr();
+  a.out = out.data_ptr();
+  a.tiles = ints(tiles, 0, "tiles");
+  a.cu = ints(cu, n_short + 2, "cu");
+  a.pos0 = ints(pos0, n_short + 1, "pos0");
+  a.cuk = ints(cuk, 2, "cuk");
+  a.n_short = (int)n_short;
+  a.tok_base = (int)tok_base;
+  a.n_tiles = (int)tiles.size(0);
+  a.H = (int)H;
+  a.dq = (int)dq;
+  a.dimp = (int)dimp;
+  a.rankp = (int)(lat.size(1) - rotp);
+  a.W = (int)lat.size(1);
+  a.St = St;
+  a.qstride = qs;
+  a.scale = (float)scale;
+  if (a.n_tiles == 0) return out;
+  if (f32)
+    launch_latent_attn_long_f32(&a, nks, ndh, stream());
+  else
+    launch_latent_attn_long_bf16(&a, nks, ndh, stream());
+  return out;
+}
+
+DeltaDims delta_dims(const Tensor& y, const Tensor& conv_w, int64_t KH,
+                     int64_t H, int64_t D, int64_t V,
+                     const std::vector<int64_t>& cols) {
+  DeltaDims d;
+  TORCH_CHECK(KH > 0 && H % KH == 0 && cols.size() == 6);
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.is_contiguous() &&
+              conv_w.size(0) == 2 * KH * D + H * V);
+  d.KH = (int)KH;
+  d.H = (int)H;
+  d.D = (int)D;
+  d.V = (int)V;
+  d.taps = (int)conv_w.size(1);
+  TORCH_CHECK(d.taps >= 1 && d.taps <= 8, "convolutions have 1 to 8 taps");
+  TORCH_CHECK(D <= 512 && delta_short_rows((int)D, (int)V, 512) > 0,
+              "state of a head is too large: ", D, " x ", V);
+  const int64_t w[6] = {KH * D, KH * D, H * V, H * V, H, H};
+  for (int i = 0; i < 6; ++i)
+    TORCH_CHECK(cols[i] >= 0 && cols[i] + w[i] <= y.size(1));
+  d.qc = (int)cols[0];
+  d.kc = (int)cols[1];
+  d.vc = (int)cols[2];
+  d.gc = (int)cols[3];
+  d.ac = (int)cols[4];
+  d.bc = (int)cols[5];
+  d.ystride = rows2(y, "y");
+  return d;
+}
+
+void check_delta(const Tensor& y, const Tensor& conv_w, const Tensor& A_log,
+                 const Tensor& dt, const Tensor& norm_w, const Tensor& state,
+                 const Tensor& conv_state, const Tensor& out,
+                 const DeltaDims& d) {
+  for (const auto* t : {&conv_w, &A_log, &dt, &norm_w, &conv_state, &out})
+    check_like(*t, y, "delta operand");
+  TORCH_CHECK(A_log.numel() == d.H && dt.numel() == d.H &&
+              norm_w.numel() == d.V && A_log.is_contiguous() &&
+              dt.is_contiguous() && norm_w.is_contiguous());
+  check_f32(state, "state");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == d.H &&
+              state.size(2) == d.D && state.size(3) == d.V);
+  TORCH_CHECK(conv_state.is_contiguous() && conv_state.dim() == 3 &&
+              conv_state.size(0) == state.size(0) &&
+              conv_state.size(1) == conv_w.size(0) &&
+              conv_state.size(2) == d.taps - 1);
+  TORCH_CHECK(out.is_contiguous() && out.size(0) == y.size(0) &&
+              out.size(1) == (long)d.H * d.V);
+}
+
+// Short portions of y's batch; rows of out that belong to them are written.
+void delta_short(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
+                 Tensor norm_w, Tensor state, Tensor conv_state, Tensor out,
+                 Tensor cu, Tensor pos0, Tensor slots, int64_t n_req,
+                 int64_t max_len, int64_t KH, int64_t H, int64_t D, int64_t V,
+                 std::vector<int64_t> cols, double eps) {
+  const bool f32 = is_f32(y, "y");
+  auto d = delta_dims(y, conv_w, KH, H, D, V, cols);
+  check_delta(y, conv_w, A_log, dt, norm_w, state, conv_state, out, d);
+  TORCH_CHECK(max_len >= 1 && max_len <= 16, "short portions have 1 to 16 "
+              "tokens");
+  if (n_req == 0) return;
+  launch_delta_short(y.data_ptr(), conv_w.data_ptr(), A_log.data_ptr(),
+                     dt.data_ptr(), norm_w.data_ptr(), state.data_ptr<float>(),
+                     conv_state.data_ptr(), out.data_ptr(),
+                     ints(cu, n_req + 1, "cu"), ints(pos0, n_req, "pos0"),
+                     ints(slots, n_req, "slots"), &d, (int)n_req, (int)max_len,
+                     (float)eps, f32, stream());
+}
+
+// Long portions: requests n_short.. of the batch, tokens tok_base..
+void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
+                Tensor norm_w, Tensor state, Tensor conv_state, Tensor out,
+                Tensor cu, Tensor pos0, Tensor slots, Tensor tok_entry,
+                Tensor chunks, Tensor chunk_cu, int64_t n_short,
+                int64_t n_long, int64_t tok_base, int64_t KH, int64_t H,
+                int64_t D, int64_t V, std::vector<int64_t> cols, double eps) {
+  const bool f32 = is_f32(y, "y");
+  auto d = delta_dims(y, conv_w, KH, H, D, V, cols);
+  check_delta(y, conv_w, A_log, dt, norm_w, state, conv_state, out, d);
+  const long n = y.size(0) - tok_base;
+  if (n <= 0 || n_long == 0) return;
+  TORCH_CHECK(chunks.dim() == 2 && chunks.size(1) == 2);
+  const long nc = chunks.size(0);
+  const long Dp = (D + 15) / 16 * 16, Vp = (V + 15) / 16 * 16;
+  auto fo = y.options().dtype(torch::kFloat32);
+  auto qn = torch::empty({n, KH, Dp}, fo), kn = torch::empty({n, KH, Dp}, fo);
+  auto vn = torch::empty({n, H, Vp}, y.options());
+  auto lg = torch::empty({n, H}, fo), bt = torch::empty({n, H}, fo);
+  auto tm = torch::empty({nc, H, 64, 64}, fo);
+  auto am = torch::empty({nc, H, 64, 64}, fo);
+  auto ge = torch::empty({nc, H, 2, 64}, fo);
+  auto o = torch::empty({n, H, Vp}, fo);
+  DeltaLongArgs a;
+  a.y = y.data_ptr();
+  a.conv_w = conv_w.data_ptr();
+  a.A_log = A_log.data_ptr();
+  a.dt_bias = dt.data_ptr();
+  a.norm_w = norm_w.data_ptr();
+  a.state = state.data_ptr<float>();
+  a.conv_state = conv_state.data_ptr();
+  a.out = out.data_ptr();
+  a.qn = qn.data_ptr<float>();
+  a.kn = kn.data_ptr<float>();
+  a.lg = lg.data_ptr<float>();
+  a.bt = bt.data_ptr<float>();
+  a.tm = tm.data_ptr<float>();
+  a.am = am.data_ptr<float>();
+  a.ge = ge.data_ptr<float>();
+  a.o = o.data_ptr<float>();
+  a.vn = vn.data_ptr();
+  a.cu = ints(cu, n_short + n_long + 1, "cu");
+  a.pos0 = ints(pos0, n_short + n_long, "pos0");
+  a.slots = ints(slots, n_short + n_long, "slots");
+  a.tok_entry = ints(tok_entry, y.size(0), "tok_entry");
+  a.chunks = ints(chunks, 0, "chunks");
+  a.chunk_cu = ints(chunk_cu, n_long + 1, "chunk_cu");
+  a.n_short = (int)n_short;
+  a.n_long = (int)n_long;
+  a.tok_base = (int)tok_base;
+  a.n_chunks = (int)nc;
+  a.Dp = (int)Dp;
+  a.Vp = (int)Vp;
+  a.n_tok = n;
+  a.eps = (float)eps;
+  launch_delta_long(&a, &d, f32, stream());
+}
+
+}  // namespace
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("glu", &glu);
+  m.def("add_norm", &add_norm);
+  m.def("latent_append", &latent_append);
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_attn_short", &latent_attn_short);
+  m.def("latent_attn_long", &latent_attn_long);
+  m.def("delta_short", &delta_short);
+  m.def("delta_long", &delta_long);
+  m.attr("PAGE") = RG_PAGE;
+}

@@ -136,6 +136,16 @@ class KVCache:
             self._k.shape[0] if self._k is not None else self.batch_size)
         self._ensure(b, cap)
 
+    # a shorter prefix of what is cached can be returned to
+    trimmable = True
+
+    def snapshot(self):
+        """What a decode step changes besides appending; nothing here."""
+        return None
+
+    def restore(self, snap):
+        pass
+
     def trim(self, n: int):
         """Roll back to the first ``n`` cached positions (prefix-cache
         reuse: a follow-up request whose prompt shares an n-token prefix

@@ -1,0 +1,356 @@
+"""Ops on ragged batches: HIP kernels on GPU, torch on CPU.
+
+The same policy as the package's other ops: GPU tensors run the hand-written
+kernels (extension ``_hip_ragged``) or fail loudly; CPU tensors run plain torch
+with the same storage layout, request by request.
+
+Layouts.  A latent row is [latent, zero padding to ``rankp`` | rotated key part,
+zero padding to ``rotp``].  A query head is [unrotated, padding | rotated,
+padding], ``dq`` wide.
+"""
+
+from __future__ import annotations
+
+import math
+from dataclasses import dataclass
+from typing import List, Optional
+
+import torch
+import torch.nn.functional as F
+
+from .paged import LayerStore, PAGE, RaggedBatch
+
+_EXT = None
+_EXT_ERR: Optional[str] = None
+_TRIED = False
+
+
+def hip_ragged():
+    """The extension module, or None where it is not built."""
+    global _EXT, _EXT_ERR, _TRIED
+    if not _TRIED:
+        _TRIED = True
+        try:
+            from mlx_sharding_amd import _hip_ragged
+            _EXT = _hip_ragged
+        except ImportError as e:
+            _EXT_ERR = repr(e)
+    return _EXT
+
+
+def _ext(op: str):
+    ext = hip_ragged()
+    if ext is None:
+        raise RuntimeError(
+            f"mlx_sharding_amd: op '{op}' called on a GPU tensor but the HIP "
+            f"extension mlx_sharding_amd._hip_ragged is not importable "
+            f"({_EXT_ERR}). Build it with `python setup.py build_ext --inplace`.")
+    return ext
+
+
+# ---------------------------------------------------------------------------
+# Norms around a 32-bit residual
+# ---------------------------------------------------------------------------
+
+def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
+    return x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def add_norm(x, y, w_post, w_next, eps: float, offset: float,
+             dtype: torch.dtype):
+    """x += rms(y) * (w_post + offset), in place, if y is given; returns
+    rms(x) * (w_next + offset) in ``dtype``, or None without w_next.
+    x is the fp32 residual [N, W]."""
+    if x.is_cuda:
+        like = w_post if w_post is not None else w_next
+        h = _ext("add_norm").add_norm(x, y, w_post, w_next, like, eps, offset)
+        return h if w_next is not None else None
+    if y is not None:
+        x += _rms(y.float(), eps) * (w_post.float() + offset)
+    if w_next is None:
+        return None
+    return (_rms(x, eps) * (w_next.float() + offset)).to(dtype)
+
+
+# ---------------------------------------------------------------------------
+# Rotation tables
+# ---------------------------------------------------------------------------
+
+@dataclass(frozen=True)
+class Rotary:
+    """Interleaved rotary positions on ``dims`` dimensions, optionally with
+    YaRN frequencies (``factor`` set): pairs that turn less than ``slow`` times
+    within ``original`` positions are slowed by ``factor``, pairs that turn more
+    than ``fast`` times are kept, with a ramp between; cos and sin are scaled
+    by 0.1 ln(factor) + 1."""
+    dims: int
+    base: float
+    factor: Optional[float] = None
+    original: float = 4096
+    fast: float = 32.0
+    slow: float = 1.0
+
+    def frequencies(self) -> torch.Tensor:
+        i = torch.arange(self.dims // 2, dtype=torch.float64)
+        f = self.base ** (-2.0 * i / self.dims)
+        if self.factor is None:
+            return f
+
+        def dim_of(turns):
+            return (self.dims * math.log(self.original / (2 * math.pi * turns))
+                    / (2 * math.log(self.base)))
+
+        lo = max(math.floor(dim_of(self.fast)), 0)
+        hi = min(math.ceil(dim_of(self.slow)), self.dims - 1)
+        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        return f / self.factor * ramp + f * (1.0 - ramp)
+
+    @property
+    def magnitude(self) -> float:
+        return 1.0 if self.factor is None else 0.1 * math.log(self.factor) + 1.0
+
+    def tables(self, n: int, device):
+        """cos, sin [n, dims / 2], fp32."""
+        a = torch.arange(n, dtype=torch.float64)[:, None] * self.frequencies()
+        return ((torch.cos(a) * self.magnitude).float().to(device).contiguous(),
+                (torch.sin(a) * self.magnitude).float().to(device).contiguous())
+
+
+# ---------------------------------------------------------------------------
+# Latent attention
+# ---------------------------------------------------------------------------
+
+def _pad(n: int, to: int) -> int:
+    return (n + to - 1) // to * to
+
+
+@dataclass(frozen=True)
+class LatentShape:
+    """Sizes of a latent-attention layer, and how they are padded: what the
+    kernels see are multiples of their tiles, filled with zeros."""
+    heads: int
+    dim: int
+    rot: int
+    vdim: int
+    rank: int
+    f32: bool = False
+
+    @property
+    def dimp(self):
+        return _pad(self.dim, 32)
+
+    @property
+    def rotp(self):
+        return _pad(self.rot, 32)
+
+    @property
+    def dq(self):
+        return self.dimp + self.rotp
+
+    @property
+    def rankp(self):
+        p = 64
+        while p < self.rank:
+            p *= 2
+        return p
+
+    @property
+    def width(self):
+        """Elements of a cached row."""
+        return self.rankp + self.rotp
+
+    @property
+    def vdp(self):
+        for p in ((64, 256) if self.f32 else (32, 64, 128, 256)):
+            if self.vdim <= p:
+                return p
+        return _pad(self.vdim, 16)
+
+    @property
+    def expandable(self) -> bool:
+        """Whether the expanded kernel has this head shape; otherwise every
+        portion takes the absorbed one."""
+        return self.dq <= 256 and self.vdim <= 256
+
+
+def latent_append(dkv, norm_w, eps: float, store: LayerStore, q, sh: LatentShape,
+                  cos, sin, batch: RaggedBatch):
+    """Rotate the queries [N, heads * dq] in place and, unless dkv is None (the
+    layer reads another layer's rows), write this batch's latent rows."""
+    if q.is_cuda:
+        _ext("latent_append").latent_append(
+            dkv, norm_w, eps, store.rows, q, sh.heads, sh.dq, sh.dimp, sh.rank,
+            sh.rankp, sh.rot, sh.rotp, cos, sin, batch.tok_pos,
+            batch.tok_entry, batch.pages)
+        return
+    pos = batch.tok_pos.long()
+    c, s = cos[pos], sin[pos]
+
+    def turn(x, c, s):
+        u, v = x[..., 0::2].float(), x[..., 1::2].float()
+        return torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2).to(x.dtype)
+
+    qh = q.view(q.shape[0], -1)[:, : sh.heads * sh.dq].unflatten(1, (sh.heads, sh.dq))
+    part = qh[..., sh.dimp: sh.dimp + sh.rot]
+    part.copy_(turn(part, c[:, None], s[:, None]))
+    if dkv is None:
+        return
+    pages = batch.pages[batch.tok_entry.long(), pos // PAGE].long()
+    row = torch.zeros(q.shape[0], sh.width, dtype=store.rows.dtype)
+    row[:, : sh.rank] = (_rms(dkv[:, : sh.rank].float(), eps)
+                         * norm_w.float()).to(row.dtype)
+    row[:, sh.rankp: sh.rankp + sh.rot] = turn(
+        dkv[:, sh.rank: sh.rank + sh.rot], c, s).to(row.dtype)
+    store.rows[pages * PAGE + pos % PAGE] = row
+
+
+def latent_attention_absorbed(q, q_abs, store: LayerStore, sh: LatentShape,
+                              scale: float, batch: RaggedBatch, n_req: int,
+                              max_len: int):
+    """Attention of the first n_req requests over the cached rows themselves.
+    q_abs [heads, tokens, rankp]; returns the same shape."""
+    if q.is_cuda:
+        return _ext("latent_attn_short").latent_attn_short(
+            q_abs, q, store.rows, batch.cu, batch.pos0, batch.pages, n_req,
+            max_len, batch.max_keys, sh.dq, sh.dimp, sh.rotp, scale)
+    out = torch.zeros_like(q_abs)
+    for t0, n, p0, held in batch.host[:n_req]:
+        rows = _gather_rows(store, held, p0 + n)
+        qr = q[t0: t0 + n, : sh.heads * sh.dq].unflatten(1, (sh.heads, sh.dq))
+        qf = torch.cat([q_abs[:, t0: t0 + n].float(),
+                        qr[..., sh.dimp:].transpose(0, 1).float()], -1)
+        s = (qf @ rows.float().T) * scale
+        dead = torch.arange(p0 + n)[None, :] > torch.arange(p0, p0 + n)[:, None]
+        p = torch.softmax(s.masked_fill(dead, float("-inf")), -1)
+        out[:, t0: t0 + n] = (p @ rows[:, : sh.rankp].float()).to(out.dtype)
+    return out
+
+
+def _gather_rows(store: LayerStore, held, n: int) -> torch.Tensor:
+    pages = torch.tensor(held.pages, dtype=torch.long)
+    idx = (pages[:, None] * PAGE + torch.arange(PAGE)[None, :]).reshape(-1)[:n]
+    return store.rows[idx]
+
+
+def latent_attention_expanded(q, store: LayerStore, w_uk, w_uv, sh: LatentShape,
+                              scale: float, batch: RaggedBatch):
+    """Attention of the long portions: keys and values of their whole prefix
+    are expanded from the gathered rows.  w_uk [heads * dimp, rankp], w_uv
+    [heads * vdp, rankp]; returns [long tokens, heads * vdp]."""
+    if q.is_cuda:
+        ext = _ext("latent_attn_long")
+        lat = ext.latent_gather(store.rows, batch.blocks, batch.key_rows)
+        c = lat[:, : sh.rankp]
+        kx = F.linear(c, w_uk)
+        vt = F.linear(w_uv, c)  # already transposed: [heads * vdp, keys]
+        return ext.latent_attn_long(
+            q, kx, lat, vt, batch.tiles, batch.cu, batch.pos0, batch.cuk,
+            batch.n_short, batch.short_tokens, sh.heads, sh.dimp, sh.rotp,
+            scale)
+    base = batch.short_tokens
+    out = q.new_zeros(batch.n_tokens - base, sh.heads * sh.vdp)
+    for t0, n, p0, held in batch.host[batch.n_short:]:
+        rows = _gather_rows(store, held, p0 + n).float()
+        c = rows[:, : sh.rankp]
+        k = (c @ w_uk.float().T).unflatten(1, (sh.heads, sh.dimp))
+        v = (c @ w_uv.float().T).unflatten(1, (sh.heads, sh.vdp))
+        qh = q[t0: t0 + n, : sh.heads * sh.dq].unflatten(1, (sh.heads, sh.dq)).float()
+        s = torch.matmul(qh[..., : sh.dimp].transpose(0, 1), k.permute(1, 2, 0))
+        s = s + torch.matmul(qh[..., sh.dimp:].transpose(0, 1), rows[:, sh.rankp:].T)
+        dead = torch.arange(p0 + n)[None, :] > torch.arange(p0, p0 + n)[:, None]
+        p = torch.softmax((s * scale).masked_fill(dead, float("-inf")), -1)
+        o = torch.matmul(p, v.transpose(0, 1)).transpose(0, 1)
+        out[t0 - base: t0 - base + n] = o.flatten(1).to(out.dtype)
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Gated delta rule
+# ---------------------------------------------------------------------------
+
+@dataclass(frozen=True)
+class DeltaShape:
+    """Sizes of a gated-delta layer and the columns of its projection row
+    [q | k | v | gate | decay | beta]."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+
+    @property
+    def widths(self) -> List[int]:
+        k, v = self.kv_heads * self.dim, self.heads * self.vdim
+        return [k, k, v, v, self.heads, self.heads]
+
+    @property
+    def columns(self) -> List[int]:
+        out, at = [], 0
+        for w in self.widths:
+            out.append(at)
+            at += w
+        return out
+
+    @property
+    def channels(self) -> int:
+        """Channels behind a short convolution: q, k and v."""
+        return sum(self.widths[:3])
+
+
+def gated_delta(y, conv_w, A_log, dt_bias, norm_w, store: LayerStore,
+                sh: DeltaShape, eps: float, batch: RaggedBatch):
+    """Projection rows y [N, sum(widths)] -> [N, heads * vdim]; state and
+    convolution inputs of every request move on."""
+    if y.is_cuda:
+        ext = _ext("gated_delta")
+        out = torch.empty(y.shape[0], sh.heads * sh.vdim, dtype=y.dtype,
+                          device=y.device)
+        sizes = (sh.kv_heads, sh.heads, sh.dim, sh.vdim, sh.columns, eps)
+        if batch.n_short:
+            ext.delta_short(y, conv_w, A_log, dt_bias, norm_w, store.state,
+                            store.conv, out, batch.cu, batch.pos0, batch.slots,
+                            batch.n_short, batch.max_short, *sizes)
+        if batch.n_long:
+            ext.delta_long(y, conv_w, A_log, dt_bias, norm_w, store.state,
+                           store.conv, out, batch.cu, batch.pos0, batch.slots,
+                           batch.tok_entry, batch.chunks, batch.chunk_cu,
+                           batch.n_short, batch.n_long, batch.short_tokens,
+                           *sizes)
+        return out
+    out = y.new_empty(y.shape[0], sh.heads * sh.vdim)
+    for t0, n, p0, held in batch.host:
+        out[t0: t0 + n] = _gated_delta_request(
+            y[t0: t0 + n], conv_w, A_log, dt_bias, norm_w, store, held.slot,
+            p0 == 0, sh, eps)
+    return out
+
+
+def _gated_delta_request(y, conv_w, A_log, dt_bias, norm_w, store, slot: int,
+                         fresh: bool, sh: DeltaShape, eps: float):
+    n, hist = y.shape[0], sh.taps - 1
+    H, KH, D, V = sh.heads, sh.kv_heads, sh.dim, sh.vdim
+    old = torch.zeros_like(store.conv[slot]) if fresh else store.conv[slot]
+    x = torch.cat([old, y[:, : sh.channels].T], 1)       # [C, hist + n]
+    store.conv[slot] = x[:, n:]
+    z = F.silu((x.float().unfold(1, sh.taps, 1) * conv_w.float()[:, None, :]).sum(-1)).T
+    q, k, v = z.split(sh.widths[:3], 1)
+    gate, a, b = y[:, sh.channels:].float().split(sh.widths[3:], 1)
+
+    def unit(t):
+        t = t.reshape(n, KH, D)
+        t = t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)
+        return t.repeat_interleave(H // KH, 1)
+
+    q, k, v = unit(q) * D ** -0.5, unit(k), v.reshape(n, H, V)
+    g = torch.exp(-torch.exp(A_log.float()) * F.softplus(a + dt_bias.float()))
+    beta = torch.sigmoid(b)
+    S = torch.zeros_like(store.state[slot]) if fresh else store.state[slot].clone()
+    o = torch.empty(n, H, V)
+    for t in range(n):
+        S *= g[t][:, None, None]
+        u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+        S += k[t][:, :, None] * u[:, None, :]
+        o[t] = torch.einsum("hdv,hd->hv", S, q[t])
+    store.state[slot] = S
+    o = _rms(o, eps) * norm_w.float() * F.silu(gate).reshape(n, H, V)
+    return o.reshape(n, H * V).to(y.dtype)

@@ -42,6 +42,69 @@ class SamplingParams:
     max_tokens: Optional[int] = None
 
 
+class Sampler:
+    """Token choice of one generation: logit bias, repetition penalty over the
+    recent context, temperature / top-p, with a generator of its own if seeded.
+    """
+
+    def __init__(self, params: SamplingParams, context: Iterable[int]):
+        self.params = params
+        self.context: List[int] = list(context)
+        self.gen = None
+        if params.seed is not None:
+            self.gen = torch.Generator(device="cpu").manual_seed(params.seed)
+
+    @property
+    def plain(self) -> bool:
+        """Greedy on the logits as they are."""
+        p = self.params
+        return (p.temperature <= 0.0 and not p.logit_bias
+                and p.repetition_penalty in (None, 0, 1.0))
+
+    def adjust(self, logits: torch.Tensor) -> torch.Tensor:
+        """logits [1, V] with bias and penalty applied."""
+        p, device = self.params, logits.device
+        if p.logit_bias:
+            idx = torch.tensor(list(p.logit_bias.keys()), device=device)
+            vals = torch.tensor(list(p.logit_bias.values()), device=device,
+                                dtype=logits.dtype)
+            logits[0, idx] += vals
+        if p.repetition_penalty and p.repetition_penalty != 1.0:
+            window = self.context[-p.repetition_context_size:] \
+                if p.repetition_context_size else self.context
+            ctx = torch.tensor(window, device=device, dtype=torch.long)
+            logits = ops.apply_repetition_penalty(logits, ctx,
+                                                  p.repetition_penalty)
+        return logits
+
+    def sample(self, logits: torch.Tensor) -> torch.Tensor:
+        """[1, V] adjusted logits -> [1] token, still on the device."""
+        return ops.sample(logits, self.params.temperature, self.params.top_p,
+                          self.gen)
+
+    @staticmethod
+    def draw_all(samplers: List["Sampler"], logits: torch.Tensor
+                 ) -> List[Tuple[int, torch.Tensor]]:
+        """One token per sampler from logits [n, V]; returns (token, logprobs).
+        Plain greedy rows are chosen together."""
+        if not samplers:
+            return []
+        if all(s.plain for s in samplers):
+            toks = logits.argmax(-1).tolist()
+        else:
+            logits = logits.clone()
+            toks = []
+            for i, s in enumerate(samplers):
+                row = s.adjust(logits[i: i + 1])
+                logits[i] = row[0]
+                # a seeded draw uses the host generator
+                toks.append(int(s.sample(row.cpu() if s.gen is not None else row)))
+        logprobs = torch.log_softmax(logits, -1)
+        for s, t in zip(samplers, toks):
+            s.context.append(t)
+        return [(t, logprobs[i]) for i, t in enumerate(toks)]
+
+
 def generate_step(
     prompt_ids: torch.Tensor,
     model: StageModel,
@@ -82,11 +145,7 @@ def generate_step(
     for r in remotes:
         r.reset_cache()
     device = prompt_ids.device
-    gen = None
-    if params.seed is not None:
-        gen = torch.Generator(device="cpu").manual_seed(params.seed)
-
-    rep_context: List[int] = prompt_ids[0].tolist()
+    sampler = Sampler(params, prompt_ids[0].tolist())
 
     def _forward(y):
         h = model(y, cache)
@@ -102,20 +161,9 @@ def generate_step(
         else:
             h = _forward(fresh)
         while True:
-            logits = h[:, -1, :].float()
-            if params.logit_bias:
-                idx = torch.tensor(list(params.logit_bias.keys()), device=device)
-                vals = torch.tensor(list(params.logit_bias.values()),
-                                    device=device, dtype=logits.dtype)
-                logits[0, idx] += vals
-            if params.repetition_penalty and params.repetition_penalty != 1.0:
-                window = rep_context[-params.repetition_context_size:] \
-                    if params.repetition_context_size else rep_context
-                ctx = torch.tensor(window, device=device, dtype=torch.long)
-                logits = ops.apply_repetition_penalty(
-                    logits, ctx, params.repetition_penalty)
+            logits = sampler.adjust(h[:, -1, :].float())
             logprobs = logits - torch.logsumexp(logits, dim=-1, keepdim=True)
-            tok = ops.sample(logits, params.temperature, params.top_p, gen)
+            tok = sampler.sample(logits)
             # one-step lookahead (the reference's mx.async_eval,
             # generate.py:82-88): enqueue the NEXT forward before the
             # host sync on .item(), hiding its launch latency behind
@@ -123,8 +171,21 @@ def generate_step(
             # wasted compute, exactly as in the reference.
             h = _forward(tok.reshape(-1, 1))
             tid = int(tok.item())
-            rep_context.append(tid)
+            sampler.context.append(tid)
             yield tid, logprobs[0]
+
+
+def batched_generate_step(prompt_ids: torch.Tensor, model: StageModel,
+                          params: Optional[SamplingParams], max_tokens: int,
+                          prefill_chunk: int = 0
+                          ) -> Generator[Tuple[int, torch.Tensor], None, None]:
+    """generate_step for a model that runs ragged batches: one request through
+    the batch scheduler, ending by itself after ``max_tokens``."""
+    from .batching import PAGE, BatchEngine, BatchScheduler
+    need = prompt_ids.shape[1] + max_tokens
+    engine = BatchEngine(model, (need + PAGE - 1) // PAGE * PAGE, 1)
+    sched = BatchScheduler(engine, prefill_chunk or 2048)
+    return sched.generate(sched.submit(prompt_ids[0].tolist(), params, max_tokens))
 
 
 @dataclass
@@ -150,12 +211,17 @@ def stream_generate(
     (prompt TPS = prompt_tokens / time-to-first-token; gen TPS =
     (n-1)/decode_time — /root/reference/generate.py:103-122)."""
     eos = set(int(e) for e in eos_token_ids)
-    cache = model.make_cache(batch_size=prompt_ids.shape[0])
+    remotes = list(remotes)
     t0 = time.perf_counter()
     n = 0
     t_first = t0
-    for tid, logprobs in generate_step(prompt_ids, model, cache, remotes,
-                                       params, wire_fp16):
+    if model.supports_ragged and not remotes and prompt_ids.shape[0] == 1:
+        tokens = batched_generate_step(prompt_ids, model, params, max_tokens)
+    else:
+        tokens = generate_step(prompt_ids, model,
+                               model.make_cache(batch_size=prompt_ids.shape[0]),
+                               remotes, params, wire_fp16)
+    for tid, logprobs in tokens:
         if n == 0:
             t_first = time.perf_counter()
         n += 1
@@ -185,7 +251,7 @@ class LocalChain:
                     device: str = "cpu") -> torch.Tensor:
         if wire_fp16 and t.dtype == torch.bfloat16:
             t = t.to(torch.float16)
-        x = t.to(self.model.fp_dtype) if t.is_floating_point() else t
+        x = t.to(self.model.hop_dtype) if t.is_floating_point() else t
         if self.cache is None or (self.cache and self.cache[0].batch_size != x.shape[0]):
             self.cache = self.model.make_cache(batch_size=x.shape[0])
         with torch.no_grad():

@@ -30,8 +30,22 @@ from ..models.base import StageModel
 from ..ops.kvcache import KVCache
 
 
-def split_layers(n_layers: int, n_stages: int) -> List[Tuple[int, int]]:
-    """Balanced contiguous split; earlier stages get the remainder."""
+def split_layers(n_layers: int, n_stages: int,
+                 allowed: Optional[List[int]] = None) -> List[Tuple[int, int]]:
+    """Balanced contiguous split; earlier stages get the remainder.
+    ``allowed``: the layers a later stage may begin at (None: any); cuts move
+    to the nearest allowed one."""
+    if allowed is not None:
+        if n_stages - 1 > len(allowed):
+            raise ValueError(f"{n_layers} layers allow at most "
+                             f"{len(allowed) + 1} stages, not {n_stages}")
+        cuts, lo = [], 0
+        for k, (s, _) in enumerate(split_layers(n_layers, n_stages)[1:], 1):
+            hi = len(allowed) - (n_stages - 1 - k)  # leave one per later stage
+            j = min(range(lo, hi), key=lambda i: abs(allowed[i] - s))
+            cuts.append(allowed[j])
+            lo = j + 1
+        return list(zip([0, *cuts], [*cuts, n_layers]))
     base = n_layers // n_stages
     rem = n_layers % n_stages
     out = []
@@ -60,7 +74,8 @@ class PipelineWorker:
         self.rank = rank
         self.world = world
         self.device = device
-        self.dtype = dtype
+        # hidden states and shipped logits travel in the model's hop type
+        self.dtype = dtype if model.hop_dtype == model.fp_dtype else model.hop_dtype
         self.group = group
         self.hidden = model.config.hidden_size
         self.caches: List[List[KVCache]] = []  # per micro-batch
@@ -316,9 +331,10 @@ def build_stage_model(config: ModelConfig, rank: int, world: int,
                       device: torch.device, seed: int = 0,
                       quant_for=None) -> StageModel:
     """Random-init one stage (synthetic-weights path for bench/tests)."""
-    ranges = split_layers(config.num_hidden_layers, world)
-    s, e = ranges[rank]
     cls = get_model_class(config.model_type)
+    ranges = split_layers(config.num_hidden_layers, world,
+                          cls.allowed_cuts(config))
+    s, e = ranges[rank]
     torch.manual_seed(seed)
     with torch.device(device):  # allocate directly on-device (big models)
         model = cls(config, config.shard(s, e), quant_for=quant_for)
@@ -409,6 +425,8 @@ class CapturedDecode:
             # warmup on a side stream (hipblaslt workspaces etc.); the two
             # garbage steps write cache slots off/off+1 — rewind pos and the
             # real steps overwrite them before they are ever attended to.
+            # a recurrent state cannot be rewound by position: keep and restore
+            kept = [c.snapshot() for c in caches]
             s = torch.cuda.Stream()
             s.wait_stream(torch.cuda.current_stream())
             with torch.cuda.stream(s):
@@ -416,6 +434,8 @@ class CapturedDecode:
                     step_fn()
             torch.cuda.current_stream().wait_stream(s)
             pos.fill_(off)
+            for c, snap in zip(caches, kept):
+                c.restore(snap)
             torch.cuda.synchronize()
 
             g = torch.cuda.CUDAGraph()

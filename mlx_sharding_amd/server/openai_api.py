@@ -29,6 +29,7 @@ from typing import List, Optional, Tuple
 
 import torch
 
+from ..parallel.batching import BatchEngine, BatchScheduler, BatchService
 from ..parallel.engine import SamplingParams, generate_step
 from ..parallel.grpc_transport import make_clients
 from ..utils import metrics
@@ -104,6 +105,8 @@ class ModelProvider:
         # shares a prefix re-uses those K/V rows (take/store under the
         # lock — a concurrent second request simply runs fresh)
         self._prefix_state: Optional[Tuple[List[int], list]] = None
+        # continuous batching, for models that run ragged batches
+        self.service: Optional[BatchService] = None
         if cli_args.model is not None:
             self.load("default_model")
 
@@ -129,6 +132,9 @@ class ModelProvider:
             self.tokenizer = None
             self.model_key = None
             self._prefix_state = None  # caches belong to the old model
+            if self.service is not None:
+                self.service.stop()
+                self.service = None
             if model_path in ("default_model", None):
                 path = self.args.model
             else:
@@ -153,6 +159,13 @@ class ModelProvider:
             self.model_key = model_path
             self.model = model
             self.tokenizer = tokenizer
+            if (model.supports_ragged and not self.remotes
+                    and model.shard.is_first and model.shard.is_last):
+                engine = BatchEngine(
+                    model, int(os.environ.get("MLXS_BATCH_TOKENS", "65536")),
+                    int(os.environ.get("MLXS_BATCH_REQUESTS", "32")))
+                chunk = int(os.environ.get("MLXS_PREFILL_CHUNK", "0"))
+                self.service = BatchService(BatchScheduler(engine, chunk or 2048))
             return self.model, self.tokenizer
 
 
@@ -329,6 +342,8 @@ class APIHandler(BaseHTTPRequestHandler):
         device = next(model.parameters()).device
         ids = torch.tensor([prompt_ids], device=device)
         chunk = int(os.environ.get("MLXS_PREFILL_CHUNK", "0"))
+        if getattr(self.provider, "service", None) is not None:
+            return self.provider.service.generate(list(prompt_ids), sp)
         use_prefix = (os.environ.get("MLXS_PREFIX_CACHE") == "1"
                       and not self.provider.remotes)
         cache = None
@@ -342,7 +357,7 @@ class APIHandler(BaseHTTPRequestHandler):
                 while p < limit and prev[p] == prompt_ids[p]:
                     p += 1
                 p = min(p, len(prompt_ids) - 1)  # must prefill >= 1 token
-                if p > 0:
+                if p > 0 and prev_cache[0].trimmable:
                     for c in prev_cache:
                         c.trim(p)
                     cache = prev_cache

@@ -27,7 +27,7 @@ class ShardWorker:
         self.model = model
         self.cache: Optional[List[KVCache]] = None
         self._device = next(model.parameters()).device
-        self._dtype = model.fp_dtype  # NOT first-param dtype: that can
+        self._dtype = model.hop_dtype  # NOT first-param dtype: that can
         #                               be a packed uint32 quant weight
         # per-stage HIP-event timing (SURVEY.md §5.1 — the reference has
         # only print statements, server.py:29-37); summary() is cheap and

@@ -154,9 +154,12 @@ def load_model(model_path: str | Path,
         bits, gs = quantize
         quantize_weights(weights, config, group_size=gs, bits=bits)
     cls = get_model_class(config.model_type)
+    if config.quantization is not None and not cls.supports_quantization:
+        raise ValueError(f"{config.model_type} has no quantized weights")
     quant_for = make_quant_predicate(config, weights)
     model = cls(config, shard, quant_for=quant_for)
     if dtype is not None:
+        model.to(dtype)
         for k in list(weights):
             if weights[k].is_floating_point():
                 weights[k] = weights[k].to(dtype)
@@ -206,8 +209,14 @@ def save_sharded_weights(model_path: str | Path, output_dir: str | Path,
     total = config.num_hidden_layers
     weights = load_weights(model_path)
     embed_on_last = config.model_type == "gemma2"  # tied head on last shard
-    kept = {k: v for k, v in weights.items()
-            if _route_key(k, start_layer, end_layer, total, embed_on_last)}
+    cls = get_model_class(config.model_type)
+    if cls.owns_key.__func__ is StageModel.owns_key.__func__ or embed_on_last:
+        mine = lambda k: _route_key(k, start_layer, end_layer, total,  # noqa: E731
+                                    embed_on_last)
+    else:  # designs with tensor names of their own
+        shard = config.shard(start_layer, end_layer)
+        mine = lambda k: cls.owns_key(k, shard)  # noqa: E731
+    kept = {k: v for k, v in weights.items() if mine(k)}
     shard_name = f"model-{start_layer:05d}-{end_layer:05d}.safetensors"
     save_file(kept, str(output_dir / shard_name), metadata={"format": "mlx"})
 

@@ -21,28 +21,34 @@ HIP_DIR = ROOT / "mlx_sharding_amd" / "ops" / "hip"
 # of ordinary float code are kept out of every kernel
 NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
+# extension -> its sources; MLXS_AMD_EXT=name[,name] builds only those
+# (bin/trace_run builds just what its model loads)
+SOURCES = {
+    "_hip_ragged": lambda name: name.startswith("ragged_") or name == "elementwise.hip",
+    "_hip_ops": lambda name: not name.startswith("ragged_"),
+}
+
 ext_modules = []
 cmdclass = {}
-hip_sources = sorted(str(p) for p in HIP_DIR.glob("*.hip") if not p.name.endswith("_hip.hip")) + \
-    sorted(str(p) for p in HIP_DIR.glob("*.cpp"))
+hip_sources = sorted(p for p in HIP_DIR.glob("*.hip") if not p.name.endswith("_hip.hip"))
 if hip_sources and os.environ.get("MLXS_AMD_SKIP_EXT", "0") != "1":
     try:
         from torch.utils.cpp_extension import BuildExtension, CUDAExtension
 
         os.environ.setdefault("PYTORCH_ROCM_ARCH", "gfx950")
-        ext_modules = [
-            CUDAExtension(
-                name="mlx_sharding_amd._hip_ops",
-                sources=hip_sources,
+        wanted = [n for n in os.environ.get("MLXS_AMD_EXT", "").split(",") if n]
+        for ext_name in wanted or sorted(SOURCES):
+            ext_modules.append(CUDAExtension(
+                name=f"mlx_sharding_amd.{ext_name}",
+                sources=[str(p) for p in hip_sources if SOURCES[ext_name](p.name)],
                 extra_compile_args={
                     "cxx": ["-O3", "-std=c++17"],
                     "nvcc": ["-O3", "-std=c++17", "--offload-arch=gfx950",
                              *NO_PACKED_FP32],
                 },
-            )
-        ]
+            ))
         cmdclass = {"build_ext": BuildExtension}
-    except Exception:  # torch missing at sdist time
+    except ImportError:  # torch missing at sdist time
         pass
 
 setup(
