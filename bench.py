@@ -50,6 +50,12 @@ def parse_args():
                    help="disable hipGraph-captured decode (debugging)")
     p.add_argument("--graph", action="store_true",
                    help="force hipGraph decode even at large batch")
+    p.add_argument("--layers", nargs="?", const="all", default=None,
+                   metavar="SIZE",
+                   help="instead of the serving benchmark: prefill and decode "
+                        "throughput of Tuvutar layers beside DeepSeek-V2's "
+                        "dense latent-attention layers of equal size, one JSON "
+                        "line per case (2048, 4096 or all)")
     return p.parse_args()
 
 
@@ -58,6 +64,9 @@ def main():
     import sys
 
     args = parse_args()
+    if args.layers is not None:
+        from mlx_sharding_amd.utils.layer_bench import run
+        return run(args.layers, steps=min(args.steps, 32))
     if args.quant is None:
         args.quant = "deepseek" in args.model
 

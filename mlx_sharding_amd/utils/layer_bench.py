@@ -1,0 +1,97 @@
+"""Prefill and decode throughput of layer stacks at real sizes (random weights).
+
+Stacks of four layers of one kind with equal width, heads, head sizes, latent
+size and feed-forward, so that their times compare directly:
+
+  mla     DeepSeek-V2 latent attention + dense MLP (the closest existing model)
+  latent  Tuvutar latent attention
+  shared  Tuvutar latent attention, three of four layers on shared rows
+  delta   Tuvutar gated delta rule
+  mixed   Tuvutar delta, delta, delta, latent
+
+All run the pipeline worker's own prefill and graph-captured decode step.
+"""
+
+from __future__ import annotations
+
+import json
+import time
+from typing import Dict
+
+import torch
+
+from ..config import ModelConfig
+from ..parallel.rccl import PipelineWorker, build_stage_model
+from .presets import _dense_mla, _tuvutar
+
+SIZES: Dict[str, dict] = {
+    "2048": dict(width=2048, heads=16, ff=8192, vocab=8192),
+    "4096": dict(width=4096, heads=32, ff=14336, vocab=8192),
+}
+KINDS = {"latent": "aaaa", "shared": "asss", "delta": "dddd", "mixed": "ddda"}
+PREFILL = ((1, 8192), (8, 1024))     # sequences, tokens each
+DECODE = ((1, 2048), (64, 2048))     # sequences, tokens cached
+
+
+def stack(kind: str, size: dict) -> ModelConfig:
+    if kind == "mla":
+        return ModelConfig.from_dict(_dense_mla(n_layers=4, **size))
+    extra = {}
+    if "d" in KINDS[kind]:
+        extra = dict(delta_heads=size["heads"], delta_kv=size["heads"] // 2)
+    return ModelConfig.from_dict(
+        _tuvutar(period=KINDS[kind], repeats=1, **size, **extra))
+
+
+def _time(fn, n: int) -> float:
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(n):
+        fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / n
+
+
+def run(which: str = "all", steps: int = 32, kinds=("mla", *KINDS)):
+    if not torch.cuda.is_available():
+        raise SystemExit("--layers needs a GPU")
+    device = torch.device("cuda", 0)
+    torch.manual_seed(0)
+    for name in (SIZES if which == "all" else [which]):
+        for kind in kinds:
+            config = stack(kind, SIZES[name])
+            model = build_stage_model(config, 0, 1, device)
+
+            def emit(phase, batch, seq, seconds, tokens):
+                print(json.dumps({
+                    "metric": f"{phase} throughput, 4 layers", "kind": kind,
+                    "width": int(name), "batch": batch, "seq_len": seq,
+                    "ms": round(seconds * 1e3, 4),
+                    "value": round(tokens / seconds, 1), "unit": "tokens/s",
+                    "dtype": "bf16", "data": "synthetic"}), flush=True)
+
+            for batch, seq in PREFILL:
+                worker = PipelineWorker(model, 0, 1, device)
+                ids = [torch.randint(0, config.vocab_size, (batch, seq),
+                                     device=device)]
+                fn = lambda: worker.prefill(ids, batch, 1, seq)  # noqa: E731
+                fn(), fn()
+                emit("prefill", batch, seq, _time(fn, 6), batch * seq)
+            for batch, seq in DECODE:
+                worker = PipelineWorker(model, 0, 1, device)
+                ids = [torch.randint(0, config.vocab_size, (batch, seq),
+                                     device=device)]
+                tokens = worker.prefill(ids, batch, 1, seq)
+                for _ in range(2):
+                    tokens = worker.decode_step(tokens, batch, 1)
+                if not worker.enable_graph_decode(tokens, batch, 1,
+                                                  seq + steps + 16):
+                    raise RuntimeError(f"{kind}: decode could not be captured")
+                for _ in range(3):
+                    tokens = worker.decode_step(tokens, batch, 1)
+                emit("decode", batch, seq,
+                     _time(lambda: worker.decode_step(tokens, batch, 1), steps),
+                     batch)
+                del worker
+            del model
+            torch.cuda.empty_cache()

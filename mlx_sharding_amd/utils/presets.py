@@ -6,6 +6,46 @@ from __future__ import annotations
 
 from ..config import ModelConfig
 
+
+def _tuvutar(width: int, heads: int, ff: int, vocab: int, period: str,
+             repeats: int, dim: int = 128, rot: int = 64, rank: int = 512,
+             delta_heads: int = 0, delta_kv: int = 0) -> dict:
+    """A Tuvutar config: ``period`` repeated, "d" a gated-delta layer, "a" a
+    latent-attention layer with rows of its own, "s" one that reads the rows of
+    the latest "a"."""
+    layers, last = [], None
+    for kind in period * repeats:
+        if kind == "d":
+            mixer = {"heads": delta_heads or 2 * heads,
+                     "kv_heads": delta_kv or heads, "dim": 128, "vdim": 128,
+                     "conv": 4}
+        else:
+            mixer = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": dim,
+                     "kv_rank": rank, "scale": (dim + rot) ** -0.5,
+                     "rot": {"base": 10000.0, "dims": rot,
+                             "scaling": {"factor": 8.0, "original": 4096,
+                                         "fast": 32.0, "slow": 1.0}}}
+            if kind == "s":
+                mixer["kv_from"] = last
+            else:
+                last = len(layers)
+        layers.append({"type": "delta" if kind == "d" else "latent_attention",
+                       "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Tuvutar", "width": width, "vocab": vocab,
+            "norm": {"eps": 1e-6}, "layers": layers}
+
+
+def _dense_mla(width: int, heads: int, ff: int, vocab: int, n_layers: int,
+               dim: int = 128, rot: int = 64, rank: int = 512) -> dict:
+    """A DeepSeek-V2 config without experts (latent attention + dense MLP)."""
+    return {"model_type": "deepseek_v2", "hidden_size": width,
+            "num_hidden_layers": n_layers, "intermediate_size": ff,
+            "num_attention_heads": heads, "vocab_size": vocab,
+            "rms_norm_eps": 1e-6, "rope_theta": 10000.0, "q_lora_rank": None,
+            "kv_lora_rank": rank, "qk_nope_head_dim": dim,
+            "qk_rope_head_dim": rot, "v_head_dim": dim}
+
+
 PRESETS = {
     # headline model: DeepSeek-Coder-V2-Lite-Instruct (15.7B total, 2.4B active)
     "deepseek-v2-lite": {
@@ -118,6 +158,33 @@ PRESETS = {
         "vocab_size": 1024,
         "rms_norm_eps": 1e-5,
         "rope_theta": 10000.0,
+    },
+    "tuvutar-2b": _tuvutar(2048, 16, 8192, 32000, "dddadds", 4),
+    "tuvutar-8b": _tuvutar(4096, 32, 14336, 32000, "dddadds", 4,
+                           delta_heads=32, delta_kv=16),
+    "debug-tuvutar": {
+        "architecture": "Tuvutar", "width": 96, "vocab": 320,
+        "norm": {"eps": 1e-6},
+        "layers": [
+            {"type": "delta", "mlp": None,
+             "mixer": {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 40,
+                       "conv": 4}},
+            {"type": "latent_attention", "mlp": {"kind": "dense", "ff": 160},
+             "mixer": {"heads": 3, "dim": 32, "rot_dim": 16, "vdim": 24,
+                       "kv_rank": 48, "scale": 0.14,
+                       "rot": {"base": 10000.0, "dims": 16,
+                               "scaling": {"factor": 4.0, "original": 512,
+                                           "fast": 32.0, "slow": 1.0}}}},
+            {"type": "delta", "mlp": {"kind": "dense", "ff": 128},
+             "mixer": {"heads": 2, "kv_heads": 2, "dim": 16, "vdim": 16,
+                       "conv": 3}},
+            {"type": "latent_attention", "mlp": {"kind": "dense", "ff": 96},
+             "mixer": {"heads": 5, "dim": 16, "rot_dim": 16, "vdim": 32,
+                       "kv_rank": 48, "scale": 0.2, "kv_from": 1,
+                       "rot": {"base": 10000.0, "dims": 16,
+                               "scaling": {"factor": 4.0, "original": 512,
+                                           "fast": 32.0, "slow": 1.0}}}},
+        ],
     },
     "debug-deepseek": {
         "model_type": "deepseek_v2",
