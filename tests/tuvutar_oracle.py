@@ -66,13 +66,13 @@ def rotary_frequencies(rot):
 def rotate(x, rot):
     """x [T, ..., dims]; pairs are neighbours; the row index is the position."""
     f, m = rotary_frequencies(rot)
+    f = torch.tensor(f, dtype=torch.float64)
     y = torch.empty_like(x)
     for p in range(x.shape[0]):
-        for i, fi in enumerate(f):
-            c, s = math.cos(p * fi) * m, math.sin(p * fi) * m
-            u, v = x[p, ..., 2 * i], x[p, ..., 2 * i + 1]
-            y[p, ..., 2 * i] = u * c - v * s
-            y[p, ..., 2 * i + 1] = v * c + u * s
+        c, s = (torch.cos(p * f) * m).to(x.dtype), (torch.sin(p * f) * m).to(x.dtype)
+        u, v = x[p, ..., 0::2], x[p, ..., 1::2]
+        y[p, ..., 0::2] = u * c - v * s
+        y[p, ..., 1::2] = v * c + u * s
     return y
 
 
@@ -92,11 +92,12 @@ def latent_attention(h, w, pre, mx, c, kr):
     k = (c @ w[pre + "uk"].T).reshape(T, H, dim)
     v = (c @ w[pre + "uv"].T).reshape(T, H, vd)
     out = torch.zeros(T, H, vd, dtype=h.dtype)
-    for t in range(T):
-        for a in range(H):
-            s = (k[: t + 1, a] @ qn[t, a] + kr[: t + 1] @ qr[t, a]) * mx["scale"]
-            p = torch.exp(s - s.max())
-            out[t, a] = (p / p.sum()) @ v[: t + 1, a]
+    seen = torch.ones(T, T).tril() > 0      # [query, key]
+    for a in range(H):
+        s = (qn[:, a] @ k[:, a].T + qr[:, a] @ kr.T) * mx["scale"]
+        s = torch.where(seen, s, torch.full_like(s, -math.inf))
+        p = torch.exp(s - s.max(-1, keepdim=True).values)
+        out[:, a] = (p / p.sum(-1, keepdim=True)) @ v[:, a]
     return out.reshape(T, H * vd) @ w[pre + "o"].T
 
 
@@ -104,11 +105,8 @@ def short_conv(x, taps):
     """x [T, C], taps [C, K], the last column meets the current token."""
     T, K = x.shape[0], taps.shape[1]
     y = torch.zeros_like(x)
-    for t in range(T):
-        for j in range(K):
-            s = t - (K - 1) + j
-            if s >= 0:
-                y[t] += taps[:, j] * x[s]
+    for back in range(min(K, T)):           # how many tokens ago
+        y[back:] += taps[:, K - 1 - back] * x[: T - back]
     return y
 
 
@@ -117,13 +115,12 @@ def delta_rule(q, k, v, beta, g):
     T, H, D = q.shape
     V = v.shape[-1]
     o = torch.zeros(T, H, V, dtype=q.dtype)
-    for a in range(H):
-        S = torch.zeros(D, V, dtype=q.dtype)
-        for t in range(T):
-            S = g[t, a] * S
-            u = beta[t, a] * (v[t, a] - S.T @ k[t, a])
-            S = S + torch.outer(k[t, a], u)
-            o[t, a] = S.T @ q[t, a]
+    S = torch.zeros(H, D, V, dtype=q.dtype)
+    for t in range(T):
+        S = g[t, :, None, None] * S
+        u = beta[t, :, None] * (v[t] - (S * k[t, :, :, None]).sum(1))
+        S = S + k[t, :, :, None] * u[:, None, :]
+        o[t] = (S * q[t, :, :, None]).sum(1)
     return o
 
 
