@@ -105,6 +105,7 @@ class StageModel(nn.Module):
         self.shard = shard
         self._rt_len = 0
         self._rt_dev = None
+        self._rt_old: List[Tuple[torch.Tensor, torch.Tensor]] = []
 
     # -- RoPE tables -------------------------------------------------------
     def _rope_tables(self, device, min_len: int):
@@ -112,6 +113,8 @@ class StageModel(nn.Module):
         no per-element trig on device); grown lazily, device-resident."""
         if self._rt_len < min_len or self._rt_dev != device:
             n = max(1024, 1 << max(int(min_len) - 1, 1).bit_length())
+            if self._rt_len:  # captured graphs may still read the old ones
+                self._rt_old.append((self._rt_cos, self._rt_sin))
             pos = torch.arange(n, device=device)
             inv = self.rope_inv_freq.to(device)
             from .. import ops as _ops

@@ -101,6 +101,7 @@ class TuvutarStageModel(StageModel):
             self.final.norm = RMSNorm(W, self.eps, NORM_OFFSET, dtype)
             self.head = Linear(W, config.vocab_size, dtype=dtype)
         self._tables: Dict = {}
+        self._old_tables: List = []  # captured graphs may still read them
 
     # -- layers ------------------------------------------------------------
     def layer(self, i: int) -> TuvutarLayer:
@@ -165,6 +166,8 @@ class TuvutarStageModel(StageModel):
     def _rotation(self, rotary: Rotary, n: int, device):
         got = self._tables.get(rotary)
         if got is None or got[0].shape[0] < n or got[0].device != device:
+            if got is not None:
+                self._old_tables.append(got)
             rows = max(1024, 1 << max(n - 1, 1).bit_length())
             got = self._tables[rotary] = rotary.tables(rows, device)
         return got

@@ -328,7 +328,7 @@ DeltaDims delta_dims(const Tensor& y, const Tensor& conv_w, int64_t KH,
   d.V = (int)V;
   d.taps = (int)conv_w.size(1);
   TORCH_CHECK(d.taps >= 1 && d.taps <= 8, "convolutions have 1 to 8 taps");
-  TORCH_CHECK(D <= 512 && delta_short_rows((int)D, (int)V, 512) > 0,
+  TORCH_CHECK(D <= 512 && V <= 512 && delta_short_rows((int)D, (int)V, 512) > 0,
               "state of a head is too large: ", D, " x ", V);
   const int64_t w[6] = {KH * D, KH * D, H * V, H * V, H, H};
   for (int i = 0; i < 6; ++i)
@@ -397,7 +397,11 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
   if (n <= 0 || n_long == 0) return;
   TORCH_CHECK(chunks.dim() == 2 && chunks.size(1) == 2);
   const long nc = chunks.size(0);
-  const long Dp = (D + 15) / 16 * 16, Vp = (V + 15) / 16 * 16;
+  // depths 16 * 2^k take the walk with a fixed depth
+  long Dp = 16;
+  while (Dp < D) Dp *= 2;
+  if (Dp > 128) Dp = (D + 15) / 16 * 16;
+  const long Vp = (V + 15) / 16 * 16;
   auto fo = y.options().dtype(torch::kFloat32);
   auto qn = torch::empty({n, KH, Dp}, fo), kn = torch::empty({n, KH, Dp}, fo);
   auto vn = torch::empty({n, H, Vp}, y.options());

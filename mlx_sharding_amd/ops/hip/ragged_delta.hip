@@ -72,6 +72,23 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
   float* red = vb + (long)n * V;               // [2][DG][VT]
   float* scratch = red + 2 * NT;               // [NT / WAVE]
 
+  const int v = tid & (VT - 1);
+  const int dg = tid / VT;
+  const int d0 = dg * RPT;
+  const int rep = dm.H / dm.KH;
+  // this thread's part of a head's state; asked for as early as possible
+  float S[RPT];
+  auto state_of = [&](int h) {
+    return state + ((slot * dm.H + h) * (long)D + d0) * V + v;
+  };
+  auto load_state = [&](int h) {
+    const float* sp = state_of(h);
+#pragma unroll
+    for (int i = 0; i < RPT; ++i)
+      S[i] = (!fresh && v < V && d0 + i < D) ? sp[(long)i * V] : 0.0f;
+  };
+  load_state(kh * rep);
+
   // convolution + silu of channel c (column col of y) for all n tokens
   auto convolve = [&](int c, int col, float* dst, int dstep) {
     float w[DR_MAXTAPS], x[DR_MAXTAPS];
@@ -123,20 +140,11 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
     if (lane == 0) kq[t] = a;
   }
 
-  const int v = tid & (VT - 1);
-  const int dg = tid / VT;
-  const int d0 = dg * RPT;
-  const int rep = dm.H / dm.KH;
   for (int hh = 0; hh < rep; ++hh) {
     const int h = kh * rep + hh;
     __syncthreads();
     for (int i = tid; i < V; i += NT)
       convolve(2 * dm.KH * D + h * V + i, dm.vc + h * V + i, vb + i, V);
-    float S[RPT];
-    float* sp = state + ((slot * dm.H + h) * (long)D + d0) * V + v;
-#pragma unroll
-    for (int i = 0; i < RPT; ++i)
-      S[i] = (!fresh && v < V && d0 + i < D) ? sp[(long)i * V] : 0.0f;
     __syncthreads();
     const float Al = (float)A_log[h], dt = (float)dt_bias[h];
     for (int t = 0; t < n; ++t) {
@@ -175,9 +183,11 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
             (T)(o / sqrtf(ss / (float)V + eps) * (float)norm_w[v] * gate);
       }
     }
+    float* sp = state_of(h);
 #pragma unroll
     for (int i = 0; i < RPT; ++i)
       if (v < V && d0 + i < D) sp[(long)i * V] = S[i];
+    if (hh + 1 < rep) load_state(h + 1);
   }
 }
 
@@ -253,14 +263,18 @@ extern "C" void launch_delta_short(const void* y, const void* conv_w,
 
 // ---------------------------------------------------------------------------
 // Long portions, step 1: convolution, silu, unit norms, gates.
-// Block per token.  q, k -> fp32 [n, KH, Dp] (zero padded), v -> T [n, H, Vp],
-// log decay and beta -> fp32 [n, H].
+// q, k -> fp32 [n, KH, Dp] (zero padded), v -> T [n, H, Vp], log decay and
+// beta -> fp32 [n, H].  One wave per (16 tokens of a chunk, piece): a piece is
+// a q or k head, 64 value channels, or the gates.  A lane keeps its channels'
+// inputs of all 16 tokens and their history in registers.
+// NU: q/k channels per lane, D <= 64 * NU.
 // ---------------------------------------------------------------------------
 
 #define DC_BLOCK 256
-#define DC_MAXD 8  // D <= 64 * DC_MAXD
+#define DC_TT 16
+#define DC_SUB (DR_CHUNK / DC_TT)
 
-template <typename T>
+template <typename T, int NU>
 __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
     const T* __restrict__ y, const T* __restrict__ conv_w,
     const T* __restrict__ A_log, const T* __restrict__ dt_bias,
@@ -268,67 +282,103 @@ __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
     float* __restrict__ ko, T* __restrict__ vo, float* __restrict__ lg,
     float* __restrict__ bt, const int* __restrict__ cu,
     const int* __restrict__ pos0, const int* __restrict__ slots,
-    const int* __restrict__ tok_entry, int tok_base, DeltaDims dm, int Dp,
-    int Vp, float q_scale) {
-  const long i = blockIdx.x;              // row among the long tokens
-  const long t = tok_base + i;
-  const int e = tok_entry[t];
-  const int rel = (int)(t - cu[e]);       // place within the portion
+    const int* __restrict__ tok_entry, const int* __restrict__ chunks,
+    int tok_base, DeltaDims dm, int Dp, int Vp, float q_scale) {
+  const int chunk = blockIdx.x / DC_SUB, sub = blockIdx.x % DC_SUB;
+  const int t0 = chunks[2 * chunk] + sub * DC_TT;
+  const int len = min(DC_TT, chunks[2 * chunk + 1] - sub * DC_TT);
+  const int lane = threadIdx.x & (WAVE - 1);
+  const int piece = blockIdx.y * (DC_BLOCK / WAVE) + threadIdx.x / WAVE;
+  const int D = dm.D, V = dm.V;
+  const int n_qk = 2 * dm.KH;
+  const int n_v = (dm.H * Vp + WAVE - 1) / WAVE;
+  if (len <= 0 || piece > n_qk + n_v) return;
+  const long i0 = t0 - tok_base;          // row among the long tokens
+  const int e = tok_entry[t0];
+  const int rel = t0 - cu[e];             // place within the portion
   const bool fresh = pos0[e] == 0;
   const int hist = dm.taps - 1;
-  const int D = dm.D, V = dm.V;
   const int C = 2 * dm.KH * D + dm.H * V;
   const T* cs = conv_state + (long)slots[e] * C * hist;
-  const T* yt = y + t * dm.ystride;
+  const T* yt = y + (long)t0 * dm.ystride;
 
-  auto conv = [&](int c, int col) {
-    float a = 0.0f;
-    for (int j = 0; j < dm.taps; ++j) {
-      const int s = rel - hist + j;
-      float x;
-      if (s >= 0)
-        x = (float)yt[col + (long)(j - hist) * dm.ystride];
-      else
-        x = fresh ? 0.0f : (float)cs[(long)c * hist + hist + s];
-      a += (float)conv_w[(long)c * dm.taps + j] * x;
+  // channel c (column col of y): convolved and silu'd values of 16 tokens
+  auto convolve = [&](int c, int col, float (&o)[DC_TT]) {
+    float x[DC_TT + DR_MAXTAPS - 1], w[DR_MAXTAPS];
+#pragma unroll
+    for (int k = 0; k < DC_TT + DR_MAXTAPS - 1; ++k) {
+      const int t = k - (DR_MAXTAPS - 1);
+      x[k] = 0.0f;
+      if (t >= 0 ? t < len : (t >= -hist && rel + t >= 0))
+        x[k] = (float)yt[(long)t * dm.ystride + col];
+      else if (t < 0 && t >= -hist && !fresh)
+        x[k] = (float)cs[(long)c * hist + hist + rel + t];
     }
-    return silu_f(a);
+    const int pad = DR_MAXTAPS - dm.taps;
+#pragma unroll
+    for (int j = 0; j < DR_MAXTAPS; ++j)
+      w[j] = j >= pad ? (float)conv_w[(long)c * dm.taps + j - pad] : 0.0f;
+#pragma unroll
+    for (int t = 0; t < DC_TT; ++t) {
+      float a = 0.0f;
+#pragma unroll
+      for (int j = 0; j < DR_MAXTAPS; ++j) a += w[j] * x[t + j];
+      o[t] = silu_f(a);
+    }
   };
 
-  const int lane = threadIdx.x & (WAVE - 1);
-  const int wid = threadIdx.x / WAVE;
-  for (int hq = wid; hq < 2 * dm.KH; hq += DC_BLOCK / WAVE) {
-    const int which = hq / dm.KH, kh = hq - which * dm.KH;
-    float x[DC_MAXD];
-    float ss = 0.0f;
+  if (piece < n_qk) {
+    const int which = piece / dm.KH, kh = piece - which * dm.KH;
+    float o[NU][DC_TT];
 #pragma unroll
-    for (int u = 0; u < DC_MAXD; ++u) {
+    for (int u = 0; u < NU; ++u) {
       const int d = lane + u * WAVE;
-      x[u] = 0.0f;
       if (d < D) {
-        x[u] = conv(which * dm.KH * D + kh * D + d,
-                    (which ? dm.kc : dm.qc) + kh * D + d);
-        ss += x[u] * x[u];
+        convolve(which * dm.KH * D + kh * D + d,
+                 (which ? dm.kc : dm.qc) + kh * D + d, o[u]);
+      } else {
+#pragma unroll
+        for (int t = 0; t < DC_TT; ++t) o[u][t] = 0.0f;
       }
     }
-    ss = wave_sum(ss);
-    const float s = (which ? 1.0f : q_scale) / sqrtf(ss + 1e-6f);
-    float* dst = (which ? ko : qo) + (i * dm.KH + kh) * Dp;
+    float* dst = (which ? ko : qo) + (i0 * dm.KH + kh) * Dp;
 #pragma unroll
-    for (int u = 0; u < DC_MAXD; ++u) {
-      const int d = lane + u * WAVE;
-      if (d < Dp) dst[d] = x[u] * s;
+    for (int t = 0; t < DC_TT; ++t) {
+      float ss = 0.0f;
+#pragma unroll
+      for (int u = 0; u < NU; ++u) ss += o[u][t] * o[u][t];
+      ss = wave_sum(ss);
+      const float s = (which ? 1.0f : q_scale) / sqrtf(ss + 1e-6f);
+      if (t < len) {
+#pragma unroll
+        for (int u = 0; u < NU; ++u) {
+          const int d = lane + u * WAVE;
+          if (d < Dp) dst[(long)t * dm.KH * Dp + d] = o[u][t] * s;
+        }
+      }
     }
-  }
-  for (int j = threadIdx.x; j < dm.H * Vp; j += DC_BLOCK) {
+  } else if (piece < n_qk + n_v) {
+    const int j = (piece - n_qk) * WAVE + lane;
+    if (j >= dm.H * Vp) return;
     const int h = j / Vp, v = j - h * Vp;
-    vo[i * ((long)dm.H * Vp) + j] =
-        v < V ? (T)conv(2 * dm.KH * D + h * V + v, dm.vc + h * V + v) : (T)0.0f;
-  }
-  for (int h = threadIdx.x; h < dm.H; h += DC_BLOCK) {
-    lg[i * dm.H + h] =
-        log_decay((float)yt[dm.ac + h], (float)A_log[h], (float)dt_bias[h]);
-    bt[i * dm.H + h] = sigmoid_f((float)yt[dm.bc + h]);
+    float o[DC_TT];
+    if (v < V) {
+      convolve(2 * dm.KH * D + h * V + v, dm.vc + h * V + v, o);
+    } else {
+#pragma unroll
+      for (int t = 0; t < DC_TT; ++t) o[t] = 0.0f;
+    }
+#pragma unroll
+    for (int t = 0; t < DC_TT; ++t)
+      if (t < len) vo[(i0 + t) * ((long)dm.H * Vp) + j] = (T)o[t];
+  } else {
+    for (int j = lane; j < len * dm.H; j += WAVE) {
+      const int t = j / dm.H, h = j - t * dm.H;
+      const T* yr = yt + (long)t * dm.ystride;
+      lg[(i0 + t) * dm.H + h] =
+          log_decay((float)yr[dm.ac + h], (float)A_log[h], (float)dt_bias[h]);
+      bt[(i0 + t) * dm.H + h] = sigmoid_f((float)yr[dm.bc + h]);
+    }
   }
 }
 
@@ -603,29 +653,232 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
   }
 }
 
+// The same walk with the state depth fixed at 16 * ND: every global operand
+// of the next chunk is fetched into registers right after the current chunk
+// used it, so its latency passes behind the products that remain.
+template <typename T, int ND>
+__global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
+    const float* __restrict__ qn, const float* __restrict__ kn,
+    const T* __restrict__ vn, const float* __restrict__ tm,
+    const float* __restrict__ am, const float* __restrict__ ge,
+    float* __restrict__ state, float* __restrict__ o,
+    const int* __restrict__ chunks, const int* __restrict__ chunk_cu,
+    const int* __restrict__ pos0, const int* __restrict__ slots, int n_short,
+    int tok_base, int KH, int H, int D, int V, int Vp) {
+  constexpr int Dp = ND * 16;
+  constexpr int NT = (ND + 3) / 4;  // state row tiles per wave
+  const int v0 = blockIdx.x * 16;
+  const int h = blockIdx.y;
+  const int e = blockIdx.z;
+  const int kh = h / (H / KH);
+  const int tid = threadIdx.x;
+  const int lane = tid & (WAVE - 1);
+  const int wid = tid / WAVE;
+  const int lr = lane & 15, g4 = lane >> 4;
+
+  __shared__ float ss[Dp * 17];  // state columns
+  __shared__ float xs[64 * 17];  // V - exp(G) K S
+  __shared__ float us[64 * 17];  // U
+  __shared__ float uw[64 * 17];  // exp(G_last - G) U
+
+  const bool fresh = pos0[n_short + e] == 0;
+  float* sg = state + ((long)slots[n_short + e] * H + h) * (long)D * V;
+  for (int i = tid; i < Dp * 16; i += 256) {
+    const int d = i >> 4, v = v0 + (i & 15);
+    ss[d * 17 + (i & 15)] =
+        (!fresh && d < D && v < V) ? sg[(long)d * V + v] : 0.0f;
+  }
+
+  const long rstride = (long)KH * Dp;
+  const f32x4 zero = {0, 0, 0, 0};
+  const int row = wid * 16 + lr;            // A-operand row
+  const int row_c = wid * 16 + g4 * 4;      // first C row
+
+  f32x4 kf[ND], qf[ND], tf[4], af[4], kt[NT][4];
+  float vf[4], gr[4], gl[4], g_all;
+
+  auto load_rows = [&](int i0, int len) {
+    const float* ka = kn + ((long)(i0 + row) * KH + kh) * Dp + g4 * 4;
+    const float* qa = qn + ((long)(i0 + row) * KH + kh) * Dp + g4 * 4;
+    const bool in = row < len;
+#pragma unroll
+    for (int d = 0; d < ND; ++d) {
+      kf[d] = in ? load4(ka + d * 16) : zero;
+      qf[d] = in ? load4(qa + d * 16) : zero;
+    }
+  };
+  auto load_misc = [&](int c, int i0, int len) {
+    const float* gc = ge + ((long)c * H + h) * 128;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = row_c + r;
+      vf[r] = i < len ? (float)vn[((long)(i0 + i) * H + h) * Vp + v0 + lr] : 0.0f;
+      gr[r] = gc[i];
+      gl[r] = gc[64 + i];
+    }
+    g_all = gc[63];
+  };
+  auto load_mat = [&](const float* m, int c, f32x4 (&f)[4]) {
+    const float* p = m + ((long)c * H + h) * 4096 + row * 64 + g4 * 4;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j <= wid) f[j] = load4(p + j * 16);
+  };
+  auto load_kt = [&](int i0, int len) {
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int d0 = wid * 16 + n * 64;
+      if (d0 >= Dp) continue;
+      const float* ka = kn + ((long)i0 * KH + kh) * Dp + d0 + lr;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          const int i = j * 16 + g4 * 4 + s;
+          kt[n][j][s] = i < len ? ka[i * rstride] : 0.0f;
+        }
+    }
+  };
+
+  const int c_end = chunk_cu[e + 1];
+  int c = chunk_cu[e];
+  int i0 = chunks[2 * c] - tok_base, len = chunks[2 * c + 1];
+  load_rows(i0, len);
+  load_misc(c, i0, len);
+  load_mat(tm, c, tf);
+  load_mat(am, c, af);
+  load_kt(i0, len);
+  __syncthreads();
+
+  for (; c < c_end; ++c) {
+    const bool more = c + 1 < c_end;
+    const int j0 = more ? chunks[2 * c + 2] - tok_base : 0;
+    const int jl = more ? chunks[2 * c + 3] : 0;
+
+    f32x4 ks = zero, qs = zero;
+#pragma unroll
+    for (int d = 0; d < ND; ++d)
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        const float sv = ss[(d * 16 + g4 * 4 + s) * 17 + lr];
+        ks = mma4(kf[d][s], sv, ks);
+        qs = mma4(qf[d][s], sv, qs);
+      }
+    if (more) load_rows(j0, jl);
+    f32x4 oc;
+    float glk[4];
+    const float g_now = g_all;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      xs[(row_c + r) * 17 + lr] = vf[r] - gr[r] * ks[r];
+      oc[r] = gr[r] * qs[r];
+      glk[r] = gl[r];
+    }
+    if (more) load_misc(c + 1, j0, jl);
+    __syncthreads();
+
+    f32x4 u = zero;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j <= wid) {
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+          u = mma4(tf[j][s], xs[(j * 16 + g4 * 4 + s) * 17 + lr], u);
+      }
+    if (more) load_mat(tm, c + 1, tf);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      us[(row_c + r) * 17 + lr] = u[r];
+      uw[(row_c + r) * 17 + lr] = u[r] * glk[r];
+    }
+    __syncthreads();
+
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j <= wid) {
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+          oc = mma4(af[j][s], us[(j * 16 + g4 * 4 + s) * 17 + lr], oc);
+      }
+    if (more) load_mat(am, c + 1, af);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (row_c + r < len)
+        o[((long)(i0 + row_c + r) * H + h) * Vp + v0 + lr] = oc[r];
+
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int d0 = wid * 16 + n * 64;
+      if (d0 >= Dp) continue;
+      f32x4 sn;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        sn[r] = g_now * ss[(d0 + g4 * 4 + r) * 17 + lr];
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+          sn = mma4(kt[n][j][s], uw[(j * 16 + g4 * 4 + s) * 17 + lr], sn);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ss[(d0 + g4 * 4 + r) * 17 + lr] = sn[r];
+    }
+    if (more) load_kt(j0, jl);
+    __syncthreads();
+    i0 = j0;
+    len = jl;
+  }
+  for (int i = tid; i < Dp * 16; i += 256) {
+    const int d = i >> 4, v = v0 + (i & 15);
+    if (d < D && v < V) sg[(long)d * V + v] = ss[d * 17 + (i & 15)];
+  }
+}
+
 // ---------------------------------------------------------------------------
 // Step 4: output norm over V, weight, silu gate.  One wave per (token, head).
 // ---------------------------------------------------------------------------
 
-template <typename T>
+// NV: channels per lane, V <= 64 * NV; DG_ROWS rows per wave in flight.
+#define DG_ROWS 4
+
+template <typename T, int NV>
 __global__ __launch_bounds__(256) void delta_gate_kernel(
     const float* __restrict__ o, const T* __restrict__ y,
     const T* __restrict__ norm_w, T* __restrict__ out, long n, int tok_base,
     DeltaDims dm, int Vp, float eps) {
-  const long wi = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
-  if (wi >= n * dm.H) return;
+  const long w0 = ((long)blockIdx.x * 4 + threadIdx.x / WAVE) * DG_ROWS;
   const int lane = threadIdx.x & (WAVE - 1);
-  const long i = wi / dm.H;
-  const int h = (int)(wi - i * dm.H);
-  const float* orow = o + wi * Vp;
-  float ss = 0.0f;
-  for (int v = lane; v < dm.V; v += WAVE) ss += orow[v] * orow[v];
-  ss = wave_sum(ss);
-  const float inv = 1.0f / sqrtf(ss / (float)dm.V + eps);
-  const T* gr = y + (tok_base + i) * dm.ystride + dm.gc + (long)h * dm.V;
-  T* dst = out + (tok_base + i) * ((long)dm.H * dm.V) + (long)h * dm.V;
-  for (int v = lane; v < dm.V; v += WAVE)
-    dst[v] = (T)(orow[v] * inv * (float)norm_w[v] * silu_f((float)gr[v]));
+  float ov[DG_ROWS][NV], gv[DG_ROWS][NV];
+#pragma unroll
+  for (int k = 0; k < DG_ROWS; ++k) {
+    const long wi = min(w0 + k, n * dm.H - 1);
+    const long i = wi / dm.H;
+    const int h = (int)(wi - i * dm.H);
+    const T* gr = y + (tok_base + i) * dm.ystride + dm.gc + (long)h * dm.V;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int v = lane + u * WAVE;
+      ov[k][u] = v < dm.V ? o[wi * Vp + v] : 0.0f;
+      gv[k][u] = v < dm.V ? (float)gr[v] : 0.0f;
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < DG_ROWS; ++k) {
+    const long wi = w0 + k;
+    if (wi >= n * dm.H) return;
+    float ss = 0.0f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) ss += ov[k][u] * ov[k][u];
+    ss = wave_sum(ss);
+    const float inv = 1.0f / sqrtf(ss / (float)dm.V + eps);
+    // row wi of [tokens * heads, V]
+    T* dst = out + (tok_base * (long)dm.H + wi) * dm.V;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int v = lane + u * WAVE;
+      if (v < dm.V)
+        dst[v] = (T)(ov[k][u] * inv * (float)norm_w[v] * silu_f(gv[k][u]));
+    }
+  }
 }
 
 struct DeltaLongArgs {
@@ -646,12 +899,20 @@ static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
   const int C = 2 * dm.KH * dm.D + dm.H * dm.V;
   const float q_scale = 1.0f / sqrtf((float)dm.D);
   dim3 block(DC_BLOCK);
-  dim3 g1((unsigned)a.n_tok);
-  delta_conv_kernel<T><<<g1, block, 0, stream>>>(
-      (const T*)a.y, (const T*)a.conv_w, (const T*)a.A_log,
-      (const T*)a.dt_bias, (const T*)a.conv_state, a.qn, a.kn, (T*)a.vn, a.lg,
-      a.bt, a.cu, a.pos0, a.slots, a.tok_entry, a.tok_base, dm, a.Dp, a.Vp,
-      q_scale);
+  const int pieces = 2 * dm.KH + (dm.H * a.Vp + WAVE - 1) / WAVE + 1;
+  dim3 g1((unsigned)(a.n_chunks * DC_SUB),
+          (unsigned)((pieces + DC_BLOCK / WAVE - 1) / (DC_BLOCK / WAVE)));
+#define DC_GO(N)                                                             \
+  delta_conv_kernel<T, N><<<g1, block, 0, stream>>>(                         \
+      (const T*)a.y, (const T*)a.conv_w, (const T*)a.A_log,                  \
+      (const T*)a.dt_bias, (const T*)a.conv_state, a.qn, a.kn, (T*)a.vn,     \
+      a.lg, a.bt, a.cu, a.pos0, a.slots, a.tok_entry, a.chunks, a.tok_base,  \
+      dm, a.Dp, a.Vp, q_scale)
+  if (a.Dp <= 64) DC_GO(1);
+  else if (a.Dp <= 128) DC_GO(2);
+  else if (a.Dp <= 256) DC_GO(4);
+  else DC_GO(8);
+#undef DC_GO
   dim3 g2((unsigned)a.n_long, (unsigned)((C + DC_BLOCK - 1) / DC_BLOCK));
   if (dm.taps > 1)
     delta_conv_state_kernel<T><<<g2, block, 0, stream>>>(
@@ -660,16 +921,34 @@ static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
   delta_chunk_kernel<<<g3, block, 0, stream>>>(
       a.qn, a.kn, a.lg, a.bt, a.tm, a.am, a.ge, a.chunks, a.tok_base, dm.KH,
       dm.H, a.Dp);
-  const size_t smem = ((size_t)a.Dp + 3 * 64) * 17 * sizeof(float);
   dim3 g4((unsigned)(a.Vp / 16), (unsigned)dm.H, (unsigned)a.n_long);
-  delta_walk_kernel<T><<<g4, block, smem, stream>>>(
-      a.qn, a.kn, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,
-      a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, dm.KH, dm.H, dm.D,
-      a.Dp, dm.V, a.Vp);
-  dim3 g5((unsigned)((a.n_tok * dm.H + 3) / 4));
-  delta_gate_kernel<T><<<g5, block, 0, stream>>>(
-      a.o, (const T*)a.y, (const T*)a.norm_w, (T*)a.out, a.n_tok, a.tok_base,
-      dm, a.Vp, a.eps);
+#define DW_GO(N)                                                             \
+  delta_walk_fixed_kernel<T, N><<<g4, block, 0, stream>>>(                   \
+      a.qn, a.kn, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,  \
+      a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, dm.KH, dm.H, dm.D, \
+      dm.V, a.Vp)
+  if (a.Dp == 16) DW_GO(1);
+  else if (a.Dp == 32) DW_GO(2);
+  else if (a.Dp == 64) DW_GO(4);
+  else if (a.Dp == 128) DW_GO(8);
+  else {
+    const size_t smem = ((size_t)a.Dp + 3 * 64) * 17 * sizeof(float);
+    delta_walk_kernel<T><<<g4, block, smem, stream>>>(
+        a.qn, a.kn, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,
+        a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, dm.KH, dm.H, dm.D,
+        a.Dp, dm.V, a.Vp);
+  }
+#undef DW_GO
+  dim3 g5((unsigned)((a.n_tok * dm.H + 4 * DG_ROWS - 1) / (4 * DG_ROWS)));
+#define DG_GO(N)                                                             \
+  delta_gate_kernel<T, N><<<g5, block, 0, stream>>>(                         \
+      a.o, (const T*)a.y, (const T*)a.norm_w, (T*)a.out, a.n_tok,            \
+      a.tok_base, dm, a.Vp, a.eps)
+  if (dm.V <= 64) DG_GO(1);
+  else if (dm.V <= 128) DG_GO(2);
+  else if (dm.V <= 256) DG_GO(4);
+  else DG_GO(8);
+#undef DG_GO
 }
 
 extern "C" void launch_delta_long(const DeltaLongArgs* a, const DeltaDims* dm,

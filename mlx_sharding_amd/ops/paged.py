@@ -255,6 +255,9 @@ class RaggedCache:
         self.held = [self.state.admit(b) for b in range(batch_size)]
         self.capacity = 0
         self._decode: Optional[RaggedBatch] = None
+        # one batch per captured position; a graph reads its arrays for as
+        # long as it may be replayed, so they are kept
+        self._graph_batches: List[Tuple[torch.Tensor, RaggedBatch]] = []
 
     def ensure_capacity(self, cap: int):
         if cap <= self.capacity:
@@ -272,20 +275,27 @@ class RaggedCache:
 
     @graph_pos.setter
     def graph_pos(self, pos):
-        if pos is not None and pos is not self._graph_pos:
+        if pos is not None and self._graph_batch(pos) is None:
             # a decode batch of its own, whose places follow the device
             # position; lengths are sized for the whole capacity
-            self._graph_batch = RaggedBatch(
+            self._graph_batches.append((pos, RaggedBatch(
                 [(h, 1) for h in self.held], self.state.device,
-                max_keys=self.capacity)
+                max_keys=self.capacity)))
         self._graph_pos = pos
+
+    def _graph_batch(self, pos: torch.Tensor) -> Optional[RaggedBatch]:
+        """The batch a graph with this position was captured on."""
+        for p, batch in self._graph_batches:
+            if p is pos:
+                return batch
+        return None
 
     def next_batch(self, T: int) -> RaggedBatch:
         """The batch of the next T tokens of every sequence."""
         if self._graph_pos is not None:
             if T != 1:
                 raise ValueError("a captured decode step has one token")
-            b = self._graph_batch
+            b = self._graph_batch(self._graph_pos)
             b.tok_pos.copy_(self._graph_pos.expand(self.batch_size))
             b.pos0.copy_(b.tok_pos)
             b.max_pos = self.capacity

@@ -406,3 +406,27 @@ def test_trace_run(checkpoint, tmp_path, monkeypatch, capsys, device, dtype):
     for k, want in ((0, ea[[18, 0]]), (2, torch.stack([ea[23], eb[3], eb[4]])), (7, eb[19:])):
         got = torch.from_numpy(np.fromfile(out / f"{k}.f32", dtype="<f4").reshape(-1, 131))
         assert cases.model_error(got, want, getattr(torch, dtype)) < 1
+
+
+def test_captured_arrays_stay(checkpoint):
+    """What a captured graph reads must outlive it: arming a graph again for
+    the next generation gets the very same batch arrays and tables."""
+    m = model()
+    cache = m.make_cache(batch_size=2)
+    x = torch.tensor([cases.tokens(CFG, 9, i) for i in (1, 2)])
+    pos, other = (torch.zeros(1, dtype=torch.int32) for _ in range(2))
+    seen = []
+    for p in (pos, other, pos):
+        cache[0].reset()
+        m(x, cache)
+        for c in cache:
+            c.graph_pos = p
+        p.fill_(9)
+        batch = cache[0].shared.next_batch(1)
+        assert batch.tok_pos.tolist() == batch.pos0.tolist() == [9, 9]
+        seen.append(batch)
+    assert seen[0] is seen[2] and seen[0] is not seen[1]
+    rotary = m.l1.mix.rotary
+    old = m._rotation(rotary, 10, x.device)
+    assert m._rotation(rotary, 5000, x.device)[0].shape[0] >= 5000
+    assert any(t is old for t in m._old_tables)
