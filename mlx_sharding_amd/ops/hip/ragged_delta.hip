@@ -42,8 +42,9 @@ __device__ __forceinline__ float log_decay(float a, float A_log, float dt) {
 // RPT state rows per thread.
 // ---------------------------------------------------------------------------
 
-template <typename T, int RPT, int NT>
-__global__ __launch_bounds__(NT) void delta_short_kernel(
+// EXACT: the threads tile the state without a remainder.
+template <typename T, int RPT, int NT, bool EXACT>
+__global__ __launch_bounds__(NT, RPT <= 32 ? 4 : 2) void delta_short_kernel(
     const T* __restrict__ y, const T* __restrict__ conv_w,
     const T* __restrict__ A_log, const T* __restrict__ dt_bias,
     const T* __restrict__ norm_w, float* __restrict__ state,
@@ -78,14 +79,16 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
   const int rep = dm.H / dm.KH;
   // this thread's part of a head's state; asked for as early as possible
   float S[RPT];
-  auto state_of = [&](int h) {
-    return state + ((slot * dm.H + h) * (long)D + d0) * V + v;
-  };
   auto load_state = [&](int h) {
-    const float* sp = state_of(h);
+    // uniform row base + one lane offset: no address per row and lane
+    const float* sp = state + ((slot * dm.H + h) * (long)D) * V;
+    const int vc = EXACT ? v : min(v, V - 1);
 #pragma unroll
-    for (int i = 0; i < RPT; ++i)
-      S[i] = (!fresh && v < V && d0 + i < D) ? sp[(long)i * V] : 0.0f;
+    for (int i = 0; i < RPT; ++i) {
+      const float x = EXACT ? sp[d0 * V + v] : sp[min(d0 + i, D - 1) * V + vc];
+      S[i] = fresh ? 0.0f : x;
+      if (EXACT) sp += V;
+    }
   };
   load_state(kh * rep);
 
@@ -156,7 +159,7 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
       float sk = 0.0f, sq = 0.0f;
 #pragma unroll
       for (int i = 0; i < RPT; ++i)
-        if (d0 + i < D) {
+        if (EXACT || d0 + i < D) {
           sk += S[i] * kr[d0 + i];
           sq += S[i] * qr[d0 + i];
         }
@@ -174,7 +177,7 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
       const float o = g * sq + kq[t] * u;
 #pragma unroll
       for (int i = 0; i < RPT; ++i)
-        if (d0 + i < D) S[i] = g * S[i] + kr[d0 + i] * u;
+        if (EXACT || d0 + i < D) S[i] = g * S[i] + kr[d0 + i] * u;
       const bool mine = dg == 0 && v < V;
       const float ss = block_sum<NT>(mine ? o * o : 0.0f, scratch);
       if (mine) {
@@ -183,10 +186,14 @@ __global__ __launch_bounds__(NT) void delta_short_kernel(
             (T)(o / sqrtf(ss / (float)V + eps) * (float)norm_w[v] * gate);
       }
     }
-    float* sp = state_of(h);
+    float* sp = state + ((slot * dm.H + h) * (long)D) * V;
+    if (EXACT || v < V) {
 #pragma unroll
-    for (int i = 0; i < RPT; ++i)
-      if (v < V && d0 + i < D) sp[(long)i * V] = S[i];
+      for (int i = 0; i < RPT; ++i) {
+        if (EXACT || d0 + i < D) sp[d0 * V + v] = S[i];
+        sp += V;
+      }
+    }
     if (hh + 1 < rep) load_state(h + 1);
   }
 }
@@ -222,16 +229,23 @@ static void delta_short_t(const void* y, const void* conv_w, const void* A_log,
                        2 * DR_NT + DR_NT / WAVE) * sizeof(float);
   const float q_scale = 1.0f / sqrtf((float)dm.D);
   dim3 grid((unsigned)n_req, (unsigned)dm.KH), block(DR_NT);
-#define DS_GO(R)                                                             \
+#define DS_ONE(R, X)                                                         \
   do {                                                                       \
     if (smem > 65536)                                                        \
       (void)hipFuncSetAttribute(                                             \
-          reinterpret_cast<const void*>(&delta_short_kernel<T, R, DR_NT>),   \
+          reinterpret_cast<const void*>(&delta_short_kernel<T, R, DR_NT, X>), \
           hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);            \
-    delta_short_kernel<T, R, DR_NT><<<grid, block, smem, stream>>>(          \
+    delta_short_kernel<T, R, DR_NT, X><<<grid, block, smem, stream>>>(       \
         (const T*)y, (const T*)conv_w, (const T*)A_log, (const T*)dt_bias,   \
         (const T*)norm_w, state, (T*)conv_state, (T*)out, cu, pos0, slots,   \
         dm, vt, q_scale, eps);                                               \
+  } while (0)
+#define DS_GO(R)                                                             \
+  do {                                                                       \
+    if (dm.V == vt && dm.D == R * (DR_NT / vt))                              \
+      DS_ONE(R, true);                                                       \
+    else                                                                     \
+      DS_ONE(R, false);                                                      \
   } while (0)
   switch (rpt) {
     case 4: DS_GO(4); break;
@@ -242,6 +256,7 @@ static void delta_short_t(const void* y, const void* conv_w, const void* A_log,
     default: break;
   }
 #undef DS_GO
+#undef DS_ONE
 }
 
 extern "C" void launch_delta_short(const void* y, const void* conv_w,
@@ -462,19 +477,19 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(
     kk[j] = f32x4{0, 0, 0, 0};
     qk[j] = f32x4{0, 0, 0, 0};
   }
-  const int ra = wid * 16 + lr;
-  const f32x4 zero = {0, 0, 0, 0};
+  // rows past the end repeat the last one: their beta is 0
+  const int ra = min(wid * 16 + lr, len - 1);
   const float* kbase = kn + ((long)i0 * KH + kh) * Dp + g4 * 4;
   const float* qbase = qn + ((long)i0 * KH + kh) * Dp + g4 * 4;
   const long rstride = (long)KH * Dp;
   for (int d = 0; d < Dp; d += 16) {
-    const f32x4 ka = ra < len ? load4(kbase + ra * rstride + d) : zero;
-    const f32x4 qa = ra < len ? load4(qbase + ra * rstride + d) : zero;
+    const f32x4 ka = load4(kbase + ra * rstride + d);
+    const f32x4 qa = load4(qbase + ra * rstride + d);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if (j > wid) continue;
-      const int rb = j * 16 + lr;
-      const f32x4 kb = rb < len ? load4(kbase + rb * rstride + d) : zero;
+      const int rb = min(j * 16 + lr, len - 1);
+      const f32x4 kb = load4(kbase + rb * rstride + d);
 #pragma unroll
       for (int s = 0; s < 4; ++s) {
         kk[j] = mma4(ka[s], kb[s], kk[j]);
@@ -655,7 +670,9 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
 
 // The same walk with the state depth fixed at 16 * ND: every global operand
 // of the next chunk is fetched into registers right after the current chunk
-// used it, so its latency passes behind the products that remain.
+// used it, so its latency passes behind the products that remain.  Rows past
+// the end of a chunk repeat its last one: their beta is 0, so they write
+// nothing, and their outputs are not stored.
 template <typename T, int ND>
 __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn,
@@ -673,7 +690,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
   const int kh = h / (H / KH);
   const int tid = threadIdx.x;
   const int lane = tid & (WAVE - 1);
-  const int wid = tid / WAVE;
+  const int wid = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int lr = lane & 15, g4 = lane >> 4;
 
   __shared__ float ss[Dp * 17];  // state columns
@@ -698,13 +715,11 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
   float vf[4], gr[4], gl[4], g_all;
 
   auto load_rows = [&](int i0, int len) {
-    const float* ka = kn + ((long)(i0 + row) * KH + kh) * Dp + g4 * 4;
-    const float* qa = qn + ((long)(i0 + row) * KH + kh) * Dp + g4 * 4;
-    const bool in = row < len;
+    const long at = ((long)(i0 + min(row, len - 1)) * KH + kh) * Dp + g4 * 4;
 #pragma unroll
     for (int d = 0; d < ND; ++d) {
-      kf[d] = in ? load4(ka + d * 16) : zero;
-      qf[d] = in ? load4(qa + d * 16) : zero;
+      kf[d] = load4(kn + at + d * 16);
+      qf[d] = load4(qn + at + d * 16);
     }
   };
   auto load_misc = [&](int c, int i0, int len) {
@@ -712,7 +727,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = row_c + r;
-      vf[r] = i < len ? (float)vn[((long)(i0 + i) * H + h) * Vp + v0 + lr] : 0.0f;
+      vf[r] = (float)vn[((long)(i0 + min(i, len - 1)) * H + h) * Vp + v0 + lr];
       gr[r] = gc[i];
       gl[r] = gc[64 + i];
     }
@@ -721,8 +736,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
   auto load_mat = [&](const float* m, int c, f32x4 (&f)[4]) {
     const float* p = m + ((long)c * H + h) * 4096 + row * 64 + g4 * 4;
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (j <= wid) f[j] = load4(p + j * 16);
+    for (int j = 0; j < 4; ++j) f[j] = load4(p + j * 16);
   };
   auto load_kt = [&](int i0, int len) {
 #pragma unroll
@@ -734,8 +748,8 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
       for (int j = 0; j < 4; ++j)
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
-          const int i = j * 16 + g4 * 4 + s;
-          kt[n][j][s] = i < len ? ka[i * rstride] : 0.0f;
+          const int i = min(j * 16 + g4 * 4 + s, len - 1);
+          kt[n][j][s] = ka[i * rstride];
         }
     }
   };
@@ -751,9 +765,9 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
   __syncthreads();
 
   for (; c < c_end; ++c) {
-    const bool more = c + 1 < c_end;
-    const int j0 = more ? chunks[2 * c + 2] - tok_base : 0;
-    const int jl = more ? chunks[2 * c + 3] : 0;
+    const int cn = min(c + 1, c_end - 1);  // the last one is fetched twice
+    const int j0 = chunks[2 * cn] - tok_base;
+    const int jl = chunks[2 * cn + 1];
 
     f32x4 ks = zero, qs = zero;
 #pragma unroll
@@ -764,7 +778,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
         ks = mma4(kf[d][s], sv, ks);
         qs = mma4(qf[d][s], sv, qs);
       }
-    if (more) load_rows(j0, jl);
+    load_rows(j0, jl);
     f32x4 oc;
     float glk[4];
     const float g_now = g_all;
@@ -774,7 +788,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
       oc[r] = gr[r] * qs[r];
       glk[r] = gl[r];
     }
-    if (more) load_misc(c + 1, j0, jl);
+    load_misc(cn, j0, jl);
     __syncthreads();
 
     f32x4 u = zero;
@@ -785,7 +799,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
         for (int s = 0; s < 4; ++s)
           u = mma4(tf[j][s], xs[(j * 16 + g4 * 4 + s) * 17 + lr], u);
       }
-    if (more) load_mat(tm, c + 1, tf);
+    load_mat(tm, cn, tf);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       us[(row_c + r) * 17 + lr] = u[r];
@@ -800,7 +814,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
         for (int s = 0; s < 4; ++s)
           oc = mma4(af[j][s], us[(j * 16 + g4 * 4 + s) * 17 + lr], oc);
       }
-    if (more) load_mat(am, c + 1, af);
+    load_mat(am, cn, af);
 #pragma unroll
     for (int r = 0; r < 4; ++r)
       if (row_c + r < len)
@@ -822,7 +836,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) ss[(d0 + g4 * 4 + r) * 17 + lr] = sn[r];
     }
-    if (more) load_kt(j0, jl);
+    load_kt(j0, jl);
     __syncthreads();
     i0 = j0;
     len = jl;

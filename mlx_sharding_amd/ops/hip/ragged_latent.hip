@@ -12,6 +12,7 @@
 
 #define LA_BLOCK 256
 #define LA_KT 32  // keys per tile, absorbed
+#define LA_MAXSPLIT WAVE
 
 // ---------------------------------------------------------------------------
 // Absorbed.  A query row is one (token, head) pair of one request; a block
@@ -187,21 +188,25 @@ __global__ __launch_bounds__(128) void latent_attn_merge_kernel(
     T* __restrict__ out, int nsplit, int rankp) {
   const long row = blockIdx.x;
   const float* ml = part_ml + row * nsplit * 2;
-  float m = -1e30f;
-  for (int s = 0; s < nsplit; ++s) m = fmaxf(m, ml[2 * s]);
-  float l = 0.0f;
-  for (int s = 0; s < nsplit; ++s) l += ml[2 * s + 1] * softmax_exp<T>(ml[2 * s] - m);
-  const float rinv = 1.0f / l;
+  __shared__ float w[LA_MAXSPLIT];  // weight of each slice
+  if (threadIdx.x < WAVE) {
+    const int s = threadIdx.x;
+    const float ms = s < nsplit ? ml[2 * s] : -1e30f;
+    const float m = wave_max(ms);
+    const float e = s < nsplit ? softmax_exp<T>(ms - m) : 0.0f;
+    const float l = wave_sum(s < nsplit ? ml[2 * s + 1] * e : 0.0f);
+    w[s] = e / l;
+  }
+  __syncthreads();
   for (int d = threadIdx.x * 4; d < rankp; d += 512) {
+    const float* p = part_o + row * nsplit * rankp + d;
     f32x4 o = {0, 0, 0, 0};
+#pragma unroll 8
     for (int s = 0; s < nsplit; ++s) {
-      const float w = softmax_exp<T>(ml[2 * s] - m);
-      const f32x4 v = load4(part_o + (row * nsplit + s) * rankp + d);
+      const f32x4 v = load4(p + (long)s * rankp);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] += v[j] * w;
+      for (int j = 0; j < 4; ++j) o[j] += v[j] * w[s];
     }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] *= rinv;
     store4(out + row * rankp + d, o);
   }
 }
