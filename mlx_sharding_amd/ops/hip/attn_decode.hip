@@ -197,13 +197,21 @@ __global__ __launch_bounds__(AD_BLOCK) void attn_decode_kernel(
       // batch 8 keys of V loads per wait (trap 4(b), as in the K loop)
       int t = 0;
       for (; t + 8 <= ntile; t += 8) {
+        bf16 raw[8][DVT];
+#pragma unroll
+        for (int tt = 0; tt < 8; ++tt)
+#pragma unroll
+          for (int u = 0; u < DVT; ++u)
+            raw[tt][u] = vbase[(long)(t + tt) * vstride + vcol[u]];
+        // all loads are issued before the first use: left to itself the
+        // scheduler may pair every load with its wait
+        __builtin_amdgcn_sched_barrier(0);
         float vv8[8][DVT];
 #pragma unroll
         for (int tt = 0; tt < 8; ++tt)
 #pragma unroll
           for (int u = 0; u < DVT; ++u)
-            vv8[tt][u] =
-                vmask[u] * bf2f(vbase[(long)(t + tt) * vstride + vcol[u]]);
+            vv8[tt][u] = vmask[u] * bf2f(raw[tt][u]);
 #pragma unroll
         for (int tt = 0; tt < 8; ++tt)
 #pragma unroll

@@ -396,6 +396,9 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
   const long n = y.size(0) - tok_base;
   if (n <= 0 || n_long == 0) return;
   TORCH_CHECK(chunks.dim() == 2 && chunks.size(1) == 2);
+  TORCH_CHECK(n * H < (1L << 31), "too many tokens in one step");
+  TORCH_CHECK(((uintptr_t)y.data_ptr()) % 8 == 0 &&
+              ((uintptr_t)norm_w.data_ptr()) % 8 == 0, "unaligned operand");
   const long nc = chunks.size(0);
   // depths 16 * 2^k take the walk with a fixed depth
   long Dp = 16;

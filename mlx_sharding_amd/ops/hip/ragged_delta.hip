@@ -280,16 +280,37 @@ extern "C" void launch_delta_short(const void* y, const void* conv_w,
 // Long portions, step 1: convolution, silu, unit norms, gates.
 // q, k -> fp32 [n, KH, Dp] (zero padded), v -> T [n, H, Vp], log decay and
 // beta -> fp32 [n, H].  One wave per (16 tokens of a chunk, piece): a piece is
-// a q or k head, 64 value channels, or the gates.  A lane keeps its channels'
-// inputs of all 16 tokens and their history in registers.
-// NU: q/k channels per lane, D <= 64 * NU.
+// a q or k head, 64 * CW value channels, or the gates.  A lane keeps its CW
+// neighbouring channels' inputs of all 16 tokens and their history in
+// registers.  NU: channel groups per lane and q/k head, D <= 64 * CW * NU.
 // ---------------------------------------------------------------------------
+
+// CW neighbouring elements at once (1 or 2)
+template <typename T, int CW>
+struct __attribute__((aligned(CW * sizeof(T)))) Lanes {
+  T v[CW];
+};
+
+template <typename T, int CW>
+__device__ __forceinline__ void load_lanes(const T* p, float (&o)[CW]) {
+  const Lanes<T, CW> t = *reinterpret_cast<const Lanes<T, CW>*>(p);
+#pragma unroll
+  for (int k = 0; k < CW; ++k) o[k] = (float)t.v[k];
+}
+
+template <typename T, int CW>
+__device__ __forceinline__ void store_lanes(T* p, const float (&o)[CW]) {
+  Lanes<T, CW> t;
+#pragma unroll
+  for (int k = 0; k < CW; ++k) t.v[k] = (T)o[k];
+  *reinterpret_cast<Lanes<T, CW>*>(p) = t;
+}
 
 #define DC_BLOCK 256
 #define DC_TT 16
 #define DC_SUB (DR_CHUNK / DC_TT)
 
-template <typename T, int NU>
+template <typename T, int NU, int CW>
 __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
     const T* __restrict__ y, const T* __restrict__ conv_w,
     const T* __restrict__ A_log, const T* __restrict__ dt_bias,
@@ -303,10 +324,11 @@ __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
   const int t0 = chunks[2 * chunk] + sub * DC_TT;
   const int len = min(DC_TT, chunks[2 * chunk + 1] - sub * DC_TT);
   const int lane = threadIdx.x & (WAVE - 1);
-  const int piece = blockIdx.y * (DC_BLOCK / WAVE) + threadIdx.x / WAVE;
+  const int piece = __builtin_amdgcn_readfirstlane(
+      blockIdx.y * (DC_BLOCK / WAVE) + threadIdx.x / WAVE);
   const int D = dm.D, V = dm.V;
   const int n_qk = 2 * dm.KH;
-  const int n_v = (dm.H * Vp + WAVE - 1) / WAVE;
+  const int n_v = (dm.H * Vp + WAVE * CW - 1) / (WAVE * CW);
   if (len <= 0 || piece > n_qk + n_v) return;
   const long i0 = t0 - tok_base;          // row among the long tokens
   const int e = tok_entry[t0];
@@ -317,43 +339,59 @@ __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
   const T* cs = conv_state + (long)slots[e] * C * hist;
   const T* yt = y + (long)t0 * dm.ystride;
 
-  // channel c (column col of y): convolved and silu'd values of 16 tokens
-  auto convolve = [&](int c, int col, float (&o)[DC_TT]) {
-    float x[DC_TT + DR_MAXTAPS - 1], w[DR_MAXTAPS];
+  // channels c.. (columns col.. of y): convolved, silu'd values of 16 tokens
+  auto convolve = [&](int c, int col, float (&o)[DC_TT][CW]) {
+    float x[DC_TT + DR_MAXTAPS - 1][CW], w[DR_MAXTAPS][CW];
 #pragma unroll
     for (int k = 0; k < DC_TT + DR_MAXTAPS - 1; ++k) {
       const int t = k - (DR_MAXTAPS - 1);
-      x[k] = 0.0f;
-      if (t >= 0 ? t < len : (t >= -hist && rel + t >= 0))
-        x[k] = (float)yt[(long)t * dm.ystride + col];
-      else if (t < 0 && t >= -hist && !fresh)
-        x[k] = (float)cs[(long)c * hist + hist + rel + t];
+#pragma unroll
+      for (int q = 0; q < CW; ++q) x[k][q] = 0.0f;
+      if (t >= 0) {
+        // tokens past the end repeat the last one and are not stored
+        load_lanes<T, CW>(yt + (long)min(t, len - 1) * dm.ystride + col, x[k]);
+      } else if (t >= -hist) {
+        if (rel + t >= 0)
+          load_lanes<T, CW>(yt + (long)t * dm.ystride + col, x[k]);
+        else if (!fresh)
+#pragma unroll
+          for (int q = 0; q < CW; ++q)
+            x[k][q] = (float)cs[(long)(c + q) * hist + hist + rel + t];
+      }
     }
     const int pad = DR_MAXTAPS - dm.taps;
 #pragma unroll
     for (int j = 0; j < DR_MAXTAPS; ++j)
-      w[j] = j >= pad ? (float)conv_w[(long)c * dm.taps + j - pad] : 0.0f;
 #pragma unroll
-    for (int t = 0; t < DC_TT; ++t) {
-      float a = 0.0f;
+      for (int q = 0; q < CW; ++q)
+        w[j][q] = j >= pad ? (float)conv_w[(long)(c + q) * dm.taps + j - pad]
+                           : 0.0f;
 #pragma unroll
-      for (int j = 0; j < DR_MAXTAPS; ++j) a += w[j] * x[t + j];
-      o[t] = silu_f(a);
-    }
+    for (int t = 0; t < DC_TT; ++t)
+#pragma unroll
+      for (int q = 0; q < CW; ++q) {
+        float a = 0.0f;
+#pragma unroll
+        for (int j = 0; j < DR_MAXTAPS; ++j)
+          if (j >= pad) a += w[j][q] * x[t + j][q];
+        o[t][q] = silu_f(a);
+      }
   };
 
   if (piece < n_qk) {
     const int which = piece / dm.KH, kh = piece - which * dm.KH;
-    float o[NU][DC_TT];
+    float o[NU][DC_TT][CW];
 #pragma unroll
     for (int u = 0; u < NU; ++u) {
-      const int d = lane + u * WAVE;
+      const int d = (lane + u * WAVE) * CW;
       if (d < D) {
         convolve(which * dm.KH * D + kh * D + d,
                  (which ? dm.kc : dm.qc) + kh * D + d, o[u]);
       } else {
 #pragma unroll
-        for (int t = 0; t < DC_TT; ++t) o[u][t] = 0.0f;
+        for (int t = 0; t < DC_TT; ++t)
+#pragma unroll
+          for (int q = 0; q < CW; ++q) o[u][t][q] = 0.0f;
       }
     }
     float* dst = (which ? ko : qo) + (i0 * dm.KH + kh) * Dp;
@@ -361,31 +399,39 @@ __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
     for (int t = 0; t < DC_TT; ++t) {
       float ss = 0.0f;
 #pragma unroll
-      for (int u = 0; u < NU; ++u) ss += o[u][t] * o[u][t];
+      for (int u = 0; u < NU; ++u)
+#pragma unroll
+        for (int q = 0; q < CW; ++q) ss += o[u][t][q] * o[u][t][q];
       ss = wave_sum(ss);
       const float s = (which ? 1.0f : q_scale) / sqrtf(ss + 1e-6f);
       if (t < len) {
 #pragma unroll
         for (int u = 0; u < NU; ++u) {
-          const int d = lane + u * WAVE;
-          if (d < Dp) dst[(long)t * dm.KH * Dp + d] = o[u][t] * s;
+          const int d = (lane + u * WAVE) * CW;
+#pragma unroll
+          for (int q = 0; q < CW; ++q) o[u][t][q] *= s;
+          if (d < Dp)
+            store_lanes<float, CW>(dst + (long)t * dm.KH * Dp + d, o[u][t]);
         }
       }
     }
   } else if (piece < n_qk + n_v) {
-    const int j = (piece - n_qk) * WAVE + lane;
+    const int j = ((piece - n_qk) * WAVE + lane) * CW;
     if (j >= dm.H * Vp) return;
     const int h = j / Vp, v = j - h * Vp;
-    float o[DC_TT];
+    float o[DC_TT][CW];
     if (v < V) {
       convolve(2 * dm.KH * D + h * V + v, dm.vc + h * V + v, o);
     } else {
 #pragma unroll
-      for (int t = 0; t < DC_TT; ++t) o[t] = 0.0f;
+      for (int t = 0; t < DC_TT; ++t)
+#pragma unroll
+        for (int q = 0; q < CW; ++q) o[t][q] = 0.0f;
     }
 #pragma unroll
     for (int t = 0; t < DC_TT; ++t)
-      if (t < len) vo[(i0 + t) * ((long)dm.H * Vp) + j] = (T)o[t];
+      if (t < len)
+        store_lanes<T, CW>(vo + (i0 + t) * ((long)dm.H * Vp) + j, o[t]);
   } else {
     for (int j = lane; j < len * dm.H; j += WAVE) {
       const int t = j / dm.H, h = j - t * dm.H;
@@ -851,46 +897,61 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
 // Step 4: output norm over V, weight, silu gate.  One wave per (token, head).
 // ---------------------------------------------------------------------------
 
-// NV: channels per lane, V <= 64 * NV; DG_ROWS rows per wave in flight.
-#define DG_ROWS 4
+// NV groups of CW channels per lane, V <= 64 * CW * NV; DG_ROWS rows per wave
+// in flight.
+#define DG_ROWS 8
 
-template <typename T, int NV>
+template <typename T, int NV, int CW>
 __global__ __launch_bounds__(256) void delta_gate_kernel(
     const float* __restrict__ o, const T* __restrict__ y,
     const T* __restrict__ norm_w, T* __restrict__ out, long n, int tok_base,
     DeltaDims dm, int Vp, float eps) {
-  const long w0 = ((long)blockIdx.x * 4 + threadIdx.x / WAVE) * DG_ROWS;
   const int lane = threadIdx.x & (WAVE - 1);
-  float ov[DG_ROWS][NV], gv[DG_ROWS][NV];
+  const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+  const long w0 = ((long)blockIdx.x * 4 + wid) * DG_ROWS;
+  const long rows = n * dm.H;
+  float ov[DG_ROWS][NV][CW], gv[DG_ROWS][NV][CW];
 #pragma unroll
   for (int k = 0; k < DG_ROWS; ++k) {
-    const long wi = min(w0 + k, n * dm.H - 1);
-    const long i = wi / dm.H;
-    const int h = (int)(wi - i * dm.H);
-    const T* gr = y + (tok_base + i) * dm.ystride + dm.gc + (long)h * dm.V;
+    const int wi = (int)min(w0 + k, rows - 1);
+    const int i = wi / dm.H;
+    const int h = wi - i * dm.H;
+    const T* gr = y + (long)(tok_base + i) * dm.ystride + dm.gc + h * dm.V;
+    const float* orow = o + (long)wi * Vp;
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int v = lane + u * WAVE;
-      ov[k][u] = v < dm.V ? o[wi * Vp + v] : 0.0f;
-      gv[k][u] = v < dm.V ? (float)gr[v] : 0.0f;
+      const int v = min((lane + u * WAVE) * CW, dm.V - CW);
+      load_lanes<float, CW>(orow + v, ov[k][u]);
+      load_lanes<T, CW>(gr + v, gv[k][u]);
     }
   }
+  float wv[NV][CW];
+#pragma unroll
+  for (int u = 0; u < NV; ++u)
+    load_lanes<T, CW>(norm_w + min((lane + u * WAVE) * CW, dm.V - CW), wv[u]);
 #pragma unroll
   for (int k = 0; k < DG_ROWS; ++k) {
     const long wi = w0 + k;
-    if (wi >= n * dm.H) return;
+    if (wi >= rows) return;
     float ss = 0.0f;
 #pragma unroll
-    for (int u = 0; u < NV; ++u) ss += ov[k][u] * ov[k][u];
+    for (int u = 0; u < NV; ++u)
+      if ((lane + u * WAVE) * CW < dm.V) {
+#pragma unroll
+        for (int q = 0; q < CW; ++q) ss += ov[k][u][q] * ov[k][u][q];
+      }
     ss = wave_sum(ss);
     const float inv = 1.0f / sqrtf(ss / (float)dm.V + eps);
     // row wi of [tokens * heads, V]
     T* dst = out + (tok_base * (long)dm.H + wi) * dm.V;
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int v = lane + u * WAVE;
-      if (v < dm.V)
-        dst[v] = (T)(ov[k][u] * inv * (float)norm_w[v] * silu_f(gv[k][u]));
+      const int v = (lane + u * WAVE) * CW;
+      float r[CW];
+#pragma unroll
+      for (int q = 0; q < CW; ++q)
+        r[q] = ov[k][u][q] * inv * wv[u][q] * silu_f(gv[k][u][q]);
+      if (v < dm.V) store_lanes<T, CW>(dst + v, r);
     }
   }
 }
@@ -913,19 +974,29 @@ static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
   const int C = 2 * dm.KH * dm.D + dm.H * dm.V;
   const float q_scale = 1.0f / sqrtf((float)dm.D);
   dim3 block(DC_BLOCK);
-  const int pieces = 2 * dm.KH + (dm.H * a.Vp + WAVE - 1) / WAVE + 1;
+  // pairs of channels per lane where the sizes allow it
+  const bool pair = dm.D % 2 == 0 && dm.V % 2 == 0 && dm.ystride % 2 == 0;
+  const int cw = pair ? 2 : 1;
+  const int pieces =
+      2 * dm.KH + (dm.H * a.Vp + WAVE * cw - 1) / (WAVE * cw) + 1;
   dim3 g1((unsigned)(a.n_chunks * DC_SUB),
           (unsigned)((pieces + DC_BLOCK / WAVE - 1) / (DC_BLOCK / WAVE)));
-#define DC_GO(N)                                                             \
-  delta_conv_kernel<T, N><<<g1, block, 0, stream>>>(                         \
+#define DC_GO(N, W)                                                          \
+  delta_conv_kernel<T, N, W><<<g1, block, 0, stream>>>(                      \
       (const T*)a.y, (const T*)a.conv_w, (const T*)a.A_log,                  \
       (const T*)a.dt_bias, (const T*)a.conv_state, a.qn, a.kn, (T*)a.vn,     \
       a.lg, a.bt, a.cu, a.pos0, a.slots, a.tok_entry, a.chunks, a.tok_base,  \
       dm, a.Dp, a.Vp, q_scale)
-  if (a.Dp <= 64) DC_GO(1);
-  else if (a.Dp <= 128) DC_GO(2);
-  else if (a.Dp <= 256) DC_GO(4);
-  else DC_GO(8);
+  if (pair) {
+    if (a.Dp <= 128) DC_GO(1, 2);
+    else if (a.Dp <= 256) DC_GO(2, 2);
+    else DC_GO(4, 2);
+  } else {
+    if (a.Dp <= 64) DC_GO(1, 1);
+    else if (a.Dp <= 128) DC_GO(2, 1);
+    else if (a.Dp <= 256) DC_GO(4, 1);
+    else DC_GO(8, 1);
+  }
 #undef DC_GO
   dim3 g2((unsigned)a.n_long, (unsigned)((C + DC_BLOCK - 1) / DC_BLOCK));
   if (dm.taps > 1)
@@ -954,14 +1025,20 @@ static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
   }
 #undef DW_GO
   dim3 g5((unsigned)((a.n_tok * dm.H + 4 * DG_ROWS - 1) / (4 * DG_ROWS)));
-#define DG_GO(N)                                                             \
-  delta_gate_kernel<T, N><<<g5, block, 0, stream>>>(                         \
+#define DG_GO(N, W)                                                          \
+  delta_gate_kernel<T, N, W><<<g5, block, 0, stream>>>(                      \
       a.o, (const T*)a.y, (const T*)a.norm_w, (T*)a.out, a.n_tok,            \
       a.tok_base, dm, a.Vp, a.eps)
-  if (dm.V <= 64) DG_GO(1);
-  else if (dm.V <= 128) DG_GO(2);
-  else if (dm.V <= 256) DG_GO(4);
-  else DG_GO(8);
+  if (pair && dm.gc % 2 == 0) {
+    if (dm.V <= 128) DG_GO(1, 2);
+    else if (dm.V <= 256) DG_GO(2, 2);
+    else DG_GO(4, 2);
+  } else {
+    if (dm.V <= 64) DG_GO(1, 1);
+    else if (dm.V <= 128) DG_GO(2, 1);
+    else if (dm.V <= 256) DG_GO(4, 1);
+    else DG_GO(8, 1);
+  }
 #undef DG_GO
 }
 
