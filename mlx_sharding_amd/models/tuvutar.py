@@ -18,7 +18,6 @@ import torch
 import torch.nn as nn
 import torch.nn.functional as F
 
-from .. import ops
 from ..config import ModelConfig, ShardSpec
 from ..ops import ragged
 from ..ops.paged import PagedState, RaggedBatch, RaggedCache, RaggedLayerCache

@@ -220,15 +220,6 @@ class RaggedBatch:
         self.host = [(int(cu[e]), int(n[e]), int(pos0[e]), held[e])
                      for e in range(E)]
 
-    def row_index(self, device) -> Optional[torch.Tensor]:
-        """Rows in the order the portions were given, None if it is theirs."""
-        if self.order == sorted(self.order):
-            return None
-        inv = np.argsort(self.order)
-        idx = np.concatenate([np.arange(s, s + n) for s, n, _, _ in
-                              (self.host[j] for j in inv)])
-        return torch.from_numpy(idx).to(device)
-
     def advance(self):
         """Turn a batch of single tokens into the next one, on the device;
         pages must not have grown since."""

@@ -4,7 +4,6 @@ import math
 
 import pytest
 import torch
-import torch.nn.functional as F
 
 import tuvutar_cases as cases
 import tuvutar_oracle as oracle
@@ -12,7 +11,6 @@ from mlx_sharding_amd.ops import ragged
 from mlx_sharding_amd.ops.paged import PagedState, RaggedBatch
 from mlx_sharding_amd.ops.ragged import Rotary
 from mlx_sharding_amd.parallel.batching import BatchEngine, CacheFull, Portion
-
 
 
 @pytest.fixture(autouse=True)

@@ -281,6 +281,22 @@ def test_stage_chain():
     assert [next(gen)[0] for _ in range(8)] == greedy(prompt, 8)
 
 
+def test_grpc_stage(checkpoint):
+    """A remote stage over the wire gets the 32-bit residual."""
+    from mlx_sharding_amd.parallel.grpc_transport import make_clients
+    from mlx_sharding_amd.server.shard_server import serve
+    prompt = cases.tokens(CFG, 18, 2)
+    server, _ = serve(str(checkpoint), 4, 6, dtype=F32, wait=False)
+    try:
+        remotes = make_clients([f"127.0.0.1:{server._mlxs_port}"])
+        m0, _ = load_model(checkpoint, 0, 4, dtype=F32)
+        for _ in range(2):
+            gen = generate_step(torch.tensor([prompt]), m0, m0.make_cache(), remotes)
+            assert [next(gen)[0] for _ in range(6)] == greedy(prompt, 8)[:6]
+    finally:
+        server.stop(0)
+
+
 def _stage(rank, world, ckpt, port, out_file, prompt, n):
     import torch.distributed as dist
 
