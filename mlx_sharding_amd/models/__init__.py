@@ -12,6 +12,7 @@ from .base import StageModel
 from .llama import LlamaStageModel
 from .gemma2 import Gemma2StageModel
 from .deepseek_v2 import DeepseekV2StageModel
+from .lepizen import LepizenStageModel
 from .tuvutar import TuvutarStageModel
 
 MODEL_REMAPPING: Dict[str, str] = {
@@ -27,6 +28,7 @@ _REGISTRY: Dict[str, Type[StageModel]] = {
     "gemma2": Gemma2StageModel,
     "deepseek_v2": DeepseekV2StageModel,
     "tuvutar": TuvutarStageModel,
+    "lepizen": LepizenStageModel,
 }
 
 

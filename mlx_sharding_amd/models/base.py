@@ -149,6 +149,11 @@ class StageModel(nn.Module):
         """Type of the hidden states handed from stage to stage."""
         return self.fp_dtype
 
+    @property
+    def hop_width(self) -> int:
+        """Width of what this stage takes from the previous one."""
+        return self.config.hidden_size
+
     @classmethod
     def allowed_cuts(cls, config: ModelConfig) -> Optional[List[int]]:
         """Layer indices a stage may begin at; None: any."""

@@ -75,7 +75,8 @@ def fuse_model(model) -> int:
     from .llama import LlamaAttention, LlamaMLP
     from .gemma2 import Gemma2Attention, Gemma2MLP
     from .deepseek_v2 import MLAAttention
-    from .mixers import GatedDelta, GatedMLP, LatentAttention
+    from .mixers import (GatedDelta, GatedMLP, LatentAttention,
+                         ParallelBlock)
 
     n = 0
     for mod in model.modules():
@@ -89,7 +90,8 @@ def fuse_model(model) -> int:
             elif isinstance(mod, MLAAttention) and not mod.q_lora_rank:
                 mod._fused_qkv = FusedColumns([mod.q_proj, mod.kv_a_proj_with_mqa])
                 n += 1
-            elif isinstance(mod, (GatedDelta, GatedMLP, LatentAttention)):
+            elif isinstance(mod, (GatedDelta, GatedMLP, LatentAttention,
+                                  ParallelBlock)):
                 mod.prepare()
                 n += 1
         except AssertionError:

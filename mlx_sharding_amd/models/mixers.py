@@ -18,12 +18,12 @@ import torch.nn.functional as F
 from .. import ops
 from ..ops import ragged
 from ..ops.paged import LayerStore, RaggedBatch, RowSpec, StateSpec
-from ..ops.ragged import DeltaShape, LatentShape, Rotary
+from ..ops.ragged import DeltaShape, GroupedShape, LatentShape, Rotary
 from .base import Linear, RMSNorm
 
 
 def _param(*shape, dtype) -> nn.Parameter:
-    return nn.Parameter(torch.empty(*shape, dtype=dtype), requires_grad=False)
+    return nn.Parameter(torch.empty(shape, dtype=dtype), requires_grad=False)
 
 
 def _share(weight: torch.Tensor, *linears: Linear):
@@ -154,6 +154,76 @@ class LatentAttention(nn.Module):
         return ops.linear(out, self.w_o)
 
 
+class GroupedAttention(nn.Module):
+    """Causal softmax attention, ``heads`` query heads over ``kv_heads`` cached
+    keys and values, without positions.
+
+    ``qk_norm``: RMS norms over the whole query and the whole key projection.
+    ``sink``: one learned score per head that enters the softmax's denominator
+    and nothing else.  ``vmix``: the share of another layer's values in this
+    layer's, where the caller passes such values.
+    """
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, scale: float, eps: float, qk_norm: bool = False,
+                 sink: bool = False, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.shape = sh = GroupedShape(heads, kv_heads, dim, vdim)
+        self.scale, self.eps = float(scale), eps
+
+        def lin(out_features):
+            if not qk_norm:
+                return Linear(width, out_features, dtype=dtype)
+            return NormedLinear(width, out_features, out_features, eps, dtype)
+
+        self.q, self.k = lin(heads * dim), lin(kv_heads * dim)
+        self.v = Linear(width, kv_heads * vdim, dtype=dtype)
+        self.vmix = _param(dtype=dtype)
+        self.sink = _param(heads, dtype=dtype) if sink else None
+        self.o = Linear(heads * vdim, width, dtype=dtype)
+        self.w_in = None
+        if max(sh.dimp, sh.vdp) > sh.MAX:
+            raise ValueError(f"head sizes {dim}/{vdim} are above {sh.MAX}")
+
+    def store_spec(self) -> RowSpec:
+        return RowSpec(self.shape.width)
+
+    @property
+    def rows(self):
+        """The projections whose outputs ``attend`` takes, in this order."""
+        return self.q, self.k, self.v
+
+    @torch.no_grad()
+    def prepare(self):
+        self.w_in = torch.cat([m.weight.data for m in self.rows]).contiguous()
+        _share(self.w_in, *self.rows)
+
+    def attend(self, y: torch.Tensor, out: torch.Tensor, batch: RaggedBatch,
+               store: LayerStore, first: Optional[torch.Tensor] = None
+               ) -> torch.Tensor:
+        """y [N, q | k | v | ...]; writes out [N, heads * vdim].  first: values
+        [N, kv_heads * vdim] to mix in.  Returns this layer's values before
+        mixing, a view of y."""
+        sh = self.shape
+        norms = [getattr(m, "norm", None) for m in (self.q, self.k)]
+        q = ragged.grouped_append(
+            y, *(None if n is None else n.weight for n in norms), self.eps,
+            None if first is None else self.vmix, first, store, sh, batch)
+        ragged.grouped_attention(q, self.sink, store, sh, self.scale, batch, out)
+        at = (sh.heads + sh.kv_heads) * sh.dim
+        return y[:, at: at + sh.kv_heads * sh.vdim]
+
+    def forward(self, h: torch.Tensor, batch: RaggedBatch, store: LayerStore,
+                first: Optional[torch.Tensor] = None):
+        """Returns (output, values before mixing)."""
+        if self.w_in is None:
+            self.prepare()
+        y = ops.linear(h, self.w_in)
+        out = y.new_empty(y.shape[0], self.o.in_features)
+        v = self.attend(y, out, batch, store, first)
+        return self.o(out), v
+
+
 class GatedDelta(nn.Module):
     """Gated delta rule: a linear recurrence with a fp32 matrix state per head
     that forgets (one decay per head) and corrects (delta write), behind short
@@ -222,3 +292,70 @@ class GatedMLP(nn.Module):
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         g, u = self.fused(h) if self.fused is not None else (self.gate(h), self.up(h))
         return self.down(self.act(g, u))
+
+
+class MLP(nn.Module):
+    """W_down act(W_up h)."""
+
+    ACTS = {"gelu": ragged.gelu}
+
+    def __init__(self, width: int, ff: int, act: str,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.act = self.ACTS[act]
+        self.up = Linear(width, ff, dtype=dtype)
+        self.down = Linear(ff, width, dtype=dtype)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return self.down(self.act(self.up(h)))
+
+
+class ParallelBlock(nn.Module):
+    """A mixer and a feed-forward (or none) that read the same rows, and the
+    sum of what they make of them: one GEMM into both, each writes its part of
+    one activation row, one GEMM out of both, whose accumulator holds the sum.
+    """
+
+    def __init__(self, mix: nn.Module, mlp: Optional[MLP]):
+        super().__init__()
+        self.mix, self.mlp = mix, mlp
+        self.w_in = self.w_out = None
+
+    @torch.no_grad()
+    def prepare(self):
+        rows, o = list(self.mix.rows), self.mix.o
+        self.mixed = o.in_features              # columns the mixer writes
+        self.taken = sum(m.out_features for m in rows)   # ... and reads
+        if self.mlp is None:
+            self.w_in = torch.cat([m.weight.data for m in rows])
+            self.w_out = o.weight.data
+        else:
+            up, down = self.mlp.up, self.mlp.down
+            # units with zero weights round the activation row up
+            extra = -(self.mixed + up.out_features) % 8
+            rows.append(up)
+            self.w_in = F.pad(torch.cat([m.weight.data for m in rows]),
+                              (0, 0, 0, extra))
+            self.w_out = F.pad(torch.cat([o.weight.data, down.weight.data], 1),
+                               (0, extra))
+            o.weight.data = self.w_out[:, : self.mixed]
+            down.weight.data = self.w_out[:, self.mixed: self.mixed
+                                          + down.in_features]
+        self.hidden = self.w_out.shape[1] - self.mixed
+        # rows of the projection start at whole vectors
+        self.w_in = F.pad(self.w_in, (0, 0, 0, -self.w_in.shape[0] % 8))
+        self.w_in = self.w_in.contiguous()
+        _share(self.w_in, *rows)
+
+    def forward(self, h: torch.Tensor, batch: RaggedBatch, store: LayerStore,
+                *extra):
+        """Returns (sum of both sublayers, what the mixer returns besides)."""
+        if self.w_in is None:
+            self.prepare()
+        y = ops.linear(h, self.w_in)
+        z = y.new_empty(y.shape[0], self.w_out.shape[1])
+        got = self.mix.attend(y, z[:, : self.mixed], batch, store, *extra)
+        if self.mlp is not None:
+            self.mlp.act(y[:, self.taken: self.taken + self.hidden],
+                         z[:, self.mixed:])
+        return ops.linear(z, self.w_out), got

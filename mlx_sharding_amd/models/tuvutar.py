@@ -16,19 +16,16 @@ from typing import Dict, List, Optional
 
 import torch
 import torch.nn as nn
-import torch.nn.functional as F
 
 from ..config import ModelConfig, ShardSpec
 from ..ops import ragged
-from ..ops.paged import PagedState, RaggedBatch, RaggedCache, RaggedLayerCache
+from ..ops.paged import PagedState, RaggedBatch
 from ..ops.ragged import Rotary
-from .base import Linear, RMSNorm, StageModel, owned_layer_indices
+from .base import RMSNorm
 from .mixers import GatedDelta, GatedMLP, LatentAttention
+from .ragged import RaggedStageModel
 
 NORM_OFFSET = 1.0  # norm weights are stored around zero
-
-# parameters that are not the ``weight`` of a module
-_BARE = ("A_log", "dt_bias")
 
 
 def _rotary(rot: dict) -> Rotary:
@@ -74,40 +71,26 @@ class TuvutarLayer(nn.Module):
             self.mlp = GatedMLP(width, int(mlp["ff"]), "gelu_tanh", dtype)
 
 
-class TuvutarStageModel(StageModel):
+class TuvutarStageModel(RaggedStageModel):
     model_type = "tuvutar"
-    supports_ragged = True
-    supports_quantization = False
+    norm_offset = NORM_OFFSET
+    bare_parameters = ("A_log", "dt_bias")
 
     def __init__(self, config: ModelConfig, shard: ShardSpec, quant_for=None,
                  dtype: torch.dtype = torch.bfloat16):
-        super().__init__(config, shard)
-        W, self.eps = config.hidden_size, float(config["norm"]["eps"])
-        specs = config["layers"]
-        if shard.is_first:
-            self.embed = nn.Embedding(config.vocab_size, W, dtype=dtype)
-        for i in owned_layer_indices(shard):
-            layer = TuvutarLayer(specs[i], W, self.eps, dtype)
-            self.add_module(f"l{i}", layer)
+        super().__init__(config, shard, quant_for, dtype)
+        for i, layer in self.layer_items():
             j = layer.source
             if j is not None and not (shard.owns(j) and j < i):
                 raise ValueError(
                     f"layer {i} reads the rows of layer {j}, which stage "
                     f"[{shard.start_layer}, {shard.end_layer}) does not run "
                     f"before it")
-        if shard.is_last:
-            self.final = nn.Module()
-            self.final.norm = RMSNorm(W, self.eps, NORM_OFFSET, dtype)
-            self.head = Linear(W, config.vocab_size, dtype=dtype)
         self._tables: Dict = {}
         self._old_tables: List = []  # captured graphs may still read them
 
-    # -- layers ------------------------------------------------------------
-    def layer(self, i: int) -> TuvutarLayer:
-        return getattr(self, f"l{i}")
-
-    def layer_items(self):
-        return [(i, self.layer(i)) for i in owned_layer_indices(self.shard)]
+    def make_layer(self, i, spec, width, dtype):
+        return TuvutarLayer(spec, width, self.eps, dtype)
 
     @classmethod
     def allowed_cuts(cls, config: ModelConfig) -> List[int]:
@@ -120,46 +103,6 @@ class TuvutarStageModel(StageModel):
             if j is not None:
                 bad.update(range(int(j) + 1, i + 1))
         return [c for c in range(1, n) if c not in bad]
-
-    @property
-    def hop_dtype(self) -> torch.dtype:
-        return torch.float32  # stages hand on the residual stream
-
-    # -- weights -----------------------------------------------------------
-    @classmethod
-    def owns_key(cls, key: str, shard: ShardSpec) -> bool:
-        top = key.split(".")[0]
-        if top == "embed":
-            return shard.is_first
-        if top in ("final", "head"):
-            return shard.is_last
-        return top[:1] == "l" and top[1:].isdigit() and shard.owns(int(top[1:]))
-
-    @classmethod
-    def sanitize(cls, weights, shard: ShardSpec):
-        out = {}
-        for k, v in weights.items():
-            if cls.owns_key(k, shard):
-                if k.rsplit(".", 1)[-1] not in (*_BARE, "weight"):
-                    k = f"{k}.weight"
-                out[k] = v
-        return out
-
-    # -- cache -------------------------------------------------------------
-    def store_specs(self) -> List:
-        return [layer.mix.store_spec() for _, layer in self.layer_items()]
-
-    def make_state(self, max_tokens: int, max_requests: int) -> PagedState:
-        p = next(self.parameters())
-        return PagedState(self.store_specs(), max_tokens, max_requests,
-                          p.dtype, p.device)
-
-    def make_cache(self, dtype: Optional[torch.dtype] = None,
-                   batch_size: int = 1, device=None) -> List[RaggedLayerCache]:
-        p = next(self.parameters())
-        shared = RaggedCache(self.store_specs(), batch_size, dtype or p.dtype,
-                             device if device is not None else p.device)
-        return [RaggedLayerCache(shared, i) for i in range(self.shard.n_layers)]
 
     # -- forward -----------------------------------------------------------
     def _rotation(self, rotary: Rotary, n: int, device):
@@ -175,13 +118,7 @@ class TuvutarStageModel(StageModel):
     def run(self, x: torch.Tensor, batch: RaggedBatch, state: PagedState,
             rows: Optional[torch.Tensor] = None,
             layer_outputs: Optional[list] = None) -> torch.Tensor:
-        """One ragged forward.  x: token ids [N] on the first stage, else the
-        residual [N, width]; rows select the tokens that go through the head.
-        Returns the residual, or fp32 logits on the last stage."""
-        if self.shard.is_first:
-            x = F.embedding(x, self.embed.weight).float()
-        else:
-            x = x.float().contiguous().clone()
+        x = self.residual(x)
         dtype = next(self.parameters()).dtype
         norm = lambda y, post, nxt: ragged.add_norm(  # noqa: E731
             x, y, None if post is None else post.weight,
@@ -213,14 +150,3 @@ class TuvutarStageModel(StageModel):
         if rows is not None:
             h = h.index_select(0, rows)
         return self.head(h).float()
-
-    def forward(self, x: torch.Tensor, cache: Optional[List] = None) -> torch.Tensor:
-        B, T = x.shape[:2]
-        if cache is None:
-            cache = self.make_cache(batch_size=B, device=x.device)
-        shared = cache[0].shared
-        if B != shared.batch_size:
-            raise ValueError(f"cache batch mismatch: {shared.batch_size} vs {B}")
-        y = self.run(x.reshape(B * T, *x.shape[2:]), shared.next_batch(T),
-                     shared.state)
-        return y.view(B, T, -1)

@@ -193,12 +193,16 @@ class RaggedBatch:
             cuk = np.zeros(self.n_long + 1, dtype=np.int32)
             np.cumsum(kpad, out=cuk[1:])
             self.key_rows = int(cuk[-1])
-            blocks, tiles, chunks, chunk_cu = [], [], [], [0]
+            blocks, fills, tiles, chunks, chunk_cu = [], [], [], [], [0]
             for j in range(self.n_long):
                 e = self.n_short + j
                 for b in range(kpad[j] // PAGE):
                     blocks.append((pages[e, b], cuk[j] + b * PAGE,
                                    min(PAGE, el[j] - b * PAGE)))
+                for b in range(pl[j] // PAGE, kpad[j] // PAGE):
+                    t = cu[e] - pl[j] + b * PAGE  # token of the first slot
+                    fills.append((pages[e, b], t, max(0, pl[j] - b * PAGE),
+                                  min(PAGE, el[j] - b * PAGE)))
                 for q0 in range(0, nl[j], QTILE):
                     tiles.append((-(pl[j] + q0), e, q0))
                 for c in range(0, nl[j], CHUNK):
@@ -207,6 +211,7 @@ class RaggedBatch:
             tiles.sort()  # most keys first
             parts.update(
                 cuk=cuk, blocks=np.array(blocks, dtype=np.int32),
+                fills=np.array(fills, dtype=np.int32),
                 tiles=np.array(tiles, dtype=np.int32)[:, 1:],
                 chunks=np.array(chunks, dtype=np.int32),
                 chunk_cu=np.array(chunk_cu, dtype=np.int32))

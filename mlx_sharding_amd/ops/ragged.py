@@ -7,6 +7,13 @@ with the same storage layout, request by request.
 Layouts.  A latent row is [latent, zero padding to ``rankp`` | rotated key part,
 zero padding to ``rotp``].  A query head is [unrotated, padding | rotated,
 padding], ``dq`` wide.
+
+A page of keys and values holds, for each key/value head, 64 keys and then 64
+values in the order in which the matrix cores take them: tiles of 16 x 32
+elements, a lane's 8 elements together, lane after lane.  A key tile is 16 keys
+by 32 dimensions, lane = (dimension / 8 % 4, key % 16).  A value tile is 16
+dimensions by 32 keys, lane = (key / 4 % 4, dimension % 16), and a lane's
+elements are keys 0..3 and 16..19 past its first.
 """
 
 from __future__ import annotations
@@ -57,16 +64,20 @@ def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
 
 
 def add_norm(x, y, w_post, w_next, eps: float, offset: float,
-             dtype: torch.dtype):
-    """x += rms(y) * (w_post + offset), in place, if y is given; returns
-    rms(x) * (w_next + offset) in ``dtype``, or None without w_next.
-    x is the fp32 residual [N, W]."""
+             dtype: torch.dtype, mult: float = 1.0):
+    """x += mult * rms(y) * (w_post + offset), in place, if y is given (without
+    w_post: x += mult * y); returns rms(x) * (w_next + offset) in ``dtype``, or
+    None without w_next.  x is the fp32 residual [N, W]."""
     if x.is_cuda:
-        like = w_post if w_post is not None else w_next
-        h = _ext("add_norm").add_norm(x, y, w_post, w_next, like, eps, offset)
+        like = next(t for t in (w_post, w_next, y) if t is not None)
+        h = _ext("add_norm").add_norm(x, y, w_post, w_next, like, eps, offset,
+                                      mult)
         return h if w_next is not None else None
     if y is not None:
-        x += _rms(y.float(), eps) * (w_post.float() + offset)
+        y = y.float()
+        if w_post is not None:
+            y = _rms(y, eps) * (w_post.float() + offset)
+        x += mult * y
     if w_next is None:
         return None
     return (_rms(x, eps) * (w_next.float() + offset)).to(dtype)
@@ -262,6 +273,159 @@ def latent_attention_expanded(q, store: LayerStore, w_uk, w_uv, sh: LatentShape,
         o = torch.matmul(p, v.transpose(0, 1)).transpose(0, 1)
         out[t0 - base: t0 - base + n] = o.flatten(1).to(out.dtype)
     return out
+
+
+# ---------------------------------------------------------------------------
+# Grouped attention
+# ---------------------------------------------------------------------------
+
+@dataclass(frozen=True)
+class GroupedShape:
+    """Sizes of a grouped-attention layer; heads are padded to whole tiles."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+
+    MAX = 512    # largest head size
+    LONG = 256   # largest head size of the prompt kernel
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads do not share "
+                             f"{self.kv_heads} key/value heads evenly")
+
+    @property
+    def dimp(self):
+        return _pad(self.dim, 32)
+
+    @property
+    def vdp(self):
+        return _pad(self.vdim, 16)
+
+    @property
+    def width(self):
+        """Cached elements per token."""
+        return self.kv_heads * (self.dimp + self.vdp)
+
+    @property
+    def prompts(self) -> bool:
+        """Whether the prompt kernel has this head shape; otherwise every
+        portion takes the decode kernel."""
+        return max(self.dimp, self.vdp) <= self.LONG
+
+    def keys(self, rows):
+        """A view of a page pool: [page, key / 16, key % 16, head, ...] with
+        the last dimensions a head's key in order."""
+        p = rows.view(-1, self.kv_heads, PAGE * (self.dimp + self.vdp))
+        k = p[..., : PAGE * self.dimp].unflatten(
+            2, (PAGE // 16, self.dimp // 32, 4, 16, 8))
+        return k.permute(0, 2, 5, 1, 3, 4, 6)
+
+    def values(self, rows):
+        """[page, key / 32, key / 16 % 2, key / 4 % 4, key % 4, head, ...]."""
+        p = rows.view(-1, self.kv_heads, PAGE * (self.dimp + self.vdp))
+        v = p[..., PAGE * self.dimp:].unflatten(
+            2, (self.vdp // 16, PAGE // 32, 4, 16, 2, 4))
+        return v.permute(0, 3, 6, 4, 7, 1, 2, 5)
+
+
+def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
+                   sh: GroupedShape, batch: RaggedBatch):
+    """From projection rows y [N, q | k | v | ...]: the queries [N, heads,
+    dimp], RMS-normed over the row if wq is given; keys (normed likewise) and
+    values go to their pages.  first: values [N, kv_heads * vdim] that are
+    blended in by vmix (one element)."""
+    H, G, D, V = sh.heads, sh.kv_heads, sh.dim, sh.vdim
+    if y.is_cuda:
+        ext = _ext("grouped_append")
+        direct = batch.short_tokens if sh.prompts else batch.n_tokens
+        q, kinv = ext.grouped_append(
+            y, wq, wk, eps, vmix, first, store.rows, H, G, D, V, sh.dimp,
+            sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages, direct)
+        if direct < batch.n_tokens:
+            ext.grouped_fill(y, wk, kinv, vmix, first, store.rows, H, G, D, V,
+                             sh.dimp, sh.vdp, batch.fills)
+        return q
+    N = y.shape[0]
+    q, k, v = (t.float() for t in y[:, : (H + G) * D + G * V].split(
+        [H * D, G * D, G * V], 1))
+    if wq is not None:
+        q = _rms(q, eps) * wq.float()
+    if wk is not None:
+        k = _rms(k, eps) * wk.float()
+    if first is not None:
+        lam = vmix.float()
+        v = (1.0 - lam) * v + lam * first.float()
+    q = F.pad(q.view(N, H, D), (0, sh.dimp - D)).to(y.dtype)
+    k = F.pad(k.view(N, G, D), (0, sh.dimp - D)).to(y.dtype)
+    v = F.pad(v.view(N, G, V), (0, sh.vdp - V)).to(y.dtype)
+    pos = batch.tok_pos.long()
+    page, r = batch.pages[batch.tok_entry.long(), pos // PAGE].long(), pos % PAGE
+    sh.keys(store.rows)[page, r // 16, r % 16] = k.view(N, G, -1, 4, 8)
+    sh.values(store.rows)[page, r // 32, r // 16 % 2, r // 4 % 4, r % 4] = \
+        v.view(N, G, -1, 16)
+    return q
+
+
+def grouped_attention(q, sink, store: LayerStore, sh: GroupedShape,
+                      scale: float, batch: RaggedBatch, out):
+    """Attention of queries [N, heads, dimp] over their requests' pages, into
+    out [N, heads * vdim].  sink [heads] (or None): a score per head that only
+    the softmax's denominator sees."""
+    if q.is_cuda:
+        ext = _ext("grouped_attention")
+        n_req, max_len = batch.n_short, batch.max_short
+        if not sh.prompts:
+            n_req, max_len = batch.n_requests, batch.max_len
+        if n_req:
+            ext.grouped_attn_short(
+                q, sink, store.rows, out, batch.cu, batch.pos0, batch.pages,
+                n_req, max_len, batch.max_keys, sh.kv_heads, sh.vdim, sh.vdp,
+                scale)
+        if n_req < batch.n_requests:
+            ext.grouped_attn_long(
+                q, sink, store.rows, out, batch.tiles, batch.cu, batch.pos0,
+                batch.pages, sh.kv_heads, sh.vdim, sh.vdp, scale)
+        return
+    H, G = sh.heads, sh.kv_heads
+    for t0, n, p0, held in batch.host:
+        S = p0 + n
+        pages = torch.tensor(held.pages, dtype=torch.long)[: (S + PAGE - 1) // PAGE]
+        k = sh.keys(store.rows)[pages].reshape(-1, G, sh.dimp)[:S].float()
+        v = sh.values(store.rows)[pages].reshape(-1, G, sh.vdp)[:S].float()
+        qg = q[t0: t0 + n].float().view(n, G, H // G, sh.dimp)
+        s = torch.matmul(qg.permute(1, 2, 0, 3), k.permute(1, 2, 0)[:, None])
+        dead = torch.arange(S)[None, :] > torch.arange(p0, S)[:, None]
+        s = (s * scale).masked_fill(dead, float("-inf"))
+        if sink is not None:
+            extra = sink.float().view(G, H // G, 1, 1).expand(-1, -1, n, -1)
+            s = torch.cat([s, extra], -1)
+        p = torch.softmax(s, -1)[..., :S]
+        o = torch.matmul(p, v.transpose(0, 1)[:, None])[..., : sh.vdim]
+        out[t0: t0 + n] = o.permute(2, 0, 1, 3).reshape(n, -1).to(out.dtype)
+
+
+# ---------------------------------------------------------------------------
+# Row-wise functions
+# ---------------------------------------------------------------------------
+
+def gelu(x, out=None):
+    """The exact (erf) gelu of rows [..., C]; out may be a column slice."""
+    if out is None:
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    if x.is_cuda:
+        _ext("gelu").gelu(x.view(-1, x.shape[-1]), out.view(-1, x.shape[-1]))
+    else:
+        out.copy_(F.gelu(x.float()))
+    return out
+
+
+def cap_logits(z, scale: float, limit: float):
+    """limit * tanh(z * scale / limit), fp32."""
+    if z.is_cuda:
+        return _ext("cap_logits").cap_logits(z, scale, limit)
+    return limit * torch.tanh(z.float() * scale / limit)
 
 
 # ---------------------------------------------------------------------------

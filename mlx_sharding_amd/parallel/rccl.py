@@ -77,7 +77,7 @@ class PipelineWorker:
         # hidden states and shipped logits travel in the model's hop type
         self.dtype = dtype if model.hop_dtype == model.fp_dtype else model.hop_dtype
         self.group = group
-        self.hidden = model.config.hidden_size
+        self.hidden = model.hop_width
         self.caches: List[List[KVCache]] = []  # per micro-batch
         self._graph: Optional["CapturedDecode"] = None
 
