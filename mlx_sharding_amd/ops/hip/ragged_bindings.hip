@@ -5,6 +5,7 @@
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 
+#include "ragged_grouped.h"
 #include "ragged_prefill.h"
 
 extern "C" {
@@ -13,7 +14,7 @@ void launch_glu_strided(const void*, const void*, void*, long, int, long, long,
 void launch_glu_any(const void*, const void*, void*, long, int, long, long,
                     bool, bool, hipStream_t);
 void launch_add_norm(void*, const void*, long, const void*, const void*, void*,
-                     long, int, float, float, bool, hipStream_t);
+                     long, int, float, float, float, bool, hipStream_t);
 void launch_latent_append(const void*, long, const void*, float, void*, void*,
                           long, int, int, int, int, int, int, int,
                           const float*, const float*, const int*, const int*,
@@ -28,6 +29,23 @@ void launch_latent_attn_long_bf16(const LatentLongArgs*, int, int,
                                   hipStream_t);
 void launch_latent_attn_long_f32(const LatentLongArgs*, int, int, hipStream_t);
 int delta_short_rows(int, int, int);
+void launch_grouped_append(const GroupedRowArgs*, void*, float*, const int*,
+                           const int*, const int*, int, int, long, bool,
+                           hipStream_t);
+void launch_grouped_fill(const GroupedRowArgs*, const float*, const int*, int,
+                         bool, hipStream_t);
+void launch_grouped_attn_short_bf16(const GroupedAttnArgs*, int, int,
+                                    hipStream_t);
+void launch_grouped_attn_short_f32(const GroupedAttnArgs*, int, int,
+                                   hipStream_t);
+void launch_grouped_attn_long_bf16(const GroupedAttnArgs*, int, int,
+                                   hipStream_t);
+void launch_grouped_attn_long_f32(const GroupedAttnArgs*, int, int,
+                                  hipStream_t);
+void launch_gelu(const void*, void*, long, int, long, long, bool, bool,
+                 hipStream_t);
+void launch_cap_logits(const void*, float*, long, float, float, bool,
+                       hipStream_t);
 }
 
 struct DeltaDims {
@@ -126,11 +144,11 @@ Tensor glu(Tensor gate, Tensor up, bool gelu) {
   return y;
 }
 
-// x [N, W] fp32 (updated in place when y is given); returns h or an empty
-// tensor when there is no following norm.
+// x [N, W] fp32 (updated in place when y is given, normed first when w_post
+// is); returns h or an empty tensor when there is no following norm.
 Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
                 c10::optional<Tensor> w_next, Tensor like, double eps,
-                double off) {
+                double off, double mult) {
   check_f32(x, "x");
   TORCH_CHECK(x.dim() == 2, "x must be [rows, width]");
   const bool f32 = is_f32(like, "like");
@@ -138,10 +156,12 @@ Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
   long ys = W;
   if (y) {
     check_like(*y, like, "y");
-    TORCH_CHECK(y->sizes() == x.sizes() && w_post, "y must match x");
+    TORCH_CHECK(y->sizes() == x.sizes(), "y must match x");
     ys = rows2(*y, "y");
-    check_like(*w_post, like, "w_post");
-    TORCH_CHECK(w_post->numel() == W && w_post->is_contiguous());
+    if (w_post) {
+      check_like(*w_post, like, "w_post");
+      TORCH_CHECK(w_post->numel() == W && w_post->is_contiguous());
+    }
   }
   Tensor h;
   if (w_next) {
@@ -153,10 +173,10 @@ Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
   }
   if (N == 0) return h;
   launch_add_norm(x.data_ptr(), y ? y->data_ptr() : nullptr, ys,
-                  y ? w_post->data_ptr() : nullptr,
+                  y && w_post ? w_post->data_ptr() : nullptr,
                   w_next ? w_next->data_ptr() : nullptr,
                   w_next ? h.data_ptr() : nullptr, N, (int)W, (float)eps,
-                  (float)off, f32, stream());
+                  (float)off, (float)mult, f32, stream());
   return h;
 }
 
@@ -448,6 +468,222 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
   launch_delta_long(&a, &d, f32, stream());
 }
 
+// ---------------------------------------------------------------------------
+// Grouped attention
+// ---------------------------------------------------------------------------
+
+bool whole8(const Tensor& t, long stride) {
+  return ((uintptr_t)t.data_ptr()) % 16 == 0 && stride % 8 == 0;
+}
+
+void check_pool(const Tensor& pool, const Tensor& like, long width) {
+  check_like(pool, like, "pool");
+  TORCH_CHECK(pool.is_contiguous() && pool.dim() == 2 &&
+                  pool.size(1) == width && pool.size(0) % RG_PAGE == 0,
+              "pool must be pages of ", width, " elements per token");
+  aligned16(pool, "pool");
+}
+
+GroupedRowArgs grouped_rows(const Tensor& y, const c10::optional<Tensor>& wq,
+                            const c10::optional<Tensor>& wk, double eps,
+                            const c10::optional<Tensor>& vmix,
+                            const c10::optional<Tensor>& first,
+                            const Tensor& pool, int64_t H, int64_t G, int64_t D,
+                            int64_t V, int64_t dimp, int64_t vdp) {
+  TORCH_CHECK(G > 0 && H > 0 && H % G == 0 && D > 0 && V > 0);
+  TORCH_CHECK(dimp % 32 == 0 && D <= dimp && vdp % 16 == 0 && V <= vdp &&
+              dimp <= 512 && vdp <= 512);
+  GroupedRowArgs a = {};
+  a.ystride = rows2(y, "y");
+  TORCH_CHECK(y.size(1) >= (H + G) * D + G * V);
+  check_pool(pool, y, G * (dimp + vdp));
+  a.vec = D % 8 == 0 && V % 8 == 0 && whole8(y, a.ystride);
+  auto weight = [&](const c10::optional<Tensor>& w, long n, const char* name) {
+    if (!w) return (const void*)nullptr;
+    check_like(*w, y, name);
+    TORCH_CHECK(w->numel() == n && w->is_contiguous());
+    a.vec = a.vec && whole8(*w, 8);
+    return (const void*)w->data_ptr();
+  };
+  a.wq = weight(wq, H * D, "wq");
+  a.wk = weight(wk, G * D, "wk");
+  if (first) {
+    TORCH_CHECK(vmix && vmix->numel() == 1);
+    check_like(*vmix, y, "vmix");
+    check_like(*first, y, "first");
+    a.fstride = rows2(*first, "first");
+    TORCH_CHECK(first->size(0) == y.size(0) && first->size(1) == G * V);
+    a.vec = a.vec && whole8(*first, a.fstride);
+    a.vmix = vmix->data_ptr();
+    a.first = first->data_ptr();
+  }
+  a.y = y.data_ptr();
+  a.pool = pool.data_ptr();
+  a.H = (int)H;
+  a.G = (int)G;
+  a.D = (int)D;
+  a.V = (int)V;
+  a.dimp = (int)dimp;
+  a.vdp = (int)vdp;
+  a.eps = (float)eps;
+  return a;
+}
+
+// y [N, q | k | v | ...] -> queries [N, H, dimp] and the keys' inverse rms [N]
+std::tuple<Tensor, Tensor> grouped_append(
+    Tensor y, c10::optional<Tensor> wq, c10::optional<Tensor> wk, double eps,
+    c10::optional<Tensor> vmix, c10::optional<Tensor> first, Tensor pool,
+    int64_t H, int64_t G, int64_t D, int64_t V, int64_t dimp, int64_t vdp,
+    Tensor tok_pos, Tensor tok_entry, Tensor pages, int64_t direct) {
+  const bool f32 = is_f32(y, "y");
+  auto a = grouped_rows(y, wq, wk, eps, vmix, first, pool, H, G, D, V, dimp,
+                        vdp);
+  const long N = y.size(0);
+  TORCH_CHECK(pages.dim() == 2 && direct >= 0 && direct <= N);
+  auto q = torch::empty({N, H, dimp}, y.options());
+  auto kinv = torch::empty({N}, y.options().dtype(torch::kFloat32));
+  if (N)
+    launch_grouped_append(&a, q.data_ptr(), kinv.data_ptr<float>(),
+                          ints(tok_pos, N, "tok_pos"),
+                          ints(tok_entry, N, "tok_entry"),
+                          ints(pages, 0, "pages"), (int)pages.size(1),
+                          (int)direct, N, f32, stream());
+  return {q, kinv};
+}
+
+// fills [*, 4]: (page, token of its first slot, first slot, end slot)
+void grouped_fill(Tensor y, c10::optional<Tensor> wk, Tensor kinv,
+                  c10::optional<Tensor> vmix, c10::optional<Tensor> first,
+                  Tensor pool, int64_t H, int64_t G, int64_t D, int64_t V,
+                  int64_t dimp, int64_t vdp, Tensor fills) {
+  const bool f32 = is_f32(y, "y");
+  auto a = grouped_rows(y, c10::nullopt, wk, 0.0, vmix, first, pool, H, G, D, V,
+                        dimp, vdp);
+  check_f32(kinv, "kinv");
+  TORCH_CHECK(kinv.numel() == y.size(0) && G <= 65535);
+  TORCH_CHECK(fills.dim() == 2 && fills.size(1) == 4);
+  if (fills.size(0))
+    launch_grouped_fill(&a, kinv.data_ptr<float>(), ints(fills, 0, "fills"),
+                        (int)fills.size(0), f32, stream());
+}
+
+int head_bucket(long n) { return n <= 64 ? 64 : n <= 128 ? 128 : n <= 256 ? 256 : 512; }
+
+GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
+                             const Tensor& pool, const Tensor& out,
+                             const Tensor& pages, int64_t G, int64_t V,
+                             int64_t vdp, double scale) {
+  TORCH_CHECK(q.dim() == 3 && q.is_contiguous());
+  const long H = q.size(1), dimp = q.size(2);
+  TORCH_CHECK(G > 0 && H % G == 0 && V > 0 && V <= vdp);
+  TORCH_CHECK(dimp % 32 == 0 && vdp % 16 == 0 && dimp <= 512 && vdp <= 512);
+  check_pool(pool, q, G * (dimp + vdp));
+  check_like(out, q, "out");
+  aligned16(q, "q");
+  GroupedAttnArgs a = {};
+  a.ostride = rows2(out, "out");
+  TORCH_CHECK(out.size(0) == q.size(0) && out.size(1) == H * V);
+  a.vec = V % 4 == 0 && a.ostride % 4 == 0 &&
+          ((uintptr_t)out.data_ptr()) % 16 == 0;
+  if (sink) {
+    check_like(*sink, q, "sink");
+    TORCH_CHECK(sink->numel() == H && sink->is_contiguous());
+    a.sink = sink->data_ptr();
+  }
+  TORCH_CHECK(pages.dim() == 2);
+  a.q = q.data_ptr();
+  a.pool = pool.data_ptr();
+  a.out = out.data_ptr();
+  a.pages = ints(pages, 0, "pages");
+  a.P = (int)pages.size(1);
+  a.H = (int)H;
+  a.G = (int)G;
+  a.dimp = (int)dimp;
+  a.V = (int)V;
+  a.vdp = (int)vdp;
+  a.scale = (float)scale;
+  return a;
+}
+
+// The first n_req requests of the batch, n_tok tokens; q [N, H, dimp], out [N, H * V].
+void grouped_attn_short(Tensor q, c10::optional<Tensor> sink, Tensor pool,
+                        Tensor out, Tensor cu, Tensor pos0, Tensor pages,
+                        int64_t n_req, int64_t n_tok, int64_t max_len,
+                        int64_t max_keys, int64_t G, int64_t V, int64_t vdp,
+                        double scale) {
+  const bool f32 = is_f32(q, "q");
+  auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale);
+  TORCH_CHECK(pages.size(0) >= n_req && n_tok <= q.size(0));
+  if (n_req == 0 || n_tok == 0) return;
+  a.cu = ints(cu, n_req + 1, "cu");
+  a.pos0 = ints(pos0, n_req, "pos0");
+  a.n_req = (int)n_req;
+  const long tiles = (max_len * (a.H / a.G) + 15) / 16;
+  TORCH_CHECK(tiles <= 65535, "portion too long");
+  a.row_tiles = (int)tiles;
+  // enough blocks for the chip, at least one step of keys per wave
+  long nsplit = std::max<long>(1, 1024 / (n_req * G * tiles));
+  nsplit = std::min<long>(nsplit, std::max<long>(1, max_keys / 128));
+  nsplit = std::min<long>(nsplit, GA_MAXSPLIT);
+  a.nsplit = (int)nsplit;
+  a.n_rows = n_tok * a.H;
+  Tensor po, ml;
+  if (nsplit > 1) {
+    auto o = q.options().dtype(torch::kFloat32);
+    po = torch::empty({a.n_rows, nsplit, vdp}, o);
+    ml = torch::empty({a.n_rows, nsplit, 2}, o);
+    a.part_o = po.data_ptr<float>();
+    a.part_ml = ml.data_ptr<float>();
+  }
+  const int kb = head_bucket(a.dimp), vb = head_bucket(vdp);
+  const bool big = kb == 512 || vb == 512;
+  (f32 ? launch_grouped_attn_short_f32 : launch_grouped_attn_short_bf16)(
+      &a, big ? 512 : kb, big ? 512 : vb, stream());
+}
+
+// The portions that tiles [*, 2] names: (request, first query).
+void grouped_attn_long(Tensor q, c10::optional<Tensor> sink, Tensor pool,
+                       Tensor out, Tensor tiles, Tensor cu, Tensor pos0,
+                       Tensor pages, int64_t G, int64_t V, int64_t vdp,
+                       double scale) {
+  const bool f32 = is_f32(q, "q");
+  auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale);
+  TORCH_CHECK(a.dimp <= 256 && vdp <= 256, "head sizes above 256");
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2 &&
+              tiles.size(0) <= 65535);
+  a.tiles = ints(tiles, 0, "tiles");
+  a.cu = ints(cu, 2, "cu");
+  a.pos0 = ints(pos0, 1, "pos0");
+  a.n_tiles = (int)tiles.size(0);
+  if (a.n_tiles == 0) return;
+  (f32 ? launch_grouped_attn_long_f32 : launch_grouped_attn_long_bf16)(
+      &a, head_bucket(a.dimp), head_bucket(vdp), stream());
+}
+
+// Rows of C columns, possibly slices of wider ones.
+void gelu(Tensor x, Tensor out) {
+  const bool f32 = is_f32(x, "x");
+  check_like(out, x, "out");
+  const long xs = rows2(x, "x"), os = rows2(out, "out");
+  TORCH_CHECK(x.sizes() == out.sizes());
+  const long rows = x.size(0), C = x.size(1);
+  if (rows == 0 || C == 0) return;
+  const bool vec = C % 8 == 0 && whole8(x, xs) && whole8(out, os);
+  launch_gelu(x.data_ptr(), out.data_ptr(), rows, (int)C, xs, os, vec, f32,
+              stream());
+}
+
+Tensor cap_logits(Tensor z, double scale, double limit) {
+  const bool f32 = is_f32(z, "z");
+  TORCH_CHECK(limit != 0.0);
+  auto c = z.contiguous();
+  auto o = torch::empty(z.sizes(), z.options().dtype(torch::kFloat32));
+  if (c.numel())
+    launch_cap_logits(c.data_ptr(), o.data_ptr<float>(), c.numel(),
+                      (float)scale, (float)limit, f32, stream());
+  return o;
+}
+
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -459,5 +695,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_attn_long", &latent_attn_long);
   m.def("delta_short", &delta_short);
   m.def("delta_long", &delta_long);
+  m.def("grouped_append", &grouped_append);
+  m.def("grouped_fill", &grouped_fill);
+  m.def("grouped_attn_short", &grouped_attn_short);
+  m.def("grouped_attn_long", &grouped_attn_long);
+  m.def("gelu", &gelu);
+  m.def("cap_logits", &cap_logits);
   m.attr("PAGE") = RG_PAGE;
 }

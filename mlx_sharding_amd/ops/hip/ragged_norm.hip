@@ -6,7 +6,8 @@
 
 // ---------------------------------------------------------------------------
 // One sublayer boundary in one kernel, one block per row:
-//   x += rms(y) * (w_post + off)      (y == null: x unchanged)
+//   x += mult * rms(y) * (w_post + off)   (y == null: x unchanged;
+//                                          w_post == null: x += mult * y)
 //   h  = rms(x) * (w_next + off)      (w_next == null: no h)
 // x is the fp32 residual; y and h are T.  NR > 0 keeps the row in registers
 // (NR groups of VEC elements per thread); NR == 0 re-reads it.
@@ -35,7 +36,7 @@ template <typename T, int VEC, int NR>
 __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y, long ystride,
     const T* __restrict__ w_post, const T* __restrict__ w_next,
-    T* __restrict__ h, int W, float eps, float off) {
+    T* __restrict__ h, int W, float eps, float off, float mult) {
   __shared__ float scratch[RN_BLOCK / WAVE];
   const long row = blockIdx.x;
   float* xr = x + row * W;
@@ -45,9 +46,17 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
   constexpr int NA = NR > 0 ? NR : 1;
   float xv[NA][VEC];
 
-  float inv_y = 0.0f;
+  float inv_y = mult;
   float yv[NA][VEC];
-  if (yr) {
+  if (yr && !w_post) {
+    if constexpr (NR > 0) {
+#pragma unroll
+      for (int i = 0; i < NR; ++i) {
+        const int c = i * step + threadIdx.x * VEC;
+        if (c < W) rn_load<T, VEC>(yr + c, yv[i]);
+      }
+    }
+  } else if (yr) {
     float ss = 0.0f;
     if constexpr (NR > 0) {
 #pragma unroll
@@ -67,13 +76,17 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
       }
     }
     ss = block_sum<RN_BLOCK>(ss, scratch);
-    inv_y = 1.0f / sqrtf(ss / (float)W + eps);
+    inv_y = mult / sqrtf(ss / (float)W + eps);
   }
 
   float ss = 0.0f;
   auto update = [&](int c, float (&xa)[VEC], float (&ya)[VEC]) {
     rn_load<float, VEC>(xr + c, xa);
-    if (yr) {
+    if (yr && !w_post) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) xa[j] += ya[j] * inv_y;
+      rn_store<float, VEC>(xr + c, xa);
+    } else if (yr) {
       float wv[VEC];
       rn_load<T, VEC>(w_post + c, wv);
 #pragma unroll
@@ -122,7 +135,7 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
 template <typename T>
 static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
                        const void* wn, void* h, long rows, int W, float eps,
-                       float off, hipStream_t stream) {
+                       float off, float mult, hipStream_t stream) {
   const bool vec = W % 4 == 0 && ystride % 4 == 0 &&
                    ((uintptr_t)y) % 16 == 0;
   const int nr = (W + RN_BLOCK * 4 - 1) / (RN_BLOCK * 4);
@@ -130,7 +143,7 @@ static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
 #define RN_GO(V, N)                                                        \
   add_norm_kernel<T, V, N><<<grid, block, 0, stream>>>(                    \
       (float*)x, (const T*)y, ystride, (const T*)wp, (const T*)wn, (T*)h, W, \
-      eps, off)
+      eps, off, mult)
   if (!vec)
     RN_GO(1, 0);
   else if (nr <= 1)
@@ -149,11 +162,11 @@ static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
 extern "C" void launch_add_norm(void* x, const void* y, long ystride,
                                 const void* wp, const void* wn, void* h,
                                 long rows, int W, float eps, float off,
-                                bool f32, hipStream_t stream) {
+                                float mult, bool f32, hipStream_t stream) {
   if (f32)
-    add_norm_t<float>(x, y, ystride, wp, wn, h, rows, W, eps, off, stream);
+    add_norm_t<float>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult, stream);
   else
-    add_norm_t<__bf16>(x, y, ystride, wp, wn, h, rows, W, eps, off, stream);
+    add_norm_t<__bf16>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult, stream);
 }
 
 // ---------------------------------------------------------------------------

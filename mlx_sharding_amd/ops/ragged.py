@@ -375,14 +375,14 @@ def grouped_attention(q, sink, store: LayerStore, sh: GroupedShape,
     the softmax's denominator sees."""
     if q.is_cuda:
         ext = _ext("grouped_attention")
-        n_req, max_len = batch.n_short, batch.max_short
+        n_req, n, max_len = batch.n_short, batch.short_tokens, batch.max_short
         if not sh.prompts:
-            n_req, max_len = batch.n_requests, batch.max_len
+            n_req, n, max_len = batch.n_requests, batch.n_tokens, batch.max_len
         if n_req:
             ext.grouped_attn_short(
                 q, sink, store.rows, out, batch.cu, batch.pos0, batch.pages,
-                n_req, max_len, batch.max_keys, sh.kv_heads, sh.vdim, sh.vdp,
-                scale)
+                n_req, n, max_len, batch.max_keys, sh.kv_heads, sh.vdim,
+                sh.vdp, scale)
         if n_req < batch.n_requests:
             ext.grouped_attn_long(
                 q, sink, store.rows, out, batch.tiles, batch.cu, batch.pos0,
