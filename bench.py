@@ -54,8 +54,12 @@ def parse_args():
                    metavar="SIZE",
                    help="instead of the serving benchmark: prefill and decode "
                         "throughput of Tuvutar layers beside DeepSeek-V2's "
-                        "dense latent-attention layers of equal size, one JSON "
-                        "line per case (2048, 4096 or all)")
+                        "dense latent-attention layers and of Lepizen layers "
+                        "beside Llama's, each of equal size, one JSON line per "
+                        "case (2048, 4096 or all)")
+    p.add_argument("--kinds", default=None, metavar="NAME,...",
+                   help="the stacks --layers times (default: all; mla, latent, "
+                        "shared, delta, mixed, llama, lepizen)")
     return p.parse_args()
 
 
@@ -66,7 +70,8 @@ def main():
     args = parse_args()
     if args.layers is not None:
         from mlx_sharding_amd.utils.layer_bench import run
-        return run(args.layers, steps=min(args.steps, 32))
+        return run(args.layers, steps=min(args.steps, 32),
+                   kinds=args.kinds.split(",") if args.kinds else None)
     if args.quant is None:
         args.quant = "deepseek" in args.model
 

@@ -42,7 +42,7 @@ def parse_args(argv=None):
     p.add_argument("--max-tokens", type=int, required=True,
                    help="most tokens that live requests hold at any time, "
                         "each rounded up to whole cache pages")
-    p.add_argument("--device", default=None, help="default: cuda, if present")
+    p.add_argument("--device", default="cuda")
     return p.parse_args(argv)
 
 
@@ -50,14 +50,13 @@ def main(argv=None) -> int:
     args = parse_args(argv)
     import torch
 
-    device = args.device or ("cuda" if torch.cuda.device_count() else "cpu")
-    if device.startswith("cuda"):
+    if args.device.startswith("cuda"):
         build_kernels()
 
     from ..parallel.batching import BatchEngine, Portion
     from ..utils.loading import load_model
 
-    model, _ = load_model(args.model, device=device,
+    model, _ = load_model(args.model, device=args.device,
                           dtype=getattr(torch, args.dtype))
     engine = BatchEngine(model, args.max_tokens, MAX_REQUESTS)
     for line in sys.stdin:

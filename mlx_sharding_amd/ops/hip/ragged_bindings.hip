@@ -688,7 +688,9 @@ Tensor cap_logits(Tensor z, double scale, double limit) {
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("glu", &glu);
-  m.def("add_norm", &add_norm);
+  m.def("add_norm", &add_norm, py::arg("x"), py::arg("y"), py::arg("w_post"),
+        py::arg("w_next"), py::arg("like"), py::arg("eps"), py::arg("offset"),
+        py::arg("mult") = 1.0);
   m.def("latent_append", &latent_append);
   m.def("latent_gather", &latent_gather);
   m.def("latent_attn_short", &latent_attn_short);

@@ -308,12 +308,18 @@ class RaggedCache:
             h.length = self.offset
         return d
 
-    def reset(self):
-        self.offset = 0
+    def trim(self, n: int):
+        """Go back to the first n tokens of every sequence."""
+        if not 0 <= n <= self.offset:
+            raise ValueError(f"trim({n}) outside [0, {self.offset}]")
+        self.offset = n
         self._graph_pos = None
         self._decode = None
         for h in self.held:
-            h.length = 0
+            h.length = n
+
+    def reset(self):
+        self.trim(0)
 
 
 class RaggedLayerCache:
@@ -323,8 +329,12 @@ class RaggedLayerCache:
         self.shared = shared
         self.layer = layer
 
-    # a recurrent state cannot be rolled back to a shorter prefix
-    trimmable = False
+    @property
+    def trimmable(self) -> bool:
+        """A recurrent state cannot be rolled back to a shorter prefix; rows
+        can."""
+        return all(s is None or s.state is None
+                   for s in self.shared.state.layers)
 
     batch_size = property(lambda self: self.shared.batch_size)
     offset = property(lambda self: self.shared.offset)
@@ -369,12 +379,10 @@ class RaggedLayerCache:
             s.conv.copy_(snap[1])
 
     def trim(self, n: int):
-        if n == self.shared.offset:
-            return
-        if n == 0:
-            self.shared.reset()
-            return
-        raise ValueError("a recurrent state has no shorter prefix to go back to")
+        if n not in (0, self.shared.offset) and not self.trimmable:
+            raise ValueError("a recurrent state has no shorter prefix to go "
+                             "back to")
+        self.shared.trim(n)
 
     def reset(self):
         self.shared.reset()

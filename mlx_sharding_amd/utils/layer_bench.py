@@ -1,13 +1,15 @@
 """Prefill and decode throughput of layer stacks at real sizes (random weights).
 
-Stacks of four layers of one kind with equal width, heads, head sizes, latent
-size and feed-forward, so that their times compare directly:
+Stacks of four layers of one kind with equal width, heads, key/value heads, head
+sizes, latent size and feed-forward, so that their times compare directly:
 
   mla     DeepSeek-V2 latent attention + dense MLP (the closest existing model)
   latent  Tuvutar latent attention
   shared  Tuvutar latent attention, three of four layers on shared rows
   delta   Tuvutar gated delta rule
   mixed   Tuvutar delta, delta, delta, latent
+  llama   Llama grouped attention + gated MLP (the closest model to the next)
+  lepizen Lepizen grouped attention beside an ungated MLP of the same width
 
 All run the pipeline worker's own prefill and graph-captured decode step.
 """
@@ -16,19 +18,20 @@ from __future__ import annotations
 
 import json
 import time
-from typing import Dict
+from typing import Dict, Optional, Sequence
 
 import torch
 
 from ..config import ModelConfig
 from ..parallel.rccl import PipelineWorker, build_stage_model
-from .presets import _dense_mla, _tuvutar
+from .presets import _dense_mla, _lepizen, _llama, _tuvutar
 
 SIZES: Dict[str, dict] = {
     "2048": dict(width=2048, heads=16, ff=8192, vocab=8192),
     "4096": dict(width=4096, heads=32, ff=14336, vocab=8192),
 }
-KINDS = {"latent": "aaaa", "shared": "asss", "delta": "dddd", "mixed": "ddda"}
+TUVUTAR = {"latent": "aaaa", "shared": "asss", "delta": "dddd", "mixed": "ddda"}
+KINDS = ("mla", *TUVUTAR, "llama", "lepizen")
 PREFILL = ((1, 8192), (8, 1024))     # sequences, tokens each
 DECODE = ((1, 2048), (64, 2048))     # sequences, tokens cached
 
@@ -36,11 +39,15 @@ DECODE = ((1, 2048), (64, 2048))     # sequences, tokens cached
 def stack(kind: str, size: dict) -> ModelConfig:
     if kind == "mla":
         return ModelConfig.from_dict(_dense_mla(n_layers=4, **size))
+    if kind in ("llama", "lepizen"):
+        make = _llama if kind == "llama" else _lepizen
+        return ModelConfig.from_dict(
+            make(n_layers=4, kv_heads=size["heads"] // 4, **size))
     extra = {}
-    if "d" in KINDS[kind]:
+    if "d" in TUVUTAR[kind]:
         extra = dict(delta_heads=size["heads"], delta_kv=size["heads"] // 2)
     return ModelConfig.from_dict(
-        _tuvutar(period=KINDS[kind], repeats=1, **size, **extra))
+        _tuvutar(period=TUVUTAR[kind], repeats=1, **size, **extra))
 
 
 def _time(fn, n: int) -> float:
@@ -52,13 +59,14 @@ def _time(fn, n: int) -> float:
     return (time.perf_counter() - t0) / n
 
 
-def run(which: str = "all", steps: int = 32, kinds=("mla", *KINDS)):
+def run(which: str = "all", steps: int = 32,
+        kinds: Optional[Sequence[str]] = None):
     if not torch.cuda.is_available():
         raise SystemExit("--layers needs a GPU")
     device = torch.device("cuda", 0)
     torch.manual_seed(0)
     for name in (SIZES if which == "all" else [which]):
-        for kind in kinds:
+        for kind in kinds or KINDS:
             config = stack(kind, SIZES[name])
             model = build_stage_model(config, 0, 1, device)
 

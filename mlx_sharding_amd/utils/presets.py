@@ -35,6 +35,26 @@ def _tuvutar(width: int, heads: int, ff: int, vocab: int, period: str,
             "norm": {"eps": 1e-6}, "layers": layers}
 
 
+def _lepizen(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
+             n_layers: int, dim: int = 128) -> dict:
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
+             "scale": dim ** -0.5, "v_mix": True}
+    return {"architecture": "Lepizen", "width": width, "vocab": vocab,
+            "norm": {"eps": 1e-6}, "residual_mult": 0.7, "logit_scale": 0.25,
+            "logit_softcap": 50.0,
+            "layers": [{"type": "attention", "mixer": dict(mixer),
+                        "mlp": {"kind": "dense", "ff": ff}}
+                       for _ in range(n_layers)]}
+
+
+def _llama(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
+           n_layers: int) -> dict:
+    return {"model_type": "llama", "hidden_size": width,
+            "num_hidden_layers": n_layers, "intermediate_size": ff,
+            "num_attention_heads": heads, "num_key_value_heads": kv_heads,
+            "vocab_size": vocab, "rms_norm_eps": 1e-6, "rope_theta": 10000.0}
+
+
 def _dense_mla(width: int, heads: int, ff: int, vocab: int, n_layers: int,
                dim: int = 128, rot: int = 64, rank: int = 512) -> dict:
     """A DeepSeek-V2 config without experts (latent attention + dense MLP)."""
@@ -162,6 +182,24 @@ PRESETS = {
     "tuvutar-2b": _tuvutar(2048, 16, 8192, 32000, "dddadds", 4),
     "tuvutar-8b": _tuvutar(4096, 32, 14336, 32000, "dddadds", 4,
                            delta_heads=32, delta_kv=16),
+    "lepizen-2b": _lepizen(2048, 16, 4, 8192, 32000, 28),
+    "lepizen-8b": _lepizen(4096, 32, 8, 16384, 32000, 36),
+    "debug-lepizen": {
+        "architecture": "Lepizen", "width": 96, "vocab": 320,
+        "norm": {"eps": 1e-6}, "residual_mult": 0.6, "logit_scale": 0.4,
+        "logit_softcap": 20.0,
+        "layers": [
+            {"type": "attention", "mlp": None,
+             "mixer": {"heads": 6, "kv_heads": 3, "dim": 24, "vdim": 40,
+                       "scale": 0.2, "v_mix": False}},
+            {"type": "attention", "mlp": {"kind": "dense", "ff": 160},
+             "mixer": {"heads": 8, "kv_heads": 2, "dim": 16, "vdim": 24,
+                       "scale": 0.25, "v_mix": True}},
+            {"type": "attention", "mlp": {"kind": "dense", "ff": 112},
+             "mixer": {"heads": 4, "kv_heads": 4, "dim": 32, "vdim": 12,
+                       "scale": 0.18, "v_mix": True}},
+        ],
+    },
     "debug-tuvutar": {
         "architecture": "Tuvutar", "width": 96, "vocab": 320,
         "norm": {"eps": 1e-6},
