@@ -677,6 +677,7 @@ Tensor cap_logits(Tensor z, double scale, double limit) {
   const bool f32 = is_f32(z, "z");
   TORCH_CHECK(limit != 0.0);
   auto c = z.contiguous();
+  aligned16(c, "z");
   auto o = torch::empty(z.sizes(), z.options().dtype(torch::kFloat32));
   if (c.numel())
     launch_cap_logits(c.data_ptr(), o.data_ptr<float>(), c.numel(),

@@ -4,82 +4,86 @@
 
 #define GR_BLOCK 256
 
-template <typename T>
-__device__ __forceinline__ void load8(const T* p, float (&o)[8]) {
-  const f32x4 a = load4(p), b = load4(p + 4);
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    o[j] = a[j];
-    o[4 + j] = b[j];
-  }
-}
+typedef float f32x8 __attribute__((ext_vector_type(8)));
 
+// eight elements as they lie in memory, and their values
 template <typename T>
-__device__ __forceinline__ void store8(T* p, const float (&v)[8]);
-template <>
-__device__ __forceinline__ void store8(__bf16* p, const float (&v)[8]) {
+using Raw8 = T __attribute__((ext_vector_type(8)));
+template <typename T>
+__device__ __forceinline__ Raw8<T> raw8(const T* p) {
+  return *reinterpret_cast<const Raw8<T>*>(p);
+}
+__device__ __forceinline__ f32x8 value8(bf16x8 v) {
+  f32x8 o;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) o[j] = (float)v[j];
+  return o;
+}
+__device__ __forceinline__ f32x8 value8(f32x8 v) { return v; }
+template <typename T>
+__device__ __forceinline__ f32x8 load8(const T* p) {
+  return value8(raw8(p));
+}
+__device__ __forceinline__ void store8(__bf16* p, f32x8 v) {
   bf16x8 o;
 #pragma unroll
   for (int j = 0; j < 8; ++j) o[j] = (__bf16)v[j];
   *reinterpret_cast<bf16x8*>(p) = o;
 }
-template <>
-__device__ __forceinline__ void store8(float* p, const float (&v)[8]) {
-  store4(p, f32x4{v[0], v[1], v[2], v[3]});
-  store4(p + 4, f32x4{v[4], v[5], v[6], v[7]});
+__device__ __forceinline__ void store8(float* p, f32x8 v) {
+  store4(p, __builtin_shufflevector(v, v, 0, 1, 2, 3));
+  store4(p + 4, __builtin_shufflevector(v, v, 4, 5, 6, 7));
 }
 
 // Columns c .. c + 7 of one head (`size` wide, zeros behind it).
 template <typename T, bool VEC>
-__device__ __forceinline__ void head8(const T* row, int c, int size,
-                                      float (&o)[8]) {
-  if (VEC && c < size) {
-    load8(row + c, o);
+__device__ __forceinline__ f32x8 head8(const T* row, int c, int size) {
+  f32x8 o = {0, 0, 0, 0, 0, 0, 0, 0};
+  if constexpr (VEC) {
+    if (c < size) o = load8(row + c);
   } else {
 #pragma unroll
     for (int j = 0; j < 8; ++j)
-      o[j] = !VEC && c + j < size ? (float)row[c + j] : 0.0f;
+      if (c + j < size) o[j] = (float)row[c + j];
   }
+  return o;
 }
 
-// normed columns: row and weight of one head, times the row's inverse rms
-template <typename T, bool VEC>
-__device__ __forceinline__ void normed8(const T* row, const T* w, int c,
-                                        int size, float inv, float (&o)[8]) {
-  head8<T, VEC>(row, c, size, o);
-  if (w) {
-    float wv[8];
-    head8<T, VEC>(w, c, size, wv);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) o[j] = o[j] * inv * wv[j];
-  }
-}
-
-template <typename T, bool VEC>
-__device__ __forceinline__ float square_sum(const T* p, int n) {
+__device__ __forceinline__ float squares(f32x8 v) {
   float s = 0.0f;
-  if constexpr (VEC) {
-    for (int i = threadIdx.x * 8; i < n; i += GR_BLOCK * 8) {
-      float v[8];
-      load8(p + i, v);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) s += v[j] * v[j];
-    }
-  } else {
-    for (int i = threadIdx.x; i < n; i += GR_BLOCK)
-      s += (float)p[i] * (float)p[i];
-  }
+  for (int j = 0; j < 8; ++j) s += v[j] * v[j];
   return s;
 }
 
-// One block per token: q out [N, H, dimp]; the first `direct` tokens' keys and
-// values go to their pages, the others only leave their keys' inverse rms.
+// The i-th chunk of eight columns of a row of heads padded to 8 * nc columns.
 template <typename T, bool VEC>
+__device__ __forceinline__ f32x8 chunk8(const T* row, int i, int size, int nc) {
+  const int h = i / nc;
+  return head8<T, VEC>(row + h * size, (i - h * nc) * 8, size);
+}
+
+// Where that chunk lies; what is past the row or in the padding reads another
+// chunk of it, so that many loads are in flight together.
+template <typename T>
+__device__ __forceinline__ const T* chunk_at(const T* row, int i, int n,
+                                             int size, int nc) {
+  i = min(i, n - 1);
+  const int h = i / nc;
+  return row + h * size + min((i - h * nc) * 8, size - 8);
+}
+
+// One block per token: queries out [N, H, dimp]; keys and values of the first
+// `direct` tokens go to their pages, the others only leave their keys' inverse
+// rms.  NQ, NK: chunks of the projections a thread keeps (whole vectors only);
+// 0: read twice.
+template <typename T, bool VEC, int NQ, int NK>
 __global__ __launch_bounds__(GR_BLOCK) void grouped_append_kernel(
     const GroupedRowArgs a, T* __restrict__ q, float* __restrict__ kinv,
     const int* __restrict__ tok_pos, const int* __restrict__ tok_entry,
     const int* __restrict__ pages, int P, int direct) {
-  __shared__ float scratch[2][GR_BLOCK / WAVE];
+  constexpr int AQ = NQ > 0 ? NQ : 1, AK = NK > 0 ? NK : 1;
+  __shared__ float sums[2][GR_BLOCK / WAVE];
   const long t = blockIdx.x;
   const int tid = threadIdx.x;
   const T* yq = (const T*)a.y + t * a.ystride;
@@ -87,47 +91,102 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_append_kernel(
   const T* yv = yk + (long)a.G * a.D;
   const T* wq = (const T*)a.wq;
   const T* wk = (const T*)a.wk;
+  const int nc = a.dimp / 8, nq = a.H * nc, nk = a.G * nc;
 
-  float sq = wq ? square_sum<T, VEC>(yq, a.H * a.D) : 0.0f;
-  float sk = wk ? square_sum<T, VEC>(yk, a.G * a.D) : 0.0f;
+  Raw8<T> rq[AQ], rqw[AQ], rk[AK], rkw[AK];
+#pragma unroll
+  for (int k = 0; k < NQ; ++k) {
+    const int i = k * GR_BLOCK + tid;
+    rq[k] = raw8(chunk_at(yq, i, nq, a.D, nc));
+    rqw[k] = raw8(chunk_at(wq ? wq : yq, i, nq, a.D, nc));
+  }
+#pragma unroll
+  for (int k = 0; k < NK; ++k) {
+    const int i = k * GR_BLOCK + tid;
+    rk[k] = raw8(chunk_at(yk, i, nk, a.D, nc));
+    rkw[k] = raw8(chunk_at(wk ? wk : yk, i, nk, a.D, nc));
+  }
+  const bool write = t < direct;
+  int r = 0;
+  long page = 0;
+  if (write) {
+    const int pos = tok_pos[t];
+    r = pos % RG_PAGE;
+    page = pages[(long)tok_entry[t] * P + pos / RG_PAGE];
+  }
+  float sq = 0.0f, sk = 0.0f;
+  f32x8 qv[AQ], kv[AK];
+  const f32x8 none = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+  for (int k = 0; k < NQ; ++k) {
+    const int i = k * GR_BLOCK + tid;
+    qv[k] = i < nq && i % nc * 8 < a.D ? value8(rq[k]) : none;
+    sq += squares(qv[k]);
+  }
+#pragma unroll
+  for (int k = 0; k < NK; ++k) {
+    const int i = k * GR_BLOCK + tid;
+    kv[k] = i < nk && i % nc * 8 < a.D ? value8(rk[k]) : none;
+    sk += squares(kv[k]);
+  }
+  if constexpr (NQ == 0)
+    for (int i = tid; i < nq; i += GR_BLOCK)
+      sq += squares(chunk8<T, VEC>(yq, i, a.D, nc));
+  if constexpr (NK == 0)
+    for (int i = tid; i < nk; i += GR_BLOCK)
+      sk += squares(chunk8<T, VEC>(yk, i, a.D, nc));
   sq = wave_sum(sq);
   sk = wave_sum(sk);
   if (tid % WAVE == 0) {
-    scratch[0][tid / WAVE] = sq;
-    scratch[1][tid / WAVE] = sk;
+    sums[0][tid / WAVE] = sq;
+    sums[1][tid / WAVE] = sk;
   }
   __syncthreads();
   sq = sk = 0.0f;
 #pragma unroll
   for (int w = 0; w < GR_BLOCK / WAVE; ++w) {
-    sq += scratch[0][w];
-    sk += scratch[1][w];
+    sq += sums[0][w];
+    sk += sums[1][w];
   }
   const float qi = 1.0f / sqrtf(sq / (float)(a.H * a.D) + a.eps);
   const float ki = 1.0f / sqrtf(sk / (float)(a.G * a.D) + a.eps);
   if (tid == 0) kinv[t] = ki;
 
-  const int nc = a.dimp / 8;
   T* qo = q + t * a.H * a.dimp;
-  for (int i = tid; i < a.H * nc; i += GR_BLOCK) {
-    const int h = i / nc, c = (i - h * nc) * 8;
-    float v[8];
-    normed8<T, VEC>(yq + h * a.D, wq ? wq + h * a.D : nullptr, c, a.D, qi, v);
-    store8(qo + (long)i * 8, v);
+#pragma unroll
+  for (int k = 0; k < NQ; ++k) {
+    const int i = k * GR_BLOCK + tid;
+    if (i < nq)
+      store8(qo + (long)i * 8, wq ? qv[k] * qi * value8(rqw[k]) : qv[k]);
   }
-  if (t >= direct) return;
+  if constexpr (NQ == 0) {
+    for (int i = tid; i < nq; i += GR_BLOCK) {
+      f32x8 v = chunk8<T, VEC>(yq, i, a.D, nc);
+      if (wq) v = v * qi * chunk8<T, VEC>(wq, i, a.D, nc);
+      store8(qo + (long)i * 8, v);
+    }
+  }
+  if (!write) return;
 
-  const int pos = tok_pos[t], r = pos % RG_PAGE;
-  const long page = pages[(long)tok_entry[t] * P + pos / RG_PAGE];
   const long PW = (long)RG_PAGE * (a.dimp + a.vdp);
   T* base = (T*)a.pool + page * a.G * PW;
-  for (int i = tid; i < a.G * nc; i += GR_BLOCK) {
+  auto key_at = [&](int i) {
     const int g = i / nc, c = (i - g * nc) * 8;
-    float v[8];
-    normed8<T, VEC>(yk + g * a.D, wk ? wk + g * a.D : nullptr, c, a.D, ki, v);
-    store8(base + g * PW +
-               ((r / 16 * (a.dimp / 32) + c / 32) * 64 + c / 8 % 4 * 16 +
-                r % 16) * 8, v);
+    return base + g * PW +
+           ((r / 16 * (a.dimp / 32) + c / 32) * 64 + c / 8 % 4 * 16 + r % 16) *
+               8;
+  };
+#pragma unroll
+  for (int k = 0; k < NK; ++k) {
+    const int i = k * GR_BLOCK + tid;
+    if (i < nk) store8(key_at(i), wk ? kv[k] * ki * value8(rkw[k]) : kv[k]);
+  }
+  if constexpr (NK == 0) {
+    for (int i = tid; i < nk; i += GR_BLOCK) {
+      f32x8 v = chunk8<T, VEC>(yk, i, a.D, nc);
+      if (wk) v = v * ki * chunk8<T, VEC>(wk, i, a.D, nc);
+      store8(key_at(i), v);
+    }
   }
   const T* first = a.first ? (const T*)a.first + t * a.fstride : nullptr;
   const float lam = first ? (float)((const T*)a.vmix)[0] : 0.0f;
@@ -170,10 +229,11 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
     const int s = tile / nk * 16 + lane % 16;
     const int c = tile % nk * 32 + lane / 16 * 8;
     if (s < lo) continue;
-    float v[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-    if (s < hi)
-      normed8<T, VEC>(y + (t + s) * a.ystride + koff, wk, c, a.D,
-                      wk ? kinv[t + s] : 1.0f, v);
+    f32x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+    if (s < hi) {
+      v = head8<T, VEC>(y + (t + s) * a.ystride + koff, c, a.D);
+      if (wk) v = v * kinv[t + s] * head8<T, VEC>(wk, c, a.D);
+    }
     store8(base + (long)i * 8, v);
   }
 
@@ -184,15 +244,13 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
     if (d0) __syncthreads();
     for (int i = tid; i < RG_PAGE * 8; i += GR_BLOCK) {
       const int s = i / 8, c = d0 + i % 8 * 8;
-      float v[8] = {0, 0, 0, 0, 0, 0, 0, 0};
+      f32x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
       if (s >= lo && s < hi) {
-        head8<T, VEC>(y + (t + s) * a.ystride + voff, c, a.V, v);
-        if (first) {
-          float u[8];
-          head8<T, VEC>(first + (t + s) * a.fstride + (long)g * a.V, c, a.V, u);
-#pragma unroll
-          for (int j = 0; j < 8; ++j) v[j] = (1.0f - lam) * v[j] + lam * u[j];
-        }
+        v = head8<T, VEC>(y + (t + s) * a.ystride + voff, c, a.V);
+        if (first)
+          v = (1.0f - lam) * v +
+              lam * head8<T, VEC>(
+                        first + (t + s) * a.fstride + (long)g * a.V, c, a.V);
       }
       T* o = &sv[s][i % 8 * 8];
       store4(o, f32x4{v[0], v[1], v[2], v[3]});
@@ -205,7 +263,7 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
       const int s = i / 64 % 2 * 32 + lane / 16 * 4;  // first key of the eight
       const int d = i / 128 * 16 + lane % 16;
       T* o = base + ((long)(d0 / 16) * 128 + i) * 8;
-      float v[8];
+      f32x8 v;
 #pragma unroll
       for (int j = 0; j < 8; ++j) v[j] = (float)sv[s + (j < 4 ? j : 12 + j)][d];
       if (s >= lo) {
@@ -225,16 +283,23 @@ extern "C" void launch_grouped_append(const GroupedRowArgs* a, void* q,
                                       int P, int direct, long n_tok, bool f32,
                                       hipStream_t stream) {
   dim3 grid((unsigned)n_tok), block(GR_BLOCK);
-#define GR_GO(T, VEC)                                        \
-  grouped_append_kernel<T, VEC><<<grid, block, 0, stream>>>( \
+  const int nq = (a->H * (a->dimp / 8) + GR_BLOCK - 1) / GR_BLOCK;
+  const int nk = (a->G * (a->dimp / 8) + GR_BLOCK - 1) / GR_BLOCK;
+#define GR_GO(T, VEC, NQ, NK)                                        \
+  grouped_append_kernel<T, VEC, NQ, NK><<<grid, block, 0, stream>>>( \
       *a, (T*)q, kinv, tok_pos, tok_entry, pages, P, direct)
-  if (f32) {
-    if (a->vec) GR_GO(float, true);
-    else GR_GO(float, false);
-  } else {
-    if (a->vec) GR_GO(__bf16, true);
-    else GR_GO(__bf16, false);
-  }
+#define GR_ROW(T)                                              \
+  do {                                                         \
+    if (!a->vec) GR_GO(T, false, 0, 0);                        \
+    else if (nq > 4) GR_GO(T, true, 0, 0);                     \
+    else if (nq <= 1) GR_GO(T, true, 1, 1);                    \
+    else if (nq <= 2 && nk <= 1) GR_GO(T, true, 2, 1);         \
+    else if (nk <= 1) GR_GO(T, true, 4, 1);                    \
+    else GR_GO(T, true, 4, 4);                                 \
+  } while (0)
+  if (f32) GR_ROW(float);
+  else GR_ROW(__bf16);
+#undef GR_ROW
 #undef GR_GO
 }
 
@@ -288,8 +353,7 @@ __global__ __launch_bounds__(GR_BLOCK) void gelu_kernel(
   if constexpr (VEC) {
     const int c = (blockIdx.x * GR_BLOCK + threadIdx.x) * 8;
     if (c >= C) return;
-    float v[8];
-    load8(xr + c, v);
+    f32x8 v = load8(xr + c);
 #pragma unroll
     for (int j = 0; j < 8; ++j) v[j] = gelu_erf<T>(v[j]);
     store8(orow + c, v);
@@ -318,20 +382,44 @@ extern "C" void launch_gelu(const void* x, void* o, long rows, int C, long xs,
 #undef GR_GO
 }
 
-// limit * tanh(z * scale / limit)
+// limit * tanh(z * scale / limit), four columns at a time.
+template <typename T>
+__device__ __forceinline__ float tanh_any(float x);
+template <>
+__device__ __forceinline__ float tanh_any<float>(float x) {
+  return tanhf(x);
+}
+// logits that come in bf16: tanh by its definition, off by 1e-7 at most
+template <>
+__device__ __forceinline__ float tanh_any<__bf16>(float x) {
+  const float e = __builtin_amdgcn_exp2f(2.88539008177792681472f * fabsf(x));
+  return copysignf(1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f), x);
+}
+
 template <typename T>
 __global__ __launch_bounds__(GR_BLOCK) void cap_logits_kernel(
     const T* __restrict__ z, float* __restrict__ o, long n, float scale,
     float limit) {
-  const long step = (long)gridDim.x * GR_BLOCK;
-  for (long i = (long)blockIdx.x * GR_BLOCK + threadIdx.x; i < n; i += step)
-    o[i] = limit * tanhf((float)z[i] * scale / limit);
+  const float by = scale / limit;
+  const long step = (long)gridDim.x * GR_BLOCK * 4;
+  for (long i = ((long)blockIdx.x * GR_BLOCK + threadIdx.x) * 4; i < n;
+       i += step) {
+    if (i + 4 <= n) {
+      f32x4 v = load4(z + i);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = limit * tanh_any<T>(v[j] * by);
+      store4(o + i, v);
+    } else {
+      for (long j = i; j < n; ++j)
+        o[j] = limit * tanh_any<T>((float)z[j] * by);
+    }
+  }
 }
 
 extern "C" void launch_cap_logits(const void* z, float* o, long n, float scale,
                                   float limit, bool f32, hipStream_t stream) {
-  const long want = (n + GR_BLOCK - 1) / GR_BLOCK;
-  dim3 grid((unsigned)(want < 8192 ? want : 8192)), block(GR_BLOCK);
+  const long want = (n + GR_BLOCK * 4 - 1) / (GR_BLOCK * 4);
+  dim3 grid((unsigned)(want < 16384 ? want : 16384)), block(GR_BLOCK);
   if (f32)
     cap_logits_kernel<float><<<grid, block, 0, stream>>>((const float*)z, o, n,
                                                          scale, limit);

@@ -149,7 +149,8 @@ def batch_of(portions, device, max_tokens=640):
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,G,D,V", [(6, 2, 24, 40), (2, 1, 17, 5), (4, 4, 128, 64),
-                                     (3, 3, 272, 8)])
+                                     (3, 3, 272, 8), (40, 5, 72, 16),
+                                     (24, 4, 256, 8), (64, 8, 160, 24)])
 def test_append(device, dtype, H, G, D, V):
     """Queries and keys normed over their whole rows, values blended, each in
     its slot; slots before a portion's start keep what they hold."""
