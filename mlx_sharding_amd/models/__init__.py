@@ -13,6 +13,7 @@ from .llama import LlamaStageModel
 from .gemma2 import Gemma2StageModel
 from .deepseek_v2 import DeepseekV2StageModel
 from .lepizen import LepizenStageModel
+from .sadosun import SadosunStageModel
 from .tuvutar import TuvutarStageModel
 
 MODEL_REMAPPING: Dict[str, str] = {
@@ -29,6 +30,7 @@ _REGISTRY: Dict[str, Type[StageModel]] = {
     "deepseek_v2": DeepseekV2StageModel,
     "tuvutar": TuvutarStageModel,
     "lepizen": LepizenStageModel,
+    "sadosun": SadosunStageModel,
 }
 
 

@@ -75,8 +75,9 @@ def fuse_model(model) -> int:
     from .llama import LlamaAttention, LlamaMLP
     from .gemma2 import Gemma2Attention, Gemma2MLP
     from .deepseek_v2 import MLAAttention
-    from .mixers import (GatedDelta, GatedMLP, LatentAttention,
-                         ParallelBlock)
+    from .mixers import (CausalConv, GatedDelta, GatedMLP, GroupedAttention,
+                         LatentAttention, ParallelBlock, RoutedExperts,
+                         SelectiveScan)
 
     n = 0
     for mod in model.modules():
@@ -90,8 +91,10 @@ def fuse_model(model) -> int:
             elif isinstance(mod, MLAAttention) and not mod.q_lora_rank:
                 mod._fused_qkv = FusedColumns([mod.q_proj, mod.kv_a_proj_with_mqa])
                 n += 1
-            elif isinstance(mod, (GatedDelta, GatedMLP, LatentAttention,
-                                  ParallelBlock)):
+            elif isinstance(mod, (CausalConv, GatedDelta, GatedMLP,
+                                  GroupedAttention, LatentAttention,
+                                  ParallelBlock, RoutedExperts,
+                                  SelectiveScan)):
                 mod.prepare()
                 n += 1
         except AssertionError:

@@ -16,9 +16,12 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from .. import ops
-from ..ops import ragged
-from ..ops.paged import LayerStore, RaggedBatch, RowSpec, StateSpec
-from ..ops.ragged import DeltaShape, GroupedShape, LatentShape, Rotary
+from ..ops import experts, ragged, recurrent
+from ..ops.experts import ExpertShape
+from ..ops.paged import (HistorySpec, LayerSpec, LayerStore, RaggedBatch,
+                         RowSpec, StateSpec)
+from ..ops.ragged import DeltaShape, GroupedShape, LatentShape, Rotary, Turns
+from ..ops.recurrent import ScanShape
 from .base import Linear, RMSNorm
 
 
@@ -38,6 +41,51 @@ class _Weight(nn.Module):
     def __init__(self, *shape, dtype):
         super().__init__()
         self.weight = _param(*shape, dtype=dtype)
+
+
+class _Biased(_Weight):
+    """A weight with a vector ``b``."""
+
+    def __init__(self, *shape, dtype):
+        super().__init__(*shape, dtype=dtype)
+        self.b = _param(shape[0], dtype=dtype)
+
+
+class CausalConv(nn.Module):
+    """A causal convolution over time per channel, ``weight`` [channels, taps],
+    the last tap on the current token, and a bias ``b`` if asked for."""
+
+    def __init__(self, channels: int, taps: int, bias: bool,
+                 dtype: torch.dtype):
+        super().__init__()
+        if not 1 <= taps <= recurrent.MAX_TAPS:
+            raise ValueError(f"convolutions have 1 to {recurrent.MAX_TAPS} "
+                             f"taps, not {taps}")
+        self.weight = _param(channels, taps, dtype=dtype)
+        self.b = _param(channels, dtype=dtype) if bias else None
+        self._by_tap = None
+
+    def prepare(self):
+        self._by_tap = self.weight.data.T.contiguous()
+
+    @property
+    def by_tap(self) -> torch.Tensor:
+        """[taps, channels], as the kernels read it."""
+        if self._by_tap is None:
+            self.prepare()
+        return self._by_tap
+
+    def history(self) -> HistorySpec:
+        channels, taps = self.weight.shape
+        return HistorySpec(channels, taps - 1)
+
+
+class ScalarNorm(nn.Module):
+    """An RMS norm whose weight is one number."""
+
+    def __init__(self, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.weight = _param(dtype=dtype)
 
 
 class ConvLinear(Linear):
@@ -156,20 +204,30 @@ class LatentAttention(nn.Module):
 
 class GroupedAttention(nn.Module):
     """Causal softmax attention, ``heads`` query heads over ``kv_heads`` cached
-    keys and values, without positions.
+    keys and values.
 
     ``qk_norm``: RMS norms over the whole query and the whole key projection.
+    ``head_norm``: every query and key divided by its own root mean square.
+    ``rotary``: positions on queries and keys; ``turn_values``: positions on the
+    values as well, undone on each output by its own position.
+    ``window``: how many tokens a token sees, up to itself.
     ``sink``: one learned score per head that enters the softmax's denominator
-    and nothing else.  ``vmix``: the share of another layer's values in this
-    layer's, where the caller passes such values.
+    and nothing else; ``zero_sink``: that score is 0 for every head.
+    ``vmix``: the share of another layer's values in this layer's, where the
+    caller passes such values.
     """
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
                  vdim: int, scale: float, eps: float, qk_norm: bool = False,
-                 sink: bool = False, dtype: torch.dtype = torch.bfloat16):
+                 sink: bool = False, dtype: torch.dtype = torch.bfloat16, *,
+                 head_norm: bool = False, rotary: Optional[Rotary] = None,
+                 turn_values: Optional[Rotary] = None,
+                 window: Optional[int] = None, zero_sink: bool = False):
         super().__init__()
         self.shape = sh = GroupedShape(heads, kv_heads, dim, vdim)
         self.scale, self.eps = float(scale), eps
+        self.head_norm, self.window = head_norm, window
+        self.rotary, self.turn_values = rotary, turn_values
 
         def lin(out_features):
             if not qk_norm:
@@ -178,12 +236,25 @@ class GroupedAttention(nn.Module):
 
         self.q, self.k = lin(heads * dim), lin(kv_heads * dim)
         self.v = Linear(width, kv_heads * vdim, dtype=dtype)
-        self.vmix = _param(dtype=dtype)
-        self.sink = _param(heads, dtype=dtype) if sink else None
+        self.vmix = None
+        if rotary is None and turn_values is None and not head_norm:
+            self.vmix = _param(dtype=dtype)
+        if zero_sink:
+            self.register_buffer("sink", torch.zeros(heads, dtype=dtype),
+                                 persistent=False)
+        else:
+            self.sink = _param(heads, dtype=dtype) if sink else None
         self.o = Linear(heads * vdim, width, dtype=dtype)
         self.w_in = None
         if max(sh.dimp, sh.vdp) > sh.MAX:
             raise ValueError(f"head sizes {dim}/{vdim} are above {sh.MAX}")
+        if rotary is not None and (rotary.dims > dim or rotary.dims % 2):
+            raise ValueError(f"{rotary.dims} of {dim} dimensions cannot be "
+                             f"rotated in pairs")
+        if turn_values is not None and (vdim % 2 or turn_values.dims != vdim):
+            raise ValueError("values are rotated whole, in pairs")
+        if window is not None and window < 1:
+            raise ValueError("a window holds at least the token itself")
 
     def store_spec(self) -> RowSpec:
         return RowSpec(self.shape.width)
@@ -195,33 +266,91 @@ class GroupedAttention(nn.Module):
 
     @torch.no_grad()
     def prepare(self):
-        self.w_in = torch.cat([m.weight.data for m in self.rows]).contiguous()
+        if self.w_in is not None:
+            return
+        w = torch.cat([m.weight.data for m in self.rows])
+        # rows of the projection start at whole vectors
+        self.w_in = F.pad(w, (0, 0, 0, -w.shape[0] % 8)).contiguous()
         _share(self.w_in, *self.rows)
 
     def attend(self, y: torch.Tensor, out: torch.Tensor, batch: RaggedBatch,
-               store: LayerStore, first: Optional[torch.Tensor] = None
-               ) -> torch.Tensor:
+               store: LayerStore, first: Optional[torch.Tensor] = None,
+               turns: Optional[Turns] = None) -> torch.Tensor:
         """y [N, q | k | v | ...]; writes out [N, heads * vdim].  first: values
-        [N, kv_heads * vdim] to mix in.  Returns this layer's values before
-        mixing, a view of y."""
+        [N, kv_heads * vdim] to mix in.  turns: the tables of this layer's
+        rotations.  Returns this layer's values before mixing, a view of y."""
         sh = self.shape
         norms = [getattr(m, "norm", None) for m in (self.q, self.k)]
         q = ragged.grouped_append(
             y, *(None if n is None else n.weight for n in norms), self.eps,
-            None if first is None else self.vmix, first, store, sh, batch)
-        ragged.grouped_attention(q, self.sink, store, sh, self.scale, batch, out)
+            None if first is None else self.vmix, first, store, sh, batch,
+            turns, self.head_norm)
+        ragged.grouped_attention(q, self.sink, store, sh, self.scale, batch, out,
+                                 self.window, turns)
         at = (sh.heads + sh.kv_heads) * sh.dim
         return y[:, at: at + sh.kv_heads * sh.vdim]
 
     def forward(self, h: torch.Tensor, batch: RaggedBatch, store: LayerStore,
-                first: Optional[torch.Tensor] = None):
+                first: Optional[torch.Tensor] = None,
+                turns: Optional[Turns] = None):
         """Returns (output, values before mixing)."""
         if self.w_in is None:
             self.prepare()
         y = ops.linear(h, self.w_in)
         out = y.new_empty(y.shape[0], self.o.in_features)
-        v = self.attend(y, out, batch, store, first)
+        v = self.attend(y, out, batch, store, first, turns)
         return self.o(out), v
+
+
+class SelectiveScan(nn.Module):
+    """Mamba: a diagonal linear recurrence per channel with ``states`` fp32
+    states, whose step size, input and read-out vectors depend on the token,
+    behind a short convolution and before a silu gate."""
+
+    def __init__(self, width: int, channels: int, states: int, rank: int,
+                 taps: int, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.shape = sh = ScanShape(channels, states, rank)
+        if states > sh.MAX:
+            raise ValueError(f"{states} states are above {sh.MAX}")
+        self.add_module("in", Linear(width, 2 * channels, dtype=dtype))
+        self.conv = CausalConv(channels, taps, True, dtype)
+        self.x = Linear(channels, rank + 2 * states, dtype=dtype)
+        self.dt = _Biased(channels, rank, dtype=dtype)
+        self.A_log = _param(channels, states, dtype=dtype)
+        self.D = _param(channels, dtype=dtype)
+        self.o = Linear(channels, width, dtype=dtype)
+        self.ready = False
+
+    def store_spec(self) -> LayerSpec:
+        sh = self.shape
+        return LayerSpec(StateSpec(1, sh.statesp, sh.channels),
+                         {"conv": self.conv.history()})
+
+    @torch.no_grad()
+    def prepare(self):
+        sh, w = self.shape, self.x.weight.data
+        # [step input | B | C], each from a whole vector on, zeros between
+        self.w_x = w.new_zeros(sh.width, w.shape[1])
+        for at, part in zip(sh.columns, w.split([sh.rank, sh.states, sh.states])):
+            self.w_x[at: at + part.shape[0]] = part
+        self.A = F.pad(-torch.exp(self.A_log.data.float()).T,
+                       (0, 0, 0, sh.statesp - sh.states)).contiguous()
+        self.D32, self.b32 = self.D.data.float(), self.dt.b.data.float()
+        self.ready = True
+
+    def forward(self, h: torch.Tensor, batch: RaggedBatch,
+                store: LayerStore) -> torch.Tensor:
+        if not self.ready:
+            self.prepare()
+        sh = self.shape
+        x, z = getattr(self, "in")(h).split(sh.channels, 1)
+        x = recurrent.causal_conv(x, self.conv.by_tap, self.conv.b,
+                                  store.histories["conv"], batch, silu=True)
+        y = ops.linear(x, self.w_x)
+        dt = ops.linear(y[:, : sh.rank], self.dt.weight)
+        return self.o(recurrent.selective_scan(x, z, dt, self.b32, y, self.A,
+                                               self.D32, store.state, sh, batch))
 
 
 class GatedDelta(nn.Module):
@@ -346,6 +475,7 @@ class ParallelBlock(nn.Module):
         self.w_in = F.pad(self.w_in, (0, 0, 0, -self.w_in.shape[0] % 8))
         self.w_in = self.w_in.contiguous()
         _share(self.w_in, *rows)
+        self.mix.w_in = self.w_in[: self.taken]
 
     def forward(self, h: torch.Tensor, batch: RaggedBatch, store: LayerStore,
                 *extra):
@@ -359,3 +489,76 @@ class ParallelBlock(nn.Module):
             self.mlp.act(y[:, self.taken: self.taken + self.hidden],
                          z[:, self.mixed:])
         return ops.linear(z, self.w_out), got
+
+
+class _Stacked(nn.Module):
+    """One matrix per expert, ``weight`` [experts, out, in]."""
+
+    def __init__(self, n: int, out_features: int, in_features: int,
+                 dtype: torch.dtype):
+        super().__init__()
+        self.weight = _param(n, out_features, in_features, dtype=dtype)
+
+    def pad(self, rows: int, cols: int) -> torch.Tensor:
+        """The weights with zeros up to this size; the parameter stays a view."""
+        n, r, c = self.weight.shape
+        w = F.pad(self.weight.data, (0, cols - c, 0, rows - r)).contiguous()
+        self.weight.data = w[:, :r, :c]
+        return w
+
+
+class RoutedExperts(nn.Module):
+    """Every token's ``top`` of ``experts`` ungated relu^2 feed-forwards and
+    ``identity`` experts that return their input.  A softmax router in 32-bit;
+    ``correction`` biases the choice but not the weights."""
+
+    def __init__(self, width: int, ff: int, experts: int, identity: int,
+                 top: int, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.shape = sh = ExpertShape(width, ff, experts, identity, top)
+        self.up = _Stacked(experts, ff, width, dtype)
+        self.down = _Stacked(experts, width, ff, dtype)
+        self.router = Linear(width, sh.total, dtype=dtype)
+        self.correction = _param(sh.total, dtype=dtype)
+        self.ready = False
+
+    @torch.no_grad()
+    def prepare(self):
+        sh = self.shape
+        self.w_up = self.up.pad(sh.ffp, sh.widthp)
+        self.w_down = self.down.pad(sh.width, sh.ffp)
+        w = F.pad(self.router.weight.data, (0, sh.widthp - sh.width)).contiguous()
+        self.router.weight.data = w[:, : sh.width]
+        self.w_router = w
+        self.ready = True
+
+    def forward(self, x: torch.Tensor, h: torch.Tensor,
+                copy: bool = False) -> Optional[torch.Tensor]:
+        """Adds to the residual x in place; h [N, width padded to a multiple of
+        ``ExpertShape.STEP``].  copy: returns the new x in h's type."""
+        if not self.ready:
+            self.prepare()
+        return experts.add_experts(x, h, self.w_router, self.correction,
+                                   self.w_up, self.w_down, self.shape, copy)
+
+
+class TokenInput(nn.Module):
+    """What a layer takes from a token's own row of an embedding table:
+    W_proj (gelu_tanh(W_gate x) * e), to be RMS-normed with ``norm`` and added
+    to the residual x."""
+
+    def __init__(self, width: int, dim: int, eps: float,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.gate = Linear(width, dim, dtype=dtype)
+        self.proj = Linear(dim, width, dtype=dtype)
+        self.norm = RMSNorm(width, eps, dtype=dtype)
+
+    def forward(self, x: torch.Tensor, e: torch.Tensor,
+                copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """x: fp32 residual; e [N, dim]; copy: x in the weights' type, where
+        the caller has it."""
+        g = experts.token_gate(x, self.gate.weight, e)
+        if g is None:
+            g = ops.geglu(self.gate(x.to(e.dtype) if copy is None else copy), e)
+        return self.proj(g)

@@ -7,7 +7,7 @@ config.json gives ``width``, ``vocab``, ``norm.eps`` and ``layers``, a list of
 
 from __future__ import annotations
 
-from typing import List, Optional, Tuple
+from typing import Dict, List, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -15,6 +15,7 @@ import torch.nn.functional as F
 
 from ..config import ModelConfig, ShardSpec
 from ..ops.paged import PagedState, RaggedBatch, RaggedCache, RaggedLayerCache
+from ..ops.ragged import Rotary
 from .base import Linear, RMSNorm, StageModel, owned_layer_indices
 
 
@@ -40,12 +41,17 @@ class RaggedStageModel(StageModel):
                                                      W, dtype))
         if shard.is_last:
             self.final = nn.Module()
-            self.final.norm = RMSNorm(W, self.eps, self.norm_offset, dtype)
+            self.final.norm = self.make_final_norm(W, dtype)
             self.head = Linear(W, config.vocab_size, dtype=dtype)
+        self._tables: Dict = {}
+        self._old_tables: List = []  # captured graphs may still read them
 
     def make_layer(self, i: int, spec: dict, width: int,
                    dtype: torch.dtype) -> nn.Module:
         raise NotImplementedError
+
+    def make_final_norm(self, width: int, dtype: torch.dtype) -> nn.Module:
+        return RMSNorm(width, self.eps, self.norm_offset, dtype)
 
     def layer(self, i: int) -> nn.Module:
         return getattr(self, f"l{i}")
@@ -79,7 +85,11 @@ class RaggedStageModel(StageModel):
 
     # -- cache -------------------------------------------------------------
     def store_specs(self) -> List:
-        return [layer.mix.store_spec() for _, layer in self.layer_items()]
+        return [self.layer_spec(layer) for _, layer in self.layer_items()]
+
+    def layer_spec(self, layer: nn.Module):
+        """What one layer keeps between steps (ops.paged)."""
+        return layer.mix.store_spec()
 
     def make_state(self, max_tokens: int, max_requests: int) -> PagedState:
         p = next(self.parameters())
@@ -94,6 +104,16 @@ class RaggedStageModel(StageModel):
         return [RaggedLayerCache(shared, i) for i in range(self.shard.n_layers)]
 
     # -- forward -----------------------------------------------------------
+    def _rotation(self, rotary: Rotary, n: int, device):
+        """(cos, sin) tables of at least n positions."""
+        got = self._tables.get(rotary)
+        if got is None or got[0].shape[0] < n or got[0].device != device:
+            if got is not None:
+                self._old_tables.append(got)
+            rows = max(1024, 1 << max(n - 1, 1).bit_length())
+            got = self._tables[rotary] = rotary.tables(rows, device)
+        return got
+
     def residual(self, x: torch.Tensor) -> torch.Tensor:
         """What the first owned layer adds to: embedded token ids, or a copy
         of the residual stream that the previous stage handed on."""

@@ -12,7 +12,7 @@ Tensors: ``embed``, ``l<i>.norm1`` / ``norm1b`` / ``norm2`` / ``norm2b``,
 
 from __future__ import annotations
 
-from typing import Dict, List, Optional
+from typing import List, Optional
 
 import torch
 import torch.nn as nn
@@ -86,8 +86,6 @@ class TuvutarStageModel(RaggedStageModel):
                     f"layer {i} reads the rows of layer {j}, which stage "
                     f"[{shard.start_layer}, {shard.end_layer}) does not run "
                     f"before it")
-        self._tables: Dict = {}
-        self._old_tables: List = []  # captured graphs may still read them
 
     def make_layer(self, i, spec, width, dtype):
         return TuvutarLayer(spec, width, self.eps, dtype)
@@ -105,15 +103,6 @@ class TuvutarStageModel(RaggedStageModel):
         return [c for c in range(1, n) if c not in bad]
 
     # -- forward -----------------------------------------------------------
-    def _rotation(self, rotary: Rotary, n: int, device):
-        got = self._tables.get(rotary)
-        if got is None or got[0].shape[0] < n or got[0].device != device:
-            if got is not None:
-                self._old_tables.append(got)
-            rows = max(1024, 1 << max(n - 1, 1).bit_length())
-            got = self._tables[rotary] = rotary.tables(rows, device)
-        return got
-
     @torch.no_grad()
     def run(self, x: torch.Tensor, batch: RaggedBatch, state: PagedState,
             rows: Optional[torch.Tensor] = None,

@@ -13,7 +13,10 @@
 // without leaving the lane.
 //
 // The optional sink is one more term of the softmax's denominator, with
-// neither key nor value; it enters once, when a row is finished.
+// neither key nor value; it enters once, when a row is finished.  With a window
+// a token sees its last `window` tokens; pages before all of a block's windows
+// are not visited.  Where values were rotated by their positions, a finished
+// row is turned back by its own.
 #pragma once
 
 #include "ragged_common.h"
@@ -25,6 +28,12 @@ struct GroupedRowArgs {
   int H, G, D, V, dimp, vdp;
   float eps;
   bool vec;  // heads, rows and bases are whole vectors of 8
+  // rotations by position, [positions, pairs]: the first 2 * qk_pairs
+  // dimensions of queries and keys, the first 2 * v_pairs of values
+  const float *qk_cos, *qk_sin, *v_cos, *v_sin;
+  int qk_pairs, v_pairs;
+  const int* tok_pos;
+  bool head_norm;  // queries and keys over their own root mean squares
 };
 
 struct GroupedAttnArgs {
@@ -37,6 +46,9 @@ struct GroupedAttnArgs {
   long n_rows, ostride;
   float scale;
   bool vec;  // rows of out take vectors of 4
+  int window;                 // 0: every earlier token is seen
+  const float *v_cos, *v_sin; // [positions, V / 2] or null
+  const int* tok_pos;
 };
 
 #define GA_BLOCK 256
@@ -101,6 +113,22 @@ __device__ __forceinline__ void store_cols(T* o, int col, int V, f32x4 v,
   }
 }
 
+// columns col .. col + 3 of a finished row at `pos`, turned back
+__device__ __forceinline__ f32x4 turn_back(const GroupedAttnArgs& a, int pos,
+                                           int col, f32x4 v) {
+  if (!a.v_cos || col >= a.V) return v;
+  const int half = a.V / 2, p = col / 2, q = min(p + 1, half - 1);
+  const float* c = a.v_cos + (long)pos * half;
+  const float* s = a.v_sin + (long)pos * half;
+  return f32x4{v[0] * c[p] + v[1] * s[p], v[1] * c[p] - v[0] * s[p],
+               v[2] * c[q] + v[3] * s[q], v[3] * c[q] - v[2] * s[q]};
+}
+
+// the first token that one at `pos` sees
+__device__ __forceinline__ int first_seen(const GroupedAttnArgs& a, int pos) {
+  return a.window ? max(0, pos - a.window + 1) : 0;
+}
+
 // ---------------------------------------------------------------------------
 // Short portions and decoding.  A query row is one (token, head) pair of one
 // request and key/value head; a block serves 16 of them over one slice of the
@@ -128,9 +156,10 @@ __global__ __launch_bounds__(GA_BLOCK) void grouped_attn_short_kernel(
   if (r0 >= rows) return;
   const int p0 = a.pos0[e];
   const int S = p0 + min(r0 + 15, rows - 1) / R + 1;  // keys these rows see
-  const int steps = (S + GA_STEP - 1) / GA_STEP;
+  const int s0 = first_seen(a, p0 + r0 / R) / GA_STEP * GA_STEP;
+  const int steps = (S - s0 + GA_STEP - 1) / GA_STEP;
   const int per = (steps + a.nsplit - 1) / a.nsplit * GA_STEP;
-  const int lo = blockIdx.y * per;
+  const int lo = s0 + blockIdx.y * per;
   const int hi = min(S, lo + per);
 
   const int tid = threadIdx.x;
@@ -145,6 +174,7 @@ __global__ __launch_bounds__(GA_BLOCK) void grouped_attn_short_kernel(
   const int my_tok = my_row / R;
   const int my_head = g * R + my_row - my_tok * R;
   const int limit = min(p0 + my_tok + 1, hi);
+  const int from = first_seen(a, p0 + my_tok);
   const float scale = a.scale * sm_unit<T>();
 
   Frag<T> qf[NK];
@@ -194,7 +224,7 @@ __global__ __launch_bounds__(GA_BLOCK) void grouped_attn_short_kernel(
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int key = t + lg * 4 + (j < 4 ? j : 12 + j);
-      p[j] = key < limit ? sc[j / 4][j % 4] * scale : GA_NONE;
+      p[j] = key < limit && key >= from ? sc[j / 4][j % 4] * scale : GA_NONE;
       mx = fmaxf(mx, p[j]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
@@ -284,7 +314,7 @@ __global__ __launch_bounds__(GA_BLOCK) void grouped_attn_short_kernel(
       const int tok = (r0 + r) / R, h = g * R + (r0 + r) % R;
       if (last)
         store_cols((T*)a.out + (long)(t0 + tok) * a.ostride + (long)h * a.V,
-                   col, a.V, v, a.vec);
+                   col, a.V, turn_back(a, p0 + tok, col, v), a.vec);
       else
         store4(a.part_o +
                    (((long)(t0 + tok) * a.H + h) * a.nsplit + blockIdx.y) *
@@ -325,6 +355,7 @@ __global__ __launch_bounds__(128) void grouped_attn_merge_kernel(
 #pragma unroll
       for (int j = 0; j < 4; ++j) o[j] += v[j] * w[s];
     }
+    if (a.v_cos) o = turn_back(a, a.tok_pos[row / a.H], d, o);
     store_cols(out, d, a.V, o, a.vec);
   }
 }
@@ -389,8 +420,9 @@ void grouped_attn_long_kernel(
 
   const int hi = p0 + min(q0 + GA_QT, n);
   const int n_pages = (hi + RG_PAGE - 1) / RG_PAGE;
-  if constexpr (BUFS == 2) stage(0, table[0]);
-  int next = table[min(1, n_pages - 1)];
+  const int first = first_seen(a, p0 + q0) / RG_PAGE;
+  if constexpr (BUFS == 2) stage(first, table[first]);
+  int next = table[min(first + 1, n_pages - 1)];
 
   const int w0 = q0 + wid * 32;  // this wave's first query
   Frag<T> qf[2][NK];
@@ -409,6 +441,10 @@ void grouped_attn_long_kernel(
   }
   const int wave_lo = p0 + min(w0, n - 1);                // positions
   const int wave_hi = w0 < n ? p0 + min(w0 + 31, n - 1) + 1 : 0;
+  const int wave_from = first_seen(a, wave_lo);
+  int qfrom[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) qfrom[i] = first_seen(a, qpos[i]);
 
   float m_run[2] = {GA_NONE, GA_NONE}, l_run[2] = {0.0f, 0.0f};
   f32x4 acc[2][ND];
@@ -417,7 +453,7 @@ void grouped_attn_long_kernel(
 #pragma unroll
     for (int d = 0; d < ND; ++d) acc[i][d] = f32x4{0, 0, 0, 0};
 
-  for (int p = 0; p < n_pages; ++p) {
+  for (int p = first; p < n_pages; ++p) {
     if constexpr (BUFS == 1) {
       __syncthreads();
       stage(p, table[p]);
@@ -430,7 +466,7 @@ void grouped_attn_long_kernel(
         next = table[min(p + 2, n_pages - 1)];
       }
     const int t = p * RG_PAGE;
-    if (t >= wave_hi) continue;
+    if (t >= wave_hi || t + RG_PAGE <= wave_from) continue;
     const T* ks = (const T*)smem + (p % BUFS) * PW + lane * 8;
     const T* vs = ks + RG_PAGE * a.dimp;
 
@@ -462,6 +498,16 @@ void grouped_attn_long_kernel(
           for (int j = 0; j < 4; ++j)
             if (t + s * 16 + lg * 4 + j > qpos[i]) sc[i][s][j] = GA_NONE;
     }
+    // the last query's window begins last
+    if (t < first_seen(a, wave_hi - 1)) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            if (t + s * 16 + lg * 4 + j < qfrom[i]) sc[i][s][j] = GA_NONE;
+    }
     float alpha[2];
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
@@ -475,13 +521,14 @@ void grouped_attn_long_kernel(
       const float m_new = fmaxf(m_run[i], mx);
       alpha[i] = sm_exp<T>(m_run[i] - m_new);
       m_run[i] = m_new;
+      // a window may begin behind its block's first page: no score yet
+      const float m_ref = m_new == GA_NONE ? 0.0f : m_new;
       float sum = 0.0f;
 #pragma unroll
       for (int s = 0; s < 4; ++s)
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          // key 0 is in the first page, so m_new is a real score
-          const float w = sm_exp<T>(sc[i][s][j] - m_new);
+          const float w = sm_exp<T>(sc[i][s][j] - m_ref);
           sc[i][s][j] = w;
           sum += w;
         }
@@ -538,6 +585,7 @@ void grouped_attn_long_kernel(
       f32x4 c4 = acc[i][d];
 #pragma unroll
       for (int j = 0; j < 4; ++j) c4[j] *= f;
+      c4 = turn_back(a, p0 + r, d * 16 + lg * 4, c4);
       store_cols(o, d * 16 + lg * 4, a.V, c4, a.vec);
     }
   }

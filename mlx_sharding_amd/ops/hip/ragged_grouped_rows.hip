@@ -1,5 +1,6 @@
-// Row work around grouped attention: norms of the projections, blended
-// values, writing keys and values to their pages; exact gelu; capped logits.
+// Row work around grouped attention: norms of the projections, rotations,
+// blended values, writing keys and values to their pages; exact gelu; capped
+// logits.
 #include "ragged_grouped.h"
 
 #define GR_BLOCK 256
@@ -56,6 +57,34 @@ __device__ __forceinline__ float squares(f32x8 v) {
   return s;
 }
 
+// Columns c .. c + 7 of one head with their pairs rotated, as far as pairs are.
+__device__ __forceinline__ f32x8 turn8(f32x8 v, const float* cos_t,
+                                       const float* sin_t, int pairs, int pos,
+                                       int c) {
+  if (!cos_t || c >= 2 * pairs) return v;
+  const float* cp = cos_t + (long)pos * pairs + c / 2;
+  const float* sp = sin_t + (long)pos * pairs + c / 2;
+  f32x4 cs = {1, 1, 1, 1}, sn = {0, 0, 0, 0};
+  if (pairs % 4 == 0) {
+    cs = load4(cp);
+    sn = load4(sp);
+  } else {
+#pragma unroll
+    for (int p = 0; p < 4; ++p)
+      if (c / 2 + p < pairs) {
+        cs[p] = cp[p];
+        sn[p] = sp[p];
+      }
+  }
+  f32x8 o;
+#pragma unroll
+  for (int p = 0; p < 4; ++p) {
+    o[2 * p] = v[2 * p] * cs[p] - v[2 * p + 1] * sn[p];
+    o[2 * p + 1] = v[2 * p + 1] * cs[p] + v[2 * p] * sn[p];
+  }
+  return o;
+}
+
 // The i-th chunk of eight columns of a row of heads padded to 8 * nc columns.
 template <typename T, bool VEC>
 __device__ __forceinline__ f32x8 chunk8(const T* row, int i, int size, int nc) {
@@ -71,6 +100,11 @@ __device__ __forceinline__ const T* chunk_at(const T* row, int i, int n,
   i = min(i, n - 1);
   const int h = i / nc;
   return row + h * size + min((i - h * nc) * 8, size - 8);
+}
+
+// Where eight columns of a key in slot r of its page go, from the head's base.
+__device__ __forceinline__ int key_place(int r, int c, int dimp) {
+  return ((r / 16 * (dimp / 32) + c / 32) * 64 + c / 8 % 4 * 16 + r % 16) * 8;
 }
 
 // One block per token: queries out [N, H, dimp]; keys and values of the first
@@ -172,9 +206,7 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_append_kernel(
   T* base = (T*)a.pool + page * a.G * PW;
   auto key_at = [&](int i) {
     const int g = i / nc, c = (i - g * nc) * 8;
-    return base + g * PW +
-           ((r / 16 * (a.dimp / 32) + c / 32) * 64 + c / 8 % 4 * 16 + r % 16) *
-               8;
+    return base + g * PW + key_place(r, c, a.dimp);
   };
 #pragma unroll
   for (int k = 0; k < NK; ++k) {
@@ -203,10 +235,67 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_append_kernel(
   }
 }
 
+// The same with rotations and norms per head: `sub` lanes (a power of two) share
+// one head of one token, each eight of its columns.  Items of a token are its
+// query heads, keys and values; keys' inverse rms [N, G].
+template <typename T, bool VEC>
+__global__ __launch_bounds__(GR_BLOCK) void grouped_turn_kernel(
+    const GroupedRowArgs a, T* __restrict__ q, float* __restrict__ kinv,
+    const int* __restrict__ tok_entry, const int* __restrict__ pages, int P,
+    int direct, int sub, long n_tok) {
+  const int items = a.H + 2 * a.G;
+  const long at = ((long)blockIdx.x * GR_BLOCK + threadIdx.x) / sub;
+  const int c = threadIdx.x % sub * 8;
+  const long t = min(at / items, n_tok - 1);
+  const bool live = at / items < n_tok;
+  const int j = (int)(at - at / items * items);
+  const int pos = a.tok_pos[t];
+  const bool value = j >= a.H + a.G;
+  const int size = value ? a.V : a.D;
+  const T* src = (const T*)a.y + t * a.ystride +
+                 (value ? (long)(a.H + a.G) * a.D + (long)(j - a.H - a.G) * a.V
+                        : (long)j * a.D);
+  f32x8 v = head8<T, VEC>(src, c, size);
+  if (value)
+    v = turn8(v, a.v_cos, a.v_sin, a.v_pairs, pos, c);
+  else
+    v = turn8(v, a.qk_cos, a.qk_sin, a.qk_pairs, pos, c);
+  if (a.head_norm) {
+    float ss = squares(v);
+    for (int o = 1; o < sub; o <<= 1) ss += __shfl_xor(ss, o, WAVE);
+    const float inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+    if (!value) v = v * inv;
+    if (live && c == 0 && !value && j >= a.H) kinv[t * a.G + j - a.H] = inv;
+  }
+  if (!live) return;
+  if (j < a.H) {
+    if (c < a.dimp) store8(q + (t * a.H + j) * a.dimp + c, v);
+    return;
+  }
+  if (t >= direct) return;
+  const int r = pos % RG_PAGE;
+  const long page = pages[(long)tok_entry[t] * P + pos / RG_PAGE];
+  const int g = value ? j - a.H - a.G : j - a.H;
+  T* base = (T*)a.pool + (page * a.G + g) * RG_PAGE * (a.dimp + a.vdp);
+  if (!value) {
+    if (c < a.dimp) store8(base + key_place(r, c, a.dimp), v);
+    return;
+  }
+  base += RG_PAGE * a.dimp;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int d = c + i;
+    if (d < a.vdp)
+      base[((d / 16 * 2 + r / 32) * 64 + r / 4 % 4 * 16 + d % 16) * 8 +
+           r / 16 % 2 * 4 + r % 4] = (T)v[i];
+  }
+}
+
 // One block per (page, key/value head): the slots lo .. hi - 1 of a page from
 // tokens t + slot; later slots become zero, earlier ones stay.
 //   fills[i] = (page, t, lo, hi)
-template <typename T, bool VEC>
+// TURN: rotations and norms per head in place of weights and blended values.
+template <typename T, bool VEC, bool TURN>
 __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
     const GroupedRowArgs a, const float* __restrict__ kinv,
     const int* __restrict__ fills) {
@@ -232,7 +321,12 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
     f32x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
     if (s < hi) {
       v = head8<T, VEC>(y + (t + s) * a.ystride + koff, c, a.D);
-      if (wk) v = v * kinv[t + s] * head8<T, VEC>(wk, c, a.D);
+      if constexpr (TURN) {
+        v = turn8(v, a.qk_cos, a.qk_sin, a.qk_pairs, a.tok_pos[t + s], c);
+        if (a.head_norm) v = v * kinv[(t + s) * a.G + g];
+      } else {
+        if (wk) v = v * kinv[t + s] * head8<T, VEC>(wk, c, a.D);
+      }
     }
     store8(base + (long)i * 8, v);
   }
@@ -247,7 +341,9 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
       f32x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
       if (s >= lo && s < hi) {
         v = head8<T, VEC>(y + (t + s) * a.ystride + voff, c, a.V);
-        if (first)
+        if constexpr (TURN)
+          v = turn8(v, a.v_cos, a.v_sin, a.v_pairs, a.tok_pos[t + s], c);
+        else if (first)
           v = (1.0f - lam) * v +
               lam * head8<T, VEC>(
                         first + (t + s) * a.fstride + (long)g * a.V, c, a.V);
@@ -303,12 +399,17 @@ extern "C" void launch_grouped_append(const GroupedRowArgs* a, void* q,
 #undef GR_GO
 }
 
-extern "C" void launch_grouped_fill(const GroupedRowArgs* a, const float* kinv,
-                                    const int* fills, int n_fills, bool f32,
-                                    hipStream_t stream) {
-  dim3 grid((unsigned)n_fills, (unsigned)a->G), block(GR_BLOCK);
-#define GR_GO(T, VEC) \
-  grouped_fill_kernel<T, VEC><<<grid, block, 0, stream>>>(*a, kinv, fills)
+extern "C" void launch_grouped_turn(const GroupedRowArgs* a, void* q,
+                                    float* kinv, const int* tok_entry,
+                                    const int* pages, int P, int direct,
+                                    long n_tok, bool f32, hipStream_t stream) {
+  int sub = 1;
+  while (sub * 8 < a->dimp || sub * 8 < a->vdp) sub *= 2;
+  const long lanes = n_tok * (a->H + 2 * a->G) * sub;
+  dim3 grid((unsigned)((lanes + GR_BLOCK - 1) / GR_BLOCK)), block(GR_BLOCK);
+#define GR_GO(T, VEC)                                                        \
+  grouped_turn_kernel<T, VEC><<<grid, block, 0, stream>>>(                   \
+      *a, (T*)q, kinv, tok_entry, pages, P, direct, sub, n_tok)
   if (f32) {
     if (a->vec) GR_GO(float, true);
     else GR_GO(float, false);
@@ -317,6 +418,30 @@ extern "C" void launch_grouped_fill(const GroupedRowArgs* a, const float* kinv,
     else GR_GO(__bf16, false);
   }
 #undef GR_GO
+}
+
+extern "C" void launch_grouped_fill(const GroupedRowArgs* a, const float* kinv,
+                                    const int* fills, int n_fills, bool f32,
+                                    hipStream_t stream) {
+  dim3 grid((unsigned)n_fills, (unsigned)a->G), block(GR_BLOCK);
+  const bool turn = a->head_norm || a->qk_cos || a->v_cos;
+#define GR_TURN(T, VEC, TURN)                                           \
+  grouped_fill_kernel<T, VEC, TURN><<<grid, block, 0, stream>>>(*a, kinv, \
+                                                               fills)
+#define GR_GO(T, VEC)               \
+  do {                              \
+    if (turn) GR_TURN(T, VEC, true); \
+    else GR_TURN(T, VEC, false);    \
+  } while (0)
+  if (f32) {
+    if (a->vec) GR_GO(float, true);
+    else GR_GO(float, false);
+  } else {
+    if (a->vec) GR_GO(__bf16, true);
+    else GR_GO(__bf16, false);
+  }
+#undef GR_GO
+#undef GR_TURN
 }
 
 // ---------------------------------------------------------------------------

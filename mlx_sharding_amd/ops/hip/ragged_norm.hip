@@ -9,7 +9,8 @@
 //   x += mult * rms(y) * (w_post + off)   (y == null: x unchanged;
 //                                          w_post == null: x += mult * y)
 //   h  = rms(x) * (w_next + off)      (w_next == null: no h)
-// x is the fp32 residual; y and h are T.  NR > 0 keeps the row in registers
+// x is the fp32 residual; y and h are T; w_next holds W weights or one for all
+// (one_next).  NR > 0 keeps the row in registers
 // (NR groups of VEC elements per thread); NR == 0 re-reads it.
 // ---------------------------------------------------------------------------
 
@@ -36,7 +37,7 @@ template <typename T, int VEC, int NR>
 __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y, long ystride,
     const T* __restrict__ w_post, const T* __restrict__ w_next,
-    T* __restrict__ h, int W, float eps, float off, float mult) {
+    T* __restrict__ h, int W, float eps, float off, float mult, bool one_next) {
   __shared__ float scratch[RN_BLOCK / WAVE];
   const long row = blockIdx.x;
   float* xr = x + row * W;
@@ -111,9 +112,15 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
   if (!hr) return;
   ss = block_sum<RN_BLOCK>(ss, scratch);
   const float inv = 1.0f / sqrtf(ss / (float)W + eps);
+  const float one = one_next ? (float)w_next[0] : 0.0f;
   auto emit = [&](int c, float (&xa)[VEC]) {
     float wv[VEC], o[VEC];
-    rn_load<T, VEC>(w_next + c, wv);
+    if (one_next) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) wv[j] = one;
+    } else {
+      rn_load<T, VEC>(w_next + c, wv);
+    }
 #pragma unroll
     for (int j = 0; j < VEC; ++j) o[j] = xa[j] * inv * (wv[j] + off);
     rn_store<T, VEC>(hr + c, o);
@@ -135,7 +142,8 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
 template <typename T>
 static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
                        const void* wn, void* h, long rows, int W, float eps,
-                       float off, float mult, hipStream_t stream) {
+                       float off, float mult, bool one_next,
+                       hipStream_t stream) {
   const bool vec = W % 4 == 0 && ystride % 4 == 0 &&
                    ((uintptr_t)y) % 16 == 0;
   const int nr = (W + RN_BLOCK * 4 - 1) / (RN_BLOCK * 4);
@@ -143,7 +151,7 @@ static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
 #define RN_GO(V, N)                                                        \
   add_norm_kernel<T, V, N><<<grid, block, 0, stream>>>(                    \
       (float*)x, (const T*)y, ystride, (const T*)wp, (const T*)wn, (T*)h, W, \
-      eps, off, mult)
+      eps, off, mult, one_next)
   if (!vec)
     RN_GO(1, 0);
   else if (nr <= 1)
@@ -162,11 +170,14 @@ static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
 extern "C" void launch_add_norm(void* x, const void* y, long ystride,
                                 const void* wp, const void* wn, void* h,
                                 long rows, int W, float eps, float off,
-                                float mult, bool f32, hipStream_t stream) {
+                                float mult, bool one_next, bool f32,
+                                hipStream_t stream) {
   if (f32)
-    add_norm_t<float>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult, stream);
+    add_norm_t<float>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult, one_next,
+                    stream);
   else
-    add_norm_t<__bf16>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult, stream);
+    add_norm_t<__bf16>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult,
+                       one_next, stream);
 }
 
 // ---------------------------------------------------------------------------

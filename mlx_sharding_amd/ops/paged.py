@@ -5,7 +5,8 @@ beside single decoded tokens, flattened to rows.  What requests keep between
 steps lives in two kinds of shared storage:
 
   * rows of a paged layer (per token), in pages of ``PAGE`` tokens;
-  * the state of a recurrent layer (per request), in slots.
+  * the state of a recurrent layer and the last inputs of short convolutions
+    (per request), in slots.
 
 Pages and slots are handed out when a request is admitted or grows and come
 back when it ends.  Nothing is cleared in between: attention reads only rows
@@ -25,6 +26,7 @@ PAGE = 64    # tokens per cache page
 SHORT = 16   # portions up to this long take the decode kernels
 CHUNK = 64   # tokens per chunk of the chunked recurrence
 QTILE = 128  # query rows per block of the expanded attention
+SPAN = 128   # tokens that one pass of the selective scan takes in sequence
 
 
 class CacheFull(RuntimeError):
@@ -40,30 +42,59 @@ class RowSpec:
 @dataclass
 class StateSpec:
     """A recurrent layer: fp32 state [heads, dim, vdim] and the last inputs
-    of a short convolution [channels, history]."""
+    of a short convolution [channels, history] (no channels: none)."""
     heads: int
     dim: int
     vdim: int
+    channels: int = 0
+    history: int = 0
+
+
+@dataclass
+class HistorySpec:
+    """The last ``history`` input rows of a causal convolution over time."""
     channels: int
     history: int
 
 
-class LayerStore:
-    """Storage of one layer: ``rows`` or ``state`` + ``conv``."""
+@dataclass
+class LayerSpec:
+    """A layer that keeps more than its mixer's storage: besides ``mix`` (a
+    RowSpec, a StateSpec or None) the histories of its convolutions by name."""
+    mix: Optional[object]
+    histories: Dict[str, HistorySpec]
 
-    __slots__ = ("spec", "rows", "state", "conv")
+
+class LayerStore:
+    """Storage of one layer: ``rows`` or ``state`` + ``conv``, and
+    ``histories`` [slots, history, channels]."""
+
+    __slots__ = ("spec", "rows", "state", "conv", "histories")
 
     def __init__(self, spec, n_pages: int, n_slots: int, dtype, device):
+        histories = {}
+        if isinstance(spec, LayerSpec):
+            spec, histories = spec.mix, spec.histories
         self.spec = spec
         self.rows = self.state = self.conv = None
+        self.histories: Dict[str, torch.Tensor] = {
+            name: torch.empty(n_slots, h.history, h.channels, dtype=dtype,
+                              device=device)
+            for name, h in histories.items()}
         if isinstance(spec, RowSpec):
             self.rows = torch.empty(n_pages * PAGE, spec.width, dtype=dtype,
                                     device=device)
-        else:
+        elif spec is not None:
             self.state = torch.empty(n_slots, spec.heads, spec.dim, spec.vdim,
                                      dtype=torch.float32, device=device)
-            self.conv = torch.empty(n_slots, spec.channels, spec.history,
-                                    dtype=dtype, device=device)
+            if spec.channels:
+                self.conv = torch.empty(n_slots, spec.channels, spec.history,
+                                        dtype=dtype, device=device)
+
+    def per_slot(self) -> List[torch.Tensor]:
+        """What moves on with every token instead of being kept per token."""
+        found = [self.state, self.conv, *self.histories.values()]
+        return [t for t in found if t is not None and t.numel()]
 
     def grow_rows(self, n_pages: int):
         if self.rows is None:
@@ -194,6 +225,7 @@ class RaggedBatch:
             np.cumsum(kpad, out=cuk[1:])
             self.key_rows = int(cuk[-1])
             blocks, fills, tiles, chunks, chunk_cu = [], [], [], [], [0]
+            spans, span_cu = [], [0]
             for j in range(self.n_long):
                 e = self.n_short + j
                 for b in range(kpad[j] // PAGE):
@@ -208,13 +240,20 @@ class RaggedBatch:
                 for c in range(0, nl[j], CHUNK):
                     chunks.append((cu[e] + c, min(CHUNK, nl[j] - c)))
                 chunk_cu.append(len(chunks))
+                for c in range(0, nl[j], SPAN):
+                    spans.append((cu[e] + c, min(SPAN, nl[j] - c), e,
+                                  c + SPAN >= nl[j]))
+                span_cu.append(len(spans))
             tiles.sort()  # most keys first
             parts.update(
                 cuk=cuk, blocks=np.array(blocks, dtype=np.int32),
                 fills=np.array(fills, dtype=np.int32),
                 tiles=np.array(tiles, dtype=np.int32)[:, 1:],
                 chunks=np.array(chunks, dtype=np.int32),
-                chunk_cu=np.array(chunk_cu, dtype=np.int32))
+                chunk_cu=np.array(chunk_cu, dtype=np.int32),
+                # (first token, tokens, request, whether the portion ends)
+                spans=np.array(spans, dtype=np.int32),
+                span_cu=np.array(span_cu, dtype=np.int32))
         flat = np.concatenate([np.ascontiguousarray(a).reshape(-1)
                                for a in parts.values()])
         dev = torch.from_numpy(flat).to(device)
@@ -331,9 +370,9 @@ class RaggedLayerCache:
 
     @property
     def trimmable(self) -> bool:
-        """A recurrent state cannot be rolled back to a shorter prefix; rows
-        can."""
-        return all(s is None or s.state is None
+        """What is kept per slot cannot be rolled back to a shorter prefix;
+        rows can."""
+        return all(s is None or not s.per_slot()
                    for s in self.shared.state.layers)
 
     batch_size = property(lambda self: self.shared.batch_size)
@@ -357,7 +396,7 @@ class RaggedLayerCache:
         if self.shared.capacity == 0:
             return None
         for s in (self._store(), *self.shared.state.layers):
-            if s is not None:
+            if s is not None and (s.rows is not None or s.state is not None):
                 return s.rows if s.rows is not None else s.state
         return None
 
@@ -368,15 +407,12 @@ class RaggedLayerCache:
 
     def snapshot(self):
         s = self._store()
-        if s is None or s.state is None:
-            return None
-        return s.state.clone(), s.conv.clone()
+        return [] if s is None else [t.clone() for t in s.per_slot()]
 
     def restore(self, snap):
-        if snap is not None:
-            s = self._store()
-            s.state.copy_(snap[0])
-            s.conv.copy_(snap[1])
+        if snap:
+            for t, kept in zip(self._store().per_slot(), snap):
+                t.copy_(kept)
 
     def trim(self, n: int):
         if n not in (0, self.shared.offset) and not self.trimmable:

@@ -20,7 +20,7 @@ from __future__ import annotations
 
 import math
 from dataclasses import dataclass
-from typing import List, Optional
+from typing import List, Optional, Tuple
 
 import torch
 import torch.nn.functional as F
@@ -330,24 +330,58 @@ class GroupedShape:
         return v.permute(0, 3, 6, 4, 7, 1, 2, 5)
 
 
+@dataclass
+class Turns:
+    """Rotations of grouped attention, as (cos, sin) tables [positions, pairs]
+    over neighbouring pairs.  ``qk``: on the first dimensions of queries and
+    keys.  ``v``: over whole values; each head's output is turned back by its
+    own position, so that only the distance to a value's token counts."""
+    qk: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
+    v: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
+
+
+def _turn(x, table, pos, sign: float = 1.0):
+    """x [N, heads, size] with its first pairs rotated, fp32."""
+    c, s = table[0][pos][:, None], sign * table[1][pos][:, None]
+    n = 2 * c.shape[-1]
+    u, v = x[..., 0:n:2].float(), x[..., 1:n:2].float()
+    turned = torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+    return torch.cat([turned, x[..., n:].float()], -1)
+
+
 def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
-                   sh: GroupedShape, batch: RaggedBatch):
+                   sh: GroupedShape, batch: RaggedBatch,
+                   turns: Optional[Turns] = None, head_norm: bool = False):
     """From projection rows y [N, q | k | v | ...]: the queries [N, heads,
     dimp], RMS-normed over the row if wq is given; keys (normed likewise) and
     values go to their pages.  first: values [N, kv_heads * vdim] that are
-    blended in by vmix (one element)."""
+    blended in by vmix (one element).  turns: rotations by position.
+    head_norm: every query and key divided by its own root mean square."""
     H, G, D, V = sh.heads, sh.kv_heads, sh.dim, sh.vdim
+    by_head = head_norm or turns is not None
+    if by_head and not (wq is None and wk is None and first is None):
+        raise ValueError("rotations and norms per head do not go together with "
+                         "norms over whole rows or blended values")
+    turns = turns or Turns()
     if y.is_cuda:
         ext = _ext("grouped_append")
         direct = batch.short_tokens if sh.prompts else batch.n_tokens
-        q, kinv = ext.grouped_append(
-            y, wq, wk, eps, vmix, first, store.rows, H, G, D, V, sh.dimp,
-            sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages, direct)
+        tables = (*(turns.qk or (None, None)), *(turns.v or (None, None)))
+        if by_head:
+            q, kinv = ext.grouped_turn(
+                y, eps, head_norm, *tables, store.rows, H, G, D, V, sh.dimp,
+                sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages, direct)
+        else:
+            q, kinv = ext.grouped_append(
+                y, wq, wk, eps, vmix, first, store.rows, H, G, D, V, sh.dimp,
+                sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages, direct)
         if direct < batch.n_tokens:
             ext.grouped_fill(y, wk, kinv, vmix, first, store.rows, H, G, D, V,
-                             sh.dimp, sh.vdp, batch.fills)
+                             sh.dimp, sh.vdp, batch.fills, head_norm, *tables,
+                             batch.tok_pos)
         return q
     N = y.shape[0]
+    pos = batch.tok_pos.long()
     q, k, v = (t.float() for t in y[:, : (H + G) * D + G * V].split(
         [H * D, G * D, G * V], 1))
     if wq is not None:
@@ -357,10 +391,16 @@ def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
     if first is not None:
         lam = vmix.float()
         v = (1.0 - lam) * v + lam * first.float()
-    q = F.pad(q.view(N, H, D), (0, sh.dimp - D)).to(y.dtype)
-    k = F.pad(k.view(N, G, D), (0, sh.dimp - D)).to(y.dtype)
-    v = F.pad(v.view(N, G, V), (0, sh.vdp - V)).to(y.dtype)
-    pos = batch.tok_pos.long()
+    q, k, v = q.view(N, H, D), k.view(N, G, D), v.view(N, G, V)
+    if turns.qk is not None:
+        q, k = _turn(q, turns.qk, pos), _turn(k, turns.qk, pos)
+    if head_norm:
+        q, k = _rms(q, eps), _rms(k, eps)
+    if turns.v is not None:
+        v = _turn(v, turns.v, pos)
+    q = F.pad(q, (0, sh.dimp - D)).to(y.dtype)
+    k = F.pad(k, (0, sh.dimp - D)).to(y.dtype)
+    v = F.pad(v, (0, sh.vdp - V)).to(y.dtype)
     page, r = batch.pages[batch.tok_entry.long(), pos // PAGE].long(), pos % PAGE
     sh.keys(store.rows)[page, r // 16, r % 16] = k.view(N, G, -1, 4, 8)
     sh.values(store.rows)[page, r // 32, r // 16 % 2, r // 4 % 4, r % 4] = \
@@ -369,24 +409,30 @@ def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
 
 
 def grouped_attention(q, sink, store: LayerStore, sh: GroupedShape,
-                      scale: float, batch: RaggedBatch, out):
+                      scale: float, batch: RaggedBatch, out,
+                      window: Optional[int] = None,
+                      turns: Optional[Turns] = None):
     """Attention of queries [N, heads, dimp] over their requests' pages, into
     out [N, heads * vdim].  sink [heads] (or None): a score per head that only
-    the softmax's denominator sees."""
+    the softmax's denominator sees.  window: how many tokens a token sees, up
+    to itself (None: all).  turns: where values are rotated, the output is
+    turned back."""
+    back = turns.v if turns is not None else None
     if q.is_cuda:
         ext = _ext("grouped_attention")
         n_req, n, max_len = batch.n_short, batch.short_tokens, batch.max_short
         if not sh.prompts:
             n_req, n, max_len = batch.n_requests, batch.n_tokens, batch.max_len
+        more = (window or 0, *(back or (None, None)), batch.tok_pos)
         if n_req:
             ext.grouped_attn_short(
                 q, sink, store.rows, out, batch.cu, batch.pos0, batch.pages,
                 n_req, n, max_len, batch.max_keys, sh.kv_heads, sh.vdim,
-                sh.vdp, scale)
+                sh.vdp, scale, *more)
         if n_req < batch.n_requests:
             ext.grouped_attn_long(
                 q, sink, store.rows, out, batch.tiles, batch.cu, batch.pos0,
-                batch.pages, sh.kv_heads, sh.vdim, sh.vdp, scale)
+                batch.pages, sh.kv_heads, sh.vdim, sh.vdp, scale, *more)
         return
     H, G = sh.heads, sh.kv_heads
     for t0, n, p0, held in batch.host:
@@ -396,14 +442,19 @@ def grouped_attention(q, sink, store: LayerStore, sh: GroupedShape,
         v = sh.values(store.rows)[pages].reshape(-1, G, sh.vdp)[:S].float()
         qg = q[t0: t0 + n].float().view(n, G, H // G, sh.dimp)
         s = torch.matmul(qg.permute(1, 2, 0, 3), k.permute(1, 2, 0)[:, None])
-        dead = torch.arange(S)[None, :] > torch.arange(p0, S)[:, None]
+        at = torch.arange(p0, S)
+        gap = at[:, None] - torch.arange(S)[None, :]
+        dead = gap < 0 if window is None else (gap < 0) | (gap >= window)
         s = (s * scale).masked_fill(dead, float("-inf"))
         if sink is not None:
             extra = sink.float().view(G, H // G, 1, 1).expand(-1, -1, n, -1)
             s = torch.cat([s, extra], -1)
         p = torch.softmax(s, -1)[..., :S]
         o = torch.matmul(p, v.transpose(0, 1)[:, None])[..., : sh.vdim]
-        out[t0: t0 + n] = o.permute(2, 0, 1, 3).reshape(n, -1).to(out.dtype)
+        o = o.permute(2, 0, 1, 3).reshape(n, H, sh.vdim)
+        if back is not None:
+            o = _turn(o, back, at, -1.0)
+        out[t0: t0 + n] = o.reshape(n, -1).to(out.dtype)
 
 
 # ---------------------------------------------------------------------------
