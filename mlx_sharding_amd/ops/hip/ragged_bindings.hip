@@ -2,9 +2,7 @@
 // Every operand's device, type, shape and alignment is checked here, before
 // anything is launched.
 
-#include <torch/extension.h>
-#include <c10/hip/HIPStream.h>
-
+#include "ragged_bindings.h"
 #include "ragged_grouped.h"
 #include "ragged_prefill.h"
 
@@ -14,7 +12,7 @@ void launch_glu_strided(const void*, const void*, void*, long, int, long, long,
 void launch_glu_any(const void*, const void*, void*, long, int, long, long,
                     bool, bool, hipStream_t);
 void launch_add_norm(void*, const void*, long, const void*, const void*, void*,
-                     long, int, float, float, float, bool, hipStream_t);
+                     long, int, float, float, float, bool, bool, hipStream_t);
 void launch_latent_append(const void*, long, const void*, float, void*, void*,
                           long, int, int, int, int, int, int, int,
                           const float*, const float*, const int*, const int*,
@@ -32,6 +30,8 @@ int delta_short_rows(int, int, int);
 void launch_grouped_append(const GroupedRowArgs*, void*, float*, const int*,
                            const int*, const int*, int, int, long, bool,
                            hipStream_t);
+void launch_grouped_turn(const GroupedRowArgs*, void*, float*, const int*,
+                         const int*, int, int, long, bool, hipStream_t);
 void launch_grouped_fill(const GroupedRowArgs*, const float*, const int*, int,
                          bool, hipStream_t);
 void launch_grouped_attn_short_bf16(const GroupedAttnArgs*, int, int,
@@ -76,49 +76,6 @@ void launch_delta_long(const DeltaLongArgs*, const DeltaDims*, bool,
 }
 
 namespace {
-
-using torch::Tensor;
-
-hipStream_t stream() { return c10::hip::getCurrentHIPStream().stream(); }
-
-bool is_f32(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda(), name, " must be on the GPU");
-  TORCH_CHECK(t.scalar_type() == torch::kFloat32 ||
-                  t.scalar_type() == torch::kBFloat16,
-              name, " must be float32 or bfloat16");
-  return t.scalar_type() == torch::kFloat32;
-}
-
-void check_like(const Tensor& t, const Tensor& as, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == as.scalar_type(), name,
-              " must be on the GPU with the activations' type");
-}
-
-void check_f32(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 &&
-                  t.is_contiguous(),
-              name, " must be contiguous float32 on the GPU");
-}
-
-const int* ints(const Tensor& t, int64_t at_least, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt32 &&
-                  t.is_contiguous() && t.numel() >= at_least,
-              name, " must be contiguous int32 on the GPU with at least ",
-              at_least, " elements");
-  return t.data_ptr<int>();
-}
-
-// [N, C] with unit column stride; returns the row stride
-long rows2(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.dim() == 2 && (t.stride(1) == 1 || t.size(1) == 1), name,
-              " must be [rows, columns] with unit column stride");
-  return t.size(0) > 1 ? t.stride(0) : std::max<long>(t.stride(0), t.size(1));
-}
-
-void aligned16(const Tensor& t, const char* name) {
-  TORCH_CHECK(((uintptr_t)t.data_ptr()) % 16 == 0, name,
-              " must be 16-byte aligned");
-}
 
 Tensor glu(Tensor gate, Tensor up, bool gelu) {
   const bool f32 = is_f32(gate, "gate");
@@ -166,7 +123,8 @@ Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
   Tensor h;
   if (w_next) {
     check_like(*w_next, like, "w_next");
-    TORCH_CHECK(w_next->numel() == W && w_next->is_contiguous());
+    TORCH_CHECK((w_next->numel() == W || w_next->numel() == 1) &&
+                w_next->is_contiguous());
     h = torch::empty({N, W}, like.options());
   } else {
     h = torch::empty({0}, like.options());
@@ -176,7 +134,8 @@ Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
                   y && w_post ? w_post->data_ptr() : nullptr,
                   w_next ? w_next->data_ptr() : nullptr,
                   w_next ? h.data_ptr() : nullptr, N, (int)W, (float)eps,
-                  (float)off, (float)mult, f32, stream());
+                  (float)off, (float)mult, w_next && w_next->numel() == 1, f32,
+                  stream());
   return h;
 }
 
@@ -472,10 +431,6 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
 // Grouped attention
 // ---------------------------------------------------------------------------
 
-bool whole8(const Tensor& t, long stride) {
-  return ((uintptr_t)t.data_ptr()) % 16 == 0 && stride % 8 == 0;
-}
-
 void check_pool(const Tensor& pool, const Tensor& like, long width) {
   check_like(pool, like, "pool");
   TORCH_CHECK(pool.is_contiguous() && pool.dim() == 2 &&
@@ -551,16 +506,72 @@ std::tuple<Tensor, Tensor> grouped_append(
   return {q, kinv};
 }
 
+using Table = c10::optional<Tensor>;
+
+// rotation tables [positions, pairs] for the first 2 * pairs of `size` columns
+void turn_tables(const Table& cos, const Table& sin, long size, const float** c,
+                 const float** s, int* pairs) {
+  TORCH_CHECK(cos.has_value() == sin.has_value());
+  if (!cos) return;
+  check_f32(*cos, "cos");
+  check_f32(*sin, "sin");
+  TORCH_CHECK(cos->dim() == 2 && cos->sizes() == sin->sizes() &&
+              2 * cos->size(1) <= size, "rotation tables do not fit");
+  *c = cos->data_ptr<float>();
+  *s = sin->data_ptr<float>();
+  *pairs = (int)cos->size(1);
+}
+
+void grouped_turns(GroupedRowArgs& a, bool head_norm, const Table& qk_cos,
+                   const Table& qk_sin, const Table& v_cos, const Table& v_sin,
+                   const Tensor& tok_pos, long n) {
+  a.head_norm = head_norm;
+  turn_tables(qk_cos, qk_sin, a.D, &a.qk_cos, &a.qk_sin, &a.qk_pairs);
+  turn_tables(v_cos, v_sin, a.V, &a.v_cos, &a.v_sin, &a.v_pairs);
+  a.tok_pos = ints(tok_pos, n, "tok_pos");
+  for (const auto* t : {&qk_cos, &qk_sin, &v_cos, &v_sin})
+    if (*t) aligned16(**t, "rotation table");
+}
+
+// y [N, q | k | v | ...] -> queries [N, H, dimp] and inverse rms of keys [N, G]
+std::tuple<Tensor, Tensor> grouped_turn(
+    Tensor y, double eps, bool head_norm, Table qk_cos, Table qk_sin,
+    Table v_cos, Table v_sin, Tensor pool, int64_t H, int64_t G, int64_t D,
+    int64_t V, int64_t dimp, int64_t vdp, Tensor tok_pos, Tensor tok_entry,
+    Tensor pages, int64_t direct) {
+  const bool f32 = is_f32(y, "y");
+  const c10::optional<Tensor> none;
+  auto a = grouped_rows(y, none, none, eps, none, none, pool, H, G, D, V, dimp,
+                        vdp);
+  const long N = y.size(0);
+  TORCH_CHECK(pages.dim() == 2 && direct >= 0 && direct <= N);
+  grouped_turns(a, head_norm, qk_cos, qk_sin, v_cos, v_sin, tok_pos, N);
+  auto q = torch::empty({N, H, dimp}, y.options());
+  auto kinv = torch::empty({N, G}, y.options().dtype(torch::kFloat32));
+  if (N)
+    launch_grouped_turn(&a, q.data_ptr(), kinv.data_ptr<float>(),
+                        ints(tok_entry, N, "tok_entry"),
+                        ints(pages, 0, "pages"), (int)pages.size(1),
+                        (int)direct, N, f32, stream());
+  return {q, kinv};
+}
+
 // fills [*, 4]: (page, token of its first slot, first slot, end slot)
 void grouped_fill(Tensor y, c10::optional<Tensor> wk, Tensor kinv,
                   c10::optional<Tensor> vmix, c10::optional<Tensor> first,
                   Tensor pool, int64_t H, int64_t G, int64_t D, int64_t V,
-                  int64_t dimp, int64_t vdp, Tensor fills) {
+                  int64_t dimp, int64_t vdp, Tensor fills, bool head_norm,
+                  Table qk_cos, Table qk_sin, Table v_cos, Table v_sin,
+                  Tensor tok_pos) {
   const bool f32 = is_f32(y, "y");
   auto a = grouped_rows(y, c10::nullopt, wk, 0.0, vmix, first, pool, H, G, D, V,
                         dimp, vdp);
   check_f32(kinv, "kinv");
-  TORCH_CHECK(kinv.numel() == y.size(0) && G <= 65535);
+  grouped_turns(a, head_norm, qk_cos, qk_sin, v_cos, v_sin, tok_pos, y.size(0));
+  const bool turns = head_norm || qk_cos || v_cos;
+  TORCH_CHECK(kinv.numel() == y.size(0) * (turns ? G : 1) && G <= 65535);
+  TORCH_CHECK(!(turns && (wk || first)), "norms per head or rotations beside "
+              "norms of whole rows or blended values");
   TORCH_CHECK(fills.dim() == 2 && fills.size(1) == 4);
   if (fills.size(0))
     launch_grouped_fill(&a, kinv.data_ptr<float>(), ints(fills, 0, "fills"),
@@ -572,7 +583,9 @@ int head_bucket(long n) { return n <= 64 ? 64 : n <= 128 ? 128 : n <= 256 ? 256 
 GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
                              const Tensor& pool, const Tensor& out,
                              const Tensor& pages, int64_t G, int64_t V,
-                             int64_t vdp, double scale) {
+                             int64_t vdp, double scale, int64_t window,
+                             const Table& v_cos, const Table& v_sin,
+                             const Tensor& tok_pos) {
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous());
   const long H = q.size(1), dimp = q.size(2);
   TORCH_CHECK(G > 0 && H % G == 0 && V > 0 && V <= vdp);
@@ -602,6 +615,12 @@ GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
   a.V = (int)V;
   a.vdp = (int)vdp;
   a.scale = (float)scale;
+  TORCH_CHECK(window >= 0 && window < (1L << 30));
+  a.window = (int)window;
+  int pairs = 0;
+  turn_tables(v_cos, v_sin, V, &a.v_cos, &a.v_sin, &pairs);
+  TORCH_CHECK(!v_cos || 2 * pairs == V, "values are turned back whole");
+  a.tok_pos = ints(tok_pos, q.size(0), "tok_pos");
   return a;
 }
 
@@ -610,9 +629,13 @@ void grouped_attn_short(Tensor q, c10::optional<Tensor> sink, Tensor pool,
                         Tensor out, Tensor cu, Tensor pos0, Tensor pages,
                         int64_t n_req, int64_t n_tok, int64_t max_len,
                         int64_t max_keys, int64_t G, int64_t V, int64_t vdp,
-                        double scale) {
+                        double scale, int64_t window, Table v_cos, Table v_sin,
+                        Tensor tok_pos) {
   const bool f32 = is_f32(q, "q");
-  auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale);
+  auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale, window,
+                        v_cos, v_sin, tok_pos);
+  // a block starts at the step that holds its first window's first key
+  if (window) max_keys = std::min(max_keys, window + max_len + GA_STEP);
   TORCH_CHECK(pages.size(0) >= n_req && n_tok <= q.size(0));
   if (n_req == 0 || n_tok == 0) return;
   a.cu = ints(cu, n_req + 1, "cu");
@@ -645,9 +668,11 @@ void grouped_attn_short(Tensor q, c10::optional<Tensor> sink, Tensor pool,
 void grouped_attn_long(Tensor q, c10::optional<Tensor> sink, Tensor pool,
                        Tensor out, Tensor tiles, Tensor cu, Tensor pos0,
                        Tensor pages, int64_t G, int64_t V, int64_t vdp,
-                       double scale) {
+                       double scale, int64_t window, Table v_cos, Table v_sin,
+                       Tensor tok_pos) {
   const bool f32 = is_f32(q, "q");
-  auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale);
+  auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale, window,
+                        v_cos, v_sin, tok_pos);
   TORCH_CHECK(a.dimp <= 256 && vdp <= 256, "head sizes above 256");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2 &&
               tiles.size(0) <= 65535);
@@ -699,10 +724,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("delta_short", &delta_short);
   m.def("delta_long", &delta_long);
   m.def("grouped_append", &grouped_append);
+  m.def("grouped_turn", &grouped_turn);
   m.def("grouped_fill", &grouped_fill);
   m.def("grouped_attn_short", &grouped_attn_short);
   m.def("grouped_attn_long", &grouped_attn_long);
   m.def("gelu", &gelu);
   m.def("cap_logits", &cap_logits);
+  bind_recurrent(m);
+  bind_experts(m);
   m.attr("PAGE") = RG_PAGE;
 }
