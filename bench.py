@@ -54,12 +54,14 @@ def parse_args():
                    metavar="SIZE",
                    help="instead of the serving benchmark: prefill and decode "
                         "throughput of Tuvutar layers beside DeepSeek-V2's "
-                        "dense latent-attention layers and of Lepizen layers "
-                        "beside Llama's, each of equal size, one JSON line per "
-                        "case (2048, 4096 or all)")
+                        "dense latent-attention layers, of Lepizen layers "
+                        "beside Llama's and of Sadosun layers beside "
+                        "DeepSeek-V2's with routed experts, each of equal size, "
+                        "one JSON line per case (2048, 4096 or all)")
     p.add_argument("--kinds", default=None, metavar="NAME,...",
                    help="the stacks --layers times (default: all; mla, latent, "
-                        "shared, delta, mixed, llama, lepizen)")
+                        "shared, delta, mixed, llama, lepizen, moe, windowed, "
+                        "scan, sadosun)")
     return p.parse_args()
 
 

@@ -585,7 +585,7 @@ GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
                              const Tensor& pages, int64_t G, int64_t V,
                              int64_t vdp, double scale, int64_t window,
                              const Table& v_cos, const Table& v_sin,
-                             const Tensor& tok_pos) {
+                             const Table& tok_pos) {
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous());
   const long H = q.size(1), dimp = q.size(2);
   TORCH_CHECK(G > 0 && H % G == 0 && V > 0 && V <= vdp);
@@ -620,7 +620,8 @@ GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
   int pairs = 0;
   turn_tables(v_cos, v_sin, V, &a.v_cos, &a.v_sin, &pairs);
   TORCH_CHECK(!v_cos || 2 * pairs == V, "values are turned back whole");
-  a.tok_pos = ints(tok_pos, q.size(0), "tok_pos");
+  TORCH_CHECK(!v_cos || tok_pos, "turning back needs positions");
+  if (tok_pos) a.tok_pos = ints(*tok_pos, q.size(0), "tok_pos");
   return a;
 }
 
@@ -630,7 +631,7 @@ void grouped_attn_short(Tensor q, c10::optional<Tensor> sink, Tensor pool,
                         int64_t n_req, int64_t n_tok, int64_t max_len,
                         int64_t max_keys, int64_t G, int64_t V, int64_t vdp,
                         double scale, int64_t window, Table v_cos, Table v_sin,
-                        Tensor tok_pos) {
+                        Table tok_pos) {
   const bool f32 = is_f32(q, "q");
   auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale, window,
                         v_cos, v_sin, tok_pos);
@@ -669,7 +670,7 @@ void grouped_attn_long(Tensor q, c10::optional<Tensor> sink, Tensor pool,
                        Tensor out, Tensor tiles, Tensor cu, Tensor pos0,
                        Tensor pages, int64_t G, int64_t V, int64_t vdp,
                        double scale, int64_t window, Table v_cos, Table v_sin,
-                       Tensor tok_pos) {
+                       Table tok_pos) {
   const bool f32 = is_f32(q, "q");
   auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale, window,
                         v_cos, v_sin, tok_pos);
@@ -726,8 +727,19 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("grouped_append", &grouped_append);
   m.def("grouped_turn", &grouped_turn);
   m.def("grouped_fill", &grouped_fill);
-  m.def("grouped_attn_short", &grouped_attn_short);
-  m.def("grouped_attn_long", &grouped_attn_long);
+  m.def("grouped_attn_short", &grouped_attn_short, py::arg("q"),
+        py::arg("sink"), py::arg("pool"), py::arg("out"), py::arg("cu"),
+        py::arg("pos0"), py::arg("pages"), py::arg("n_req"), py::arg("n_tok"),
+        py::arg("max_len"), py::arg("max_keys"), py::arg("kv_heads"),
+        py::arg("vdim"), py::arg("vdp"), py::arg("scale"),
+        py::arg("window") = 0, py::arg("v_cos") = py::none(),
+        py::arg("v_sin") = py::none(), py::arg("tok_pos") = py::none());
+  m.def("grouped_attn_long", &grouped_attn_long, py::arg("q"),
+        py::arg("sink"), py::arg("pool"), py::arg("out"), py::arg("tiles"),
+        py::arg("cu"), py::arg("pos0"), py::arg("pages"), py::arg("kv_heads"),
+        py::arg("vdim"), py::arg("vdp"), py::arg("scale"),
+        py::arg("window") = 0, py::arg("v_cos") = py::none(),
+        py::arg("v_sin") = py::none(), py::arg("tok_pos") = py::none());
   m.def("gelu", &gelu);
   m.def("cap_logits", &cap_logits);
   bind_recurrent(m);

@@ -10,19 +10,26 @@
 #define EX_WAVES (EX_BLOCK / WAVE)
 
 // ---------------------------------------------------------------------------
-// Router.  A block has 16 tokens; its waves split the contraction and meet in
-// LDS, 64 experts at a time; then a wave per token softmaxes and picks.
+// Router.  A block has 16 tokens and 16 waves: 128 experts at a time, half of
+// the waves for each 64 of them, eight parts of the contraction, which meet in
+// LDS.  Then a wave per token softmaxes and picks.
 // ---------------------------------------------------------------------------
 
+#define RT_BLOCK 1024
+#define RT_WAVES (RT_BLOCK / WAVE)
+#define RT_PARTS 8
+#define RT_LS (128 + 4)
+
 template <typename T>
-__global__ __launch_bounds__(EX_BLOCK) void expert_route_kernel(
+__global__ __launch_bounds__(RT_BLOCK) void expert_route_kernel(
     const RouteArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  __shared__ float part[EX_WAVES][EX_TOK][64 + 4];
   const int totalp = (a.total + 63) / 64 * 64;
-  float* logits = reinterpret_cast<float*>(smem);             // [16][totalp]
-  float* choices = logits + EX_TOK * totalp;                  // [waves][totalp]
-  int* counts = reinterpret_cast<int*>(choices + EX_WAVES * totalp);  // [experts]
+  float* part = reinterpret_cast<float*>(smem);        // [parts][16][RT_LS]
+  float* choices = part;                               // later: [waves][totalp]
+  const int shared_n = max(RT_PARTS * EX_TOK * RT_LS, RT_WAVES * totalp);
+  float* logits = part + shared_n;                     // [16][totalp]
+  int* counts = reinterpret_cast<int*>(logits + EX_TOK * totalp);  // [experts]
   const int tid = threadIdx.x;
   const int lane = tid & (WAVE - 1);
   const int wid = __builtin_amdgcn_readfirstlane(tid / WAVE);
@@ -30,14 +37,16 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_route_kernel(
   const long t0 = (long)blockIdx.x * EX_TOK;
   const int n = (int)min((long)EX_TOK, a.n - t0);
 
-  for (int e = tid; e < a.experts; e += EX_BLOCK) counts[e] = 0;
+  for (int e = tid; e < a.experts; e += RT_BLOCK) counts[e] = 0;
   const T* hrow =
       (const T*)a.h + (t0 + min(lr, n - 1)) * a.hstride + lg * 8;
   const int steps = a.K / 32;
-  const int per = (steps + EX_WAVES - 1) / EX_WAVES;
-  const int s0 = wid * per, s1 = min(steps, s0 + per);
-  for (int e0 = 0; e0 < a.total; e0 += 64) {
-    const int tiles = min(4, (a.total - e0 + 15) / 16);
+  const int per = (steps + RT_PARTS - 1) / RT_PARTS;
+  const int half = wid / RT_PARTS, which = wid % RT_PARTS;
+  const int s0 = which * per, s1 = min(steps, s0 + per);
+  for (int e0 = 0; e0 < a.total; e0 += 128) {
+    const int first = e0 + half * 64;
+    const int tiles = max(0, min(4, (a.total - first + 15) / 16));
     f32x4 acc[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0, 0, 0, 0};
@@ -45,32 +54,38 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_route_kernel(
 #pragma unroll
     for (int i = 0; i < 4; ++i)
       wrow[i] = (const T*)a.w +
-                (long)min(e0 + i * 16 + lr, a.total - 1) * a.K + lg * 8;
+                (long)min(first + i * 16 + lr, a.total - 1) * a.K + lg * 8;
+    if (tiles) {
 #pragma unroll 4
-    for (int s = s0; s < s1; ++s) {
-      Frag<T> b;
-      b.load(hrow + s * 32);
+      for (int s = s0; s < s1; ++s) {
+        Frag<T> b, w[4];
+        b.load(hrow + s * 32);
+        // tiles past the last repeat it
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        if (i >= tiles) continue;
-        Frag<T> w;
-        w.load(wrow[i] + s * 32);
-        acc[i] = mma(w, b, acc[i]);
+        for (int i = 0; i < 4; ++i) w[i].load(wrow[min(i, tiles - 1)] + s * 32);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[i] = mma(w[i], b, acc[i]);
       }
     }
+    __syncthreads();  // the sums of the last round are read
 #pragma unroll
-    for (int i = 0; i < 4; ++i) store4(&part[wid][lr][i * 16 + lg * 4], acc[i]);
+    for (int i = 0; i < 4; ++i)
+      store4(part + (which * EX_TOK + lr) * RT_LS + half * 64 + i * 16 + lg * 4,
+             acc[i]);
     __syncthreads();
-    for (int i = tid; i < EX_TOK * 64; i += EX_BLOCK) {
+    for (int i = tid; i < EX_TOK * 128; i += RT_BLOCK) {
+      const int t = i / 128, e = i % 128;
+      if (e0 + e >= totalp) continue;
       float z = 0.0f;
 #pragma unroll
-      for (int w = 0; w < EX_WAVES; ++w) z += part[w][i / 64][i % 64];
-      logits[i / 64 * totalp + e0 + i % 64] = z;
+      for (int w = 0; w < RT_PARTS; ++w)
+        z += part[(w * EX_TOK + t) * RT_LS + e];
+      logits[t * totalp + e0 + e] = z;
     }
-    __syncthreads();
   }
+  __syncthreads();
 
-  for (int t = wid; t < n; t += EX_WAVES) {
+  for (int t = wid; t < n; t += RT_WAVES) {
     const float* z = logits + t * totalp;
     float* choice = choices + wid * totalp;
     float mx = -INFINITY;
@@ -126,22 +141,23 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_route_kernel(
       a.weight[(t0 + t) * a.top + k] *= by;
   }
   __syncthreads();
-  for (int e = tid; e < a.experts; e += EX_BLOCK)
+  for (int e = tid; e < a.experts; e += RT_BLOCK)
     a.hist[(long)blockIdx.x * a.experts + e] = counts[e];
 }
 
 extern "C" void launch_expert_route(const RouteArgs* a, bool f32,
                                     hipStream_t stream) {
   const int totalp = (a->total + 63) / 64 * 64;
-  const size_t smem = (size_t)((EX_TOK + EX_WAVES) * totalp + a->experts) * 4;
+  const int parts = RT_PARTS * EX_TOK * RT_LS, picks = RT_WAVES * totalp;
+  const size_t smem = (size_t)((parts > picks ? parts : picks) +
+                               EX_TOK * totalp + a->experts) * 4;
   const dim3 grid((unsigned)((a->n + EX_TOK - 1) / EX_TOK));
 #define EX_GO(T)                                                            \
   do {                                                                      \
-    if (smem > 40000)                                                       \
-      (void)hipFuncSetAttribute(                                            \
-          reinterpret_cast<const void*>(&expert_route_kernel<T>),           \
-          hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);           \
-    expert_route_kernel<T><<<grid, dim3(EX_BLOCK), smem, stream>>>(*a);     \
+    (void)hipFuncSetAttribute(                                              \
+        reinterpret_cast<const void*>(&expert_route_kernel<T>),             \
+        hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);             \
+    expert_route_kernel<T><<<grid, dim3(RT_BLOCK), smem, stream>>>(*a);     \
   } while (0)
   if (f32) EX_GO(float);
   else EX_GO(__bf16);
@@ -549,7 +565,8 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_combine_kernel(
   const float* weight = a.weight + t * a.top;
   const T* h = (const T*)a.h + t * a.hstride;
   float* x = a.x + t * a.W;
-  for (int c = threadIdx.x * V; c < a.W; c += EX_BLOCK * V) {
+  const int c = (blockIdx.y * EX_BLOCK + threadIdx.x) * V;
+  if (c < a.W) {
     float s[V];
 #pragma unroll
     for (int i = 0; i < V; ++i) s[i] = 0.0f;
@@ -582,8 +599,10 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_combine_kernel(
 
 extern "C" void launch_expert_combine(const CombineArgs* a, bool f32,
                                       hipStream_t stream) {
-  const dim3 grid((unsigned)a->n), block(EX_BLOCK);
   const bool vec = a->W % 4 == 0;
+  const int per = EX_BLOCK * (vec ? 4 : 1);
+  const dim3 grid((unsigned)a->n, (unsigned)((a->W + per - 1) / per));
+  const dim3 block(EX_BLOCK);
 #define EX_GO(T)                                                  \
   do {                                                            \
     if (vec) \

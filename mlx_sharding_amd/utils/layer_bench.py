@@ -10,6 +10,11 @@ sizes, latent size and feed-forward, so that their times compare directly:
   mixed   Tuvutar delta, delta, delta, latent
   llama   Llama grouped attention + gated MLP (the closest model to the next)
   lepizen Lepizen grouped attention beside an ungated MLP of the same width
+  moe     DeepSeek-V2 latent attention + routed experts (the closest model to
+          the rest: equal experts, gated there and ungated here)
+  windowed  Sadosun windowed attention + routed experts
+  scan    Sadosun selective scan + routed experts
+  sadosun Sadosun scan, windowed, windowed, scan
 
 All run the pipeline worker's own prefill and graph-captured decode step.
 """
@@ -24,14 +29,17 @@ import torch
 
 from ..config import ModelConfig
 from ..parallel.rccl import PipelineWorker, build_stage_model
-from .presets import _dense_mla, _lepizen, _llama, _tuvutar
+from .presets import (_dense_mla, _lepizen, _llama, _moe_mla, _sadosun,
+                      _tuvutar)
 
 SIZES: Dict[str, dict] = {
     "2048": dict(width=2048, heads=16, ff=8192, vocab=8192),
     "4096": dict(width=4096, heads=32, ff=14336, vocab=8192),
 }
 TUVUTAR = {"latent": "aaaa", "shared": "asss", "delta": "dddd", "mixed": "ddda"}
-KINDS = ("mla", *TUVUTAR, "llama", "lepizen")
+SADOSUN = {"windowed": "aaaa", "scan": "mmmm", "sadosun": "maam"}
+EXPERT_FF = {"2048": 1408, "4096": 1536}
+KINDS = ("mla", *TUVUTAR, "llama", "lepizen", "moe", *SADOSUN)
 PREFILL = ((1, 8192), (8, 1024))     # sequences, tokens each
 DECODE = ((1, 2048), (64, 2048))     # sequences, tokens cached
 
@@ -43,11 +51,27 @@ def stack(kind: str, size: dict) -> ModelConfig:
         make = _llama if kind == "llama" else _lepizen
         return ModelConfig.from_dict(
             make(n_layers=4, kv_heads=size["heads"] // 4, **size))
+    if kind == "moe" or kind in SADOSUN:
+        size = {**size, "ff": EXPERT_FF[str(size["width"])]}
+        if kind == "moe":
+            return ModelConfig.from_dict(_moe_mla(n_layers=4, **size))
+        return ModelConfig.from_dict(
+            _sadosun(period=SADOSUN[kind], kv_heads=size["heads"] // 4, **size))
     extra = {}
     if "d" in TUVUTAR[kind]:
         extra = dict(delta_heads=size["heads"], delta_kv=size["heads"] // 2)
     return ModelConfig.from_dict(
         _tuvutar(period=TUVUTAR[kind], repeats=1, **size, **extra))
+
+
+def _spread(model):
+    """Random router weights, not random biases of the choice, pick the experts;
+    they see normed rows."""
+    for name, p in model.named_parameters():
+        if name.endswith(".correction"):
+            p.data.zero_()
+        elif p.dim() == 0 and ".norm" in name:
+            p.data.fill_(1.0)
 
 
 def _time(fn, n: int) -> float:
@@ -69,6 +93,8 @@ def run(which: str = "all", steps: int = 32,
         for kind in kinds or KINDS:
             config = stack(kind, SIZES[name])
             model = build_stage_model(config, 0, 1, device)
+            if kind in SADOSUN:
+                _spread(model)
 
             def emit(phase, batch, seq, seconds, tokens):
                 print(json.dumps({

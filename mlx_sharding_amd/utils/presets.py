@@ -47,6 +47,33 @@ def _lepizen(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
                        for _ in range(n_layers)]}
 
 
+def _sadosun(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
+             period: str, repeats: int = 1, dim: int = 128, window: int = 1024,
+             experts: int = 64, identity: int = 8, top: int = 6,
+             inner: int = 0, state: int = 16, side: int = 256) -> dict:
+    """A Sadosun config: ``period`` repeated, "a" a windowed-attention layer,
+    "m" a selective-scan layer; ff: units of one expert."""
+    layers = []
+    for kind in period * repeats:
+        if kind == "m":
+            mixer = {"inner": inner or 2 * width, "state": state,
+                     "dt_rank": width // 16, "conv": 4}
+        else:
+            mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                     "vdim": dim, "scale": dim ** -0.5,
+                     "rot": {"base": 10000.0, "dims": dim},
+                     "mask": {"size": window}}
+        layers.append({
+            "type": "mamba1" if kind == "m" else "attention", "mixer": mixer,
+            "mlp": {"kind": "moe", "expert": {"ff": ff},
+                    "router": {"experts": experts, "identity": identity,
+                               "top": top}}})
+    return {"architecture": "Sadosun", "width": width, "vocab": vocab,
+            "norm": {"eps": 1e-6}, "embedding": {"scale": 12.0},
+            "canon": {"taps": 4}, "token_side": {"dim": side},
+            "layers": layers}
+
+
 def _llama(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
            n_layers: int) -> dict:
     return {"model_type": "llama", "hidden_size": width,
@@ -64,6 +91,15 @@ def _dense_mla(width: int, heads: int, ff: int, vocab: int, n_layers: int,
             "rms_norm_eps": 1e-6, "rope_theta": 10000.0, "q_lora_rank": None,
             "kv_lora_rank": rank, "qk_nope_head_dim": dim,
             "qk_rope_head_dim": rot, "v_head_dim": dim}
+
+
+def _moe_mla(width: int, heads: int, ff: int, vocab: int, n_layers: int,
+             experts: int = 64, top: int = 6) -> dict:
+    """A DeepSeek-V2 config with routed experts of ``ff`` units everywhere."""
+    return {**_dense_mla(width, heads, ff, vocab, n_layers),
+            "moe_intermediate_size": ff, "n_routed_experts": experts,
+            "num_experts_per_tok": top, "n_shared_experts": 0,
+            "first_k_dense_replace": 0, "moe_layer_freq": 1}
 
 
 PRESETS = {
@@ -184,6 +220,23 @@ PRESETS = {
                            delta_heads=32, delta_kv=16),
     "lepizen-2b": _lepizen(2048, 16, 4, 8192, 32000, 28),
     "lepizen-8b": _lepizen(4096, 32, 8, 16384, 32000, 36),
+    "sadosun-7b": _sadosun(2048, 16, 4, 1024, 32000, "maamaa", 4),
+    "debug-sadosun": {
+        "architecture": "Sadosun", "width": 80, "vocab": 320,
+        "norm": {"eps": 1e-6}, "embedding": {"scale": 4.0},
+        "canon": {"taps": 3}, "token_side": {"dim": 20},
+        "layers": [
+            {"type": "attention",
+             "mixer": {"heads": 6, "kv_heads": 2, "dim": 24, "vdim": 16,
+                       "scale": 0.2, "rot": {"base": 1000.0, "dims": 16},
+                       "mask": {"size": 50}},
+             "mlp": {"kind": "moe", "expert": {"ff": 48},
+                     "router": {"experts": 6, "identity": 1, "top": 2}}},
+            {"type": "mamba1",
+             "mixer": {"inner": 120, "state": 10, "dt_rank": 6, "conv": 4},
+             "mlp": None},
+        ],
+    },
     "debug-lepizen": {
         "architecture": "Lepizen", "width": 96, "vocab": 320,
         "norm": {"eps": 1e-6}, "residual_mult": 0.6, "logit_scale": 0.4,
