@@ -77,7 +77,7 @@ def fuse_model(model) -> int:
     from .deepseek_v2 import MLAAttention
     from .mixers import (CausalConv, GatedDelta, GatedMLP, GroupedAttention,
                          LatentAttention, ParallelBlock, RoutedExperts,
-                         SelectiveScan)
+                         SelectiveScan, TokenInput)
 
     n = 0
     for mod in model.modules():
@@ -94,7 +94,7 @@ def fuse_model(model) -> int:
             elif isinstance(mod, (CausalConv, GatedDelta, GatedMLP,
                                   GroupedAttention, LatentAttention,
                                   ParallelBlock, RoutedExperts,
-                                  SelectiveScan)):
+                                  SelectiveScan, TokenInput)):
                 mod.prepare()
                 n += 1
         except AssertionError:

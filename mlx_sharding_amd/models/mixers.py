@@ -527,9 +527,7 @@ class RoutedExperts(nn.Module):
         sh = self.shape
         self.w_up = self.up.pad(sh.ffp, sh.widthp)
         self.w_down = self.down.pad(sh.width, sh.ffp)
-        w = F.pad(self.router.weight.data, (0, sh.widthp - sh.width)).contiguous()
-        self.router.weight.data = w[:, : sh.width]
-        self.w_router = w
+        self.w_router = experts.pack(self.router.weight.data, sh.widthp)
         self.ready = True
 
     def forward(self, x: torch.Tensor, h: torch.Tensor,
@@ -553,12 +551,21 @@ class TokenInput(nn.Module):
         self.gate = Linear(width, dim, dtype=dtype)
         self.proj = Linear(dim, width, dtype=dtype)
         self.norm = RMSNorm(width, eps, dtype=dtype)
+        self.w_gate = None
+
+    @torch.no_grad()
+    def prepare(self):
+        if self.gate.in_features % ExpertShape.STEP == 0:
+            self.w_gate = experts.pack(self.gate.weight.data,
+                                       self.gate.in_features)
 
     def forward(self, x: torch.Tensor, e: torch.Tensor,
                 copy: Optional[torch.Tensor] = None) -> torch.Tensor:
         """x: fp32 residual; e [N, dim]; copy: x in the weights' type, where
         the caller has it."""
-        g = experts.token_gate(x, self.gate.weight, e)
-        if g is None:
+        if (self.w_gate is not None and x.is_cuda
+                and x.shape[0] <= experts.FEW):
+            g = experts.token_gate(x, self.w_gate, e)
+        else:
             g = ops.geglu(self.gate(x.to(e.dtype) if copy is None else copy), e)
         return self.proj(g)

@@ -26,7 +26,7 @@ import torch.nn.functional as F
 
 from ..config import ModelConfig, ShardSpec
 from ..ops import ragged
-from ..ops.experts import ExpertShape
+from ..ops.experts import FEW, ExpertShape
 from ..ops.paged import LayerSpec, PagedState, RaggedBatch
 from ..ops.ragged import Rotary, Turns
 from ..ops.recurrent import norm_conv
@@ -170,7 +170,7 @@ class SadosunStageModel(RaggedStageModel):
             copy = None
             if layer.mlp is not None:
                 h = enter(k, 2, y, pad_to=ExpertShape.STEP)
-                copy = layer.mlp(x, h, copy=batch.n_tokens > 64)
+                copy = layer.mlp(x, h, copy=batch.n_tokens > FEW)
             else:
                 ragged.add_norm(x, y, None, None, self.eps, 0.0, dtype)
             at = k * n

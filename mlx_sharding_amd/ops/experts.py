@@ -11,6 +11,7 @@ from __future__ import annotations
 from dataclasses import dataclass
 
 import torch
+import torch.nn.functional as F
 
 from .ragged import _ext, _pad
 
@@ -56,11 +57,25 @@ class ExpertShape:
         return TILE_SHORT if few else TILE_LONG
 
 
+def pack(w, width: int):
+    """Weights [rows, columns], the columns padded to ``width``, as matrix-core
+    operands of 16 rows by 32 columns, lane = (column / 8 % 4, row % 16)."""
+    rows, cols = w.shape
+    w = F.pad(w, (0, width - cols, 0, -rows % 16))
+    w = w.view(-1, 16, width // 32, 4, 8).permute(0, 2, 3, 1, 4)
+    return w.reshape(-1, width // 32, 64, 8).contiguous()
+
+
+def unpack(w, rows: int, cols: int):
+    w = w.view(-1, w.shape[1], 4, 16, 8).permute(0, 3, 1, 2, 4)
+    return w.reshape(w.shape[0] * 16, -1)[:rows, :cols]
+
+
 def route(h, router, correction, sh: ExpertShape):
     """Softmax router: chosen experts [N, top] and their weights (fp32).  The
     choice is by score + correction, the weights are the scores alone, divided
     by their sum."""
-    z = h[:, : sh.width].float() @ router[:, : sh.width].float().T
+    z = h[:, : sh.width].float() @ unpack(router, sh.total, sh.width).float().T
     s = torch.softmax(z, -1)
     idx = torch.topk(s + correction.float(), sh.top, dim=-1).indices
     w = s.gather(-1, idx)
@@ -71,8 +86,7 @@ def add_experts(x, h, router, correction, up, down, sh: ExpertShape,
                 copy: bool = False):
     """x [N, width] (fp32) += the weighted sum of the chosen experts of rows h
     [N, width padded], each W_down relu(W_up h)^2.  up [experts, ff padded,
-    width padded], down [experts, width, ff padded], router [total, width
-    padded].  copy: returns x in h's type as well."""
+    width padded], down [experts, width, ff padded], router packed.  copy: returns x in h's type as well."""
     if x.is_cuda:
         ext = _ext("experts")
         N = x.shape[0]
@@ -99,9 +113,10 @@ def add_experts(x, h, router, correction, up, down, sh: ExpertShape,
     return x.to(h.dtype) if copy else None
 
 
+FEW = 64  # rows that one skinny product takes
+
+
 def token_gate(x, gate, e):
-    """gelu_tanh(gate x) * e for rows of the fp32 residual x: one kernel for a
-    few rows, or None where it does not apply."""
-    if x.is_cuda and x.shape[0] <= 64 and x.shape[1] % 64 == 0:
-        return _ext("token_gate").token_gate(x, gate, e)
-    return None
+    """gelu_tanh(gate x) * e for a few rows of the fp32 residual x, in one
+    kernel; gate packed."""
+    return _ext("token_gate").token_gate(x, gate, e)

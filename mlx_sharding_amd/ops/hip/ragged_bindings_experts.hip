@@ -16,7 +16,7 @@ Tensor int_rows(const Tensor& like, std::vector<int64_t> sizes) {
   return torch::empty(sizes, like.options().dtype(torch::kInt32));
 }
 
-// h [N, K], w [total, K], correction [total]
+// h [N, K], w [total / 16, K / 32, 64, 8], correction [total]
 // -> chosen [N, top], weights [N, top], ranks [N, top], histograms
 std::tuple<Tensor, Tensor, Tensor, Tensor> expert_route(Tensor h, Tensor w,
                                                         Tensor correction,
@@ -29,16 +29,18 @@ std::tuple<Tensor, Tensor, Tensor, Tensor> expert_route(Tensor h, Tensor w,
   a.hstride = rows2(h, "h");
   a.n = h.size(0);
   a.K = (int)h.size(1);
-  TORCH_CHECK(w.dim() == 2 && w.is_contiguous() && w.size(1) == a.K &&
-              a.K % EX_STEP == 0 && a.hstride % 8 == 0);
+  a.total = (int)correction.numel();
+  TORCH_CHECK(a.K % EX_STEP == 0 && a.hstride % 8 == 0);
+  TORCH_CHECK(w.dim() == 4 && w.is_contiguous() &&
+              w.size(0) == (a.total + 15) / 16 && w.size(1) == a.K / 32 &&
+              w.size(2) == 64 && w.size(3) == 8, "router not packed for h");
   aligned16(h, "h");
   aligned16(w, "router");
-  a.total = (int)w.size(0);
   a.experts = (int)experts;
   a.top = (int)top;
   TORCH_CHECK(a.total <= EX_MAXTOTAL && experts >= 1 && experts <= a.total &&
               top >= 1 && top <= a.total);
-  TORCH_CHECK(correction.numel() == a.total && correction.is_contiguous());
+  TORCH_CHECK(correction.is_contiguous());
   const long blocks = (a.n + EX_TOK - 1) / EX_TOK;
   auto idx = int_rows(h, {a.n, top}), rank = int_rows(h, {a.n, top});
   auto hist = int_rows(h, {blocks, experts});
@@ -148,7 +150,8 @@ c10::optional<Tensor> expert_combine(Tensor x, Tensor h, Tensor d, Tensor where,
   return out;
 }
 
-// gelu_tanh(x w^T) * e for a few rows of the fp32 residual
+// gelu_tanh(x w^T) * e for a few rows of the fp32 residual; w packed for e's
+// columns
 Tensor token_gate(Tensor x, Tensor w, Tensor e) {
   check_f32(x, "x");
   const bool f32 = is_f32(w, "w");
@@ -156,13 +159,14 @@ Tensor token_gate(Tensor x, Tensor w, Tensor e) {
   TokenGateArgs a = {};
   a.n = (int)x.size(0);
   a.K = (int)x.size(1);
-  a.O = (int)w.size(0);
-  TORCH_CHECK(w.dim() == 2 && w.is_contiguous() && w.size(1) == a.K &&
-              a.K % EX_STEP == 0);
+  a.O = (int)e.size(1);
+  TORCH_CHECK(a.K % EX_STEP == 0 && w.dim() == 4 && w.is_contiguous() &&
+              w.size(0) == (a.O + 15) / 16 && w.size(1) == a.K / 32 &&
+              w.size(2) == 64 && w.size(3) == 8, "w not packed for x");
   aligned16(x, "x");
   aligned16(w, "w");
   a.estride = rows2(e, "e");
-  TORCH_CHECK(e.size(0) == a.n && e.size(1) == a.O);
+  TORCH_CHECK(e.size(0) == a.n);
   auto out = torch::empty({a.n, a.O}, w.options());
   a.x = x.data_ptr<float>();
   a.w = w.data_ptr();

@@ -8,6 +8,8 @@
 #define EX_MAXTOTAL 1024
 #define EX_STEP 64     // contractions are padded to this many elements
 
+// w: matrix-core operands of 16 experts by 32 columns, [tiles, K / 32, 64, 8],
+// lane = (column / 8 % 4, expert % 16)
 struct RouteArgs {
   const void *h, *w, *correction;
   int* idx;        // [tokens, top], >= experts: an identity expert
@@ -49,7 +51,7 @@ struct CombineArgs {
 
 struct TokenGateArgs {
   const float* x;             // [n, K]
-  const void *w, *e;          // [O, K], [n, O]
+  const void *w, *e;          // operands as the router's, [n, O]
   void* out;                  // [n, O]
   long estride;
   int n, O, K;

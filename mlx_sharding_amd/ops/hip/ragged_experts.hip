@@ -50,22 +50,19 @@ __global__ __launch_bounds__(RT_BLOCK) void expert_route_kernel(
     f32x4 acc[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0, 0, 0, 0};
-    const T* wrow[4];
+    // operands of 16 experts by 32 columns lie together, lane after lane
+    const T* w = (const T*)a.w + (long)first / 16 * steps * 512 + lane * 8;
+    const long next = (long)steps * 512;
+#pragma unroll 8
+    for (int s = s0; s < s1; ++s) {
+      Frag<T> b, f[4];
+      b.load(hrow + s * 32);
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      wrow[i] = (const T*)a.w +
-                (long)min(first + i * 16 + lr, a.total - 1) * a.K + lg * 8;
-    if (tiles) {
-#pragma unroll 4
-      for (int s = s0; s < s1; ++s) {
-        Frag<T> b, w[4];
-        b.load(hrow + s * 32);
-        // tiles past the last repeat it
+      for (int i = 0; i < 4; ++i)
+        if (i < tiles) f[i].load(w + i * next + s * 512);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) w[i].load(wrow[min(i, tiles - 1)] + s * 32);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) acc[i] = mma(w[i], b, acc[i]);
-      }
+      for (int i = 0; i < 4; ++i)
+        if (i < tiles) acc[i] = mma(f[i], b, acc[i]);
     }
     __syncthreads();  // the sums of the last round are read
 #pragma unroll
@@ -289,9 +286,9 @@ __device__ __forceinline__ void load_as(Frag<__bf16>& f, const float* p) {
   }
 }
 
-// red[wave][token][output] <- partial sums; w0, w1: this lane's weight rows,
-// xr: its row of X, each at the lane's first element
-template <typename T, typename X>
+// red[wave][token][output] <- partial sums; w0, w1: this lane's weights of two
+// tiles, WS elements from step to step; xr: its row of X
+template <typename T, typename X, int WS>
 __device__ __forceinline__ void skinny_sums(const T* w0, const T* w1,
                                             const X* xr, int K, int wid, int lr,
                                             int lg,
@@ -306,8 +303,8 @@ __device__ __forceinline__ void skinny_sums(const T* w0, const T* w1,
     Frag<T> a0[U], a1[U], b[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      a0[u].load(w0 + (s + u) * 32);
-      a1[u].load(w1 + (s + u) * 32);
+      a0[u].load(w0 + (s + u) * WS);
+      a1[u].load(w1 + (s + u) * WS);
       load_as(b[u], xr + (s + u) * 32);
     }
     __builtin_amdgcn_sched_barrier(0);
@@ -319,8 +316,8 @@ __device__ __forceinline__ void skinny_sums(const T* w0, const T* w1,
   }
   for (; s < s1; ++s) {
     Frag<T> a0, a1, b;
-    a0.load(w0 + s * 32);
-    a1.load(w1 + s * 32);
+    a0.load(w0 + s * WS);
+    a1.load(w1 + s * WS);
     load_as(b, xr + s * 32);
     c0 = mma(a0, b, c0);
     c1 = mma(a1, b, c1);
@@ -346,10 +343,10 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_skinny_kernel(
   const T* w = (const T*)a.w + (long)e * a.O * a.K + lg * 8;
   const long p = p0 + min(lr, n - 1);
   const long row = a.tokens ? a.tokens[p] : p;
-  skinny_sums<T, T>(w + (long)min(o0 + lr, a.O - 1) * a.K,
-                    w + (long)min(o0 + 16 + lr, a.O - 1) * a.K,
-                    (const T*)a.x + row * a.xstride + lg * 8, a.K, wid, lr, lg,
-                    red);
+  skinny_sums<T, T, 32>(
+      w + (long)min(o0 + lr, a.O - 1) * a.K,
+      w + (long)min(o0 + 16 + lr, a.O - 1) * a.K,
+      (const T*)a.x + row * a.xstride + lg * 8, a.K, wid, lr, lg, red);
   for (int i = tid; i < n * SK_OUT; i += EX_BLOCK) {
     const int t = i / SK_OUT, o = i % SK_OUT;
     if (o0 + o >= a.O) continue;
@@ -381,11 +378,13 @@ __global__ __launch_bounds__(EX_BLOCK) void token_gate_kernel(
   const int lr = lane & 15, lg = lane >> 4;
   const int o0 = blockIdx.x * SK_OUT, t0 = blockIdx.y * 16;
   const int n = min(16, a.n - t0);
-  const T* w = (const T*)a.w + lg * 8;
-  skinny_sums<T, float>(w + (long)min(o0 + lr, a.O - 1) * a.K,
-                        w + (long)min(o0 + 16 + lr, a.O - 1) * a.K,
-                        a.x + (long)(t0 + min(lr, n - 1)) * a.K + lg * 8, a.K,
-                        wid, lr, lg, red);
+  // operands of 16 outputs by 32 columns lie together, lane after lane
+  const int tiles = (a.O + 15) / 16;
+  const T* w = (const T*)a.w + lane * 8;
+  skinny_sums<T, float, 512>(
+      w + (long)(o0 / 16) * a.K * 16,
+      w + (long)min(o0 / 16 + 1, tiles - 1) * a.K * 16,
+      a.x + (long)(t0 + min(lr, n - 1)) * a.K + lg * 8, a.K, wid, lr, lg, red);
   for (int i = tid; i < n * SK_OUT; i += EX_BLOCK) {
     const int t = i / SK_OUT, o = o0 + i % SK_OUT;
     if (o >= a.O) continue;
@@ -501,10 +500,13 @@ __global__ __launch_bounds__(EX_BLOCK, 2) void expert_wide_kernel(
         read_row(fw[i], wb, wo + i * 16 + lr, kk, lg);
         read_row(fx[i], xb, wt + i * 16 + lr, kk, lg);
       }
+      // the block that multiplies goes before the one that loads
+      __builtin_amdgcn_s_setprio(1);
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = mma(fw[i], fx[j], acc[i][j]);
+      __builtin_amdgcn_s_setprio(0);
     }
   }
 #pragma unroll

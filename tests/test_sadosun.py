@@ -282,6 +282,15 @@ def test_experts(device, dtype, kind, n):
     assert m(x2, hp) is None and torch.equal(x2, xd)
 
 
+def test_operand_layout():
+    w = torch.arange(23 * 70).float().view(23, 70)
+    p = experts.pack(w, 128)
+    assert p.shape == (2, 4, 64, 8)
+    e, c = 21, 61
+    assert float(p[e // 16, c // 32, c // 8 % 4 * 16 + e % 16, c % 8]) == float(w[e, c])
+    assert torch.equal(experts.unpack(p, 23, 70), w)
+
+
 @pytest.mark.gpu
 @pytest.mark.parametrize("tile", [16, 128])
 def test_tile_sizes_agree(tile, monkeypatch):
@@ -312,7 +321,8 @@ def test_correction_biases_the_choice_only(device, dtype):
     want = (a * y2 + b * h.double()) / (a + b + 1e-20)
     pad = torch.nn.functional.pad
     x = torch.zeros(20, 32, device=device)
-    experts.add_experts(x, pad(h, (0, 32)).to(device), pad(router, (0, 32)).to(device),
+    experts.add_experts(x, pad(h, (0, 32)).to(device),
+                        experts.pack(router, 64).to(device),
                         corr.to(device), pad(up, (0, 32, 0, 48)).to(device),
                         pad(down, (0, 48)).to(device), sh)
     assert cases.error(x, want) < (1e-5 if dtype == F32 else 2e-2)
@@ -333,7 +343,7 @@ def test_token_input(device, dtype, W, dim, n):
     w = {"s." + k.replace(".weight", ""): v.double() for k, v in m.state_dict().items()}
     e = table[:, dim: 2 * dim]
     want = x.double() + oracle.token_input(x.double(), e.double(), w, "s.", 1e-2)
-    m.to(device)
+    m.to(device).prepare()
     xd, td = x.to(device), table.to(device)
     for copy in (None, xd.to(dtype)):
         y = m(xd, td[:, dim: 2 * dim], copy)
@@ -827,6 +837,7 @@ def test_kernels_refuse_bad_operands():
     idx = torch.zeros(20, 2, dtype=torch.int32, **dev)
     tiles = torch.zeros(4, 3, dtype=torch.int32, **dev)
     up = torch.zeros(3, 64, 64, **dev)
+    router = torch.zeros(1, 2, 64, 8, **dev)
     tab = torch.zeros(64, 8, **dev)
     pool = torch.zeros(640, 2 * 48, **dev)
     sizes = (4, 2, 32, 16, 32, 16, batch.tok_pos, batch.tok_entry, batch.pages, 20)
@@ -843,14 +854,14 @@ def test_kernels_refuse_bad_operands():
         lambda: scan(A=torch.zeros(12, 8, **dev)),
         lambda: scan(bc=torch.zeros(20, 32, **dev)),
         lambda: scan(state=torch.zeros(2, 1, 8, 16, **dev)),
-        lambda: ext.expert_route(h[:, :48], torch.zeros(5, 48, **dev), torch.zeros(5, **dev), 4, 2),
-        lambda: ext.expert_route(h, torch.zeros(5, 64, **dev), torch.zeros(4, **dev), 4, 2),
-        lambda: ext.expert_route(h, torch.zeros(5, 64, **dev), torch.zeros(5, **dev), 4, 6),
+        lambda: ext.expert_route(h[:, :32], router, torch.zeros(5, **dev), 4, 2),
+        lambda: ext.expert_route(h, router, torch.zeros(17, **dev), 4, 2),
+        lambda: ext.expert_route(h, router, torch.zeros(5, **dev), 4, 6),
         lambda: ext.expert_plan(idx, idx, torch.zeros(1, 3, dtype=torch.int32, **dev), 3, 16),
         lambda: ext.expert_gemm(h, idx.view(-1), tiles, up, 32, 40, False),
         lambda: ext.expert_gemm(h, None, tiles, up, 16, 40, False),
         lambda: ext.expert_gemm(h[:, :32], idx.view(-1), tiles, up, 16, 40, False),
-        lambda: ext.token_gate(h, torch.zeros(3, 32, **dev), torch.zeros(20, 3, **dev)),
+        lambda: ext.token_gate(h, router, torch.zeros(20, 17, **dev)),
         lambda: ext.grouped_turn(y, 1e-6, True, tab[:, :4], tab[:, :4], None, None, pool, *sizes),
         lambda: ext.grouped_turn(y, 1e-6, True, torch.zeros(64, 20, **dev), torch.zeros(64, 20, **dev),
                                  None, None, pool, *sizes),
