@@ -380,7 +380,7 @@ __device__ __forceinline__ float decay_exp<float>(float x) {
 }
 
 // ln(1 + e^d).  For bf16 operands: the logarithm of 1 + u from the instruction
-// where u is not small, else its series; both to about 1e-7 of the result.
+// where u is not small, else its series; both to about 1e-6 of the result.
 template <typename T>
 __device__ __forceinline__ float step_size(float d);
 template <>
