@@ -5,7 +5,7 @@
 #include "ragged_recurrent.h"
 
 #define RC_BLOCK 256
-#define RC_TT 16       // tokens per block of a long portion
+#define RC_TT 8        // tokens per block of a long portion
 #define RC_CHUNK 64    // tokens per entry of `chunks`
 #define RC_SUB (RC_CHUNK / RC_TT)
 
@@ -37,6 +37,18 @@ struct Raw<T, 1> {
   __device__ __forceinline__ void set(int, float x) { v = (T)x; }
 };
 
+template <typename T>
+__device__ __forceinline__ float silu_of(float z);
+template <>
+__device__ __forceinline__ float silu_of<float>(float z) {
+  return silu_f(z);
+}
+template <>
+__device__ __forceinline__ float silu_of<__bf16>(float z) {
+  return z * __builtin_amdgcn_rcpf(
+                 1.0f + __builtin_amdgcn_exp2f(-1.44269504088896340736f * z));
+}
+
 // What one token's convolution gives from the last HT + 1 rows, newest last;
 // rows and weights past the real taps are zero.
 template <typename T, int V, int HT>
@@ -50,7 +62,7 @@ __device__ __forceinline__ Raw<T, V> convolved(const Raw<T, V>* rows,
     float s = bias.at(i);
 #pragma unroll
     for (int j = 0; j <= HT; ++j) s += w[j].at(i) * rows[j].at(i);
-    if (a.silu) s = silu_f(s);
+    if (a.silu) s = silu_of<T>(s);
     if (a.add) s += rows[HT].at(i);
     o.set(i, s);
   }
@@ -108,7 +120,7 @@ __global__ __launch_bounds__(RC_BLOCK) void conv_short_kernel(const ConvArgs a) 
     if (j >= HT - hist) rows[j].store(hp + (long)(j - HT + hist) * a.C);
 }
 
-// Long portions: 16 tokens by V channels a thread, all rows asked for first.
+// Long portions: RC_TT tokens by V channels a thread, all rows asked for first.
 // grid (chunks * RC_SUB, channel groups)
 template <typename T, int V, int HT>
 __global__ __launch_bounds__(RC_BLOCK) void conv_long_kernel(const ConvArgs a) {
@@ -397,18 +409,6 @@ __device__ __forceinline__ float step_size<__bf16>(float d) {
   small = fmaf(u, small, -0.5f);
   small = fmaf(u, small * u, u);
   return fmaxf(d, 0.0f) + (u < 0.04f ? small : large);
-}
-
-template <typename T>
-__device__ __forceinline__ float silu_of(float z);
-template <>
-__device__ __forceinline__ float silu_of<float>(float z) {
-  return silu_f(z);
-}
-template <>
-__device__ __forceinline__ float silu_of<__bf16>(float z) {
-  return z * __builtin_amdgcn_rcpf(
-                 1.0f + __builtin_amdgcn_exp2f(-1.44269504088896340736f * z));
 }
 
 typedef const __attribute__((address_space(4))) unsigned* ScalarWords;
