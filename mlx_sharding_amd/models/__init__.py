@@ -12,6 +12,7 @@ from .base import StageModel
 from .llama import LlamaStageModel
 from .gemma2 import Gemma2StageModel
 from .deepseek_v2 import DeepseekV2StageModel
+from .dufinex import DufinexStageModel
 from .lepizen import LepizenStageModel
 from .sadosun import SadosunStageModel
 from .tuvutar import TuvutarStageModel
@@ -31,6 +32,7 @@ _REGISTRY: Dict[str, Type[StageModel]] = {
     "tuvutar": TuvutarStageModel,
     "lepizen": LepizenStageModel,
     "sadosun": SadosunStageModel,
+    "dufinex": DufinexStageModel,
 }
 
 

@@ -180,6 +180,11 @@ class StageModel(nn.Module):
 
     # -- weights ----------------------------------------------------------
     @classmethod
+    def complete_config(cls, config: ModelConfig,
+                        weights: Dict[str, torch.Tensor]):
+        """Enter sizes that only the checkpoint's tensors tell."""
+
+    @classmethod
     def owns_key(cls, key: str, shard: ShardSpec) -> bool:
         """Key-routing rule — identical to the reference splitter
         (/root/reference/sharding_weight.py:17-24): layer keys by index

@@ -9,7 +9,7 @@ GEMM, head sizes padded to the kernels' tiles) once they are on their device.
 
 from __future__ import annotations
 
-from typing import Optional
+from typing import Optional, Tuple, Union
 
 import torch
 import torch.nn as nn
@@ -17,10 +17,11 @@ import torch.nn.functional as F
 
 from .. import ops
 from ..ops import experts, ragged, recurrent
-from ..ops.experts import ExpertShape
+from ..ops.experts import ExpertShape, Routing
 from ..ops.paged import (HistorySpec, LayerSpec, LayerStore, RaggedBatch,
                          RowSpec, StateSpec)
-from ..ops.ragged import DeltaShape, GroupedShape, LatentShape, Rotary, Turns
+from ..ops.ragged import (ClampedGLU, DeltaShape, GroupedShape, LatentShape,
+                          Rotary, Turns)
 from ..ops.recurrent import ScanShape
 from .base import Linear, RMSNorm
 
@@ -207,12 +208,18 @@ class GroupedAttention(nn.Module):
     keys and values.
 
     ``qk_norm``: RMS norms over the whole query and the whole key projection.
-    ``head_norm``: every query and key divided by its own root mean square.
+    ``head_norm``: every query and key divided by its own root mean square;
+    ``head_weights``: and multiplied by a weight per dimension that the heads
+    share.
     ``rotary``: positions on queries and keys; ``turn_values``: positions on the
     values as well, undone on each output by its own position.
     ``window``: how many tokens a token sees, up to itself.
     ``sink``: one learned score per head that enters the softmax's denominator
     and nothing else; ``zero_sink``: that score is 0 for every head.
+    ``gate``: every head's output times the sigmoid of a number that a
+    projection of the input gives.
+    ``own_rows``: otherwise the layer has no keys and values of its own and
+    attends to the pages of another layer's store.
     ``vmix``: the share of another layer's values in this layer's, where the
     caller passes such values.
     """
@@ -222,22 +229,31 @@ class GroupedAttention(nn.Module):
                  sink: bool = False, dtype: torch.dtype = torch.bfloat16, *,
                  head_norm: bool = False, rotary: Optional[Rotary] = None,
                  turn_values: Optional[Rotary] = None,
-                 window: Optional[int] = None, zero_sink: bool = False):
+                 window: Optional[int] = None, zero_sink: bool = False,
+                 head_weights: bool = False, gate: bool = False,
+                 own_rows: bool = True):
         super().__init__()
         self.shape = sh = GroupedShape(heads, kv_heads, dim, vdim)
         self.scale, self.eps = float(scale), eps
-        self.head_norm, self.window = head_norm, window
+        self.head_norm, self.window = head_norm or head_weights, window
         self.rotary, self.turn_values = rotary, turn_values
+        if qk_norm and self.head_norm:
+            raise ValueError("queries and keys are normed whole or per head")
 
         def lin(out_features):
-            if not qk_norm:
+            if not (qk_norm or head_weights):
                 return Linear(width, out_features, dtype=dtype)
-            return NormedLinear(width, out_features, out_features, eps, dtype)
+            normed = dim if head_weights else out_features
+            return NormedLinear(width, out_features, normed, eps, dtype)
 
-        self.q, self.k = lin(heads * dim), lin(kv_heads * dim)
-        self.v = Linear(width, kv_heads * vdim, dtype=dtype)
+        self.q, self.k, self.v = lin(heads * dim), None, None
+        if own_rows:
+            self.k = lin(kv_heads * dim)
+            self.v = Linear(width, kv_heads * vdim, dtype=dtype)
+        self.g = Linear(width, heads, dtype=dtype) if gate else None
         self.vmix = None
-        if rotary is None and turn_values is None and not head_norm:
+        if (rotary is None and turn_values is None and not self.head_norm
+                and own_rows):
             self.vmix = _param(dtype=dtype)
         if zero_sink:
             self.register_buffer("sink", torch.zeros(heads, dtype=dtype),
@@ -256,13 +272,14 @@ class GroupedAttention(nn.Module):
         if window is not None and window < 1:
             raise ValueError("a window holds at least the token itself")
 
-    def store_spec(self) -> RowSpec:
-        return RowSpec(self.shape.width)
+    def store_spec(self) -> Optional[RowSpec]:
+        return None if self.k is None else RowSpec(self.shape.width)
 
     @property
     def rows(self):
         """The projections whose outputs ``attend`` takes, in this order."""
-        return self.q, self.k, self.v
+        return tuple(m for m in (self.q, self.k, self.v, self.g)
+                     if m is not None)
 
     @torch.no_grad()
     def prepare(self):
@@ -275,20 +292,24 @@ class GroupedAttention(nn.Module):
 
     def attend(self, y: torch.Tensor, out: torch.Tensor, batch: RaggedBatch,
                store: LayerStore, first: Optional[torch.Tensor] = None,
-               turns: Optional[Turns] = None) -> torch.Tensor:
-        """y [N, q | k | v | ...]; writes out [N, heads * vdim].  first: values
-        [N, kv_heads * vdim] to mix in.  turns: the tables of this layer's
-        rotations.  Returns this layer's values before mixing, a view of y."""
-        sh = self.shape
+               turns: Optional[Turns] = None) -> Optional[torch.Tensor]:
+        """y [N, q | k | v | gate | ...], what there is of them; writes out [N,
+        heads * vdim].  store: the layer's own, or that of the layer it reads.
+        first: values [N, kv_heads * vdim] to mix in.  turns: the tables of
+        this layer's rotations.  Returns this layer's values before mixing, a
+        view of y."""
+        sh, own = self.shape, self.k is not None
         norms = [getattr(m, "norm", None) for m in (self.q, self.k)]
         q = ragged.grouped_append(
             y, *(None if n is None else n.weight for n in norms), self.eps,
             None if first is None else self.vmix, first, store, sh, batch,
-            turns, self.head_norm)
+            turns, self.head_norm, own)
+        values = (sh.heads + sh.kv_heads) * sh.dim
+        end = values + sh.kv_heads * sh.vdim if own else sh.heads * sh.dim
+        gate = None if self.g is None else y[:, end: end + sh.heads]
         ragged.grouped_attention(q, self.sink, store, sh, self.scale, batch, out,
-                                 self.window, turns)
-        at = (sh.heads + sh.kv_heads) * sh.dim
-        return y[:, at: at + sh.kv_heads * sh.vdim]
+                                 self.window, turns, gate)
+        return y[:, values: end] if own else None
 
     def forward(self, h: torch.Tensor, batch: RaggedBatch, store: LayerStore,
                 first: Optional[torch.Tensor] = None,
@@ -355,25 +376,40 @@ class SelectiveScan(nn.Module):
 
 class GatedDelta(nn.Module):
     """Gated delta rule: a linear recurrence with a fp32 matrix state per head
-    that forgets (one decay per head) and corrects (delta write), behind short
-    convolutions, with a normed and gated output."""
+    that forgets and corrects (delta write), behind short convolutions, with a
+    normed and gated output.
+
+    The decay is one number per head (projection ``a``) and the gate a
+    projection ``g``.  ``ranks``: the decay is one number per head and key
+    channel, and both come through low-rank projections, ``a2`` of ``a1`` and
+    ``g2`` of ``g1``.  ``gate``: silu or sigmoid."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
                  vdim: int, taps: int, eps: float,
-                 dtype: torch.dtype = torch.bfloat16):
+                 dtype: torch.dtype = torch.bfloat16, *,
+                 ranks: Optional[Tuple[int, int]] = None, gate: str = "silu"):
         super().__init__()
-        self.shape = DeltaShape(heads, kv_heads, dim, vdim, taps)
-        self.eps = eps
+        if heads % kv_heads:
+            raise ValueError(f"{heads} heads do not share {kv_heads} query/key "
+                             f"heads evenly")
+        if gate not in ("silu", "sigmoid"):
+            raise ValueError(f"unknown gate {gate!r}")
+        self.shape = DeltaShape(heads, kv_heads, dim, vdim, taps, ranks)
+        self.eps, self.sigmoid = eps, gate == "sigmoid"
+        lin = lambda i, o: Linear(i, o, dtype=dtype)  # noqa: E731
         self.q = ConvLinear(width, kv_heads * dim, taps, dtype)
         self.k = ConvLinear(width, kv_heads * dim, taps, dtype)
         self.v = ConvLinear(width, heads * vdim, taps, dtype)
-        self.g = Linear(width, heads * vdim, dtype=dtype)
-        self.a = Linear(width, heads, dtype=dtype)
-        self.b = Linear(width, heads, dtype=dtype)
+        if ranks is None:
+            self.g, self.a = lin(width, heads * vdim), lin(width, heads)
+        else:
+            self.a1, self.a2 = lin(width, ranks[0]), lin(ranks[0], heads * dim)
+            self.g1, self.g2 = lin(width, ranks[1]), lin(ranks[1], heads * vdim)
+        self.b = lin(width, heads)
         self.A_log = _param(heads, dtype=dtype)
-        self.dt_bias = _param(heads, dtype=dtype)
+        self.dt_bias = _param(heads * (1 if ranks is None else dim), dtype=dtype)
         self.norm = RMSNorm(vdim, eps, dtype=dtype)
-        self.o = Linear(heads * vdim, width, dtype=dtype)
+        self.o = lin(heads * vdim, width)
         self.ready = False
 
     def store_spec(self) -> StateSpec:
@@ -382,36 +418,59 @@ class GatedDelta(nn.Module):
 
     @torch.no_grad()
     def prepare(self):
-        rows = (self.q, self.k, self.v, self.g, self.a, self.b)
-        self.w_in = torch.cat([m.weight.data for m in rows]).contiguous()
-        _share(self.w_in, *rows)
-        convs = (self.q, self.k, self.v)
+        sh, convs = self.shape, (self.q, self.k, self.v)
         self.w_conv = torch.cat([m.conv.weight.data for m in convs]).contiguous()
+        if sh.ranks is None:
+            rows = (*convs, self.g, self.a, self.b)
+            self.w_in = torch.cat([m.weight.data for m in rows]).contiguous()
+            _share(self.w_in, *rows)
+        else:
+            rows = (*convs, self.a1, self.g1, self.b)
+            w = self.q.weight.data
+            self.w_in = w.new_zeros(-(-(sh.columns[5] + sh.heads) // 8) * 8,
+                                    w.shape[1])
+            for at, m in zip(sh.columns, rows):
+                self.w_in[at: at + m.out_features] = m.weight.data
+                m.weight.data = self.w_in[at: at + m.out_features]
+            # both second projections in one product, zeros where they do not
+            # read
+            lo, hi = sh.inputs
+            mid, cut = sh.columns[4] - lo, self.a2.out_features
+            self.w_low = w.new_zeros(cut + self.g2.out_features, hi - lo)
+            for m, part in ((self.a2, self.w_low[:cut, :mid]),
+                            (self.g2, self.w_low[cut:, mid:])):
+                part = part[:, : m.in_features]
+                part.copy_(m.weight.data)
+                m.weight.data = part
         self.ready = True
 
     def forward(self, h: torch.Tensor, batch: RaggedBatch,
                 store: LayerStore) -> torch.Tensor:
         if not self.ready:
             self.prepare()
-        y = ops.linear(h, self.w_in)
+        y, z = ops.linear(h, self.w_in), None
+        if self.shape.ranks is not None:
+            lo, hi = self.shape.inputs
+            z = ops.linear(y[:, lo: hi], self.w_low)
         o = ragged.gated_delta(y, self.w_conv, self.A_log, self.dt_bias,
                                self.norm.weight, store, self.shape, self.eps,
-                               batch)
+                               batch, z, self.sigmoid)
         return self.o(o)
 
 
 class GatedMLP(nn.Module):
-    """W_down (act(W_gate h) * W_up h)."""
+    """W_down (act(W_gate h) * W_up h), or W_down of any other function of the
+    two (``act``), with or without biases."""
 
     ACTS = {"gelu_tanh": ops.geglu, "silu": ops.swiglu}
 
-    def __init__(self, width: int, ff: int, act: str,
-                 dtype: torch.dtype = torch.bfloat16):
+    def __init__(self, width: int, ff: int, act: Union[str, ClampedGLU],
+                 dtype: torch.dtype = torch.bfloat16, bias: bool = False):
         super().__init__()
-        self.act = self.ACTS[act]
-        self.gate = Linear(width, ff, dtype=dtype)
-        self.up = Linear(width, ff, dtype=dtype)
-        self.down = Linear(ff, width, dtype=dtype)
+        self.act = self.ACTS[act] if isinstance(act, str) else act
+        self.gate = Linear(width, ff, bias=bias, dtype=dtype)
+        self.up = Linear(width, ff, bias=bias, dtype=dtype)
+        self.down = Linear(ff, width, bias=bias, dtype=dtype)
         self.fused = None
 
     def prepare(self):
@@ -508,36 +567,62 @@ class _Stacked(nn.Module):
 
 
 class RoutedExperts(nn.Module):
-    """Every token's ``top`` of ``experts`` ungated relu^2 feed-forwards and
-    ``identity`` experts that return their input.  A softmax router in 32-bit;
+    """Every token's ``top`` of ``experts`` feed-forwards and ``identity``
+    experts that return their input.  A feed-forward is ungated with relu^2,
+    or gated with ``glu``.  ``routing``: what the router's 32-bit logits become;
     ``correction`` biases the choice but not the weights."""
 
     def __init__(self, width: int, ff: int, experts: int, identity: int,
-                 top: int, dtype: torch.dtype = torch.bfloat16):
+                 top: int, dtype: torch.dtype = torch.bfloat16, *,
+                 glu: Optional[ClampedGLU] = None, routing: Routing = Routing(),
+                 correction: bool = True):
         super().__init__()
         self.shape = sh = ExpertShape(width, ff, experts, identity, top)
+        self.glu, self.routing = glu, routing
+        if glu is not None:
+            self.gate = _Stacked(experts, ff, width, dtype)
         self.up = _Stacked(experts, ff, width, dtype)
         self.down = _Stacked(experts, width, ff, dtype)
         self.router = Linear(width, sh.total, dtype=dtype)
-        self.correction = _param(sh.total, dtype=dtype)
+        self.correction = _param(sh.total, dtype=dtype) if correction else None
         self.ready = False
 
     @torch.no_grad()
     def prepare(self):
         sh = self.shape
-        self.w_up = self.up.pad(sh.ffp, sh.widthp)
+        if self.glu is None:
+            self.w_up = self.up.pad(sh.ffp, sh.widthp)
+        else:  # the gate's rows, then the up projection's
+            w = self.up.weight.data
+            self.w_up = w.new_zeros(w.shape[0], 2 * sh.ffp, sh.widthp)
+            for at, m in ((0, self.gate), (sh.ffp, self.up)):
+                part = self.w_up[:, at: at + sh.ff, : sh.width]
+                part.copy_(m.weight.data)
+                m.weight.data = part
         self.w_down = self.down.pad(sh.width, sh.ffp)
         self.w_router = experts.pack(self.router.weight.data, sh.widthp)
         self.ready = True
 
+    def rows(self, h: torch.Tensor):
+        """What a token's experts give, to be summed per token: (rows, where
+        [N, top]); h [N, width padded to a multiple of ``ExpertShape.STEP``]."""
+        if not self.ready:
+            self.prepare()
+        if self.shape.identity or not self.routing.on_input:
+            raise ValueError("these experts' rows still need their weights")
+        return experts.expert_rows(h, self.w_router, self.correction, self.w_up,
+                                   self.w_down, self.shape, self.routing,
+                                   self.glu)[:2]
+
     def forward(self, x: torch.Tensor, h: torch.Tensor,
                 copy: bool = False) -> Optional[torch.Tensor]:
-        """Adds to the residual x in place; h [N, width padded to a multiple of
-        ``ExpertShape.STEP``].  copy: returns the new x in h's type."""
+        """Adds to the residual x in place; h as above.  copy: returns the new
+        x in h's type."""
         if not self.ready:
             self.prepare()
         return experts.add_experts(x, h, self.w_router, self.correction,
-                                   self.w_up, self.w_down, self.shape, copy)
+                                   self.w_up, self.w_down, self.shape, copy,
+                                   self.routing, self.glu)
 
 
 class TokenInput(nn.Module):

@@ -2,17 +2,21 @@
 
 config.json gives ``width``, ``vocab``, ``norm.eps`` and ``layers``, a list of
 {"type", "mixer", "mlp"}.  Tensors: ``embed``, ``l<i>.*``, ``final.norm``,
-``head``.  The residual stream is 32-bit, also between pipeline stages.
+``head`` (where it is not the embedding table).  The residual stream is 32-bit,
+also between pipeline stages.  A layer whose mixer has ``kv_from`` reads the rows
+that layer cached, so both live on one stage.
 """
 
 from __future__ import annotations
 
+import re
 from typing import Dict, List, Optional, Tuple
 
 import torch
 import torch.nn as nn
 import torch.nn.functional as F
 
+from .. import ops
 from ..config import ModelConfig, ShardSpec
 from ..ops.paged import PagedState, RaggedBatch, RaggedCache, RaggedLayerCache
 from ..ops.ragged import Rotary
@@ -27,6 +31,7 @@ class RaggedStageModel(StageModel):
     supports_ragged = True
     supports_quantization = False
     norm_offset = 0.0  # norm weights are stored around 1 - norm_offset
+    tied_head = False  # the embedding table makes the logits
     # parameters that are not the ``weight`` of a module
     bare_parameters: Tuple[str, ...] = ()
 
@@ -34,7 +39,7 @@ class RaggedStageModel(StageModel):
                  dtype: torch.dtype = torch.bfloat16):
         super().__init__(config, shard)
         W, self.eps = config.hidden_size, float(config["norm"]["eps"])
-        if shard.is_first:
+        if shard.is_first or (self.tied_head and shard.is_last):
             self.embed = nn.Embedding(config.vocab_size, W, dtype=dtype)
         for i in owned_layer_indices(shard):
             self.add_module(f"l{i}", self.make_layer(i, config["layers"][i],
@@ -42,9 +47,17 @@ class RaggedStageModel(StageModel):
         if shard.is_last:
             self.final = nn.Module()
             self.final.norm = self.make_final_norm(W, dtype)
-            self.head = Linear(W, config.vocab_size, dtype=dtype)
+            if not self.tied_head:
+                self.head = Linear(W, config.vocab_size, dtype=dtype)
         self._tables: Dict = {}
         self._old_tables: List = []  # captured graphs may still read them
+        for i in owned_layer_indices(shard):
+            j = self.row_source(config, i)
+            if j != i and not (shard.owns(j) and j < i):
+                raise ValueError(
+                    f"layer {i} reads the rows of layer {j}, which stage "
+                    f"[{shard.start_layer}, {shard.end_layer}) does not run "
+                    f"before it")
 
     def make_layer(self, i: int, spec: dict, width: int,
                    dtype: torch.dtype) -> nn.Module:
@@ -52,6 +65,23 @@ class RaggedStageModel(StageModel):
 
     def make_final_norm(self, width: int, dtype: torch.dtype) -> nn.Module:
         return RMSNorm(width, self.eps, self.norm_offset, dtype)
+
+    # -- layers that read another layer's rows -----------------------------
+    @staticmethod
+    def row_source(config: ModelConfig, i: int) -> int:
+        """The layer whose rows layer i reads."""
+        j = config["layers"][i]["mixer"].get("kv_from")
+        return i if j is None else int(j)
+
+    @classmethod
+    def allowed_cuts(cls, config: ModelConfig) -> Optional[List[int]]:
+        """Layer indices a pipeline stage may begin at: not between a layer
+        and one that reads its rows (None: any)."""
+        n = config.num_hidden_layers
+        bad = set()
+        for i in range(n):
+            bad.update(range(cls.row_source(config, i) + 1, i + 1))
+        return [c for c in range(1, n) if c not in bad] if bad else None
 
     def layer(self, i: int) -> nn.Module:
         return getattr(self, f"l{i}")
@@ -68,7 +98,7 @@ class RaggedStageModel(StageModel):
     def owns_key(cls, key: str, shard: ShardSpec) -> bool:
         top = key.split(".")[0]
         if top == "embed":
-            return shard.is_first
+            return shard.is_first or (cls.tied_head and shard.is_last)
         if top in ("final", "head"):
             return shard.is_last
         return top[:1] == "l" and top[1:].isdigit() and shard.owns(int(top[1:]))
@@ -76,11 +106,26 @@ class RaggedStageModel(StageModel):
     @classmethod
     def sanitize(cls, weights, shard: ShardSpec):
         out = {}
-        for k, v in weights.items():
+        for k, v in cls.stack_experts(weights, shard).items():
             if cls.owns_key(k, shard):
                 if k.rsplit(".", 1)[-1] not in (*cls.bare_parameters, "weight"):
                     k = f"{k}.weight"
                 out[k] = v
+        return out
+
+    @classmethod
+    def stack_experts(cls, weights, shard: ShardSpec):
+        """One stacked matrix per kind in place of those of the experts."""
+        found: Dict[str, Dict[int, str]] = {}
+        out = dict(weights)
+        for k in weights:
+            m = re.fullmatch(r"(l\d+\.mlp)\.e(\d+)\.(gate|up|down)", k)
+            if m and cls.owns_key(k, shard):
+                found.setdefault(f"{m[1]}.{m[3]}", {})[int(m[2])] = k
+        for name, keys in found.items():
+            if sorted(keys) == list(range(len(keys))):  # else: reported
+                out[name] = torch.stack([out.pop(keys[e])
+                                         for e in range(len(keys))])
         return out
 
     # -- cache -------------------------------------------------------------
@@ -120,6 +165,12 @@ class RaggedStageModel(StageModel):
         if self.shard.is_first:
             return F.embedding(x, self.embed.weight).float()
         return x[:, : self.config.hidden_size].float().contiguous().clone()
+
+    def logits(self, h: torch.Tensor) -> torch.Tensor:
+        """fp32 logits of rows that went through the final norm."""
+        if self.tied_head:
+            return ops.linear(h, self.embed.weight).float()
+        return self.head(h).float()
 
     def run(self, x: torch.Tensor, batch: RaggedBatch, state: PagedState,
             rows: Optional[torch.Tensor] = None,

@@ -17,8 +17,7 @@ Tensors: ``embed``, ``side.embed``, ``l<i>.norm1`` / ``norm2``, ``l<i>.canon1`` 
 
 from __future__ import annotations
 
-import re
-from typing import Dict, Optional
+from typing import Optional
 
 import torch
 import torch.nn as nn
@@ -117,21 +116,6 @@ class SadosunStageModel(RaggedStageModel):
             return shard.is_first
         return super().owns_key(key, shard)
 
-    @classmethod
-    def sanitize(cls, weights, shard):
-        """One stacked matrix per kind in place of those of the experts."""
-        found: Dict[str, Dict[int, str]] = {}
-        out = dict(weights)
-        for k in weights:
-            m = re.fullmatch(r"(l\d+\.mlp)\.e(\d+)\.(up|down)", k)
-            if m and cls.owns_key(k, shard):
-                found.setdefault(f"{m[1]}.{m[3]}", {})[int(m[2])] = k
-        for name, keys in found.items():
-            if sorted(keys) == list(range(len(keys))):  # else: reported
-                out[name] = torch.stack([out.pop(keys[e])
-                                         for e in range(len(keys))])
-        return super().sanitize(out, shard)
-
     # -- forward -----------------------------------------------------------
     def _turns(self, layer, batch: RaggedBatch, device) -> Turns:
         n = batch.max_pos
@@ -187,4 +171,4 @@ class SadosunStageModel(RaggedStageModel):
             return torch.cat([x, side[:, len(items) * n:].float()], 1)
         if rows is not None:
             h = h.index_select(0, rows)
-        return self.head(h).float()
+        return self.logits(h)

@@ -12,12 +12,11 @@ Tensors: ``embed``, ``l<i>.norm1`` / ``norm1b`` / ``norm2`` / ``norm2b``,
 
 from __future__ import annotations
 
-from typing import List, Optional
+from typing import Optional
 
 import torch
 import torch.nn as nn
 
-from ..config import ModelConfig, ShardSpec
 from ..ops import ragged
 from ..ops.paged import PagedState, RaggedBatch
 from ..ops.ragged import Rotary
@@ -59,8 +58,6 @@ class TuvutarLayer(nn.Module):
         self.norm1 = RMSNorm(width, eps, NORM_OFFSET, dtype)
         self.norm1b = RMSNorm(width, eps, NORM_OFFSET, dtype)
         self.mix = _mixer(spec["type"], mx, width, eps, dtype)
-        src = mx.get("kv_from")
-        self.source: Optional[int] = None if src is None else int(src)
         mlp = spec.get("mlp")
         self.mlp = None
         if mlp is not None:
@@ -76,31 +73,8 @@ class TuvutarStageModel(RaggedStageModel):
     norm_offset = NORM_OFFSET
     bare_parameters = ("A_log", "dt_bias")
 
-    def __init__(self, config: ModelConfig, shard: ShardSpec, quant_for=None,
-                 dtype: torch.dtype = torch.bfloat16):
-        super().__init__(config, shard, quant_for, dtype)
-        for i, layer in self.layer_items():
-            j = layer.source
-            if j is not None and not (shard.owns(j) and j < i):
-                raise ValueError(
-                    f"layer {i} reads the rows of layer {j}, which stage "
-                    f"[{shard.start_layer}, {shard.end_layer}) does not run "
-                    f"before it")
-
     def make_layer(self, i, spec, width, dtype):
         return TuvutarLayer(spec, width, self.eps, dtype)
-
-    @classmethod
-    def allowed_cuts(cls, config: ModelConfig) -> List[int]:
-        """Layer indices a pipeline stage may begin at: not between a layer
-        and one that reads its rows."""
-        n = config.num_hidden_layers
-        bad = set()
-        for i, spec in enumerate(config["layers"]):
-            j = spec["mixer"].get("kv_from")
-            if j is not None:
-                bad.update(range(int(j) + 1, i + 1))
-        return [c for c in range(1, n) if c not in bad]
 
     # -- forward -----------------------------------------------------------
     @torch.no_grad()
@@ -121,7 +95,7 @@ class TuvutarStageModel(RaggedStageModel):
             else:
                 after = self.final.norm if self.shard.is_last else None
             if isinstance(layer.mix, LatentAttention):
-                src = i if layer.source is None else layer.source
+                src = self.row_source(self.config, i)
                 y = layer.mix(h, batch, state.layers[src - first],
                               self._rotation(layer.mix.rotary, batch.max_pos,
                                              x.device))
@@ -138,4 +112,4 @@ class TuvutarStageModel(RaggedStageModel):
             return x
         if rows is not None:
             h = h.index_select(0, rows)
-        return self.head(h).float()
+        return self.logits(h)

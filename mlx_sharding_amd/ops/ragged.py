@@ -55,6 +55,10 @@ def _ext(op: str):
     return ext
 
 
+def _pad(n: int, to: int) -> int:
+    return (n + to - 1) // to * to
+
+
 # ---------------------------------------------------------------------------
 # Norms around a 32-bit residual
 # ---------------------------------------------------------------------------
@@ -64,23 +68,35 @@ def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
 
 
 def add_norm(x, y, w_post, w_next, eps: float, offset: float,
-             dtype: torch.dtype, mult: float = 1.0):
+             dtype: torch.dtype, mult: float = 1.0, *, where=None,
+             copy: bool = False, pad_to: int = 1):
     """x += mult * rms(y) * (w_post + offset), in place, if y is given (without
     w_post: x += mult * y); returns rms(x) * (w_next + offset) in ``dtype``, or
-    None without w_next.  x is the fp32 residual [N, W]."""
+    None without w_next.  x is the fp32 residual [N, W].
+
+    where [N, top]: row i of y is the sum of the rows y[where[i]].  copy: without
+    w_next, returns x itself in ``dtype``.  What is returned is padded with
+    zeros to a multiple of ``pad_to`` columns."""
+    wide = _pad(x.shape[1], pad_to)
     if x.is_cuda:
-        like = next(t for t in (w_post, w_next, y) if t is not None)
-        h = _ext("add_norm").add_norm(x, y, w_post, w_next, like, eps, offset,
-                                      mult)
-        return h if w_next is not None else None
+        out = w_next is not None or copy
+        h = _ext("add_norm").add_norm(x, y, w_post, w_next,
+                                      dtype == torch.float32, eps, offset,
+                                      mult, where, wide if out else 0)
+        return h if out else None
     if y is not None:
-        y = y.float()
+        y = y.float() if where is None else y[where.long()].float().sum(1)
+        y = y[:, : x.shape[1]]
         if w_post is not None:
             y = _rms(y, eps) * (w_post.float() + offset)
         x += mult * y
     if w_next is None:
-        return None
-    return (_rms(x, eps) * (w_next.float() + offset)).to(dtype)
+        if not copy:
+            return None
+        h = x
+    else:
+        h = _rms(x, eps) * (w_next.float() + offset)
+    return F.pad(h, (0, wide - h.shape[1])).to(dtype, copy=True)
 
 
 # ---------------------------------------------------------------------------
@@ -130,10 +146,6 @@ class Rotary:
 # ---------------------------------------------------------------------------
 # Latent attention
 # ---------------------------------------------------------------------------
-
-def _pad(n: int, to: int) -> int:
-    return (n + to - 1) // to * to
-
 
 @dataclass(frozen=True)
 class LatentShape:
@@ -351,17 +363,23 @@ def _turn(x, table, pos, sign: float = 1.0):
 
 def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
                    sh: GroupedShape, batch: RaggedBatch,
-                   turns: Optional[Turns] = None, head_norm: bool = False):
+                   turns: Optional[Turns] = None, head_norm: bool = False,
+                   own: bool = True):
     """From projection rows y [N, q | k | v | ...]: the queries [N, heads,
     dimp], RMS-normed over the row if wq is given; keys (normed likewise) and
     values go to their pages.  first: values [N, kv_heads * vdim] that are
     blended in by vmix (one element).  turns: rotations by position.
-    head_norm: every query and key divided by its own root mean square."""
+    head_norm: every query and key is divided by its own root mean square
+    (before it is rotated), and wq, wk are weights [dim] that all heads share.
+    own: otherwise y is [N, q | ...] and nothing is written."""
     H, G, D, V = sh.heads, sh.kv_heads, sh.dim, sh.vdim
-    by_head = head_norm or turns is not None
-    if by_head and not (wq is None and wk is None and first is None):
+    by_head = head_norm or turns is not None or not own
+    if by_head and first is not None:
         raise ValueError("rotations and norms per head do not go together with "
-                         "norms over whole rows or blended values")
+                         "blended values")
+    if by_head and not head_norm and not (wq is None and wk is None):
+        raise ValueError("rotations do not go together with norms over whole "
+                         "rows")
     turns = turns or Turns()
     if y.is_cuda:
         ext = _ext("grouped_append")
@@ -369,37 +387,44 @@ def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
         tables = (*(turns.qk or (None, None)), *(turns.v or (None, None)))
         if by_head:
             q, kinv = ext.grouped_turn(
-                y, eps, head_norm, *tables, store.rows, H, G, D, V, sh.dimp,
-                sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages, direct)
+                y, wq, wk, eps, head_norm, *tables, store.rows, H, G, D, V,
+                sh.dimp, sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages,
+                direct, own)
         else:
             q, kinv = ext.grouped_append(
                 y, wq, wk, eps, vmix, first, store.rows, H, G, D, V, sh.dimp,
                 sh.vdp, batch.tok_pos, batch.tok_entry, batch.pages, direct)
-        if direct < batch.n_tokens:
+        if own and direct < batch.n_tokens:
             ext.grouped_fill(y, wk, kinv, vmix, first, store.rows, H, G, D, V,
                              sh.dimp, sh.vdp, batch.fills, head_norm, *tables,
                              batch.tok_pos)
         return q
     N = y.shape[0]
     pos = batch.tok_pos.long()
-    q, k, v = (t.float() for t in y[:, : (H + G) * D + G * V].split(
-        [H * D, G * D, G * V], 1))
-    if wq is not None:
-        q = _rms(q, eps) * wq.float()
-    if wk is not None:
-        k = _rms(k, eps) * wk.float()
+
+    def ready(x, w, heads):
+        if not head_norm and w is not None:
+            x = _rms(x, eps) * w.float()
+        x = x.view(N, heads, D)
+        if head_norm:
+            x = _rms(x, eps)
+            x = x if w is None else x * w.float()
+        if turns.qk is not None:
+            x = _turn(x, turns.qk, pos)
+        return F.pad(x, (0, sh.dimp - D)).to(y.dtype)
+
+    q = ready(y[:, : H * D].float(), wq, H)
+    if not own:
+        return q
+    k, v = (t.float() for t in y[:, H * D: (H + G) * D + G * V].split(
+        [G * D, G * V], 1))
+    k = ready(k, wk, G)
     if first is not None:
         lam = vmix.float()
         v = (1.0 - lam) * v + lam * first.float()
-    q, k, v = q.view(N, H, D), k.view(N, G, D), v.view(N, G, V)
-    if turns.qk is not None:
-        q, k = _turn(q, turns.qk, pos), _turn(k, turns.qk, pos)
-    if head_norm:
-        q, k = _rms(q, eps), _rms(k, eps)
+    v = v.view(N, G, V)
     if turns.v is not None:
         v = _turn(v, turns.v, pos)
-    q = F.pad(q, (0, sh.dimp - D)).to(y.dtype)
-    k = F.pad(k, (0, sh.dimp - D)).to(y.dtype)
     v = F.pad(v, (0, sh.vdp - V)).to(y.dtype)
     page, r = batch.pages[batch.tok_entry.long(), pos // PAGE].long(), pos % PAGE
     sh.keys(store.rows)[page, r // 16, r % 16] = k.view(N, G, -1, 4, 8)
@@ -411,19 +436,20 @@ def grouped_append(y, wq, wk, eps: float, vmix, first, store: LayerStore,
 def grouped_attention(q, sink, store: LayerStore, sh: GroupedShape,
                       scale: float, batch: RaggedBatch, out,
                       window: Optional[int] = None,
-                      turns: Optional[Turns] = None):
+                      turns: Optional[Turns] = None, gate=None):
     """Attention of queries [N, heads, dimp] over their requests' pages, into
     out [N, heads * vdim].  sink [heads] (or None): a score per head that only
     the softmax's denominator sees.  window: how many tokens a token sees, up
     to itself (None: all).  turns: where values are rotated, the output is
-    turned back."""
+    turned back.  gate [N, heads] (may be columns of wider rows): every head's
+    output is multiplied by the sigmoid of its number."""
     back = turns.v if turns is not None else None
     if q.is_cuda:
         ext = _ext("grouped_attention")
         n_req, n, max_len = batch.n_short, batch.short_tokens, batch.max_short
         if not sh.prompts:
             n_req, n, max_len = batch.n_requests, batch.n_tokens, batch.max_len
-        more = (window or 0, *(back or (None, None)), batch.tok_pos)
+        more = (window or 0, *(back or (None, None)), batch.tok_pos, gate)
         if n_req:
             ext.grouped_attn_short(
                 q, sink, store.rows, out, batch.cu, batch.pos0, batch.pages,
@@ -454,6 +480,8 @@ def grouped_attention(q, sink, store: LayerStore, sh: GroupedShape,
         o = o.permute(2, 0, 1, 3).reshape(n, H, sh.vdim)
         if back is not None:
             o = _turn(o, back, at, -1.0)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[t0: t0 + n].float())[..., None]
         out[t0: t0 + n] = o.reshape(n, -1).to(out.dtype)
 
 
@@ -472,6 +500,25 @@ def gelu(x, out=None):
     return out
 
 
+@dataclass(frozen=True)
+class ClampedGLU:
+    """g sigmoid(alpha g) (u + 1) with g = min(gate, limit) and u = up within
+    +-limit."""
+    limit: float
+    alpha: float = 1.702
+
+    def __call__(self, gate, up):
+        """Rows [N, C], which may be columns of wider ones."""
+        if gate.is_cuda:
+            return _ext("clamped_glu").clamped_glu(gate, up, self.limit,
+                                                   self.alpha)
+        return self.of(gate.float(), up.float()).to(gate.dtype)
+
+    def of(self, gate, up):
+        g, u = gate.clamp(max=self.limit), up.clamp(-self.limit, self.limit)
+        return g * torch.sigmoid(self.alpha * g) * (u + 1.0)
+
+
 def cap_logits(z, scale: float, limit: float):
     """limit * tanh(z * scale / limit), fp32."""
     if z.is_cuda:
@@ -486,25 +533,49 @@ def cap_logits(z, scale: float, limit: float):
 @dataclass(frozen=True)
 class DeltaShape:
     """Sizes of a gated-delta layer and the columns of its projection row
-    [q | k | v | gate | decay | beta]."""
+    [q | k | v | gate | decay | beta].
+
+    ``ranks``: one decay per head and key channel, and decay and gate are made
+    by a second projection of (decay, gate) ``ranks`` columns each.  The row is
+    [q | k | v | decay inputs | gate inputs | beta] then, inputs from whole
+    vectors on, and a second one [decay | gate] has what comes of them."""
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     taps: int
+    ranks: Optional[Tuple[int, int]] = None
 
     @property
     def widths(self) -> List[int]:
         k, v = self.kv_heads * self.dim, self.heads * self.vdim
-        return [k, k, v, v, self.heads, self.heads]
+        if self.ranks is None:
+            return [k, k, v, v, self.heads, self.heads]
+        return [k, k, v, *self.ranks, self.heads]
 
     @property
     def columns(self) -> List[int]:
         out, at = [], 0
-        for w in self.widths:
+        for i, w in enumerate(self.widths):
+            if self.ranks is not None and i >= 3:
+                at = _pad(at, 8)
             out.append(at)
             at += w
         return out
+
+    @property
+    def inputs(self) -> Tuple[int, int]:
+        """Columns of the inputs of the second projection, from and to."""
+        at = self.columns
+        return at[3], at[5]
+
+    @property
+    def places(self) -> List[int]:
+        """Columns of q, k, v, gate, decay and beta, each in its row."""
+        at = self.columns
+        if self.ranks is not None:
+            at = [*at[:3], self.heads * self.dim, 0, at[5]]
+        return at
 
     @property
     def channels(self) -> int:
@@ -513,43 +584,51 @@ class DeltaShape:
 
 
 def gated_delta(y, conv_w, A_log, dt_bias, norm_w, store: LayerStore,
-                sh: DeltaShape, eps: float, batch: RaggedBatch):
-    """Projection rows y [N, sum(widths)] -> [N, heads * vdim]; state and
-    convolution inputs of every request move on."""
+                sh: DeltaShape, eps: float, batch: RaggedBatch, z=None,
+                sigmoid_gate: bool = False):
+    """Projection rows y [N, *] -> [N, heads * vdim]; state and convolution
+    inputs of every request move on.  z: the second rows of a shape with
+    ``ranks``.  The output gate is silu, or sigmoid if asked for."""
     if y.is_cuda:
         ext = _ext("gated_delta")
         out = torch.empty(y.shape[0], sh.heads * sh.vdim, dtype=y.dtype,
                           device=y.device)
-        sizes = (sh.kv_heads, sh.heads, sh.dim, sh.vdim, sh.columns, eps)
+        more = (sh.kv_heads, sh.heads, sh.dim, sh.vdim, sh.places, eps, z,
+                sigmoid_gate)
         if batch.n_short:
             ext.delta_short(y, conv_w, A_log, dt_bias, norm_w, store.state,
                             store.conv, out, batch.cu, batch.pos0, batch.slots,
-                            batch.n_short, batch.max_short, *sizes)
+                            batch.n_short, batch.max_short, *more)
         if batch.n_long:
             ext.delta_long(y, conv_w, A_log, dt_bias, norm_w, store.state,
                            store.conv, out, batch.cu, batch.pos0, batch.slots,
                            batch.tok_entry, batch.chunks, batch.chunk_cu,
                            batch.n_short, batch.n_long, batch.short_tokens,
-                           *sizes)
+                           *more)
         return out
     out = y.new_empty(y.shape[0], sh.heads * sh.vdim)
     for t0, n, p0, held in batch.host:
         out[t0: t0 + n] = _gated_delta_request(
-            y[t0: t0 + n], conv_w, A_log, dt_bias, norm_w, store, held.slot,
-            p0 == 0, sh, eps)
+            y[t0: t0 + n], None if z is None else z[t0: t0 + n], conv_w, A_log,
+            dt_bias, norm_w, store, held.slot, p0 == 0, sh, eps, sigmoid_gate)
     return out
 
 
-def _gated_delta_request(y, conv_w, A_log, dt_bias, norm_w, store, slot: int,
-                         fresh: bool, sh: DeltaShape, eps: float):
+def _gated_delta_request(y, z, conv_w, A_log, dt_bias, norm_w, store, slot: int,
+                         fresh: bool, sh: DeltaShape, eps: float,
+                         sigmoid_gate: bool):
     n, hist = y.shape[0], sh.taps - 1
     H, KH, D, V = sh.heads, sh.kv_heads, sh.dim, sh.vdim
     old = torch.zeros_like(store.conv[slot]) if fresh else store.conv[slot]
     x = torch.cat([old, y[:, : sh.channels].T], 1)       # [C, hist + n]
     store.conv[slot] = x[:, n:]
-    z = F.silu((x.float().unfold(1, sh.taps, 1) * conv_w.float()[:, None, :]).sum(-1)).T
-    q, k, v = z.split(sh.widths[:3], 1)
-    gate, a, b = y[:, sh.channels:].float().split(sh.widths[3:], 1)
+    c = F.silu((x.float().unfold(1, sh.taps, 1) * conv_w.float()[:, None, :]).sum(-1)).T
+    q, k, v = c.split(sh.widths[:3], 1)
+    gc, ac, bc = sh.places[3:]
+    rows, steps = (y, 1) if z is None else (z, D)     # decays per head
+    gate, a = (rows[:, i: i + w].float()
+               for i, w in ((gc, H * V), (ac, H * steps)))
+    beta = torch.sigmoid(y[:, bc: bc + H].float())
 
     def unit(t):
         t = t.reshape(n, KH, D)
@@ -557,15 +636,16 @@ def _gated_delta_request(y, conv_w, A_log, dt_bias, norm_w, store, slot: int,
         return t.repeat_interleave(H // KH, 1)
 
     q, k, v = unit(q) * D ** -0.5, unit(k), v.reshape(n, H, V)
-    g = torch.exp(-torch.exp(A_log.float()) * F.softplus(a + dt_bias.float()))
-    beta = torch.sigmoid(b)
+    step = F.softplus(a + dt_bias.float(), threshold=80).view(n, H, steps)
+    g = torch.exp(-torch.exp(A_log.float())[:, None] * step)[..., None]
     S = torch.zeros_like(store.state[slot]) if fresh else store.state[slot].clone()
     o = torch.empty(n, H, V)
     for t in range(n):
-        S *= g[t][:, None, None]
+        S *= g[t]
         u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
         S += k[t][:, :, None] * u[:, None, :]
         o[t] = torch.einsum("hdv,hd->hv", S, q[t])
     store.state[slot] = S
-    o = _rms(o, eps) * norm_w.float() * F.silu(gate).reshape(n, H, V)
+    act = torch.sigmoid if sigmoid_gate else F.silu
+    o = _rms(o, eps) * norm_w.float() * act(gate).reshape(n, H, V)
     return o.reshape(n, H * V).to(y.dtype)

@@ -157,6 +157,7 @@ def load_model(model_path: str | Path,
     if config.quantization is not None and not cls.supports_quantization:
         raise ValueError(f"{config.model_type} has no quantized weights")
     quant_for = make_quant_predicate(config, weights)
+    cls.complete_config(config, weights)
     model = cls(config, shard, quant_for=quant_for)
     if dtype is not None:
         model.to(dtype)
