@@ -6,13 +6,25 @@
 #include "ragged_grouped.h"
 #include "ragged_prefill.h"
 
+struct AddNormArgs {
+  float* x;
+  const void *y, *w_post, *w_next;
+  void* h;
+  const int* where;
+  long rows, ystride;
+  int W, Wh, top;
+  float eps, off, mult;
+  bool one_next;
+};
+
 extern "C" {
+void launch_clamped_glu(const void*, const void*, void*, long, int, long, long,
+                        float, float, bool, bool, hipStream_t);
 void launch_glu_strided(const void*, const void*, void*, long, int, long, long,
                         bool, hipStream_t);
 void launch_glu_any(const void*, const void*, void*, long, int, long, long,
                     bool, bool, hipStream_t);
-void launch_add_norm(void*, const void*, long, const void*, const void*, void*,
-                     long, int, float, float, float, bool, bool, hipStream_t);
+void launch_add_norm(const AddNormArgs*, bool, hipStream_t);
 void launch_latent_append(const void*, long, const void*, float, void*, void*,
                           long, int, int, int, int, int, int, int,
                           const float*, const float*, const int*, const int*,
@@ -31,7 +43,7 @@ void launch_grouped_append(const GroupedRowArgs*, void*, float*, const int*,
                            const int*, const int*, int, int, long, bool,
                            hipStream_t);
 void launch_grouped_turn(const GroupedRowArgs*, void*, float*, const int*,
-                         const int*, int, int, long, bool, hipStream_t);
+                         const int*, int, int, long, bool, bool, hipStream_t);
 void launch_grouped_fill(const GroupedRowArgs*, const float*, const int*, int,
                          bool, hipStream_t);
 void launch_grouped_attn_short_bf16(const GroupedAttnArgs*, int, int,
@@ -51,14 +63,15 @@ void launch_cap_logits(const void*, float*, long, float, float, bool,
 struct DeltaDims {
   int KH, H, D, V, taps;
   int qc, kc, vc, gc, ac, bc;
-  long ystride;
+  long ystride, zstride;
+  bool channels, sigmoid;
 };
 
 struct DeltaLongArgs {
-  const void *y, *conv_w, *A_log, *dt_bias, *norm_w;
+  const void *y, *z, *conv_w, *A_log, *dt_bias, *norm_w;
   float* state;
   void *conv_state, *out;
-  float *qn, *kn, *lg, *bt, *tm, *am, *ge, *o;
+  float *qn, *kn, *lg, *bt, *tm, *am, *ge, *o, *qg, *kg, *kl;
   void* vn;
   const int *cu, *pos0, *slots, *tok_entry, *chunks, *chunk_cu;
   int n_short, n_long, tok_base, n_chunks, Dp, Vp;
@@ -68,7 +81,7 @@ struct DeltaLongArgs {
 
 extern "C" {
 void launch_delta_short(const void*, const void*, const void*, const void*,
-                        const void*, float*, void*, void*, const int*,
+                        const void*, const void*, float*, void*, void*, const int*,
                         const int*, const int*, const DeltaDims*, int, int,
                         float, bool, hipStream_t);
 void launch_delta_long(const DeltaLongArgs*, const DeltaDims*, bool,
@@ -101,41 +114,72 @@ Tensor glu(Tensor gate, Tensor up, bool gelu) {
   return y;
 }
 
+// gate and up [rows, C], possibly slices of wider rows
+Tensor clamped_glu(Tensor gate, Tensor up, double limit, double alpha) {
+  const bool f32 = is_f32(gate, "gate");
+  check_like(up, gate, "up");
+  const long gs = rows2(gate, "gate"), us = rows2(up, "up");
+  TORCH_CHECK(gate.sizes() == up.sizes());
+  const long rows = gate.size(0), C = gate.size(1);
+  auto out = torch::empty({rows, C}, gate.options());
+  if (rows == 0 || C == 0) return out;
+  const bool vec = C % 8 == 0 && whole8(gate, gs) && whole8(up, us);
+  launch_clamped_glu(gate.data_ptr(), up.data_ptr(), out.data_ptr(), rows,
+                     (int)C, gs, us, (float)limit, (float)alpha, vec, f32,
+                     stream());
+  return out;
+}
+
 // x [N, W] fp32 (updated in place when y is given, normed first when w_post
-// is); returns h or an empty tensor when there is no following norm.
+// is; where [N, top]: sums of rows of y); returns h, `wide` columns of the next
+// norm's rows or of x itself, or an empty tensor for wide == 0.
 Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
-                c10::optional<Tensor> w_next, Tensor like, double eps,
-                double off, double mult) {
+                c10::optional<Tensor> w_next, bool f32, double eps,
+                double off, double mult, c10::optional<Tensor> where,
+                int64_t wide) {
   check_f32(x, "x");
   TORCH_CHECK(x.dim() == 2, "x must be [rows, width]");
-  const bool f32 = is_f32(like, "like");
-  const long N = x.size(0), W = x.size(1);
-  long ys = W;
+  const auto type = x.options().dtype(f32 ? torch::kFloat32 : torch::kBFloat16);
+  auto h = torch::empty({wide ? x.size(0) : 0, wide}, type);
+  AddNormArgs a = {};
+  a.rows = x.size(0);
+  a.W = (int)x.size(1);
+  a.Wh = (int)wide;
+  a.ystride = a.W;
+  TORCH_CHECK(wide == 0 || wide >= a.W);
   if (y) {
-    check_like(*y, like, "y");
-    TORCH_CHECK(y->sizes() == x.sizes(), "y must match x");
-    ys = rows2(*y, "y");
+    check_like(*y, h, "y");
+    a.ystride = rows2(*y, "y");
+    if (where) {
+      TORCH_CHECK(where->dim() == 2 && where->size(0) == a.rows &&
+                  y->size(1) >= a.W && y->size(0) == where->numel(),
+                  "rows of y do not fit x");
+      a.where = ints(*where, where->numel(), "where");
+      a.top = (int)where->size(1);
+    } else {
+      TORCH_CHECK(y->sizes() == x.sizes(), "y must match x");
+    }
+    a.y = y->data_ptr();
     if (w_post) {
-      check_like(*w_post, like, "w_post");
-      TORCH_CHECK(w_post->numel() == W && w_post->is_contiguous());
+      check_like(*w_post, h, "w_post");
+      TORCH_CHECK(w_post->numel() == a.W && w_post->is_contiguous());
+      a.w_post = w_post->data_ptr();
     }
   }
-  Tensor h;
   if (w_next) {
-    check_like(*w_next, like, "w_next");
-    TORCH_CHECK((w_next->numel() == W || w_next->numel() == 1) &&
+    check_like(*w_next, h, "w_next");
+    TORCH_CHECK((w_next->numel() == a.W || w_next->numel() == 1) &&
                 w_next->is_contiguous());
-    h = torch::empty({N, W}, like.options());
-  } else {
-    h = torch::empty({0}, like.options());
+    a.w_next = w_next->data_ptr();
+    a.one_next = w_next->numel() == 1;
   }
-  if (N == 0) return h;
-  launch_add_norm(x.data_ptr(), y ? y->data_ptr() : nullptr, ys,
-                  y && w_post ? w_post->data_ptr() : nullptr,
-                  w_next ? w_next->data_ptr() : nullptr,
-                  w_next ? h.data_ptr() : nullptr, N, (int)W, (float)eps,
-                  (float)off, (float)mult, w_next && w_next->numel() == 1, f32,
-                  stream());
+  if (a.rows == 0) return h;
+  a.x = x.data_ptr<float>();
+  a.h = wide ? h.data_ptr() : nullptr;
+  a.eps = (float)eps;
+  a.off = (float)off;
+  a.mult = (float)mult;
+  launch_add_norm(&a, f32, stream());
   return h;
 }
 
@@ -294,9 +338,12 @@ Tensor latent_attn_long(Tensor q, Tensor kx, Tensor lat, Tensor vt,
   return out;
 }
 
-DeltaDims delta_dims(const Tensor& y, const Tensor& conv_w, int64_t KH,
-                     int64_t H, int64_t D, int64_t V,
-                     const std::vector<int64_t>& cols) {
+// y [N, *] has q, k, v and beta; gate and decay are columns of y as well (one
+// decay per head), or of z (one per head and key channel)
+DeltaDims delta_dims(const Tensor& y, const c10::optional<Tensor>& z,
+                     const Tensor& conv_w, int64_t KH, int64_t H, int64_t D,
+                     int64_t V, const std::vector<int64_t>& cols,
+                     bool sigmoid) {
   DeltaDims d;
   TORCH_CHECK(KH > 0 && H % KH == 0 && cols.size() == 6);
   TORCH_CHECK(conv_w.dim() == 2 && conv_w.is_contiguous() &&
@@ -309,16 +356,25 @@ DeltaDims delta_dims(const Tensor& y, const Tensor& conv_w, int64_t KH,
   TORCH_CHECK(d.taps >= 1 && d.taps <= 8, "convolutions have 1 to 8 taps");
   TORCH_CHECK(D <= 512 && V <= 512 && delta_short_rows((int)D, (int)V, 512) > 0,
               "state of a head is too large: ", D, " x ", V);
-  const int64_t w[6] = {KH * D, KH * D, H * V, H * V, H, H};
-  for (int i = 0; i < 6; ++i)
-    TORCH_CHECK(cols[i] >= 0 && cols[i] + w[i] <= y.size(1));
+  d.channels = z.has_value();
+  d.sigmoid = sigmoid;
+  const int64_t w[6] = {KH * D, KH * D, H * V, H * V, d.channels ? H * D : H, H};
+  for (int i = 0; i < 6; ++i) {
+    const Tensor& rows = d.channels && (i == 3 || i == 4) ? *z : y;
+    TORCH_CHECK(cols[i] >= 0 && cols[i] + w[i] <= rows.size(1));
+  }
   d.qc = (int)cols[0];
   d.kc = (int)cols[1];
   d.vc = (int)cols[2];
   d.gc = (int)cols[3];
   d.ac = (int)cols[4];
   d.bc = (int)cols[5];
-  d.ystride = rows2(y, "y");
+  d.ystride = d.zstride = rows2(y, "y");
+  if (z) {
+    check_like(*z, y, "z");
+    TORCH_CHECK(z->size(0) == y.size(0));
+    d.zstride = rows2(*z, "z");
+  }
   return d;
 }
 
@@ -328,7 +384,8 @@ void check_delta(const Tensor& y, const Tensor& conv_w, const Tensor& A_log,
                  const DeltaDims& d) {
   for (const auto* t : {&conv_w, &A_log, &dt, &norm_w, &conv_state, &out})
     check_like(*t, y, "delta operand");
-  TORCH_CHECK(A_log.numel() == d.H && dt.numel() == d.H &&
+  TORCH_CHECK(A_log.numel() == d.H &&
+              dt.numel() == (d.channels ? (long)d.H * d.D : d.H) &&
               norm_w.numel() == d.V && A_log.is_contiguous() &&
               dt.is_contiguous() && norm_w.is_contiguous());
   check_f32(state, "state");
@@ -347,14 +404,16 @@ void delta_short(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
                  Tensor norm_w, Tensor state, Tensor conv_state, Tensor out,
                  Tensor cu, Tensor pos0, Tensor slots, int64_t n_req,
                  int64_t max_len, int64_t KH, int64_t H, int64_t D, int64_t V,
-                 std::vector<int64_t> cols, double eps) {
+                 std::vector<int64_t> cols, double eps, c10::optional<Tensor> z,
+                 bool sigmoid) {
   const bool f32 = is_f32(y, "y");
-  auto d = delta_dims(y, conv_w, KH, H, D, V, cols);
+  auto d = delta_dims(y, z, conv_w, KH, H, D, V, cols, sigmoid);
   check_delta(y, conv_w, A_log, dt, norm_w, state, conv_state, out, d);
   TORCH_CHECK(max_len >= 1 && max_len <= 16, "short portions have 1 to 16 "
               "tokens");
   if (n_req == 0) return;
-  launch_delta_short(y.data_ptr(), conv_w.data_ptr(), A_log.data_ptr(),
+  launch_delta_short(y.data_ptr(), z ? z->data_ptr() : y.data_ptr(),
+                     conv_w.data_ptr(), A_log.data_ptr(),
                      dt.data_ptr(), norm_w.data_ptr(), state.data_ptr<float>(),
                      conv_state.data_ptr(), out.data_ptr(),
                      ints(cu, n_req + 1, "cu"), ints(pos0, n_req, "pos0"),
@@ -368,16 +427,17 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
                 Tensor cu, Tensor pos0, Tensor slots, Tensor tok_entry,
                 Tensor chunks, Tensor chunk_cu, int64_t n_short,
                 int64_t n_long, int64_t tok_base, int64_t KH, int64_t H,
-                int64_t D, int64_t V, std::vector<int64_t> cols, double eps) {
+                int64_t D, int64_t V, std::vector<int64_t> cols, double eps,
+                c10::optional<Tensor> z, bool sigmoid) {
   const bool f32 = is_f32(y, "y");
-  auto d = delta_dims(y, conv_w, KH, H, D, V, cols);
+  auto d = delta_dims(y, z, conv_w, KH, H, D, V, cols, sigmoid);
   check_delta(y, conv_w, A_log, dt, norm_w, state, conv_state, out, d);
   const long n = y.size(0) - tok_base;
   if (n <= 0 || n_long == 0) return;
   TORCH_CHECK(chunks.dim() == 2 && chunks.size(1) == 2);
   TORCH_CHECK(n * H < (1L << 31), "too many tokens in one step");
-  TORCH_CHECK(((uintptr_t)y.data_ptr()) % 8 == 0 &&
-              ((uintptr_t)norm_w.data_ptr()) % 8 == 0, "unaligned operand");
+  for (const Tensor* t : {&y, &norm_w, z ? &*z : &y})
+    TORCH_CHECK(((uintptr_t)t->data_ptr()) % 8 == 0, "unaligned operand");
   const long nc = chunks.size(0);
   // depths 16 * 2^k take the walk with a fixed depth
   long Dp = 16;
@@ -387,13 +447,27 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
   auto fo = y.options().dtype(torch::kFloat32);
   auto qn = torch::empty({n, KH, Dp}, fo), kn = torch::empty({n, KH, Dp}, fo);
   auto vn = torch::empty({n, H, Vp}, y.options());
-  auto lg = torch::empty({n, H}, fo), bt = torch::empty({n, H}, fo);
+  auto bt = torch::empty({n, H}, fo);
   auto tm = torch::empty({nc, H, 64, 64}, fo);
   auto am = torch::empty({nc, H, 64, 64}, fo);
-  auto ge = torch::empty({nc, H, 2, 64}, fo);
   auto o = torch::empty({n, H, Vp}, fo);
-  DeltaLongArgs a;
+  DeltaLongArgs a = {};
+  Tensor lg, ge, qg, kg, kl;
+  if (d.channels) {
+    qg = torch::empty({n, H, Dp}, fo);
+    kg = torch::empty({n, H, Dp}, fo);
+    kl = torch::empty({n, H, Dp}, fo);
+    ge = torch::empty({nc, H, Dp}, fo);
+    a.qg = qg.data_ptr<float>();
+    a.kg = kg.data_ptr<float>();
+    a.kl = kl.data_ptr<float>();
+  } else {
+    lg = torch::empty({n, H}, fo);
+    ge = torch::empty({nc, H, 2, 64}, fo);
+    a.lg = lg.data_ptr<float>();
+  }
   a.y = y.data_ptr();
+  a.z = z ? z->data_ptr() : y.data_ptr();
   a.conv_w = conv_w.data_ptr();
   a.A_log = A_log.data_ptr();
   a.dt_bias = dt.data_ptr();
@@ -403,7 +477,6 @@ void delta_long(Tensor y, Tensor conv_w, Tensor A_log, Tensor dt,
   a.out = out.data_ptr();
   a.qn = qn.data_ptr<float>();
   a.kn = kn.data_ptr<float>();
-  a.lg = lg.data_ptr<float>();
   a.bt = bt.data_ptr<float>();
   a.tm = tm.data_ptr<float>();
   a.am = am.data_ptr<float>();
@@ -444,13 +517,14 @@ GroupedRowArgs grouped_rows(const Tensor& y, const c10::optional<Tensor>& wq,
                             const c10::optional<Tensor>& vmix,
                             const c10::optional<Tensor>& first,
                             const Tensor& pool, int64_t H, int64_t G, int64_t D,
-                            int64_t V, int64_t dimp, int64_t vdp) {
+                            int64_t V, int64_t dimp, int64_t vdp,
+                            bool own = true, bool by_head = false) {
   TORCH_CHECK(G > 0 && H > 0 && H % G == 0 && D > 0 && V > 0);
   TORCH_CHECK(dimp % 32 == 0 && D <= dimp && vdp % 16 == 0 && V <= vdp &&
               dimp <= 512 && vdp <= 512);
   GroupedRowArgs a = {};
   a.ystride = rows2(y, "y");
-  TORCH_CHECK(y.size(1) >= (H + G) * D + G * V);
+  TORCH_CHECK(y.size(1) >= (own ? (H + G) * D + G * V : H * D));
   check_pool(pool, y, G * (dimp + vdp));
   a.vec = D % 8 == 0 && V % 8 == 0 && whole8(y, a.ystride);
   auto weight = [&](const c10::optional<Tensor>& w, long n, const char* name) {
@@ -460,8 +534,8 @@ GroupedRowArgs grouped_rows(const Tensor& y, const c10::optional<Tensor>& wq,
     a.vec = a.vec && whole8(*w, 8);
     return (const void*)w->data_ptr();
   };
-  a.wq = weight(wq, H * D, "wq");
-  a.wk = weight(wk, G * D, "wk");
+  a.wq = weight(wq, by_head ? D : H * D, "wq");
+  a.wk = weight(wk, by_head ? D : G * D, "wk");
   if (first) {
     TORCH_CHECK(vmix && vmix->numel() == 1);
     check_like(*vmix, y, "vmix");
@@ -533,16 +607,20 @@ void grouped_turns(GroupedRowArgs& a, bool head_norm, const Table& qk_cos,
     if (*t) aligned16(**t, "rotation table");
 }
 
-// y [N, q | k | v | ...] -> queries [N, H, dimp] and inverse rms of keys [N, G]
+// y [N, q | k | v | ...] -> queries [N, H, dimp] and inverse rms of keys [N, G];
+// wq, wk [D] weights of the norms per head; not own: y [N, q | ...], the queries
+// alone
 std::tuple<Tensor, Tensor> grouped_turn(
-    Tensor y, double eps, bool head_norm, Table qk_cos, Table qk_sin,
-    Table v_cos, Table v_sin, Tensor pool, int64_t H, int64_t G, int64_t D,
-    int64_t V, int64_t dimp, int64_t vdp, Tensor tok_pos, Tensor tok_entry,
-    Tensor pages, int64_t direct) {
+    Tensor y, c10::optional<Tensor> wq, c10::optional<Tensor> wk, double eps,
+    bool head_norm, Table qk_cos, Table qk_sin, Table v_cos, Table v_sin,
+    Tensor pool, int64_t H, int64_t G, int64_t D, int64_t V, int64_t dimp,
+    int64_t vdp, Tensor tok_pos, Tensor tok_entry, Tensor pages, int64_t direct,
+    bool own) {
   const bool f32 = is_f32(y, "y");
   const c10::optional<Tensor> none;
-  auto a = grouped_rows(y, none, none, eps, none, none, pool, H, G, D, V, dimp,
-                        vdp);
+  TORCH_CHECK(head_norm || !(wq || wk), "weights without norms per head");
+  auto a = grouped_rows(y, wq, wk, eps, none, none, pool, H, G, D, V, dimp, vdp,
+                        own, true);
   const long N = y.size(0);
   TORCH_CHECK(pages.dim() == 2 && direct >= 0 && direct <= N);
   grouped_turns(a, head_norm, qk_cos, qk_sin, v_cos, v_sin, tok_pos, N);
@@ -552,7 +630,7 @@ std::tuple<Tensor, Tensor> grouped_turn(
     launch_grouped_turn(&a, q.data_ptr(), kinv.data_ptr<float>(),
                         ints(tok_entry, N, "tok_entry"),
                         ints(pages, 0, "pages"), (int)pages.size(1),
-                        (int)direct, N, f32, stream());
+                        (int)direct, N, own, f32, stream());
   return {q, kinv};
 }
 
@@ -564,14 +642,15 @@ void grouped_fill(Tensor y, c10::optional<Tensor> wk, Tensor kinv,
                   Table qk_cos, Table qk_sin, Table v_cos, Table v_sin,
                   Tensor tok_pos) {
   const bool f32 = is_f32(y, "y");
+  const bool turns = head_norm || qk_cos || v_cos;
   auto a = grouped_rows(y, c10::nullopt, wk, 0.0, vmix, first, pool, H, G, D, V,
-                        dimp, vdp);
+                        dimp, vdp, true, turns);
   check_f32(kinv, "kinv");
   grouped_turns(a, head_norm, qk_cos, qk_sin, v_cos, v_sin, tok_pos, y.size(0));
-  const bool turns = head_norm || qk_cos || v_cos;
   TORCH_CHECK(kinv.numel() == y.size(0) * (turns ? G : 1) && G <= 65535);
-  TORCH_CHECK(!(turns && (wk || first)), "norms per head or rotations beside "
-              "norms of whole rows or blended values");
+  TORCH_CHECK(!(turns && first) && !(turns && !head_norm && wk),
+              "norms per head or rotations beside norms of whole rows or "
+              "blended values");
   TORCH_CHECK(fills.dim() == 2 && fills.size(1) == 4);
   if (fills.size(0))
     launch_grouped_fill(&a, kinv.data_ptr<float>(), ints(fills, 0, "fills"),
@@ -585,7 +664,7 @@ GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
                              const Tensor& pages, int64_t G, int64_t V,
                              int64_t vdp, double scale, int64_t window,
                              const Table& v_cos, const Table& v_sin,
-                             const Table& tok_pos) {
+                             const Table& tok_pos, const Table& gate) {
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous());
   const long H = q.size(1), dimp = q.size(2);
   TORCH_CHECK(G > 0 && H % G == 0 && V > 0 && V <= vdp);
@@ -622,6 +701,12 @@ GroupedAttnArgs grouped_attn(const Tensor& q, const c10::optional<Tensor>& sink,
   TORCH_CHECK(!v_cos || 2 * pairs == V, "values are turned back whole");
   TORCH_CHECK(!v_cos || tok_pos, "turning back needs positions");
   if (tok_pos) a.tok_pos = ints(*tok_pos, q.size(0), "tok_pos");
+  if (gate) {
+    check_like(*gate, q, "gate");
+    a.gstride = rows2(*gate, "gate");
+    TORCH_CHECK(gate->size(0) == q.size(0) && gate->size(1) == H);
+    a.gate = gate->data_ptr();
+  }
   return a;
 }
 
@@ -631,10 +716,10 @@ void grouped_attn_short(Tensor q, c10::optional<Tensor> sink, Tensor pool,
                         int64_t n_req, int64_t n_tok, int64_t max_len,
                         int64_t max_keys, int64_t G, int64_t V, int64_t vdp,
                         double scale, int64_t window, Table v_cos, Table v_sin,
-                        Table tok_pos) {
+                        Table tok_pos, Table gate) {
   const bool f32 = is_f32(q, "q");
   auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale, window,
-                        v_cos, v_sin, tok_pos);
+                        v_cos, v_sin, tok_pos, gate);
   // a block starts at the step that holds its first window's first key
   if (window) max_keys = std::min(max_keys, window + max_len + GA_STEP);
   TORCH_CHECK(pages.size(0) >= n_req && n_tok <= q.size(0));
@@ -670,10 +755,10 @@ void grouped_attn_long(Tensor q, c10::optional<Tensor> sink, Tensor pool,
                        Tensor out, Tensor tiles, Tensor cu, Tensor pos0,
                        Tensor pages, int64_t G, int64_t V, int64_t vdp,
                        double scale, int64_t window, Table v_cos, Table v_sin,
-                       Table tok_pos) {
+                       Table tok_pos, Table gate) {
   const bool f32 = is_f32(q, "q");
   auto a = grouped_attn(q, sink, pool, out, pages, G, V, vdp, scale, window,
-                        v_cos, v_sin, tok_pos);
+                        v_cos, v_sin, tok_pos, gate);
   TORCH_CHECK(a.dimp <= 256 && vdp <= 256, "head sizes above 256");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2 &&
               tiles.size(0) <= 65535);
@@ -715,9 +800,8 @@ Tensor cap_logits(Tensor z, double scale, double limit) {
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("glu", &glu);
-  m.def("add_norm", &add_norm, py::arg("x"), py::arg("y"), py::arg("w_post"),
-        py::arg("w_next"), py::arg("like"), py::arg("eps"), py::arg("offset"),
-        py::arg("mult") = 1.0);
+  m.def("clamped_glu", &clamped_glu);
+  m.def("add_norm", &add_norm);
   m.def("latent_append", &latent_append);
   m.def("latent_gather", &latent_gather);
   m.def("latent_attn_short", &latent_attn_short);
@@ -733,13 +817,15 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("max_len"), py::arg("max_keys"), py::arg("kv_heads"),
         py::arg("vdim"), py::arg("vdp"), py::arg("scale"),
         py::arg("window") = 0, py::arg("v_cos") = py::none(),
-        py::arg("v_sin") = py::none(), py::arg("tok_pos") = py::none());
+        py::arg("v_sin") = py::none(), py::arg("tok_pos") = py::none(),
+        py::arg("gate") = py::none());
   m.def("grouped_attn_long", &grouped_attn_long, py::arg("q"),
         py::arg("sink"), py::arg("pool"), py::arg("out"), py::arg("tiles"),
         py::arg("cu"), py::arg("pos0"), py::arg("pages"), py::arg("kv_heads"),
         py::arg("vdim"), py::arg("vdp"), py::arg("scale"),
         py::arg("window") = 0, py::arg("v_cos") = py::none(),
-        py::arg("v_sin") = py::none(), py::arg("tok_pos") = py::none());
+        py::arg("v_sin") = py::none(), py::arg("tok_pos") = py::none(),
+        py::arg("gate") = py::none());
   m.def("gelu", &gelu);
   m.def("cap_logits", &cap_logits);
   bind_recurrent(m);

@@ -16,20 +16,20 @@ Tensor int_rows(const Tensor& like, std::vector<int64_t> sizes) {
   return torch::empty(sizes, like.options().dtype(torch::kInt32));
 }
 
-// h [N, K], w [total / 16, K / 32, 64, 8], correction [total]
+// h [N, K], w [total / 16, K / 32, 64, 8], correction [total] or none
 // -> chosen [N, top], weights [N, top], ranks [N, top], histograms
-std::tuple<Tensor, Tensor, Tensor, Tensor> expert_route(Tensor h, Tensor w,
-                                                        Tensor correction,
-                                                        int64_t experts,
-                                                        int64_t top) {
+std::tuple<Tensor, Tensor, Tensor, Tensor> expert_route(
+    Tensor h, Tensor w, c10::optional<Tensor> correction, int64_t total,
+    int64_t experts, int64_t top, bool sigmoid, bool normalize) {
   const bool f32 = is_f32(h, "h");
   check_like(w, h, "router");
-  check_like(correction, h, "correction");
   RouteArgs a = {};
+  a.sigmoid = sigmoid;
+  a.normalize = normalize;
   a.hstride = rows2(h, "h");
   a.n = h.size(0);
   a.K = (int)h.size(1);
-  a.total = (int)correction.numel();
+  a.total = (int)total;
   TORCH_CHECK(a.K % EX_STEP == 0 && a.hstride % 8 == 0);
   TORCH_CHECK(w.dim() == 4 && w.is_contiguous() &&
               w.size(0) == (a.total + 15) / 16 && w.size(1) == a.K / 32 &&
@@ -40,14 +40,17 @@ std::tuple<Tensor, Tensor, Tensor, Tensor> expert_route(Tensor h, Tensor w,
   a.top = (int)top;
   TORCH_CHECK(a.total <= EX_MAXTOTAL && experts >= 1 && experts <= a.total &&
               top >= 1 && top <= a.total);
-  TORCH_CHECK(correction.is_contiguous());
+  if (correction) {
+    check_like(*correction, h, "correction");
+    TORCH_CHECK(correction->is_contiguous() && correction->numel() == total);
+    a.correction = correction->data_ptr();
+  }
   const long blocks = (a.n + EX_TOK - 1) / EX_TOK;
   auto idx = int_rows(h, {a.n, top}), rank = int_rows(h, {a.n, top});
   auto hist = int_rows(h, {blocks, experts});
   auto weight = torch::empty({a.n, top}, h.options().dtype(torch::kFloat32));
   a.h = h.data_ptr();
   a.w = w.data_ptr();
-  a.correction = correction.data_ptr();
   a.idx = idx.data_ptr<int>();
   a.weight = weight.data_ptr<float>();
   a.rank = rank.data_ptr<int>();
@@ -56,10 +59,11 @@ std::tuple<Tensor, Tensor, Tensor, Tensor> expert_route(Tensor h, Tensor w,
   return {idx, weight, rank, hist};
 }
 
-// -> rows of the pairs [N, top], tokens of the rows [N * top], tiles [*, 3]
-std::tuple<Tensor, Tensor, Tensor> expert_plan(Tensor idx, Tensor rank,
-                                               Tensor hist, int64_t experts,
-                                               int64_t tile) {
+// -> rows of the pairs [N, top], tokens of the rows [N * top], tiles [*, 3], and
+// the rows' weights [N * top] if weight is given
+std::tuple<Tensor, Tensor, Tensor, c10::optional<Tensor>> expert_plan(
+    Tensor idx, Tensor rank, Tensor hist, c10::optional<Tensor> weight,
+    int64_t experts, int64_t tile) {
   PlanArgs a = {};
   TORCH_CHECK(idx.dim() == 2 && hist.dim() == 2);
   a.n = idx.size(0);
@@ -83,14 +87,23 @@ std::tuple<Tensor, Tensor, Tensor> expert_plan(Tensor idx, Tensor rank,
   a.where = where.data_ptr<int>();
   a.tokens = tokens.data_ptr<int>();
   a.tiles = tiles.data_ptr<int>();
+  c10::optional<Tensor> scale;
+  if (weight) {
+    check_f32(*weight, "weight");
+    TORCH_CHECK(weight->numel() == pairs);
+    scale = torch::empty({pairs}, weight->options());
+    a.weight = weight->data_ptr<float>();
+    a.scale = scale->data_ptr<float>();
+  }
   if (a.n) launch_expert_plan(&a, stream());
-  return {where, tokens, tiles};
+  return {where, tokens, tiles, scale};
 }
 
-// x rows (of `tokens`, or the pairs' own) times w [experts, O, K] -> [pairs, O],
-// rows padded to whole vectors
+// x rows (of `tokens`, or the pairs' own) times w [experts, O, K] and the rows'
+// scale -> [pairs, O], half of it for gated units; rows padded to whole vectors
 Tensor expert_gemm(Tensor x, c10::optional<Tensor> tokens, Tensor tiles,
-                   Tensor w, int64_t tile, int64_t pairs, bool act) {
+                   Tensor w, c10::optional<Tensor> scale, int64_t tile,
+                   int64_t pairs, int64_t act, double limit, double alpha) {
   const bool f32 = is_f32(x, "x");
   check_like(w, x, "w");
   ExpertGemmArgs a = {};
@@ -107,13 +120,27 @@ Tensor expert_gemm(Tensor x, c10::optional<Tensor> tokens, Tensor tiles,
   aligned16(w, "w");
   if (tokens) a.tokens = ints(*tokens, pairs, "tokens");
   else TORCH_CHECK(x.size(0) >= pairs);
-  a.ostride = (a.O + 7) / 8 * 8;
+  TORCH_CHECK(act == EX_NONE || act == EX_RELU2 || act == EX_CLAMPED_GLU);
+  a.act = (int)act;
+  a.limit = (float)limit;
+  a.alpha = (float)alpha;
+  int outs = a.O;
+  if (act == EX_CLAMPED_GLU) {
+    // gate and up projection are padded to whole 16-row tiles each
+    TORCH_CHECK(a.O % 32 == 0, "gated units come in tiles of 16");
+    outs /= 2;
+  }
+  if (scale) {
+    check_f32(*scale, "scale");
+    TORCH_CHECK(scale->numel() >= pairs);
+    a.scale = scale->data_ptr<float>();
+  }
+  a.ostride = (outs + 7) / 8 * 8;
   auto out = torch::empty({pairs, a.ostride}, x.options());
   a.x = x.data_ptr();
   a.w = w.data_ptr();
   a.out = out.data_ptr();
   a.tiles = ints(tiles, 0, "tiles");
-  a.act = act;
   if (a.n_tiles) launch_expert_gemm(&a, (int)tile, f32, stream());
   return out;
 }

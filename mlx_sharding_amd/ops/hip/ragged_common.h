@@ -170,3 +170,45 @@ __device__ __forceinline__ float sigmoid_f(float x) {
 __device__ __forceinline__ float softplus_f(float x) {
   return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x)));
 }
+
+// sigmoid for bf16 results from the hardware's power of two, off by about 1e-7
+template <typename T>
+__device__ __forceinline__ float sigmoid_of(float x);
+template <>
+__device__ __forceinline__ float sigmoid_of<float>(float x) {
+  return sigmoid_f(x);
+}
+template <>
+__device__ __forceinline__ float sigmoid_of<__bf16>(float x) {
+  return __builtin_amdgcn_rcpf(
+      1.0f + __builtin_amdgcn_exp2f(-1.44269504088896340736f * x));
+}
+
+// ln(1 + e^x).  For bf16 operands: the logarithm of 1 + u from the instruction
+// where u is not small, else its series; both to about 1e-6 of the result.
+template <typename T>
+__device__ __forceinline__ float softplus_of(float x);
+template <>
+__device__ __forceinline__ float softplus_of<float>(float x) {
+  return softplus_f(x);
+}
+template <>
+__device__ __forceinline__ float softplus_of<__bf16>(float d) {
+  const float u = __builtin_amdgcn_exp2f(-1.44269504088896340736f * fabsf(d));
+  const float large = 0.69314718055994530942f * __builtin_amdgcn_logf(1.0f + u);
+  // u - u^2/2 + ... + u^5/5, off by u^6/6
+  float small = fmaf(u, 0.2f, -0.25f);
+  small = fmaf(u, small, 0.33333333333333333333f);
+  small = fmaf(u, small, -0.5f);
+  small = fmaf(u, small * u, u);
+  return fmaxf(d, 0.0f) + (u < 0.04f ? small : large);
+}
+
+// g sigmoid(alpha g) (u + 1), g at most `limit`, u within +-limit
+template <typename T>
+__device__ __forceinline__ float clamped_glu_of(float g, float u, float limit,
+                                                float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * sigmoid_of<T>(alpha * g) * (u + 1.0f);
+}

@@ -3,8 +3,9 @@
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //
 // with q, k, v behind a short causal convolution and silu, q and k unit
-// vectors, one decay g per head.  The state [D, V] and everything that enters
-// the recurrence are fp32 in either element type.
+// vectors, and one decay g per head, or one per head and key channel (rows of
+// S).  The state [D, V] and everything that enters the recurrence are fp32 in
+// either element type.
 //
 //  * short portions (decoding): one kernel does convolution, norms, gates,
 //    recurrence, output norm and gate; the state lives in registers.
@@ -18,6 +19,13 @@
 //    (I + L)^-1 diag(beta) and A of all chunks at once, a second walks the
 //    chunks of a (request, head, 16 value columns).  All products run on the
 //    fp32 matrix cores.
+//  * decays per channel: exp(G) is a vector then, and L and A sum
+//    k_i[d] k_j[d] exp(G_i[d] - G_j[d]) over channels.  Between the tokens of two
+//    neighbouring blocks, with the second block's begin as reference, that is a
+//    product of two factors, the decay from there to i and the one from j to
+//    there; both are running products of decays of at most 1, so nothing
+//    overflows and no difference of large logarithms is taken.  Every pair of a
+//    chunk lies in two such blocks of 1, 2, 4, 8, 16 or more tokens.
 //
 // A request at position 0 starts from a zero state whatever its slot holds.
 #include "ragged_common.h"
@@ -28,12 +36,32 @@
 
 struct DeltaDims {
   int KH, H, D, V, taps;
-  int qc, kc, vc, gc, ac, bc;  // column offsets in a projection row
-  long ystride;
+  int qc, kc, vc, gc, ac, bc;  // column offsets in a projection row; gate (gc)
+  long ystride, zstride;       // and decay (ac) in rows z of their own
+  bool channels;               // decays per head and key channel
+  bool sigmoid;                // the output gate; else silu
 };
 
 __device__ __forceinline__ float log_decay(float a, float A_log, float dt) {
   return -expf(A_log) * softplus_f(a + dt);
+}
+
+// the factor of one step
+template <typename T>
+__device__ __forceinline__ float decay_of(float a, float rate, float dt);
+template <>
+__device__ __forceinline__ float decay_of<float>(float a, float rate, float dt) {
+  return expf(-rate * softplus_of<float>(a + dt));
+}
+template <>
+__device__ __forceinline__ float decay_of<__bf16>(float a, float rate, float dt) {
+  return __builtin_amdgcn_exp2f(-1.44269504088896340736f * rate *
+                                softplus_of<__bf16>(a + dt));
+}
+
+__device__ __forceinline__ float out_gate(float x, bool sigmoid) {
+  const float s = sigmoid_f(x);
+  return sigmoid ? s : x * s;
 }
 
 // ---------------------------------------------------------------------------
@@ -42,10 +70,11 @@ __device__ __forceinline__ float log_decay(float a, float A_log, float dt) {
 // RPT state rows per thread.
 // ---------------------------------------------------------------------------
 
-// EXACT: the threads tile the state without a remainder.
-template <typename T, int RPT, int NT, bool EXACT>
+// EXACT: the threads tile the state without a remainder.  CH: decays per channel.
+template <typename T, int RPT, int NT, bool EXACT, bool CH>
 __global__ __launch_bounds__(NT, RPT <= 32 ? 4 : 2) void delta_short_kernel(
-    const T* __restrict__ y, const T* __restrict__ conv_w,
+    const T* __restrict__ y, const T* __restrict__ z,
+    const T* __restrict__ conv_w,
     const T* __restrict__ A_log, const T* __restrict__ dt_bias,
     const T* __restrict__ norm_w, float* __restrict__ state,
     T* __restrict__ conv_state, T* __restrict__ out,
@@ -72,6 +101,7 @@ __global__ __launch_bounds__(NT, RPT <= 32 ? 4 : 2) void delta_short_kernel(
   float* vb = kq + DR_SHORT;                   // [n][V]
   float* red = vb + (long)n * V;               // [2][DG][VT]
   float* scratch = red + 2 * NT;               // [NT / WAVE]
+  float* gd = scratch + NT / WAVE;             // [n][D], decays per channel
 
   const int v = tid & (VT - 1);
   const int dg = tid / VT;
@@ -148,11 +178,21 @@ __global__ __launch_bounds__(NT, RPT <= 32 ? 4 : 2) void delta_short_kernel(
     __syncthreads();
     for (int i = tid; i < V; i += NT)
       convolve(2 * dm.KH * D + h * V + i, dm.vc + h * V + i, vb + i, V);
+    const float Al = (float)A_log[h], dt = CH ? 0.0f : (float)dt_bias[h];
+    if constexpr (CH) {
+      const float rate = expf(Al);
+      for (int i = tid; i < n * D; i += NT) {
+        const int t = i / D, d = i - t * D;
+        gd[i] = decay_of<T>((float)z[(t0 + t) * dm.zstride + dm.ac + h * D + d],
+                            rate, (float)dt_bias[h * D + d]);
+      }
+    }
     __syncthreads();
-    const float Al = (float)A_log[h], dt = (float)dt_bias[h];
     for (int t = 0; t < n; ++t) {
       const T* yt = y + (long)(t0 + t) * dm.ystride;
-      const float g = expf(log_decay((float)yt[dm.ac + h], Al, dt));
+      const T* zt = z + (long)(t0 + t) * dm.zstride;
+      const float g =
+          CH ? 1.0f : expf(log_decay((float)zt[dm.ac + h], Al, dt));
       const float beta = sigmoid_f((float)yt[dm.bc + h]);
       const float* qr = qk + (long)t * 2 * D;
       const float* kr = qr + D;
@@ -160,6 +200,7 @@ __global__ __launch_bounds__(NT, RPT <= 32 ? 4 : 2) void delta_short_kernel(
 #pragma unroll
       for (int i = 0; i < RPT; ++i)
         if (EXACT || d0 + i < D) {
+          if (CH) S[i] *= gd[t * D + d0 + i];
           sk += S[i] * kr[d0 + i];
           sq += S[i] * qr[d0 + i];
         }
@@ -181,7 +222,7 @@ __global__ __launch_bounds__(NT, RPT <= 32 ? 4 : 2) void delta_short_kernel(
       const bool mine = dg == 0 && v < V;
       const float ss = block_sum<NT>(mine ? o * o : 0.0f, scratch);
       if (mine) {
-        const float gate = silu_f((float)yt[dm.gc + h * V + v]);
+        const float gate = out_gate((float)zt[dm.gc + h * V + v], dm.sigmoid);
         out[(long)(t0 + t) * ((long)dm.H * V) + h * V + v] =
             (T)(o / sqrtf(ss / (float)V + eps) * (float)norm_w[v] * gate);
       }
@@ -216,29 +257,30 @@ extern "C" int delta_short_rows(int D, int V, int nt) {
 
 #define DR_NT 512
 
-template <typename T>
-static void delta_short_t(const void* y, const void* conv_w, const void* A_log,
-                          const void* dt_bias, const void* norm_w,
-                          float* state, void* conv_state, void* out,
-                          const int* cu, const int* pos0, const int* slots,
-                          const DeltaDims& dm, int n_req, int max_len,
-                          float eps, hipStream_t stream) {
+template <typename T, bool CH>
+static void delta_short_t(const void* y, const void* z, const void* conv_w,
+                          const void* A_log, const void* dt_bias,
+                          const void* norm_w, float* state, void* conv_state,
+                          void* out, const int* cu, const int* pos0,
+                          const int* slots, const DeltaDims& dm, int n_req,
+                          int max_len, float eps, hipStream_t stream) {
   const int vt = pow2_at_least(dm.V);
   const int rpt = delta_short_rows(dm.D, dm.V, DR_NT);
-  const size_t smem = ((size_t)max_len * (2 * dm.D + dm.V) + DR_SHORT +
-                       2 * DR_NT + DR_NT / WAVE) * sizeof(float);
+  const size_t smem = ((size_t)max_len * ((CH ? 3 : 2) * dm.D + dm.V) +
+                       DR_SHORT + 2 * DR_NT + DR_NT / WAVE) * sizeof(float);
   const float q_scale = 1.0f / sqrtf((float)dm.D);
   dim3 grid((unsigned)n_req, (unsigned)dm.KH), block(DR_NT);
 #define DS_ONE(R, X)                                                         \
   do {                                                                       \
     if (smem > 65536)                                                        \
       (void)hipFuncSetAttribute(                                             \
-          reinterpret_cast<const void*>(&delta_short_kernel<T, R, DR_NT, X>), \
+          reinterpret_cast<const void*>(                                     \
+              &delta_short_kernel<T, R, DR_NT, X, CH>),                      \
           hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);            \
-    delta_short_kernel<T, R, DR_NT, X><<<grid, block, smem, stream>>>(       \
-        (const T*)y, (const T*)conv_w, (const T*)A_log, (const T*)dt_bias,   \
-        (const T*)norm_w, state, (T*)conv_state, (T*)out, cu, pos0, slots,   \
-        dm, vt, q_scale, eps);                                               \
+    delta_short_kernel<T, R, DR_NT, X, CH><<<grid, block, smem, stream>>>(   \
+        (const T*)y, (const T*)z, (const T*)conv_w, (const T*)A_log,         \
+        (const T*)dt_bias, (const T*)norm_w, state, (T*)conv_state, (T*)out, \
+        cu, pos0, slots, dm, vt, q_scale, eps);                              \
   } while (0)
 #define DS_GO(R)                                                             \
   do {                                                                       \
@@ -259,21 +301,26 @@ static void delta_short_t(const void* y, const void* conv_w, const void* A_log,
 #undef DS_ONE
 }
 
-extern "C" void launch_delta_short(const void* y, const void* conv_w,
-                                   const void* A_log, const void* dt_bias,
-                                   const void* norm_w, float* state,
-                                   void* conv_state, void* out, const int* cu,
-                                   const int* pos0, const int* slots,
-                                   const DeltaDims* dm, int n_req, int max_len,
-                                   float eps, bool f32, hipStream_t stream) {
-  if (f32)
-    delta_short_t<float>(y, conv_w, A_log, dt_bias, norm_w, state, conv_state,
-                         out, cu, pos0, slots, *dm, n_req, max_len, eps,
-                         stream);
-  else
-    delta_short_t<__bf16>(y, conv_w, A_log, dt_bias, norm_w, state, conv_state,
-                          out, cu, pos0, slots, *dm, n_req, max_len, eps,
-                          stream);
+extern "C" void launch_delta_short(const void* y, const void* z,
+                                   const void* conv_w, const void* A_log,
+                                   const void* dt_bias, const void* norm_w,
+                                   float* state, void* conv_state, void* out,
+                                   const int* cu, const int* pos0,
+                                   const int* slots, const DeltaDims* dm,
+                                   int n_req, int max_len, float eps, bool f32,
+                                   hipStream_t stream) {
+#define DS_TYPE(T, CH)                                                        \
+  delta_short_t<T, CH>(y, z, conv_w, A_log, dt_bias, norm_w, state,           \
+                       conv_state, out, cu, pos0, slots, *dm, n_req, max_len, \
+                       eps, stream)
+  if (dm->channels) {
+    if (f32) DS_TYPE(float, true);
+    else DS_TYPE(__bf16, true);
+  } else {
+    if (f32) DS_TYPE(float, false);
+    else DS_TYPE(__bf16, false);
+  }
+#undef DS_TYPE
 }
 
 // ---------------------------------------------------------------------------
@@ -436,8 +483,9 @@ __global__ __launch_bounds__(DC_BLOCK) void delta_conv_kernel(
     for (int j = lane; j < len * dm.H; j += WAVE) {
       const int t = j / dm.H, h = j - t * dm.H;
       const T* yr = yt + (long)t * dm.ystride;
-      lg[(i0 + t) * dm.H + h] =
-          log_decay((float)yr[dm.ac + h], (float)A_log[h], (float)dt_bias[h]);
+      if (!dm.channels)
+        lg[(i0 + t) * dm.H + h] =
+            log_decay((float)yr[dm.ac + h], (float)A_log[h], (float)dt_bias[h]);
       bt[(i0 + t) * dm.H + h] = sigmoid_f((float)yr[dm.bc + h]);
     }
   }
@@ -480,6 +528,29 @@ __global__ __launch_bounds__(DC_BLOCK) void delta_conv_state_kernel(
 // ---------------------------------------------------------------------------
 
 #define DR_LS 68
+
+// (I + L)^-1 times `by`, one column per lane; ls: L, rows of DR_LS
+__device__ __forceinline__ void invert_unit(const float* ls, float by, float* tm,
+                                            int lane) {
+  float x[DR_CHUNK];
+#pragma unroll
+  for (int i = 0; i < DR_CHUNK; ++i) {
+    float a0 = i == lane ? 1.0f : 0.0f, a1 = 0.0f, a2 = 0.0f, a3 = 0.0f;
+    const float* row = ls + i * DR_LS;
+#pragma unroll
+    for (int j = 0; j + 4 <= i; j += 4) {
+      const f32x4 l4 = load4(row + j);
+      a0 -= l4[0] * x[j];
+      a1 -= l4[1] * x[j + 1];
+      a2 -= l4[2] * x[j + 2];
+      a3 -= l4[3] * x[j + 3];
+    }
+#pragma unroll
+    for (int j = i & ~3; j < i; ++j) a0 -= row[j] * x[j];
+    x[i] = (a0 + a1) + (a2 + a3);
+    tm[i * 64 + lane] = x[i] * by;
+  }
+}
 
 __global__ __launch_bounds__(256) void delta_chunk_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn,
@@ -557,39 +628,193 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(
     }
   }
   __syncthreads();
-  if (wid != 0) return;
-  float x[DR_CHUNK];
-  const float bc = bs[lane];
+  if (wid == 0) invert_unit(ls, bs[lane], tm + ch * 4096, lane);
+}
+
+// The same for decays per channel, and what the walk multiplies the state with:
+//   qg, kg [tokens, H, Dp]  q and k with the decay from the chunk's begin
+//   kl     [tokens, H, Dp]  k with the decay to the chunk's end
+//   gl     [chunks, H, Dp]  the decay of the whole chunk
+// Wave w has token rows 16w..16w+15, a lane one of them and four of each 16
+// channels.  Per 16 channels, running products over blocks of 1, 2, 4, 8 and 16
+// rows grow by one exchange between lanes each: `from` decays from the row's
+// block's begin to the row, `to` from the row to its block's end.
+#define DCH_STEPS 4                    // steps of 16 channels between barriers
+#define DCH_LS (DCH_STEPS * 16 + 4)
+
+template <typename T>
+__global__ __launch_bounds__(256) void delta_chunk_channels_kernel(
+    const float* __restrict__ qn, const float* __restrict__ kn,
+    const T* __restrict__ z, const T* __restrict__ A_log,
+    const T* __restrict__ dt_bias, const float* __restrict__ bt,
+    float* __restrict__ tm, float* __restrict__ am, float* __restrict__ qg,
+    float* __restrict__ kg, float* __restrict__ kl, float* __restrict__ gl,
+    const int* __restrict__ chunks, int tok_base, DeltaDims dm, int Dp) {
+  const int c = blockIdx.x, h = blockIdx.y;
+  const int H = dm.H, KH = dm.KH, D = dm.D;
+  const int kh = h / (H / KH);
+  const int i0 = chunks[2 * c] - tok_base;
+  const int len = chunks[2 * c + 1];
+  const int tid = threadIdx.x;
+  const int lane = tid & (WAVE - 1);
+  const int wid = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int lr = lane & 15, g4 = lane >> 4;
+
+  __shared__ float bs[DR_CHUNK];
+  __shared__ __attribute__((aligned(16))) float ms[4][DCH_STEPS * 16];
+  // k with the decay to its wave's last row; later I + L
+  __shared__ __attribute__((aligned(16))) float ls[DR_CHUNK * DR_LS];
+  static_assert(DCH_LS <= DR_LS, "");
+
+  const long ch = (long)c * H + h;
+  if (wid == 0) bs[lane] = lane < len ? bt[(long)(i0 + lane) * H + h] : 0.0f;
+
+  const int row = wid * 16 + lr;
+  const bool in = row < len;
+  // rows past the end repeat the last one with k = q = 0, decay 1 and beta 0
+  const long tok = i0 + min(row, len - 1);
+  const float* kp = kn + (tok * KH + kh) * Dp + g4 * 4;
+  const float* qp = qn + (tok * KH + kh) * Dp + g4 * 4;
+  const T* zp = z + (tok_base + tok) * dm.zstride + dm.ac + (long)h * D;
+  const T* dp = dt_bias + (long)h * D;
+  const long at = ((long)(i0 + row) * H + h) * Dp + g4 * 4;
+  const float rate = expf((float)A_log[h]);
+  const f32x4 zero = {0, 0, 0, 0}, one = {1, 1, 1, 1};
+
+  f32x4 kk[4], qk[4], kko[3], qko[3];
 #pragma unroll
-  for (int i = 0; i < DR_CHUNK; ++i) {
-    float a0 = i == lane ? 1.0f : 0.0f, a1 = 0.0f, a2 = 0.0f, a3 = 0.0f;
-    const float* row = ls + i * DR_LS;
+  for (int i = 0; i < 4; ++i) kk[i] = qk[i] = zero;
 #pragma unroll
-    for (int j = 0; j + 4 <= i; j += 4) {
-      const f32x4 l4 = load4(row + j);
-      a0 -= l4[0] * x[j];
-      a1 -= l4[1] * x[j + 1];
-      a2 -= l4[2] * x[j + 2];
-      a3 -= l4[3] * x[j + 3];
+  for (int i = 0; i < 3; ++i) kko[i] = qko[i] = zero;
+  float diag = 0.0f;
+
+  for (int d0 = 0; d0 < Dp; d0 += DCH_STEPS * 16) {
+    f32x4 ka[DCH_STEPS], qa[DCH_STEPS], kb[DCH_STEPS];
+#pragma unroll
+    for (int s = 0; s < DCH_STEPS; ++s) {
+      const int ds = d0 + s * 16;
+      if (ds >= Dp) continue;
+      const f32x4 k = in ? load4(kp + ds) : zero;
+      const f32x4 q = in ? load4(qp + ds) : zero;
+      f32x4 from, to = one;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = ds + g4 * 4 + j;
+        const int dc = min(d, D - 1);
+        const float g = decay_of<T>((float)zp[dc], rate, (float)dp[dc]);
+        from[j] = in && d < D ? g : 1.0f;
+        diag += q[j] * k[j];
+      }
+#pragma unroll
+      for (int l = 0; l < 4; ++l) {
+        const int half = 1 << l;
+        const f32x4 kf = k * from, qf = q * from, kt = k * to;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          kk[l] = mma4(kf[j], kt[j], kk[l]);
+          qk[l] = mma4(qf[j], kt[j], qk[l]);
+        }
+        // the other half's whole decay: of the first for rows of the second
+        const bool second = lr & half;
+        const int src = (lane & ~(2 * half - 1)) + (second ? half : 2 * half) - 1;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float other = __shfl(from[j], src, WAVE);
+          if (second) from[j] *= other;
+          else to[j] *= other;
+        }
+      }
+      ka[s] = k * from;
+      qa[s] = q * from;
+      kb[s] = k * to;
+      store4(ls + row * DCH_LS + s * 16 + g4 * 4, kb[s]);
+      if (lr == 15) store4(&ms[wid][s * 16 + g4 * 4], from);
     }
+    __syncthreads();
+    // blocks before this wave's, the nearest first
 #pragma unroll
-    for (int j = i & ~3; j < i; ++j) a0 -= row[j] * x[j];
-    x[i] = (a0 + a1) + (a2 + a3);
-    tm[ch * 4096 + i * 64 + lane] = x[i] * bc;
+    for (int b = 2; b >= 0; --b) {
+      if (b >= wid) continue;
+#pragma unroll
+      for (int s = 0; s < DCH_STEPS; ++s) {
+        if (d0 + s * 16 >= Dp) continue;
+        const f32x4 k = load4(ls + (b * 16 + lr) * DCH_LS + s * 16 + g4 * 4);
+        const f32x4 m = load4(&ms[b][s * 16 + g4 * 4]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          kko[b] = mma4(ka[s][j], k[j], kko[b]);
+          qko[b] = mma4(qa[s][j], k[j], qko[b]);
+        }
+        ka[s] = ka[s] * m;
+        qa[s] = qa[s] * m;
+      }
+    }
+    // and those behind it
+#pragma unroll
+    for (int b = 1; b < 4; ++b) {
+      if (b <= wid) continue;
+#pragma unroll
+      for (int s = 0; s < DCH_STEPS; ++s)
+        if (d0 + s * 16 < Dp)
+          kb[s] = kb[s] * load4(&ms[b][s * 16 + g4 * 4]);
+    }
+    if (in) {
+#pragma unroll
+      for (int s = 0; s < DCH_STEPS; ++s) {
+        const int ds = d0 + s * 16;
+        if (ds >= Dp) continue;
+        store4(kg + at + ds, ka[s]);
+        store4(qg + at + ds, qa[s]);
+        store4(kl + at + ds, kb[s]);
+      }
+    }
+    if (tid < DCH_STEPS * 16 && d0 + tid < Dp)
+      gl[ch * Dp + d0 + tid] =
+          (ms[0][tid] * ms[1][tid]) * (ms[2][tid] * ms[3][tid]);
+    __syncthreads();
   }
+  diag += __shfl_xor(diag, 16, WAVE);
+  diag += __shfl_xor(diag, 32, WAVE);  // of this lane's row: q.k
+
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int i = wid * 16 + g4 * 4 + r;
+    const float b = bs[i];
+#pragma unroll
+    for (int j = 0; j < 3; ++j) {
+      if (j >= wid) continue;
+      ls[i * DR_LS + j * 16 + lr] = b * kko[j][r];
+      am[ch * 4096 + i * 64 + j * 16 + lr] = qko[j][r];
+    }
+    // the level that separates the row from the column
+    const int local = g4 * 4 + r;
+    float kv = 0.0f, qv = local == lr ? diag : 0.0f;
+#pragma unroll
+    for (int l = 0; l < 4; ++l)
+      if (local > lr && (local ^ lr) >> l == 1) {
+        kv = kk[l][r];
+        qv = qk[l][r];
+      }
+    ls[i * DR_LS + row] = b * kv;
+    am[ch * 4096 + i * 64 + row] = qv;
+  }
+  __syncthreads();
+  if (wid == 0) invert_unit(ls, bs[lane], tm + ch * 4096, lane);
 }
 
 // ---------------------------------------------------------------------------
 // Step 3: the walk.  Block = (value column tile, head, request), 4 waves;
 // wave w owns token rows 16w..16w+15 of a chunk and state row tiles w, w+4,...
 // A operands come straight from global memory as vectors (the contraction
-// order inside 16 is permuted the same way on both sides).
+// order inside 16 is permuted the same way on both sides).  CH: decays per
+// channel; q, k and kt (k as the state takes it up) come with their decays, one
+// row per value head (KH == H), and ge is the chunk's decay [chunks, H, Dp].
 // ---------------------------------------------------------------------------
 
-template <typename T>
+template <typename T, bool CH>
 __global__ __launch_bounds__(256) void delta_walk_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn,
-    const T* __restrict__ vn, const float* __restrict__ tm,
+    const float* __restrict__ kt, const T* __restrict__ vn, const float* __restrict__ tm,
     const float* __restrict__ am, const float* __restrict__ ge,
     float* __restrict__ state, float* __restrict__ o,
     const int* __restrict__ chunks, const int* __restrict__ chunk_cu,
@@ -628,7 +853,8 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
     const long ch = (long)c * H + h;
     const float* kp = kn + ((long)i0 * KH + kh) * Dp;
     const float* qp = qn + ((long)i0 * KH + kh) * Dp;
-    const float* gc = ge + ch * 128;
+    const float* tp = kt + ((long)i0 * KH + kh) * Dp;
+    const float* gc = ge + ch * (CH ? Dp : 128);
 
     f32x4 ks = zero, qs = zero;
     {
@@ -651,8 +877,8 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = wid * 16 + g4 * 4 + r;
-      gr[r] = gc[i];
-      gl[r] = gc[64 + i];
+      gr[r] = CH ? 1.0f : gc[i];
+      gl[r] = CH ? 1.0f : gc[64 + i];
       const float v =
           i < len ? (float)vn[((long)(i0 + i) * H + h) * Vp + v0 + lr] : 0.0f;
       xs[i * 17 + lr] = v - gr[r] * ks[r];
@@ -688,13 +914,12 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
       const int i = wid * 16 + g4 * 4 + r;
       if (i < len) o[((long)(i0 + i) * H + h) * Vp + v0 + lr] = oc[r];
     }
-    const float g_all = gc[63];
     for (int d0 = wid * 16; d0 < Dp; d0 += 64) {
       f32x4 sn;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        sn[r] = g_all * ss[(d0 + g4 * 4 + r) * 17 + lr];
-      const float* ka = kp + d0 + lr;
+        sn[r] = gc[CH ? d0 + g4 * 4 + r : 63] * ss[(d0 + g4 * 4 + r) * 17 + lr];
+      const float* ka = tp + d0 + lr;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -719,10 +944,10 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
 // used it, so its latency passes behind the products that remain.  Rows past
 // the end of a chunk repeat its last one: their beta is 0, so they write
 // nothing, and their outputs are not stored.
-template <typename T, int ND>
+template <typename T, int ND, bool CH>
 __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn,
-    const T* __restrict__ vn, const float* __restrict__ tm,
+    const float* __restrict__ ktn, const T* __restrict__ vn, const float* __restrict__ tm,
     const float* __restrict__ am, const float* __restrict__ ge,
     float* __restrict__ state, float* __restrict__ o,
     const int* __restrict__ chunks, const int* __restrict__ chunk_cu,
@@ -759,6 +984,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
 
   f32x4 kf[ND], qf[ND], tf[4], af[4], kt[NT][4];
   float vf[4], gr[4], gl[4], g_all;
+  f32x4 gd[NT];  // decays of this lane's state rows
 
   auto load_rows = [&](int i0, int len) {
     const long at = ((long)(i0 + min(row, len - 1)) * KH + kh) * Dp + g4 * 4;
@@ -769,15 +995,24 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
     }
   };
   auto load_misc = [&](int c, int i0, int len) {
-    const float* gc = ge + ((long)c * H + h) * 128;
+    const float* gc = ge + ((long)c * H + h) * (CH ? Dp : 128);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = row_c + r;
       vf[r] = (float)vn[((long)(i0 + min(i, len - 1)) * H + h) * Vp + v0 + lr];
-      gr[r] = gc[i];
-      gl[r] = gc[64 + i];
+      gr[r] = CH ? 1.0f : gc[i];
+      gl[r] = CH ? 1.0f : gc[64 + i];
     }
-    g_all = gc[63];
+    if (!CH) g_all = gc[63];
+  };
+  auto load_decay = [&](int c) {
+    if constexpr (CH) {
+#pragma unroll
+      for (int n = 0; n < NT; ++n) {
+        const int d0 = wid * 16 + n * 64;
+        if (d0 < Dp) gd[n] = load4(ge + ((long)c * H + h) * Dp + d0 + g4 * 4);
+      }
+    }
   };
   auto load_mat = [&](const float* m, int c, f32x4 (&f)[4]) {
     const float* p = m + ((long)c * H + h) * 4096 + row * 64 + g4 * 4;
@@ -789,7 +1024,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
     for (int n = 0; n < NT; ++n) {
       const int d0 = wid * 16 + n * 64;
       if (d0 >= Dp) continue;
-      const float* ka = kn + ((long)i0 * KH + kh) * Dp + d0 + lr;
+      const float* ka = ktn + ((long)i0 * KH + kh) * Dp + d0 + lr;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -808,6 +1043,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
   load_mat(tm, c, tf);
   load_mat(am, c, af);
   load_kt(i0, len);
+  load_decay(c);
   __syncthreads();
 
   for (; c < c_end; ++c) {
@@ -873,7 +1109,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
       f32x4 sn;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        sn[r] = g_now * ss[(d0 + g4 * 4 + r) * 17 + lr];
+        sn[r] = (CH ? gd[n][r] : g_now) * ss[(d0 + g4 * 4 + r) * 17 + lr];
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -883,6 +1119,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
       for (int r = 0; r < 4; ++r) ss[(d0 + g4 * 4 + r) * 17 + lr] = sn[r];
     }
     load_kt(j0, jl);
+    load_decay(cn);
     __syncthreads();
     i0 = j0;
     len = jl;
@@ -894,7 +1131,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// Step 4: output norm over V, weight, silu gate.  One wave per (token, head).
+// Step 4: output norm over V, weight, gate.  One wave per (token, head).
 // ---------------------------------------------------------------------------
 
 // NV groups of CW channels per lane, V <= 64 * CW * NV; DG_ROWS rows per wave
@@ -903,7 +1140,7 @@ __global__ __launch_bounds__(256, 1) void delta_walk_fixed_kernel(
 
 template <typename T, int NV, int CW>
 __global__ __launch_bounds__(256) void delta_gate_kernel(
-    const float* __restrict__ o, const T* __restrict__ y,
+    const float* __restrict__ o, const T* __restrict__ z,
     const T* __restrict__ norm_w, T* __restrict__ out, long n, int tok_base,
     DeltaDims dm, int Vp, float eps) {
   const int lane = threadIdx.x & (WAVE - 1);
@@ -916,7 +1153,7 @@ __global__ __launch_bounds__(256) void delta_gate_kernel(
     const int wi = (int)min(w0 + k, rows - 1);
     const int i = wi / dm.H;
     const int h = wi - i * dm.H;
-    const T* gr = y + (long)(tok_base + i) * dm.ystride + dm.gc + h * dm.V;
+    const T* gr = z + (long)(tok_base + i) * dm.zstride + dm.gc + h * dm.V;
     const float* orow = o + (long)wi * Vp;
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
@@ -950,23 +1187,48 @@ __global__ __launch_bounds__(256) void delta_gate_kernel(
       float r[CW];
 #pragma unroll
       for (int q = 0; q < CW; ++q)
-        r[q] = ov[k][u][q] * inv * wv[u][q] * silu_f(gv[k][u][q]);
+        r[q] = ov[k][u][q] * inv * wv[u][q] * out_gate(gv[k][u][q], dm.sigmoid);
       if (v < dm.V) store_lanes<T, CW>(dst + v, r);
     }
   }
 }
 
 struct DeltaLongArgs {
-  const void *y, *conv_w, *A_log, *dt_bias, *norm_w;
+  const void *y, *z, *conv_w, *A_log, *dt_bias, *norm_w;
   float* state;
   void *conv_state, *out;
-  float *qn, *kn, *lg, *bt, *tm, *am, *ge, *o;
+  float *qn, *kn, *lg, *bt, *tm, *am, *ge, *o, *qg, *kg, *kl;
   void* vn;
   const int *cu, *pos0, *slots, *tok_entry, *chunks, *chunk_cu;
   int n_short, n_long, tok_base, n_chunks, Dp, Vp;
   long n_tok;
   float eps;
 };
+
+// KH: heads that q, k and kt have
+template <typename T, bool CH>
+static void delta_walk_t(const DeltaLongArgs& a, const DeltaDims& dm,
+                         const float* q, const float* k, const float* kt, int KH,
+                         dim3 grid, hipStream_t stream) {
+  const dim3 block(256);
+#define DW_GO(N)                                                              \
+  delta_walk_fixed_kernel<T, N, CH><<<grid, block, 0, stream>>>(              \
+      q, k, kt, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,     \
+      a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, KH, dm.H, dm.D,     \
+      dm.V, a.Vp)
+  if (a.Dp == 16) DW_GO(1);
+  else if (a.Dp == 32) DW_GO(2);
+  else if (a.Dp == 64) DW_GO(4);
+  else if (a.Dp == 128) DW_GO(8);
+  else {
+    const size_t smem = ((size_t)a.Dp + 3 * 64) * 17 * sizeof(float);
+    delta_walk_kernel<T, CH><<<grid, block, smem, stream>>>(
+        q, k, kt, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,
+        a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, KH, dm.H, dm.D,
+        a.Dp, dm.V, a.Vp);
+  }
+#undef DW_GO
+}
 
 template <typename T>
 static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
@@ -1003,33 +1265,24 @@ static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
     delta_conv_state_kernel<T><<<g2, block, 0, stream>>>(
         (const T*)a.y, (T*)a.conv_state, a.cu, a.pos0, a.slots, a.n_short, dm);
   dim3 g3((unsigned)a.n_chunks, (unsigned)dm.H);
-  delta_chunk_kernel<<<g3, block, 0, stream>>>(
-      a.qn, a.kn, a.lg, a.bt, a.tm, a.am, a.ge, a.chunks, a.tok_base, dm.KH,
-      dm.H, a.Dp);
   dim3 g4((unsigned)(a.Vp / 16), (unsigned)dm.H, (unsigned)a.n_long);
-#define DW_GO(N)                                                             \
-  delta_walk_fixed_kernel<T, N><<<g4, block, 0, stream>>>(                   \
-      a.qn, a.kn, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,  \
-      a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, dm.KH, dm.H, dm.D, \
-      dm.V, a.Vp)
-  if (a.Dp == 16) DW_GO(1);
-  else if (a.Dp == 32) DW_GO(2);
-  else if (a.Dp == 64) DW_GO(4);
-  else if (a.Dp == 128) DW_GO(8);
-  else {
-    const size_t smem = ((size_t)a.Dp + 3 * 64) * 17 * sizeof(float);
-    delta_walk_kernel<T><<<g4, block, smem, stream>>>(
-        a.qn, a.kn, (const T*)a.vn, a.tm, a.am, a.ge, a.state, a.o, a.chunks,
-        a.chunk_cu, a.pos0, a.slots, a.n_short, a.tok_base, dm.KH, dm.H, dm.D,
-        a.Dp, dm.V, a.Vp);
+  if (dm.channels) {
+    delta_chunk_channels_kernel<T><<<g3, block, 0, stream>>>(
+        a.qn, a.kn, (const T*)a.z, (const T*)a.A_log, (const T*)a.dt_bias, a.bt,
+        a.tm, a.am, a.qg, a.kg, a.kl, a.ge, a.chunks, a.tok_base, dm, a.Dp);
+    delta_walk_t<T, true>(a, dm, a.qg, a.kg, a.kl, dm.H, g4, stream);
+  } else {
+    delta_chunk_kernel<<<g3, block, 0, stream>>>(
+        a.qn, a.kn, a.lg, a.bt, a.tm, a.am, a.ge, a.chunks, a.tok_base, dm.KH,
+        dm.H, a.Dp);
+    delta_walk_t<T, false>(a, dm, a.qn, a.kn, a.kn, dm.KH, g4, stream);
   }
-#undef DW_GO
   dim3 g5((unsigned)((a.n_tok * dm.H + 4 * DG_ROWS - 1) / (4 * DG_ROWS)));
 #define DG_GO(N, W)                                                          \
   delta_gate_kernel<T, N, W><<<g5, block, 0, stream>>>(                      \
-      a.o, (const T*)a.y, (const T*)a.norm_w, (T*)a.out, a.n_tok,            \
+      a.o, (const T*)a.z, (const T*)a.norm_w, (T*)a.out, a.n_tok,            \
       a.tok_base, dm, a.Vp, a.eps)
-  if (pair && dm.gc % 2 == 0) {
+  if (pair && dm.gc % 2 == 0 && dm.zstride % 2 == 0) {
     if (dm.V <= 128) DG_GO(1, 2);
     else if (dm.V <= 256) DG_GO(2, 2);
     else DG_GO(4, 2);

@@ -12,7 +12,7 @@
 // ---------------------------------------------------------------------------
 // Router.  A block has 16 tokens and 16 waves: 128 experts at a time, half of
 // the waves for each 64 of them, eight parts of the contraction, which meet in
-// LDS.  Then a wave per token softmaxes and picks.
+// LDS.  Then a wave per token makes scores and picks.
 // ---------------------------------------------------------------------------
 
 #define RT_BLOCK 1024
@@ -85,16 +85,22 @@ __global__ __launch_bounds__(RT_BLOCK) void expert_route_kernel(
   for (int t = wid; t < n; t += RT_WAVES) {
     const float* z = logits + t * totalp;
     float* choice = choices + wid * totalp;
-    float mx = -INFINITY;
-    for (int e = lane; e < a.total; e += WAVE) mx = fmaxf(mx, z[e]);
-    mx = wave_max(mx);
-    float sum = 0.0f;
-    for (int e = lane; e < a.total; e += WAVE) sum += expf(z[e] - mx);
-    sum = wave_sum(sum);
-    const float inv = 1.0f / sum;
-    // a lane writes and reads only its own choices
+    float mx = -INFINITY, inv = 1.0f;
+    if (!a.sigmoid) {
+      for (int e = lane; e < a.total; e += WAVE) mx = fmaxf(mx, z[e]);
+      mx = wave_max(mx);
+      float sum = 0.0f;
+      for (int e = lane; e < a.total; e += WAVE) sum += expf(z[e] - mx);
+      inv = 1.0f / wave_sum(sum);
+    }
+    auto score = [&](int e) {
+      return a.sigmoid ? sigmoid_f(z[e]) : expf(z[e] - mx) * inv;
+    };
+    // a lane writes and reads only its own choices; logits order uncorrected
+    // scores, also where those round to the same
     for (int e = lane; e < a.total; e += WAVE)
-      choice[e] = expf(z[e] - mx) * inv + (float)((const T*)a.correction)[e];
+      choice[e] = a.correction ? score(e) + (float)((const T*)a.correction)[e]
+                               : z[e];
     float picked = 0.0f, mine = 0.0f;
     int my_e = 0;
     for (int k = 0; k < a.top; ++k) {
@@ -116,7 +122,7 @@ __global__ __launch_bounds__(RT_BLOCK) void expert_route_kernel(
       }
       at = min(at, a.total - 1);
       if (at % WAVE == lane) choice[at] = -INFINITY;
-      const float s = expf(z[at] - mx) * inv;  // without the correction
+      const float s = score(at);  // without the correction
       picked += s;
       if (lane == k % WAVE) {
         mine = s;
@@ -133,6 +139,7 @@ __global__ __launch_bounds__(RT_BLOCK) void expert_route_kernel(
         }
       }
     }
+    if (!a.normalize) continue;
     const float by = 1.0f / (picked + 1e-20f);
     for (int k = lane; k < a.top; k += WAVE)
       a.weight[(t0 + t) * a.top + k] *= by;
@@ -253,6 +260,7 @@ __global__ __launch_bounds__(PB) void expert_plan_kernel(const PlanArgs a,
     for (int r = b0; r < b; ++r) at += a.hist[(long)r * a.experts + x];
     a.where[p] = at;
     a.tokens[at] = (int)(p / a.top);
+    if (a.weight) a.scale[at] = a.weight[p];
   }
 }
 
@@ -327,8 +335,9 @@ __device__ __forceinline__ void skinny_sums(const T* w0, const T* w1,
   __syncthreads();
 }
 
-// grid (output blocks, tiles)
-template <typename T>
+// grid (output blocks, tiles).  GLU: 16 gated units, the first weight tile is
+// their gate's, the second their up projection's.
+template <typename T, bool GLU>
 __global__ __launch_bounds__(EX_BLOCK) void expert_skinny_kernel(
     const ExpertGemmArgs a) {
   __shared__ __attribute__((aligned(16))) float red[EX_WAVES][16][SK_OUT + 4];
@@ -339,21 +348,31 @@ __global__ __launch_bounds__(EX_BLOCK) void expert_skinny_kernel(
   const int lane = tid & (WAVE - 1);
   const int wid = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int lr = lane & 15, lg = lane >> 4;
-  const int o0 = blockIdx.x * SK_OUT;
+  constexpr int OUT = GLU ? SK_OUT / 2 : SK_OUT;
+  const int outs = GLU ? a.O / 2 : a.O;
+  const int o0 = blockIdx.x * OUT;
   const T* w = (const T*)a.w + (long)e * a.O * a.K + lg * 8;
   const long p = p0 + min(lr, n - 1);
   const long row = a.tokens ? a.tokens[p] : p;
-  skinny_sums<T, T, 32>(
-      w + (long)min(o0 + lr, a.O - 1) * a.K,
-      w + (long)min(o0 + 16 + lr, a.O - 1) * a.K,
-      (const T*)a.x + row * a.xstride + lg * 8, a.K, wid, lr, lg, red);
-  for (int i = tid; i < n * SK_OUT; i += EX_BLOCK) {
-    const int t = i / SK_OUT, o = i % SK_OUT;
-    if (o0 + o >= a.O) continue;
-    float v = 0.0f;
+  const int r0 = min(o0 + lr, outs - 1);
+  const int r1 = GLU ? outs + r0 : min(o0 + 16 + lr, outs - 1);
+  skinny_sums<T, T, 32>(w + (long)r0 * a.K, w + (long)r1 * a.K,
+                        (const T*)a.x + row * a.xstride + lg * 8, a.K, wid, lr,
+                        lg, red);
+  for (int i = tid; i < n * OUT; i += EX_BLOCK) {
+    const int t = i / OUT, o = i % OUT;
+    if (o0 + o >= outs) continue;
+    float v = 0.0f, u = 0.0f;
 #pragma unroll
-    for (int k = 0; k < EX_WAVES; ++k) v += red[k][t][o];
-    if (a.act) {
+    for (int k = 0; k < EX_WAVES; ++k) {
+      v += red[k][t][o];
+      if (GLU) u += red[k][t][16 + o];
+    }
+    const float scale = a.scale ? a.scale[p0 + t] : 1.0f;
+    v *= scale;
+    if constexpr (GLU) {
+      v = clamped_glu_of<T>(v, u * scale, a.limit, a.alpha);
+    } else if (a.act == EX_RELU2) {
       v = fmaxf(v, 0.0f);
       v *= v;
     }
@@ -407,8 +426,9 @@ extern "C" void launch_token_gate(const TokenGateArgs* a, bool f32,
 }
 
 // ---------------------------------------------------------------------------
-// Many tokens per expert.  A block makes 128 outputs of up to 128 pairs, a wave
-// 64 x 64 of them.  Rows of 128 bytes go to LDS without passing registers, the
+// Many tokens per expert.  A block takes 128 weight rows to up to 128 pairs, a
+// wave 64 x 64 of them; of a gated unit, 16 rows of the gate and 16 of the up
+// projection by turns, so that a lane has both halves of its outputs.  Rows of 128 bytes go to LDS without passing registers, the
 // next step while this one is worked on; 16-byte pieces are swapped within a
 // row (by the source address) so that reads of a column meet different banks.
 // ---------------------------------------------------------------------------
@@ -437,7 +457,7 @@ __device__ __forceinline__ void read_row(Frag<float>& f, const char* base,
 }
 
 // grid: one row of blocks per XCD, so that neighbouring tiles share an L2
-template <typename T>
+template <typename T, bool GLU>
 __global__ __launch_bounds__(EX_BLOCK, 2) void expert_wide_kernel(
     const ExpertGemmArgs a) {
   constexpr int STEP = WT_BYTES / (int)sizeof(T);   // elements per step
@@ -463,7 +483,10 @@ __global__ __launch_bounds__(EX_BLOCK, 2) void expert_wide_kernel(
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int r = wid * 32 + i * 8 + (lane >> 3);
-    ws[i] = (const T*)a.w + ((long)e * a.O + min(o0 + r, a.O - 1)) * a.K + piece;
+    int o = min(o0 + r, a.O - 1);
+    if (GLU)
+      o = r / 16 % 2 * (a.O / 2) + min(o0 / 2 + r / 32 * 16 + r % 16, a.O / 2 - 1);
+    ws[i] = (const T*)a.w + ((long)e * a.O + o) * a.K + piece;
     const long p = p0 + min(r, n - 1);
     const long row = a.tokens ? a.tokens[p] : p;
     xs[i] = (const T*)a.x + row * a.xstride + piece;
@@ -514,22 +537,29 @@ __global__ __launch_bounds__(EX_BLOCK, 2) void expert_wide_kernel(
     const int t = wt + j * 16 + lr;
     if (t >= n) continue;
     T* out = (T*)a.out + (long)(p0 + t) * a.ostride;
+    const float scale = a.scale ? a.scale[p0 + t] : 1.0f;
+    const int outs = GLU ? a.O / 2 : a.O;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int o = o0 + wo + i * 16 + lg * 4;
+    for (int i = 0; i < 4; i += GLU ? 2 : 1) {
+      const int o = GLU ? (o0 + wo) / 2 + i * 8 + lg * 4
+                        : o0 + wo + i * 16 + lg * 4;
       f32x4 v = acc[i][j];
-      if (a.act)
 #pragma unroll
-        for (int k = 0; k < 4; ++k) {
+      for (int k = 0; k < 4; ++k) {
+        v[k] *= scale;
+        if constexpr (GLU) {
+          v[k] = clamped_glu_of<T>(v[k], acc[i + 1][j][k] * scale, a.limit, a.alpha);
+        } else if (a.act == EX_RELU2) {
           v[k] = fmaxf(v[k], 0.0f);
           v[k] *= v[k];
         }
-      if (o + 4 <= a.O) {
+      }
+      if (o + 4 <= outs) {
         store4(out + o, v);  // rows of out begin at whole vectors
       } else {
 #pragma unroll
         for (int k = 0; k < 4; ++k)
-          if (o + k < a.O) out[o + k] = (T)v[k];
+          if (o + k < outs) out[o + k] = (T)v[k];
       }
     }
   }
@@ -537,22 +567,36 @@ __global__ __launch_bounds__(EX_BLOCK, 2) void expert_wide_kernel(
 
 extern "C" void launch_expert_gemm(const ExpertGemmArgs* a, int tile, bool f32,
                                    hipStream_t stream) {
+  const bool glu = a->act == EX_CLAMPED_GLU;
+  const dim3 block(EX_BLOCK);
   if (tile == 16) {
     const dim3 grid((unsigned)((a->O + SK_OUT - 1) / SK_OUT),
                     (unsigned)a->n_tiles);
-    if (f32)
-      expert_skinny_kernel<float><<<grid, dim3(EX_BLOCK), 0, stream>>>(*a);
-    else
-      expert_skinny_kernel<__bf16><<<grid, dim3(EX_BLOCK), 0, stream>>>(*a);
+#define EX_GO(T)                                                     \
+  do {                                                               \
+    if (glu)                                                         \
+      expert_skinny_kernel<T, true><<<grid, block, 0, stream>>>(*a); \
+    else                                                             \
+      expert_skinny_kernel<T, false><<<grid, block, 0, stream>>>(*a); \
+  } while (0)
+    if (f32) EX_GO(float);
+    else EX_GO(__bf16);
+#undef EX_GO
     return;
   }
   const size_t smem = 2 * 2 * WT_OUT * WT_BYTES;
   const long work = (long)((a->O + WT_OUT - 1) / WT_OUT) * a->n_tiles;
   const dim3 grid((unsigned)((work + 7) / 8 * 8));
-  if (f32)
-    expert_wide_kernel<float><<<grid, dim3(EX_BLOCK), smem, stream>>>(*a);
-  else
-    expert_wide_kernel<__bf16><<<grid, dim3(EX_BLOCK), smem, stream>>>(*a);
+#define EX_GO(T)                                                      \
+  do {                                                                \
+    if (glu)                                                          \
+      expert_wide_kernel<T, true><<<grid, block, smem, stream>>>(*a); \
+    else                                                              \
+      expert_wide_kernel<T, false><<<grid, block, smem, stream>>>(*a); \
+  } while (0)
+  if (f32) EX_GO(float);
+  else EX_GO(__bf16);
+#undef EX_GO
 }
 
 // ---------------------------------------------------------------------------

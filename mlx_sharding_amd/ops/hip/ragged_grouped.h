@@ -16,7 +16,8 @@
 // neither key nor value; it enters once, when a row is finished.  With a window
 // a token sees its last `window` tokens; pages before all of a block's windows
 // are not visited.  Where values were rotated by their positions, a finished
-// row is turned back by its own.
+// row is turned back by its own.  A gate multiplies a finished row of a head by
+// the sigmoid of one number.
 #pragma once
 
 #include "ragged_common.h"
@@ -33,7 +34,8 @@ struct GroupedRowArgs {
   const float *qk_cos, *qk_sin, *v_cos, *v_sin;
   int qk_pairs, v_pairs;
   const int* tok_pos;
-  bool head_norm;  // queries and keys over their own root mean squares
+  bool head_norm;  // queries and keys over their own root mean squares, times
+                   // weights [D] if wq, wk are given
 };
 
 struct GroupedAttnArgs {
@@ -49,6 +51,8 @@ struct GroupedAttnArgs {
   int window;                 // 0: every earlier token is seen
   const float *v_cos, *v_sin; // [positions, V / 2] or null
   const int* tok_pos;
+  const void* gate;           // [tokens, H] or null
+  long gstride;
 };
 
 #define GA_BLOCK 256
@@ -122,6 +126,14 @@ __device__ __forceinline__ f32x4 turn_back(const GroupedAttnArgs& a, int pos,
   const float* s = a.v_sin + (long)pos * half;
   return f32x4{v[0] * c[p] + v[1] * s[p], v[1] * c[p] - v[0] * s[p],
                v[2] * c[q] + v[3] * s[q], v[3] * c[q] - v[2] * s[q]};
+}
+
+// what a head's finished row of a token is multiplied by
+template <typename T>
+__device__ __forceinline__ float gate_of(const GroupedAttnArgs& a, long tok,
+                                         int h) {
+  return a.gate ? sigmoid_f((float)((const T*)a.gate)[tok * a.gstride + h])
+                : 1.0f;
 }
 
 // the first token that one at `pos` sees
@@ -276,7 +288,7 @@ __global__ __launch_bounds__(GA_BLOCK) void grouped_attn_short_kernel(
   const float mine = sm_exp<T>(m_run - M);
   if (tid < 16) {
     if (last) {
-      sw[lr] = 1.0f / L;
+      sw[lr] = gate_of<T>(a, t0 + my_tok, my_head) / L;
     } else {
       sw[lr] = 1.0f;
       if (r0 + lr < rows) {
@@ -342,7 +354,7 @@ __global__ __launch_bounds__(128) void grouped_attn_merge_kernel(
     const float e = s < n ? sm_exp<T>(ms - M) : 0.0f;
     float L = wave_sum(s < n ? ml[2 * s + 1] * e : 0.0f);
     if (a.sink) L += sm_exp<T>(sink - M);
-    w[s] = e / L;
+    w[s] = e / L * gate_of<T>(a, row / a.H, h);
   }
   __syncthreads();
   T* out = (T*)a.out + row / a.H * a.ostride + (long)h * a.V;
@@ -579,6 +591,7 @@ void grouped_attn_long_kernel(
       f = sm_exp<T>(m_run[i] - M);
       f /= l_run[i] * f + sm_exp<T>(sink - M);
     }
+    f *= gate_of<T>(a, t0 + r, h);
     T* o = (T*)a.out + (long)(t0 + r) * a.ostride + (long)h * a.V;
 #pragma unroll
     for (int d = 0; d < ND; ++d) {

@@ -1,6 +1,6 @@
 // Row work around grouped attention: norms of the projections, rotations,
-// blended values, writing keys and values to their pages; exact gelu; capped
-// logits.
+// blended values, writing keys and values to their pages; exact gelu; clamped
+// gated units; capped logits.
 #include "ragged_grouped.h"
 
 #define GR_BLOCK 256
@@ -235,15 +235,15 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_append_kernel(
   }
 }
 
-// The same with rotations and norms per head: `sub` lanes (a power of two) share
+// The same with norms per head and rotations: `sub` lanes (a power of two) share
 // one head of one token, each eight of its columns.  Items of a token are its
-// query heads, keys and values; keys' inverse rms [N, G].
+// query heads, keys and values, or the query heads alone; keys' inverse rms
+// [N, G].
 template <typename T, bool VEC>
 __global__ __launch_bounds__(GR_BLOCK) void grouped_turn_kernel(
     const GroupedRowArgs a, T* __restrict__ q, float* __restrict__ kinv,
     const int* __restrict__ tok_entry, const int* __restrict__ pages, int P,
-    int direct, int sub, long n_tok) {
-  const int items = a.H + 2 * a.G;
+    int direct, int sub, long n_tok, int items) {
   const long at = ((long)blockIdx.x * GR_BLOCK + threadIdx.x) / sub;
   const int c = threadIdx.x % sub * 8;
   const long t = min(at / items, n_tok - 1);
@@ -256,17 +256,21 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_turn_kernel(
                  (value ? (long)(a.H + a.G) * a.D + (long)(j - a.H - a.G) * a.V
                         : (long)j * a.D);
   f32x8 v = head8<T, VEC>(src, c, size);
-  if (value)
-    v = turn8(v, a.v_cos, a.v_sin, a.v_pairs, pos, c);
-  else
-    v = turn8(v, a.qk_cos, a.qk_sin, a.qk_pairs, pos, c);
   if (a.head_norm) {
     float ss = squares(v);
     for (int o = 1; o < sub; o <<= 1) ss += __shfl_xor(ss, o, WAVE);
     const float inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
-    if (!value) v = v * inv;
+    if (!value) {
+      v = v * inv;
+      const T* w = (const T*)(j < a.H ? a.wq : a.wk);
+      if (w) v = v * head8<T, VEC>(w, c, a.D);
+    }
     if (live && c == 0 && !value && j >= a.H) kinv[t * a.G + j - a.H] = inv;
   }
+  if (value)
+    v = turn8(v, a.v_cos, a.v_sin, a.v_pairs, pos, c);
+  else
+    v = turn8(v, a.qk_cos, a.qk_sin, a.qk_pairs, pos, c);
   if (!live) return;
   if (j < a.H) {
     if (c < a.dimp) store8(q + (t * a.H + j) * a.dimp + c, v);
@@ -294,7 +298,8 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_turn_kernel(
 // One block per (page, key/value head): the slots lo .. hi - 1 of a page from
 // tokens t + slot; later slots become zero, earlier ones stay.
 //   fills[i] = (page, t, lo, hi)
-// TURN: rotations and norms per head in place of weights and blended values.
+// TURN: norms per head (wk is one head's weights) and rotations in place of
+// norms of rows and blended values.
 template <typename T, bool VEC, bool TURN>
 __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
     const GroupedRowArgs a, const float* __restrict__ kinv,
@@ -306,7 +311,7 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
   const int lo = f[2], hi = f[3];
   const int tid = threadIdx.x;
   const T* y = (const T*)a.y;
-  const T* wk = a.wk ? (const T*)a.wk + g * a.D : nullptr;
+  const T* wk = a.wk ? (const T*)a.wk + (TURN ? 0 : g * a.D) : nullptr;
   const long koff = (long)(a.H + g) * a.D;
   const long voff = (long)(a.H + a.G) * a.D + (long)g * a.V;
   T* base = (T*)a.pool +
@@ -322,8 +327,9 @@ __global__ __launch_bounds__(GR_BLOCK) void grouped_fill_kernel(
     if (s < hi) {
       v = head8<T, VEC>(y + (t + s) * a.ystride + koff, c, a.D);
       if constexpr (TURN) {
-        v = turn8(v, a.qk_cos, a.qk_sin, a.qk_pairs, a.tok_pos[t + s], c);
         if (a.head_norm) v = v * kinv[(t + s) * a.G + g];
+        if (wk) v = v * head8<T, VEC>(wk, c, a.D);
+        v = turn8(v, a.qk_cos, a.qk_sin, a.qk_pairs, a.tok_pos[t + s], c);
       } else {
         if (wk) v = v * kinv[t + s] * head8<T, VEC>(wk, c, a.D);
       }
@@ -402,14 +408,16 @@ extern "C" void launch_grouped_append(const GroupedRowArgs* a, void* q,
 extern "C" void launch_grouped_turn(const GroupedRowArgs* a, void* q,
                                     float* kinv, const int* tok_entry,
                                     const int* pages, int P, int direct,
-                                    long n_tok, bool f32, hipStream_t stream) {
+                                    long n_tok, bool own, bool f32,
+                                    hipStream_t stream) {
   int sub = 1;
   while (sub * 8 < a->dimp || sub * 8 < a->vdp) sub *= 2;
-  const long lanes = n_tok * (a->H + 2 * a->G) * sub;
+  const int items = a->H + (own ? 2 * a->G : 0);
+  const long lanes = n_tok * items * sub;
   dim3 grid((unsigned)((lanes + GR_BLOCK - 1) / GR_BLOCK)), block(GR_BLOCK);
 #define GR_GO(T, VEC)                                                        \
   grouped_turn_kernel<T, VEC><<<grid, block, 0, stream>>>(                   \
-      *a, (T*)q, kinv, tok_entry, pages, P, direct, sub, n_tok)
+      *a, (T*)q, kinv, tok_entry, pages, P, direct, sub, n_tok, items)
   if (f32) {
     if (a->vec) GR_GO(float, true);
     else GR_GO(float, false);
@@ -503,6 +511,53 @@ extern "C" void launch_gelu(const void* x, void* o, long rows, int C, long xs,
     if (vec) { GR_GO(float, true) } else { GR_GO(float, false) }
   } else {
     if (vec) { GR_GO(__bf16, true) } else { GR_GO(__bf16, false) }
+  }
+#undef GR_GO
+}
+
+// ---------------------------------------------------------------------------
+// Clamped gated unit on strided rows: g sigmoid(alpha g) (u + 1), g at most
+// limit, u within +-limit.
+// ---------------------------------------------------------------------------
+
+template <typename T, bool VEC>
+__global__ __launch_bounds__(GR_BLOCK) void clamped_glu_kernel(
+    const T* __restrict__ gate, const T* __restrict__ up, T* __restrict__ o,
+    long rows, int C, long gs, long us, float limit, float alpha) {
+  constexpr int V = VEC ? 8 : 1;
+  const int per = C / V;  // whole vectors, or elements
+  const long total = rows * per, step = (long)gridDim.x * GR_BLOCK;
+  for (long i = (long)blockIdx.x * GR_BLOCK + threadIdx.x; i < total; i += step) {
+    const long r = i / per;
+    const int c = (int)(i - r * per) * V;
+    if constexpr (VEC) {
+      f32x8 g = load8(gate + r * gs + c);
+      const f32x8 u = load8(up + r * us + c);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) g[j] = clamped_glu_of<T>(g[j], u[j], limit, alpha);
+      store8(o + r * C + c, g);
+    } else {
+      o[r * C + c] = (T)clamped_glu_of<T>((float)gate[r * gs + c],
+                                       (float)up[r * us + c], limit, alpha);
+    }
+  }
+}
+
+extern "C" void launch_clamped_glu(const void* gate, const void* up, void* o,
+                                   long rows, int C, long gs, long us,
+                                   float limit, float alpha, bool vec, bool f32,
+                                   hipStream_t stream) {
+  const long want = (rows * (vec ? C / 8 : C) + GR_BLOCK - 1) / GR_BLOCK;
+  dim3 grid((unsigned)(want < 16384 ? want : 16384)), block(GR_BLOCK);
+#define GR_GO(T, VEC)                                                     \
+  clamped_glu_kernel<T, VEC><<<grid, block, 0, stream>>>(                 \
+      (const T*)gate, (const T*)up, (T*)o, rows, C, gs, us, limit, alpha)
+  if (f32) {
+    if (vec) GR_GO(float, true);
+    else GR_GO(float, false);
+  } else {
+    if (vec) GR_GO(__bf16, true);
+    else GR_GO(__bf16, false);
   }
 #undef GR_GO
 }

@@ -8,10 +8,12 @@
 // One sublayer boundary in one kernel, one block per row:
 //   x += mult * rms(y) * (w_post + off)   (y == null: x unchanged;
 //                                          w_post == null: x += mult * y)
-//   h  = rms(x) * (w_next + off)      (w_next == null: no h)
+//   h  = rms(x) * (w_next + off)      (w_next == null: h = x; h == null: no h)
 // x is the fp32 residual; y and h are T; w_next holds W weights or one for all
-// (one_next).  NR > 0 keeps the row in registers
-// (NR groups of VEC elements per thread); NR == 0 re-reads it.
+// (one_next).  Rows of h have Wh columns, those past W become zero.  NR > 0
+// keeps the row in registers (NR groups of VEC elements per thread); NR == 0
+// re-reads it.  SUM: row i of y is the sum of its rows where[i, 0 .. top - 1],
+// -1 for none.
 // ---------------------------------------------------------------------------
 
 template <typename T, int VEC>
@@ -33,65 +35,95 @@ __device__ __forceinline__ void rn_store(T* p, const float (&o)[VEC]) {
   }
 }
 
-template <typename T, int VEC, int NR>
+struct AddNormArgs {
+  float* x;
+  const void *y, *w_post, *w_next;
+  void* h;
+  const int* where;
+  long rows, ystride;
+  int W, Wh, top;
+  float eps, off, mult;
+  bool one_next;
+};
+
+template <typename T, int VEC, int NR, bool SUM>
 __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
-    float* __restrict__ x, const T* __restrict__ y, long ystride,
-    const T* __restrict__ w_post, const T* __restrict__ w_next,
-    T* __restrict__ h, int W, float eps, float off, float mult, bool one_next) {
+    const AddNormArgs a) {
   __shared__ float scratch[RN_BLOCK / WAVE];
   const long row = blockIdx.x;
-  float* xr = x + row * W;
-  const T* yr = y ? y + row * ystride : nullptr;
-  T* hr = h ? h + row * W : nullptr;
+  const int W = a.W;
+  float* xr = a.x + row * W;
+  const T* y = (const T*)a.y;
+  const T* w_post = (const T*)a.w_post;
+  const T* w_next = (const T*)a.w_next;
+  T* hr = a.h ? (T*)a.h + row * a.Wh : nullptr;
   const int step = RN_BLOCK * VEC;
   constexpr int NA = NR > 0 ? NR : 1;
   float xv[NA][VEC];
 
-  float inv_y = mult;
+  auto load_y = [&](int c, float (&o)[VEC]) {
+    if constexpr (SUM) {
+      const int* from = a.where + row * a.top;
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = 0.0f;
+#pragma unroll 4
+      for (int k = 0; k < a.top; ++k) {
+        if (from[k] < 0) continue;
+        float part[VEC];
+        rn_load<T, VEC>(y + from[k] * a.ystride + c, part);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) o[j] += part[j];
+      }
+    } else {
+      rn_load<T, VEC>(y + row * a.ystride + c, o);
+    }
+  };
+
+  float inv_y = a.mult;
   float yv[NA][VEC];
-  if (yr && !w_post) {
+  if (y && !w_post) {
     if constexpr (NR > 0) {
 #pragma unroll
       for (int i = 0; i < NR; ++i) {
         const int c = i * step + threadIdx.x * VEC;
-        if (c < W) rn_load<T, VEC>(yr + c, yv[i]);
+        if (c < W) load_y(c, yv[i]);
       }
     }
-  } else if (yr) {
+  } else if (y) {
     float ss = 0.0f;
     if constexpr (NR > 0) {
 #pragma unroll
       for (int i = 0; i < NR; ++i) {
         const int c = i * step + threadIdx.x * VEC;
         if (c < W) {
-          rn_load<T, VEC>(yr + c, yv[i]);
+          load_y(c, yv[i]);
 #pragma unroll
           for (int j = 0; j < VEC; ++j) ss += yv[i][j] * yv[i][j];
         }
       }
     } else {
       for (int c = threadIdx.x * VEC; c < W; c += step) {
-        rn_load<T, VEC>(yr + c, yv[0]);
+        load_y(c, yv[0]);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) ss += yv[0][j] * yv[0][j];
       }
     }
     ss = block_sum<RN_BLOCK>(ss, scratch);
-    inv_y = mult / sqrtf(ss / (float)W + eps);
+    inv_y = a.mult / sqrtf(ss / (float)W + a.eps);
   }
 
   float ss = 0.0f;
   auto update = [&](int c, float (&xa)[VEC], float (&ya)[VEC]) {
     rn_load<float, VEC>(xr + c, xa);
-    if (yr && !w_post) {
+    if (y && !w_post) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) xa[j] += ya[j] * inv_y;
       rn_store<float, VEC>(xr + c, xa);
-    } else if (yr) {
+    } else if (y) {
       float wv[VEC];
       rn_load<T, VEC>(w_post + c, wv);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) xa[j] += ya[j] * inv_y * (wv[j] + off);
+      for (int j = 0; j < VEC; ++j) xa[j] += ya[j] * inv_y * (wv[j] + a.off);
       rn_store<float, VEC>(xr + c, xa);
     }
 #pragma unroll
@@ -105,24 +137,32 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
     }
   } else {
     for (int c = threadIdx.x * VEC; c < W; c += step) {
-      if (yr) rn_load<T, VEC>(yr + c, yv[0]);
+      if (y) load_y(c, yv[0]);
       update(c, xv[0], yv[0]);
     }
   }
   if (!hr) return;
-  ss = block_sum<RN_BLOCK>(ss, scratch);
-  const float inv = 1.0f / sqrtf(ss / (float)W + eps);
-  const float one = one_next ? (float)w_next[0] : 0.0f;
+  for (int c = W + threadIdx.x; c < a.Wh; c += RN_BLOCK) hr[c] = (T)0.0f;
+  float inv = 1.0f;
+  if (w_next) {
+    ss = block_sum<RN_BLOCK>(ss, scratch);
+    inv = 1.0f / sqrtf(ss / (float)W + a.eps);
+  }
+  const float one = a.one_next ? (float)w_next[0] : 0.0f;
   auto emit = [&](int c, float (&xa)[VEC]) {
+    if (!w_next) {
+      rn_store<T, VEC>(hr + c, xa);
+      return;
+    }
     float wv[VEC], o[VEC];
-    if (one_next) {
+    if (a.one_next) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) wv[j] = one;
     } else {
       rn_load<T, VEC>(w_next + c, wv);
     }
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) o[j] = xa[j] * inv * (wv[j] + off);
+    for (int j = 0; j < VEC; ++j) o[j] = xa[j] * inv * (wv[j] + a.off);
     rn_store<T, VEC>(hr + c, o);
   };
   if constexpr (NR > 0) {
@@ -140,18 +180,18 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
 }
 
 template <typename T>
-static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
-                       const void* wn, void* h, long rows, int W, float eps,
-                       float off, float mult, bool one_next,
-                       hipStream_t stream) {
-  const bool vec = W % 4 == 0 && ystride % 4 == 0 &&
-                   ((uintptr_t)y) % 16 == 0;
-  const int nr = (W + RN_BLOCK * 4 - 1) / (RN_BLOCK * 4);
-  dim3 grid((unsigned)rows), block(RN_BLOCK);
-#define RN_GO(V, N)                                                        \
-  add_norm_kernel<T, V, N><<<grid, block, 0, stream>>>(                    \
-      (float*)x, (const T*)y, ystride, (const T*)wp, (const T*)wn, (T*)h, W, \
-      eps, off, mult, one_next)
+static void add_norm_t(const AddNormArgs& a, hipStream_t stream) {
+  const bool vec = a.W % 4 == 0 && a.Wh % 4 == 0 && a.ystride % 4 == 0 &&
+                   ((uintptr_t)a.y) % 16 == 0;
+  const int nr = (a.W + RN_BLOCK * 4 - 1) / (RN_BLOCK * 4);
+  dim3 grid((unsigned)a.rows), block(RN_BLOCK);
+#define RN_GO(V, N)                                                 \
+  do {                                                              \
+    if (a.where)                                                    \
+      add_norm_kernel<T, V, N, true><<<grid, block, 0, stream>>>(a); \
+    else                                                            \
+      add_norm_kernel<T, V, N, false><<<grid, block, 0, stream>>>(a); \
+  } while (0)
   if (!vec)
     RN_GO(1, 0);
   else if (nr <= 1)
@@ -167,17 +207,12 @@ static void add_norm_t(void* x, const void* y, long ystride, const void* wp,
 #undef RN_GO
 }
 
-extern "C" void launch_add_norm(void* x, const void* y, long ystride,
-                                const void* wp, const void* wn, void* h,
-                                long rows, int W, float eps, float off,
-                                float mult, bool one_next, bool f32,
+extern "C" void launch_add_norm(const AddNormArgs* a, bool f32,
                                 hipStream_t stream) {
   if (f32)
-    add_norm_t<float>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult, one_next,
-                    stream);
+    add_norm_t<float>(*a, stream);
   else
-    add_norm_t<__bf16>(x, y, ystride, wp, wn, h, rows, W, eps, off, mult,
-                       one_next, stream);
+    add_norm_t<__bf16>(*a, stream);
 }
 
 // ---------------------------------------------------------------------------

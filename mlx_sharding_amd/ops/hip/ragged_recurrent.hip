@@ -391,26 +391,6 @@ __device__ __forceinline__ float decay_exp<float>(float x) {
   return expf(x);
 }
 
-// ln(1 + e^d).  For bf16 operands: the logarithm of 1 + u from the instruction
-// where u is not small, else its series; both to about 1e-6 of the result.
-template <typename T>
-__device__ __forceinline__ float step_size(float d);
-template <>
-__device__ __forceinline__ float step_size<float>(float d) {
-  return softplus_f(d);
-}
-template <>
-__device__ __forceinline__ float step_size<__bf16>(float d) {
-  const float u = __builtin_amdgcn_exp2f(-1.44269504088896340736f * fabsf(d));
-  const float large = 0.69314718055994530942f * __builtin_amdgcn_logf(1.0f + u);
-  // u - u^2/2 + ... + u^5/5, off by u^6/6
-  float small = fmaf(u, 0.2f, -0.25f);
-  small = fmaf(u, small, 0.33333333333333333333f);
-  small = fmaf(u, small, -0.5f);
-  small = fmaf(u, small * u, u);
-  return fmaxf(d, 0.0f) + (u < 0.04f ? small : large);
-}
-
 typedef const __attribute__((address_space(4))) unsigned* ScalarWords;
 
 template <int NS>
@@ -523,7 +503,7 @@ struct ScanLane {
 #pragma unroll
       for (int u = 0; u < SS_AHEAD; ++u) {
         if (t + u >= n) break;
-        const float step = step_size<T>(d[u]);
+        const float step = softplus_of<T>(d[u]);
         const float in = step * x[u];
         float B[NS], C[NS];
         load_coeffs<T, NS, PARTS>(bp + (long)(t + u) * a.bs + a.b0, part, B);

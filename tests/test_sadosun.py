@@ -842,7 +842,10 @@ def test_kernels_refuse_bad_operands():
     pool = torch.zeros(640, 2 * 48, **dev)
     sizes = (4, 2, 32, 16, 32, 16, batch.tok_pos, batch.tok_entry, batch.pages, 20)
     y = torch.zeros(20, 4 * 32 + 2 * 32 + 2 * 16, **dev)
-    conv(), scan()
+    turn = lambda cos, sin: ext.grouped_turn(  # noqa: E731
+        y, None, None, 1e-6, True, cos, sin, None, None, pool, *sizes, True)
+    soft, none = (False, True), (0, 0.0, 0.0)
+    conv(), scan(), turn(tab, tab)
     bad = (
         lambda: conv(w=torch.zeros(9, 64, **dev)),
         lambda: conv(hist=hist[:, :2].contiguous()),
@@ -854,18 +857,18 @@ def test_kernels_refuse_bad_operands():
         lambda: scan(A=torch.zeros(12, 8, **dev)),
         lambda: scan(bc=torch.zeros(20, 32, **dev)),
         lambda: scan(state=torch.zeros(2, 1, 8, 16, **dev)),
-        lambda: ext.expert_route(h[:, :32], router, torch.zeros(5, **dev), 4, 2),
-        lambda: ext.expert_route(h, router, torch.zeros(17, **dev), 4, 2),
-        lambda: ext.expert_route(h, router, torch.zeros(5, **dev), 4, 6),
-        lambda: ext.expert_plan(idx, idx, torch.zeros(1, 3, dtype=torch.int32, **dev), 3, 16),
-        lambda: ext.expert_gemm(h, idx.view(-1), tiles, up, 32, 40, False),
-        lambda: ext.expert_gemm(h, None, tiles, up, 16, 40, False),
-        lambda: ext.expert_gemm(h[:, :32], idx.view(-1), tiles, up, 16, 40, False),
+        lambda: ext.expert_route(h[:, :32], router, torch.zeros(5, **dev), 5, 4, 2, *soft),
+        lambda: ext.expert_route(h, router, torch.zeros(17, **dev), 5, 4, 2, *soft),
+        lambda: ext.expert_route(h, router, torch.zeros(17, **dev), 17, 4, 2, *soft),
+        lambda: ext.expert_route(h, router, torch.zeros(5, **dev), 5, 4, 6, *soft),
+        lambda: ext.expert_plan(idx, idx, torch.zeros(1, 3, dtype=torch.int32, **dev), None, 3, 16),
+        lambda: ext.expert_gemm(h, idx.view(-1), tiles, up, None, 32, 40, *none),
+        lambda: ext.expert_gemm(h, None, tiles, up, None, 16, 40, *none),
+        lambda: ext.expert_gemm(h[:, :32], idx.view(-1), tiles, up, None, 16, 40, *none),
         lambda: ext.token_gate(h, router, torch.zeros(20, 17, **dev)),
-        lambda: ext.grouped_turn(y, 1e-6, True, tab[:, :4], tab[:, :4], None, None, pool, *sizes),
-        lambda: ext.grouped_turn(y, 1e-6, True, torch.zeros(64, 20, **dev), torch.zeros(64, 20, **dev),
-                                 None, None, pool, *sizes),
-        lambda: ext.grouped_turn(y, 1e-6, True, tab, None, None, None, pool, *sizes),
+        lambda: turn(tab[:, :4], tab[:, :4]),
+        lambda: turn(torch.zeros(64, 20, **dev), torch.zeros(64, 20, **dev)),
+        lambda: turn(tab, None),
         lambda: ext.grouped_attn_short(
             torch.zeros(20, 4, 32, **dev), None, pool, torch.zeros(20, 64, **dev), batch.cu,
             batch.pos0, batch.pages, 1, 20, 20, 20, 2, 16, 16, 1.0, 0, tab[:, :4].contiguous(),

@@ -441,9 +441,9 @@ def test_kernels_refuse_bad_operands():
     x = torch.randn(4, 64, device="cuda")
     w = torch.randn(64, device="cuda")
     with pytest.raises(RuntimeError):
-        ext.add_norm(x, x.bfloat16(), w, w, w, 1e-6, 1.0)
+        ext.add_norm(x, x.bfloat16(), w, w, True, 1e-6, 1.0, 1.0, None, 64)
     with pytest.raises(RuntimeError):
-        ext.add_norm(x, None, None, w[:32], w, 1e-6, 1.0)
+        ext.add_norm(x, None, None, w[:32], True, 1e-6, 1.0, 1.0, None, 64)
     with pytest.raises(RuntimeError):
         ext.latent_gather(torch.zeros(100, 64, device="cuda"),
                           torch.zeros(1, 3, device="cuda", dtype=torch.int32), 64)
