@@ -55,13 +55,15 @@ def parse_args():
                    help="instead of the serving benchmark: prefill and decode "
                         "throughput of Tuvutar layers beside DeepSeek-V2's "
                         "dense latent-attention layers, of Lepizen layers "
-                        "beside Llama's and of Sadosun layers beside "
-                        "DeepSeek-V2's with routed experts, each of equal size, "
+                        "beside Llama's, of Sadosun layers beside "
+                        "DeepSeek-V2's with routed experts and of Dufinex "
+                        "layers beside all of these, each of equal size, "
                         "one JSON line per case (2048, 4096 or all)")
     p.add_argument("--kinds", default=None, metavar="NAME,...",
                    help="the stacks --layers times (default: all; mla, latent, "
                         "shared, delta, mixed, llama, lepizen, moe, windowed, "
-                        "scan, sadosun)")
+                        "scan, sadosun, gated, reader, channel, routed, "
+                        "dufinex)")
     return p.parse_args()
 
 

@@ -15,6 +15,11 @@ sizes, latent size and feed-forward, so that their times compare directly:
   windowed  Sadosun windowed attention + routed experts
   scan    Sadosun selective scan + routed experts
   sadosun Sadosun scan, windowed, windowed, scan
+  gated   Dufinex attention + dense MLP (beside llama)
+  reader  the same, three of four layers on another's keys and values
+  channel Dufinex delta rule with decays per channel + dense MLP (beside delta)
+  routed  Dufinex attention + routed experts (beside moe: equal experts)
+  dufinex Dufinex delta, attention, attention on shared keys, delta + experts
 
 All run the pipeline worker's own prefill and graph-captured decode step.
 """
@@ -29,8 +34,8 @@ import torch
 
 from ..config import ModelConfig
 from ..parallel.rccl import PipelineWorker, build_stage_model
-from .presets import (_dense_mla, _lepizen, _llama, _moe_mla, _sadosun,
-                      _tuvutar)
+from .presets import (_dense_mla, _dufinex, _lepizen, _llama, _moe_mla,
+                      _sadosun, _tuvutar)
 
 SIZES: Dict[str, dict] = {
     "2048": dict(width=2048, heads=16, ff=8192, vocab=8192),
@@ -38,8 +43,11 @@ SIZES: Dict[str, dict] = {
 }
 TUVUTAR = {"latent": "aaaa", "shared": "asss", "delta": "dddd", "mixed": "ddda"}
 SADOSUN = {"windowed": "aaaa", "scan": "mmmm", "sadosun": "maam"}
+DUFINEX = {"gated": "aaaa", "reader": "asss", "channel": "dddd",
+           "routed": "AAAA", "dufinex": "dasD"}
 EXPERT_FF = {"2048": 1408, "4096": 1536}
-KINDS = ("mla", *TUVUTAR, "llama", "lepizen", "moe", *SADOSUN)
+KINDS = ("mla", *TUVUTAR, "llama", "lepizen", "moe", *SADOSUN,
+         *DUFINEX)
 PREFILL = ((1, 8192), (8, 1024))     # sequences, tokens each
 DECODE = ((1, 2048), (64, 2048))     # sequences, tokens cached
 
@@ -51,6 +59,11 @@ def stack(kind: str, size: dict) -> ModelConfig:
         make = _llama if kind == "llama" else _lepizen
         return ModelConfig.from_dict(
             make(n_layers=4, kv_heads=size["heads"] // 4, **size))
+    if kind in DUFINEX:
+        heads = size["heads"]
+        return ModelConfig.from_dict(_dufinex(
+            period=DUFINEX[kind], kv_heads=heads // 4, delta_heads=heads,
+            delta_kv=heads // 2, expert_ff=EXPERT_FF[str(size["width"])], **size))
     if kind == "moe" or kind in SADOSUN:
         size = {**size, "ff": EXPERT_FF[str(size["width"])]}
         if kind == "moe":
@@ -66,11 +79,11 @@ def stack(kind: str, size: dict) -> ModelConfig:
 
 def _spread(model):
     """Random router weights, not random biases of the choice, pick the experts;
-    they see normed rows."""
+    they see rows of an ordinary size."""
     for name, p in model.named_parameters():
         if name.endswith(".correction"):
             p.data.zero_()
-        elif p.dim() == 0 and ".norm" in name:
+        elif p.dim() <= 1 and ".norm" in name:
             p.data.fill_(1.0)
 
 
@@ -93,7 +106,7 @@ def run(which: str = "all", steps: int = 32,
         for kind in kinds or KINDS:
             config = stack(kind, SIZES[name])
             model = build_stage_model(config, 0, 1, device)
-            if kind in SADOSUN:
+            if kind in SADOSUN or kind in DUFINEX:
                 _spread(model)
 
             def emit(phase, batch, seq, seconds, tokens):

@@ -74,6 +74,38 @@ def _sadosun(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
             "layers": layers}
 
 
+def _dufinex(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
+             period: str, repeats: int = 1, dim: int = 128, expert_ff: int = 0,
+             experts: int = 64, top: int = 6, delta_heads: int = 0,
+             delta_kv: int = 0, rank: int = 128, scale: float = 50.0) -> dict:
+    """A Dufinex config: ``period`` repeated, "d" a delta layer, "a" an attention
+    layer, "s" one that reads the keys and values of the latest "a"; capitals
+    have routed experts in place of a dense feed-forward."""
+    layers, last = [], None
+    for kind in period * repeats:
+        low = kind.lower()
+        if low == "d":
+            mixer = {"heads": delta_heads or heads, "kv_heads": delta_kv or heads,
+                     "dim": 128, "vdim": 128, "conv": 4, "decay_rank": rank,
+                     "gate_rank": rank}
+        else:
+            mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                     "vdim": dim, "scale": dim ** -0.5}
+            if low == "s":
+                mixer["kv_from"] = last
+            else:
+                last = len(layers)
+        mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+        if kind != low:
+            mlp = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0},
+                   "router": {"experts": experts, "top": top}}
+        layers.append({"type": "channel_delta" if low == "d" else "attention",
+                       "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Dufinex", "width": width, "vocab": vocab,
+            "norm": {"eps": 1e-6}, "embedding": {"scale": scale},
+            "layers": layers}
+
+
 def _llama(width: int, heads: int, kv_heads: int, ff: int, vocab: int,
            n_layers: int) -> dict:
     return {"model_type": "llama", "hidden_size": width,
@@ -221,6 +253,27 @@ PRESETS = {
     "lepizen-2b": _lepizen(2048, 16, 4, 8192, 32000, 28),
     "lepizen-8b": _lepizen(4096, 32, 8, 16384, 32000, 36),
     "sadosun-7b": _sadosun(2048, 16, 4, 1024, 32000, "maamaa", 4),
+    "dufinex-7b": _dufinex(2048, 16, 4, 8192, 32000, "dDaDdDsD", 3,
+                           expert_ff=1024),
+    "debug-dufinex": {
+        "architecture": "Dufinex", "width": 80, "vocab": 320,
+        "norm": {"eps": 1e-5}, "embedding": {"scale": 0.8},
+        "layers": [
+            {"type": "attention",
+             "mixer": {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 16,
+                       "scale": 0.2},
+             "mlp": {"kind": "moe", "expert": {"ff": 40, "limit": 2.0},
+                     "router": {"experts": 5, "top": 2}}},
+            {"type": "channel_delta",
+             "mixer": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24,
+                       "conv": 3, "decay_rank": 12, "gate_rank": 8},
+             "mlp": {"kind": "dense", "ff": 112, "limit": 3.0}},
+            {"type": "attention",
+             "mixer": {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 16,
+                       "scale": 0.2, "kv_from": 0},
+             "mlp": None},
+        ],
+    },
     "debug-sadosun": {
         "architecture": "Sadosun", "width": 80, "vocab": 320,
         "norm": {"eps": 1e-6}, "embedding": {"scale": 4.0},
