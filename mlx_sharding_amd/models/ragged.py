@@ -52,8 +52,8 @@ class RaggedStageModel(StageModel):
         self._tables: Dict = {}
         self._old_tables: List = []  # captured graphs may still read them
         for i in owned_layer_indices(shard):
-            j = self.row_source(config, i)
-            if j != i and not (shard.owns(j) and j < i):
+            j = config["layers"][i]["mixer"].get("kv_from")
+            if j is not None and not (shard.owns(int(j)) and int(j) < i):
                 raise ValueError(
                     f"layer {i} reads the rows of layer {j}, which stage "
                     f"[{shard.start_layer}, {shard.end_layer}) does not run "

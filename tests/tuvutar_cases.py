@@ -125,8 +125,10 @@ def build(cfg, w, device="cpu", dtype=torch.float32, start=None, end=None):
     from mlx_sharding_amd.config import ModelConfig
     from mlx_sharding_amd.models import get_model_class
     from mlx_sharding_amd.models.fuse import fuse_model
-    mc = ModelConfig.from_dict(cfg)
-    m = get_model_class(mc.model_type)(mc, mc.shard(start, end))
+    mc = ModelConfig.from_dict(json.loads(json.dumps(cfg)))
+    cls = get_model_class(mc.model_type)
+    cls.complete_config(mc, w)
+    m = cls(mc, mc.shard(start, end))
     m.to(dtype)
     m.load_weights(w)
     m.to(device).eval()
