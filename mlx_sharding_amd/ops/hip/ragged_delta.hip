@@ -642,8 +642,9 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(
 #define DCH_STEPS 4                    // steps of 16 channels between barriers
 #define DCH_LS (DCH_STEPS * 16 + 4)
 
-template <typename T>
-__global__ __launch_bounds__(256) void delta_chunk_channels_kernel(
+// VEC: channels and rows of z are whole vectors of 4.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256, 2) void delta_chunk_channels_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn,
     const T* __restrict__ z, const T* __restrict__ A_log,
     const T* __restrict__ dt_bias, const float* __restrict__ bt,
@@ -690,19 +691,36 @@ __global__ __launch_bounds__(256) void delta_chunk_channels_kernel(
 
   for (int d0 = 0; d0 < Dp; d0 += DCH_STEPS * 16) {
     f32x4 ka[DCH_STEPS], qa[DCH_STEPS], kb[DCH_STEPS];
+    f32x4 za[DCH_STEPS], dt[DCH_STEPS];
+    // everything a slice reads is asked for first
+#pragma unroll
+    for (int s = 0; s < DCH_STEPS; ++s) {
+      const int ds = min(d0 + s * 16, Dp - 16), d = ds + g4 * 4;
+      ka[s] = load4(kp + ds);
+      qa[s] = load4(qp + ds);
+      if constexpr (VEC) {
+        const int dc = min(d, D - 4);
+        za[s] = load4(zp + dc);
+        dt[s] = load4(dp + dc);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int dc = min(d + j, D - 1);
+          za[s][j] = (float)zp[dc];
+          dt[s][j] = (float)dp[dc];
+        }
+      }
+    }
 #pragma unroll
     for (int s = 0; s < DCH_STEPS; ++s) {
       const int ds = d0 + s * 16;
       if (ds >= Dp) continue;
-      const f32x4 k = in ? load4(kp + ds) : zero;
-      const f32x4 q = in ? load4(qp + ds) : zero;
+      const f32x4 k = in ? ka[s] : zero, q = in ? qa[s] : zero;
       f32x4 from, to = one;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const int d = ds + g4 * 4 + j;
-        const int dc = min(d, D - 1);
-        const float g = decay_of<T>((float)zp[dc], rate, (float)dp[dc]);
-        from[j] = in && d < D ? g : 1.0f;
+        const float g = decay_of<T>(za[s][j], rate, dt[s][j]);
+        from[j] = in && ds + g4 * 4 + j < D ? g : 1.0f;
         diag += q[j] * k[j];
       }
 #pragma unroll
@@ -1267,9 +1285,15 @@ static void delta_long_t(const DeltaLongArgs& a, const DeltaDims& dm,
   dim3 g3((unsigned)a.n_chunks, (unsigned)dm.H);
   dim3 g4((unsigned)(a.Vp / 16), (unsigned)dm.H, (unsigned)a.n_long);
   if (dm.channels) {
-    delta_chunk_channels_kernel<T><<<g3, block, 0, stream>>>(
-        a.qn, a.kn, (const T*)a.z, (const T*)a.A_log, (const T*)a.dt_bias, a.bt,
-        a.tm, a.am, a.qg, a.kg, a.kl, a.ge, a.chunks, a.tok_base, dm, a.Dp);
+    const bool vec = dm.D % 4 == 0 && dm.ac % 4 == 0 && dm.zstride % 4 == 0 &&
+                     ((uintptr_t)a.z | (uintptr_t)a.dt_bias) % 16 == 0;
+#define DCH_GO(V)                                                              \
+  delta_chunk_channels_kernel<T, V><<<g3, block, 0, stream>>>(                 \
+      a.qn, a.kn, (const T*)a.z, (const T*)a.A_log, (const T*)a.dt_bias, a.bt, \
+      a.tm, a.am, a.qg, a.kg, a.kl, a.ge, a.chunks, a.tok_base, dm, a.Dp)
+    if (vec) DCH_GO(true);
+    else DCH_GO(false);
+#undef DCH_GO
     delta_walk_t<T, true>(a, dm, a.qg, a.kg, a.kl, dm.H, g4, stream);
   } else {
     delta_chunk_kernel<<<g3, block, 0, stream>>>(
