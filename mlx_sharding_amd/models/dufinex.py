@@ -25,7 +25,7 @@ from ..ops.experts import ExpertShape, Routing
 from ..ops.paged import PagedState, RaggedBatch
 from ..ops.ragged import ClampedGLU
 from .base import RMSNorm
-from .mixers import GatedDelta, GatedMLP, GroupedAttention, RoutedExperts
+from .mixers import BiasedMLP, GatedDelta, GroupedAttention, RoutedExperts
 from .ragged import RaggedStageModel
 
 ROUTING = Routing(score="sigmoid", normalize=False, on_input=True)
@@ -48,8 +48,8 @@ def _mixer(kind: str, mx: dict, width: int, eps: float, dtype: torch.dtype):
 
 def _mlp(spec: dict, width: int, dtype: torch.dtype):
     if spec["kind"] == "dense":
-        return GatedMLP(width, int(spec["ff"]), ClampedGLU(float(spec["limit"])),
-                        dtype, bias=True)
+        return BiasedMLP(width, int(spec["ff"]),
+                         ClampedGLU(float(spec["limit"])), dtype)
     if spec["kind"] == "moe":
         expert, router = spec["expert"], spec["router"]
         return RoutedExperts(
@@ -121,14 +121,14 @@ class DufinexStageModel(RaggedStageModel):
         items = self.layer_items()
         first = self.shard.start_layer
 
-        def add(y, norm, after=None, where=None):
+        def add(y, norm, after=None, **of_y):
             """The residual moves on; returns what the next sublayer reads, or
             the rows of the norm that follows."""
             return ragged.add_norm(
                 x, y, None if norm is None else norm.weight,
                 None if after is None else after.weight, self.eps, 0.0, dtype,
-                where=where, copy=True,
-                pad_to=1 if after is not None else ExpertShape.STEP)
+                copy=True, pad_to=1 if after is not None else ExpertShape.STEP,
+                **of_y)
 
         h = add(None, None)
         for k, (i, layer) in enumerate(items):
@@ -144,9 +144,10 @@ class DufinexStageModel(RaggedStageModel):
                 h = add(y, layer.norm1)
                 if isinstance(layer.mlp, RoutedExperts):
                     y, where = layer.mlp.rows(h)
-                    h = add(y, layer.norm2, end, where)
+                    h = add(y, layer.norm2, end, where=where)
                 else:
-                    h = add(layer.mlp(h[:, :W]), layer.norm2, end)
+                    y, bias = layer.mlp.rows(h[:, :W])
+                    h = add(y, layer.norm2, end, y_bias=bias)
             if layer_outputs is not None:
                 layer_outputs.append(x.clone())
         if not self.shard.is_last:

@@ -75,7 +75,7 @@ def fuse_model(model) -> int:
     from .llama import LlamaAttention, LlamaMLP
     from .gemma2 import Gemma2Attention, Gemma2MLP
     from .deepseek_v2 import MLAAttention
-    from .mixers import (CausalConv, GatedDelta, GatedMLP, GroupedAttention,
+    from .mixers import (BiasedMLP, CausalConv, GatedDelta, GatedMLP, GroupedAttention,
                          LatentAttention, ParallelBlock, RoutedExperts,
                          SelectiveScan, TokenInput)
 
@@ -91,7 +91,7 @@ def fuse_model(model) -> int:
             elif isinstance(mod, MLAAttention) and not mod.q_lora_rank:
                 mod._fused_qkv = FusedColumns([mod.q_proj, mod.kv_a_proj_with_mqa])
                 n += 1
-            elif isinstance(mod, (CausalConv, GatedDelta, GatedMLP,
+            elif isinstance(mod, (BiasedMLP, CausalConv, GatedDelta, GatedMLP,
                                   GroupedAttention, LatentAttention,
                                   ParallelBlock, RoutedExperts,
                                   SelectiveScan, TokenInput)):

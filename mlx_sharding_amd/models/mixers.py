@@ -9,7 +9,7 @@ GEMM, head sizes padded to the kernels' tiles) once they are on their device.
 
 from __future__ import annotations
 
-from typing import Optional, Tuple, Union
+from typing import Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -459,18 +459,17 @@ class GatedDelta(nn.Module):
 
 
 class GatedMLP(nn.Module):
-    """W_down (act(W_gate h) * W_up h), or W_down of any other function of the
-    two (``act``), with or without biases."""
+    """W_down (act(W_gate h) * W_up h)."""
 
     ACTS = {"gelu_tanh": ops.geglu, "silu": ops.swiglu}
 
-    def __init__(self, width: int, ff: int, act: Union[str, ClampedGLU],
-                 dtype: torch.dtype = torch.bfloat16, bias: bool = False):
+    def __init__(self, width: int, ff: int, act: str,
+                 dtype: torch.dtype = torch.bfloat16):
         super().__init__()
-        self.act = self.ACTS[act] if isinstance(act, str) else act
-        self.gate = Linear(width, ff, bias=bias, dtype=dtype)
-        self.up = Linear(width, ff, bias=bias, dtype=dtype)
-        self.down = Linear(ff, width, bias=bias, dtype=dtype)
+        self.act = self.ACTS[act]
+        self.gate = Linear(width, ff, dtype=dtype)
+        self.up = Linear(width, ff, dtype=dtype)
+        self.down = Linear(ff, width, dtype=dtype)
         self.fused = None
 
     def prepare(self):
@@ -480,6 +479,46 @@ class GatedMLP(nn.Module):
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         g, u = self.fused(h) if self.fused is not None else (self.gate(h), self.up(h))
         return self.down(self.act(g, u))
+
+
+class BiasedMLP(nn.Module):
+    """W_down glu(W_gate h + b, W_up h + b) + b.  The products are plain ones;
+    the unit adds its biases itself, and the last one is left to what comes
+    next."""
+
+    def __init__(self, width: int, ff: int, glu: ClampedGLU,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.glu = glu
+        self.gate = Linear(width, ff, bias=True, dtype=dtype)
+        self.up = Linear(width, ff, bias=True, dtype=dtype)
+        self.down = Linear(ff, width, bias=True, dtype=dtype)
+        self.w_in = None
+
+    @torch.no_grad()
+    def prepare(self):
+        # both halves of a row begin at whole vectors
+        ff = self.gate.out_features
+        self.half = -(-ff // 8) * 8
+        w = self.gate.weight.data
+        self.w_in = w.new_zeros(2 * self.half, w.shape[1])
+        for at, m in ((0, self.gate), (self.half, self.up)):
+            part = self.w_in[at: at + ff]
+            part.copy_(m.weight.data)
+            m.weight.data = part
+
+    def rows(self, h: torch.Tensor):
+        """(output without the last bias, that bias)."""
+        if self.w_in is None:
+            self.prepare()
+        y, ff = ops.linear(h, self.w_in), self.gate.out_features
+        u = self.glu(y[:, :ff], y[:, self.half: self.half + ff],
+                     self.gate.bias, self.up.bias)
+        return ops.linear(u, self.down.weight), self.down.bias
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        y, bias = self.rows(h)
+        return y + bias
 
 
 class MLP(nn.Module):

@@ -8,7 +8,7 @@
 
 struct AddNormArgs {
   float* x;
-  const void *y, *w_post, *w_next;
+  const void *y, *y_bias, *w_post, *w_next;
   void* h;
   const int* where;
   long rows, ystride;
@@ -18,8 +18,9 @@ struct AddNormArgs {
 };
 
 extern "C" {
-void launch_clamped_glu(const void*, const void*, void*, long, int, long, long,
-                        float, float, bool, bool, hipStream_t);
+void launch_clamped_glu(const void*, const void*, const void*, const void*,
+                        void*, long, int, long, long, float, float, bool, bool,
+                        hipStream_t);
 void launch_glu_strided(const void*, const void*, void*, long, int, long, long,
                         bool, hipStream_t);
 void launch_glu_any(const void*, const void*, void*, long, int, long, long,
@@ -114,8 +115,10 @@ Tensor glu(Tensor gate, Tensor up, bool gelu) {
   return y;
 }
 
-// gate and up [rows, C], possibly slices of wider rows
-Tensor clamped_glu(Tensor gate, Tensor up, double limit, double alpha) {
+// gate and up [rows, C], possibly slices of wider rows; biases [C] or none
+Tensor clamped_glu(Tensor gate, Tensor up, double limit, double alpha,
+                   c10::optional<Tensor> gate_bias,
+                   c10::optional<Tensor> up_bias) {
   const bool f32 = is_f32(gate, "gate");
   check_like(up, gate, "up");
   const long gs = rows2(gate, "gate"), us = rows2(up, "up");
@@ -123,20 +126,28 @@ Tensor clamped_glu(Tensor gate, Tensor up, double limit, double alpha) {
   const long rows = gate.size(0), C = gate.size(1);
   auto out = torch::empty({rows, C}, gate.options());
   if (rows == 0 || C == 0) return out;
-  const bool vec = C % 8 == 0 && whole8(gate, gs) && whole8(up, us);
-  launch_clamped_glu(gate.data_ptr(), up.data_ptr(), out.data_ptr(), rows,
-                     (int)C, gs, us, (float)limit, (float)alpha, vec, f32,
+  bool vec = C % 8 == 0 && whole8(gate, gs) && whole8(up, us);
+  auto bias = [&](const c10::optional<Tensor>& b) {
+    if (!b) return (const void*)nullptr;
+    check_like(*b, gate, "bias");
+    TORCH_CHECK(b->numel() == C && b->is_contiguous());
+    vec = vec && whole8(*b, 8);
+    return (const void*)b->data_ptr();
+  };
+  const void *gb = bias(gate_bias), *ub = bias(up_bias);
+  launch_clamped_glu(gate.data_ptr(), up.data_ptr(), gb, ub, out.data_ptr(),
+                     rows, (int)C, gs, us, (float)limit, (float)alpha, vec, f32,
                      stream());
   return out;
 }
 
 // x [N, W] fp32 (updated in place when y is given, normed first when w_post
-// is; where [N, top]: sums of rows of y); returns h, `wide` columns of the next
+// is; where [N, top]: sums of rows of y; y_bias [W] added to y); returns h, `wide` columns of the next
 // norm's rows or of x itself, or an empty tensor for wide == 0.
 Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
                 c10::optional<Tensor> w_next, bool f32, double eps,
                 double off, double mult, c10::optional<Tensor> where,
-                int64_t wide) {
+                int64_t wide, c10::optional<Tensor> y_bias) {
   check_f32(x, "x");
   TORCH_CHECK(x.dim() == 2, "x must be [rows, width]");
   const auto type = x.options().dtype(f32 ? torch::kFloat32 : torch::kBFloat16);
@@ -160,6 +171,11 @@ Tensor add_norm(Tensor x, c10::optional<Tensor> y, c10::optional<Tensor> w_post,
       TORCH_CHECK(y->sizes() == x.sizes(), "y must match x");
     }
     a.y = y->data_ptr();
+    if (y_bias) {
+      check_like(*y_bias, h, "y_bias");
+      TORCH_CHECK(y_bias->numel() == a.W && y_bias->is_contiguous());
+      a.y_bias = y_bias->data_ptr();
+    }
     if (w_post) {
       check_like(*w_post, h, "w_post");
       TORCH_CHECK(w_post->numel() == a.W && w_post->is_contiguous());
@@ -800,8 +816,13 @@ Tensor cap_logits(Tensor z, double scale, double limit) {
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("glu", &glu);
-  m.def("clamped_glu", &clamped_glu);
-  m.def("add_norm", &add_norm);
+  m.def("clamped_glu", &clamped_glu, py::arg("gate"), py::arg("up"),
+        py::arg("limit"), py::arg("alpha"), py::arg("gate_bias") = py::none(),
+        py::arg("up_bias") = py::none());
+  m.def("add_norm", &add_norm, py::arg("x"), py::arg("y"), py::arg("w_post"),
+        py::arg("w_next"), py::arg("f32"), py::arg("eps"), py::arg("offset"),
+        py::arg("mult"), py::arg("where"), py::arg("wide"),
+        py::arg("y_bias") = py::none());
   m.def("latent_append", &latent_append);
   m.def("latent_gather", &latent_gather);
   m.def("latent_attn_short", &latent_attn_short);

@@ -516,13 +516,14 @@ extern "C" void launch_gelu(const void* x, void* o, long rows, int C, long xs,
 }
 
 // ---------------------------------------------------------------------------
-// Clamped gated unit on strided rows: g sigmoid(alpha g) (u + 1), g at most
-// limit, u within +-limit.
+// Clamped gated unit on strided rows (and biases, if there are any):
+// g sigmoid(alpha g) (u + 1), g at most limit, u within +-limit.
 // ---------------------------------------------------------------------------
 
 template <typename T, bool VEC>
 __global__ __launch_bounds__(GR_BLOCK) void clamped_glu_kernel(
-    const T* __restrict__ gate, const T* __restrict__ up, T* __restrict__ o,
+    const T* __restrict__ gate, const T* __restrict__ up,
+    const T* __restrict__ gate_b, const T* __restrict__ up_b, T* __restrict__ o,
     long rows, int C, long gs, long us, float limit, float alpha) {
   constexpr int V = VEC ? 8 : 1;
   const int per = C / V;  // whole vectors, or elements
@@ -531,27 +532,31 @@ __global__ __launch_bounds__(GR_BLOCK) void clamped_glu_kernel(
     const long r = i / per;
     const int c = (int)(i - r * per) * V;
     if constexpr (VEC) {
-      f32x8 g = load8(gate + r * gs + c);
-      const f32x8 u = load8(up + r * us + c);
+      f32x8 g = load8(gate + r * gs + c), u = load8(up + r * us + c);
+      if (gate_b) g = g + load8(gate_b + c);
+      if (up_b) u = u + load8(up_b + c);
 #pragma unroll
       for (int j = 0; j < 8; ++j) g[j] = clamped_glu_of<T>(g[j], u[j], limit, alpha);
       store8(o + r * C + c, g);
     } else {
-      o[r * C + c] = (T)clamped_glu_of<T>((float)gate[r * gs + c],
-                                       (float)up[r * us + c], limit, alpha);
+      const float g = (float)gate[r * gs + c] + (gate_b ? (float)gate_b[c] : 0.0f);
+      const float u = (float)up[r * us + c] + (up_b ? (float)up_b[c] : 0.0f);
+      o[r * C + c] = (T)clamped_glu_of<T>(g, u, limit, alpha);
     }
   }
 }
 
-extern "C" void launch_clamped_glu(const void* gate, const void* up, void* o,
-                                   long rows, int C, long gs, long us,
+extern "C" void launch_clamped_glu(const void* gate, const void* up,
+                                   const void* gate_b, const void* up_b,
+                                   void* o, long rows, int C, long gs, long us,
                                    float limit, float alpha, bool vec, bool f32,
                                    hipStream_t stream) {
   const long want = (rows * (vec ? C / 8 : C) + GR_BLOCK - 1) / GR_BLOCK;
   dim3 grid((unsigned)(want < 16384 ? want : 16384)), block(GR_BLOCK);
 #define GR_GO(T, VEC)                                                     \
   clamped_glu_kernel<T, VEC><<<grid, block, 0, stream>>>(                 \
-      (const T*)gate, (const T*)up, (T*)o, rows, C, gs, us, limit, alpha)
+      (const T*)gate, (const T*)up, (const T*)gate_b, (const T*)up_b, (T*)o, \
+      rows, C, gs, us, limit, alpha)
   if (f32) {
     if (vec) GR_GO(float, true);
     else GR_GO(float, false);

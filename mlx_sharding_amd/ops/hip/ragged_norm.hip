@@ -6,6 +6,7 @@
 
 // ---------------------------------------------------------------------------
 // One sublayer boundary in one kernel, one block per row:
+//   y += y_bias                           (y_bias == null: y as it is)
 //   x += mult * rms(y) * (w_post + off)   (y == null: x unchanged;
 //                                          w_post == null: x += mult * y)
 //   h  = rms(x) * (w_next + off)      (w_next == null: h = x; h == null: no h)
@@ -37,7 +38,7 @@ __device__ __forceinline__ void rn_store(T* p, const float (&o)[VEC]) {
 
 struct AddNormArgs {
   float* x;
-  const void *y, *w_post, *w_next;
+  const void *y, *y_bias, *w_post, *w_next;
   void* h;
   const int* where;
   long rows, ystride;
@@ -76,6 +77,12 @@ __global__ __launch_bounds__(RN_BLOCK) void add_norm_kernel(
       }
     } else {
       rn_load<T, VEC>(y + row * a.ystride + c, o);
+    }
+    if (a.y_bias) {
+      float b[VEC];
+      rn_load<T, VEC>((const T*)a.y_bias + c, b);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] += b[j];
     }
   };
 

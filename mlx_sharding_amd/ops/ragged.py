@@ -68,13 +68,14 @@ def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
 
 
 def add_norm(x, y, w_post, w_next, eps: float, offset: float,
-             dtype: torch.dtype, mult: float = 1.0, *, where=None,
+             dtype: torch.dtype, mult: float = 1.0, *, where=None, y_bias=None,
              copy: bool = False, pad_to: int = 1):
     """x += mult * rms(y) * (w_post + offset), in place, if y is given (without
     w_post: x += mult * y); returns rms(x) * (w_next + offset) in ``dtype``, or
     None without w_next.  x is the fp32 residual [N, W].
 
-    where [N, top]: row i of y is the sum of the rows y[where[i]].  copy: without
+    where [N, top]: row i of y is the sum of the rows y[where[i]].  y_bias [W] is
+    added to y's rows before all else.  copy: without
     w_next, returns x itself in ``dtype``.  What is returned is padded with
     zeros to a multiple of ``pad_to`` columns."""
     wide = _pad(x.shape[1], pad_to)
@@ -82,11 +83,13 @@ def add_norm(x, y, w_post, w_next, eps: float, offset: float,
         out = w_next is not None or copy
         h = _ext("add_norm").add_norm(x, y, w_post, w_next,
                                       dtype == torch.float32, eps, offset,
-                                      mult, where, wide if out else 0)
+                                      mult, where, wide if out else 0, y_bias)
         return h if out else None
     if y is not None:
         y = y.float() if where is None else y[where.long()].float().sum(1)
         y = y[:, : x.shape[1]]
+        if y_bias is not None:
+            y = y + y_bias.float()
         if w_post is not None:
             y = _rms(y, eps) * (w_post.float() + offset)
         x += mult * y
@@ -507,12 +510,18 @@ class ClampedGLU:
     limit: float
     alpha: float = 1.702
 
-    def __call__(self, gate, up):
-        """Rows [N, C], which may be columns of wider ones."""
+    def __call__(self, gate, up, gate_bias=None, up_bias=None):
+        """Rows [N, C], which may be columns of wider ones; biases [C] are
+        added first."""
         if gate.is_cuda:
             return _ext("clamped_glu").clamped_glu(gate, up, self.limit,
-                                                   self.alpha)
-        return self.of(gate.float(), up.float()).to(gate.dtype)
+                                                   self.alpha, gate_bias, up_bias)
+        g, u = gate.float(), up.float()
+        if gate_bias is not None:
+            g = g + gate_bias.float()
+        if up_bias is not None:
+            u = u + up_bias.float()
+        return self.of(g, u).to(gate.dtype)
 
     def of(self, gate, up):
         g, u = gate.clamp(max=self.limit), up.clamp(-self.limit, self.limit)

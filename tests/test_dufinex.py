@@ -9,7 +9,7 @@ import torch.nn.functional as F
 
 import dufinex_cases as cases
 import dufinex_oracle as oracle
-from mlx_sharding_amd.models.mixers import (GatedDelta, GatedMLP,
+from mlx_sharding_amd.models.mixers import (BiasedMLP, GatedDelta,
                                             GroupedAttention, RoutedExperts)
 from mlx_sharding_amd.ops import experts, ragged
 from mlx_sharding_amd.ops.experts import ExpertShape, Routing
@@ -73,9 +73,9 @@ def test_clamped_glu(device, dtype, C, limit):
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("ff", [64, 33, 1])
-def test_gated_mlp_with_biases(device, dtype, ff):
+def test_mlp_with_biases(device, dtype, ff):
     g = torch.Generator().manual_seed(2)
-    m = GatedMLP(48, ff, ClampedGLU(1.5), dtype, bias=True)
+    m = BiasedMLP(48, ff, ClampedGLU(1.5), dtype)
     for p in m.parameters():
         p.data = (torch.randn(p.shape, generator=g) * 0.2).to(dtype)
     w = {}
@@ -87,7 +87,17 @@ def test_gated_mlp_with_biases(device, dtype, ff):
     # rows of the residual's copy are wider than the model
     wide = F.pad(h, (0, 16)).to(device)[:, :48]
     want = oracle.dense(h.double(), w, "m.", 1.5)
-    assert cases.error(m(wide), want) < (2e-6 if dtype == F32 else 2e-2)
+    tol = 2e-6 if dtype == F32 else 2e-2
+    assert cases.error(m(wide), want) < tol
+    # the last bias goes with the residual update
+    x = torch.randn(7, 48, generator=g)
+    y, bias = m.rows(wide)
+    xd = x.clone().to(device)
+    ragged.add_norm(xd, y, None, None, 1e-5, 0.0, dtype, y_bias=bias)
+    assert cases.error(xd, x.double() + want) < tol
+    xd = x.clone().to(device)
+    ragged.add_norm(xd, y, bias, None, 1e-2, 0.0, dtype, y_bias=bias)
+    assert cases.error(xd, x.double() + oracle.rms(want, 1e-2) * w["m.down.b"]) < tol
 
 
 @pytest.mark.parametrize("device", DEVICES)
