@@ -464,7 +464,7 @@ DELTAS = {
     "one": cases.delta(1, 1, 1, 1, 1, (1, 1)),
     "shared keys": cases.delta(8, 1, 16, 32, 4, (4, 24)),
     "odd": cases.delta(3, 1, 33, 17, 2, (5, 3)),
-    "64/32": cases.delta(2, 1, 64, 32, 4),
+    "64/48": cases.delta(4, 2, 64, 48, 3),
     "128": cases.delta(2, 2, 128, 128, 4, (32, 32)),
     "100/50": cases.delta(2, 1, 100, 50, 5),
     "deep": cases.delta(2, 1, 200, 24, 8),
